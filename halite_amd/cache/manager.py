@@ -193,7 +193,9 @@ class CacheManager:
                 if slot not in live:
                     raise AssertionError(f"group {g.group_id}: table of dead slot {slot}")
                 done = g.released.get(slot, 0)
-                if any(p >= 0 for p in table[:done]) or any(p < 0 for p in table[done:]):
+                kept = min(g.kept_pages, done)
+                if (any(p >= 0 for p in table[kept:done]) or any(p < 0 for p in table[done:])
+                        or any(p < 0 for p in table[:kept])):
                     raise AssertionError(
                         f"group {g.group_id}: slot {slot} has a hole behind its first held page "
                         f"(released {done}, table {table})"

@@ -114,8 +114,16 @@ class CacheGroup:
             oldest_key = max(oldest_key, next_position - next_position % chunk)
         return max(0, oldest_key // self.page_size)
 
-    # A request's table has no holes behind its first held page: ``released[slot]``
-    # leading entries were given back (they are -1), every later entry holds a page.
+    @property
+    def kept_pages(self) -> int:
+        """Leading pages that a request keeps although a window or chunk has passed them."""
+        if self._span() is None:
+            return 0
+        return -(-getattr(self.need, "keep", 0) // self.page_size)
+
+    # A request's table has no holes behind its first held page: of its ``released[slot]``
+    # leading entries all but the first ``kept_pages`` were given back (they are -1), every
+    # later entry holds a page.
     def pages_missing(self, slot: int, start: int, new_len: int) -> int:
         """Pages to allocate so that the tokens ``[start, new_len)`` can be run:
         their own positions, and nothing that the window has passed."""
@@ -127,7 +135,8 @@ class CacheGroup:
         last = (new_len - 1) // self.page_size
         if first >= self.released.get(slot, 0):  # nothing that was given back is asked for again
             return range(max(first, len(table)), last + 1)
-        return [i for i in range(first, last + 1) if i >= len(table) or table[i] < 0]
+        kept = range(min(self.kept_pages, first))
+        return [i for i in (*kept, *range(first, last + 1)) if i >= len(table) or table[i] < 0]
 
     def reserve(self, slot: int, start: int, new_len: int) -> None:
         want = self._wanted(slot, start, new_len)
@@ -150,8 +159,9 @@ class CacheGroup:
         done = self.released.get(slot, 0)
         if first <= done:
             return 0
-        dead = [p for p in table[done:first] if p >= 0]
-        for i in range(done, first):
+        passed = range(max(done, self.kept_pages), first)
+        dead = [table[i] for i in passed if table[i] >= 0]
+        for i in passed:
             table[i] = -1
         self.released[slot] = first
         self.pool.free(dead)
@@ -182,14 +192,14 @@ class CacheGroup:
         span = self._span()
         if span is None:
             return n_tokens
-        return min(n_tokens, (-(-span // self.page_size) + 1) * self.page_size)
+        return min(n_tokens, (-(-span // self.page_size) + 1 + self.kept_pages) * self.page_size)
 
     def pages_per_token_span(self, n_tokens: int) -> int:
         """Upper bound of the pages a request of ``n_tokens`` holds at once."""
         span = self._span()
         if span is None:
             return -(-n_tokens // self.page_size)
-        return min(-(-n_tokens // self.page_size), -(-span // self.page_size) + 1)
+        return min(-(-n_tokens // self.page_size), -(-span // self.page_size) + 1 + self.kept_pages)
 
     def _span(self) -> int | None:
         """The most keys that a query reaches back over (a window, a chunk, the smaller of

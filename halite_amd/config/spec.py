@@ -58,11 +58,13 @@ class LayerRun(BaseModel):
 
     ``layer`` names an entry of ``ModelSpec.layers`` (the weights).  Every run
     has a cache of its own unless ``cache_from`` gives the index of an earlier
-    run: then the mixer appends nothing and reads that run's cache.
+    run: then the mixer appends nothing and reads that run's cache.  ``junction`` names an
+    entry of ``ModelSpec.junctions``, which makes the residual stream anew right before the run.
     """
 
     layer: str
     cache_from: StrictInt | None = None
+    junction: str | None = None
 
 
 class ModelSpec(BaseModel):
@@ -76,12 +78,15 @@ class ModelSpec(BaseModel):
     order: list[LayerRun]
     final_norm: PartSpec
     head: PartSpec
+    junctions: dict[str, PartSpec] = {}
 
     @model_validator(mode="after")
     def _check(self):
         for i, run in enumerate(self.order):
             if run.layer not in self.layers:
                 raise ValueError(f"order[{i}] names unknown layer {run.layer!r}")
+            if run.junction is not None and run.junction not in self.junctions:
+                raise ValueError(f"order[{i}] names unknown junction {run.junction!r}")
             if run.cache_from is not None:
                 if not 0 <= run.cache_from < i:
                     raise ValueError(

@@ -104,7 +104,10 @@ __device__ __forceinline__ void load_to_lds(const bf16_t* src, void* lds) {
 // tokens and number of keys in the last three of the eight instead, so that the wave need
 // not wait for the item before it can ask for them; then the first partial slot of its tile
 // and the number of pieces of the tile's key range, if the kernel is to merge them itself
-// (else 0, 0), and two unused.
+// (else 0, 0); then the first and the number of the kept first keys (multiples of 32) that this
+// wave walks before the keys of its range (0, 0: none).  An item of the kernel for long segments
+// says at 13 how many kept keys its workgroup walks in front (from key 0 on; a multiple of 64),
+// and at 14 up to which key they count for this item (0: not for this one).
 // A wave works on up to RT tiles of 16 rows of one segment; the keys and values it
 // loads serve all of them.  The tiles need not be neighbours (the host lists neighbours:
 // they share nearly all of their keys).  A tile skips the steps whose keys lie wholly
@@ -117,8 +120,9 @@ __device__ __forceinline__ void load_to_lds(const bf16_t* src, void* lds) {
 #define MIN_WAVES_PER_SIMD (D > 160 ? 1 : 2)
 // RULED: the scores follow a rule beyond scale, causal mask and window (`hal_score_rule`): a
 // bias by distance (the table comes multiplied by log2 e), a sink in the denominator; a
-// chunked mask needs no build of its own.
-template <int RT, bool POW2, bool PAGE32, bool SHARED, bool TILED, int KB, int HALVES, bool RULED>
+// chunked mask needs no build of its own.  KEPT: the first `rule.keep` keys stay visible under the
+// window, and the items say which of them a wave walks in front of its range.
+template <int RT, bool POW2, bool PAGE32, bool SHARED, bool TILED, int KB, int HALVES, bool RULED, bool KEPT>
 __global__ void __launch_bounds__(256 * HALVES, MIN_WAVES_PER_SIMD)
 attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __restrict__ out,
                       int out_row_stride, const int* __restrict__ items,
@@ -163,7 +167,7 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   // segment's scalars and the key range that the workgroup's four items walk together)
   constexpr bool INLINE_SEG = SHARED || RT == 1;
   constexpr int STRIDE_INTS = SHARED ? BIG_ITEM_INTS : SMALL_ITEM_INTS;
-  constexpr int PRE_INTS = SHARED ? 13 : 10;
+  constexpr int PRE_INTS = KEPT ? (SHARED ? 15 : 12) : (SHARED ? 13 : 10);
   int pre[PRE_INTS];
   if constexpr (INLINE_SEG) {
     const int* ip = items + (size_t)(item < max_items ? item : max_items - 1) * STRIDE_INTS;
@@ -192,6 +196,22 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
     walk_begin = uniform(pre[11]), walk_end = uniform(pre[12]);
     if (walk_begin >= walk_end) return;  // the same for all four waves
   }
+  // Kept first keys: the walk takes n_pre keys from pre0 on before those of its range; of these
+  // the item's own are the ones from kept_begin to kept_end.
+  int pre0 = 0, n_pre = 0;
+  // the item's own keys below `keep` (its kept ones, or those of its range): from kept_begin to kept_end
+  int kept_begin = 0, kept_end = 0;
+  if constexpr (KEPT) {
+    if constexpr (SHARED) {
+      n_pre = uniform(pre[13]);
+      kept_end = have_item ? uniform(pre[14]) : 0;
+    } else if (have_item) {
+      pre0 = uniform(pre[10]), n_pre = uniform(pre[11]);
+      kept_begin = pre0, kept_end = pre0 + n_pre;
+    }
+    if (kept_end == 0) kept_begin = kv_begin, kept_end = kv_end;
+    kept_end = min(kept_end, rule.keep);
+  }
   const int G = H / K;
   int q_start, q_len, kv_len;
   if constexpr (SHARED) {
@@ -209,6 +229,12 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   static_assert(KB == 32 || (SHARED && KB == 64), "keys per step");
   constexpr int SUBS = KB / 32;
   const int j_first = walk_begin & ~31;
+  // the keys of the walk in their order: x counts from the walk's start, in steps of 32
+  auto key_at = [&](int x) {
+    if constexpr (KEPT) return x < n_pre ? pre0 + x : j_first + (x - n_pre);
+    else return j_first + x;
+  };
+  const int walk_keys = n_pre + (walk_end > walk_begin ? walk_end - j_first : 0);
   // PAGE32: page numbers are looked up (scalar loads) well before the loads that need them
   auto page_at = [&](int j0) {
     // (an entry of a page that a window has passed is -1: never an address)
@@ -221,10 +247,10 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   if constexpr (SHARED) {
 #pragma unroll
     for (int u = 0; u < SUBS; ++u) {
-      const int j_mine = j_first + half_id * KB + 32 * u;
-      pages_0[u] = page_at(j_mine);
-      pages_1[u] = page_at(j_mine + KB * HALVES);
-      pages_2[u] = page_at(j_mine + 2 * KB * HALVES);
+      const int x_mine = half_id * KB + 32 * u;
+      pages_0[u] = page_at(key_at(x_mine));
+      pages_1[u] = page_at(key_at(x_mine + KB * HALVES));
+      pages_2[u] = page_at(key_at(x_mine + 2 * KB * HALVES));
     }
   }
 
@@ -232,6 +258,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   // this lane's query row in every row tile
   bool row_ok[RT];
   int qi[RT], head[RT], p_row[RT], lo_row[RT];
+  // (KEPT) the row sees the item's keys from see_from on, see_span more of them, and n_kept from kept_begin on
+  int see_from[RT], see_span[RT], n_kept[RT];
   bf16x8 bq[RT][KT];  // Q^T as the B operand: lane holds Q[row][ks*32 + quad*8 .. +8]
   f32x4 o[RT][DT];
   float m[RT], l[RT];
@@ -244,6 +272,12 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
     head[rt] = g * G + (row_ok[rt] ? rho % G : 0);
     p_row[rt] = pos0 + qi[rt];  // the row's position: it sees keys <= p_row
     lo_row[rt] = hal_rule_lo(rule, p_row[rt]);
+    if constexpr (KEPT) {
+      const int from = max(lo_row[rt], kv_begin), to = min(p_row[rt], kv_end - 1);
+      const bool some = row_ok[rt] && from <= to;
+      see_from[rt] = some ? from : 0x7fffffff, see_span[rt] = some ? to - from : 0;
+      n_kept[rt] = row_ok[rt] ? max(min(kept_end, p_row[rt] + 1) - kept_begin, 0) : 0;
+    }
     const bf16_t* qp = q + (size_t)(q_start + qi[rt]) * q_row_stride + (size_t)head[rt] * D;
 #pragma unroll
     for (int ks = 0; ks < KT; ++ks) {
@@ -298,14 +332,16 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   // [walk_begin, last_key] are clamped for the address only.
   const int koff0 = ((col / 4) * 8 + (col % 4)) * D + quad * 8;  // tile 1 is 4 keys on
   const int voff = col * page_size + quad * 8;
+  // (a block of kept keys: all of them are held)
+  auto kept_block = [&](int j0) { return KEPT && j0 >= pre0 && j0 < pre0 + n_pre; };
   auto key_index = [&](int j0, int t) {
     const int j = j0 + (col / 4) * 8 + t * 4 + (col % 4);
-    return j < walk_begin ? walk_begin : (j > last_key ? last_key : j);
+    return (j < walk_begin && !kept_block(j0)) ? walk_begin : (j > last_key ? last_key : j);
   };
   auto value_index = [&](int j0) {
     int jv = j0 + quad * 8;
     if constexpr (!PAGE32) {
-      if (jv < (walk_begin & ~7)) jv = walk_begin & ~7;
+      if (jv < (walk_begin & ~7) && !kept_block(j0)) jv = walk_begin & ~7;
       if (jv > (last_key & ~7)) jv = last_key & ~7;
     }
     return jv;
@@ -382,8 +418,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
       if (!active[rt]) continue;
       float sv[SUBS * 8];
       float m_raw = -INFINITY;
-      const bool full = j0 >= kv_begin && j0 + KB <= kv_end && j0 + KB - 1 <= p_first[rt] &&
-                        j0 >= lo_last[rt];
+      bool full = j0 >= kv_begin && j0 + KB <= kv_end && j0 + KB - 1 <= p_first[rt] && j0 >= lo_last[rt];
+      if constexpr (KEPT) full = full || (j0 >= kept_begin && j0 + KB <= kept_end && j0 + KB - 1 <= p_first[rt]);
       // (RULED: sv holds scaled scores, in units of log2, with the bias added)
       const bool far = RULED && p_first[rt] - (j0 + KB - 1) >= rule.bias_len - 1;  // (the same for the wave)
       // (a capped score: 2 s / cap in units of log2 going in, cap in units of log2 coming out)
@@ -428,8 +464,11 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
 #pragma unroll
         for (int e = 0; e < SUBS * 8; ++e) {
           const int j = j0 + (e / 8) * 32 + quad * 8 + e % 8;
-          const bool ok =
-              row_ok[rt] && j >= kv_begin && j < kv_end && j >= lo_row[rt] && j <= p_row[rt];
+          bool ok;
+          if constexpr (KEPT)
+            ok = (unsigned)(j - see_from[rt]) <= (unsigned)see_span[rt] || (unsigned)(j - kept_begin) < (unsigned)n_kept[rt];
+          else
+            ok = row_ok[rt] && j >= kv_begin && j < kv_end && j >= lo_row[rt] && j <= p_row[rt];
           sv[e] = ok ? ruled(s[rt][e / 8][(e % 8) / 4][e % 4], j) : -INFINITY;
           m_raw = fmaxf(m_raw, sv[e]);
         }
@@ -475,8 +514,10 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   // a step wholly after the tile's last row or before its first row's window does nothing
   // for this tile
   auto tile_active = [&](int j0, int rt) {
-    return j0 <= p_last[rt] && j0 + KB - 1 >= lo_first[rt] && j0 < kv_end && j0 + KB > kv_begin &&
-           j0 < walk_end;
+    const bool in_range = j0 <= p_last[rt] && j0 + KB - 1 >= lo_first[rt] && j0 < kv_end && j0 + KB > kv_begin &&
+                          j0 < walk_end;
+    if constexpr (KEPT) return in_range || (j0 <= p_last[rt] && j0 < walk_end && j0 < kept_end && j0 + KB > kept_begin);
+    else return in_range;
   };
 
   constexpr int FK = 2 * KT;                       // key fragments of a block of 32 keys
@@ -513,8 +554,8 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
     frag_t* const kbuf = (frag_t*)lds_raw + (size_t)half_id * 2 * (NFK + NFV);
     frag_t* const vbuf = kbuf + 2 * NFK;
     constexpr int STRIDE = KB * HALVES;
-    const int n_steps = (walk_end - j_first + STRIDE - 1) / STRIDE;
-    auto j_of = [&](int i) { return j_first + i * STRIDE + half_id * KB; };
+    const int n_steps = (walk_keys + STRIDE - 1) / STRIDE;
+    auto j_of = [&](int i) { return key_at(i * STRIDE + half_id * KB); };
     auto pages_of = [&](int j0, int (&pages)[SUBS]) {
 #pragma unroll
       for (int u = 0; u < SUBS; ++u) pages[u] = page_at(j0 + 32 * u);
@@ -670,24 +711,25 @@ attention_mfma_kernel(const bf16_t* __restrict__ q, int q_row_stride, bf16_t* __
   } else {
     // Without LDS: this block's values and the next block's keys (a second buffer) are asked
     // for at the block's start; deeper or shallower schedules measured the same or worse.
-    int page_0 = page_at(j_first), page_1 = page_at(j_first + 32), page_2 = page_at(j_first + 64);
+    int page_0 = page_at(key_at(0)), page_1 = page_at(key_at(32)), page_2 = page_at(key_at(64));
     bf16x8 kcur[2][KT], knext[2][KT], vf[DT];
 #pragma unroll
     for (int t = 0; t < 2; ++t)
 #pragma unroll
-      for (int ks = 0; ks < KT; ++ks) kcur[t][ks] = load_key_frag(j_first, page_0, t, ks);
+      for (int ks = 0; ks < KT; ++ks) kcur[t][ks] = load_key_frag(key_at(0), page_0, t, ks);
 
-    for (int j0 = j_first; j0 < walk_end; j0 += KB) {
+    for (int x = 0; x < walk_keys; x += KB) {
+      const int j0 = key_at(x);
       const bool tail = j0 + KB > kv_len;  // some of the keys are not written yet
-      const bool more = j0 + KB < walk_end;
-      const int page_3 = page_at(j0 + 96);
+      const bool more = x + KB < walk_keys;
+      const int page_3 = page_at(key_at(x + 96));
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) vf[dt] = load_value_frag(j0, page_0, dt);
       if (more) {
 #pragma unroll
         for (int t = 0; t < 2; ++t)
 #pragma unroll
-          for (int ks = 0; ks < KT; ++ks) knext[t][ks] = load_key_frag(j0 + 32, page_1, t, ks);
+          for (int ks = 0; ks < KT; ++ks) knext[t][ks] = load_key_frag(key_at(x + 32), page_1, t, ks);
       }
 
       // ---- S^T = K Q^T for 32 keys (two tiles of 16), all row tiles -------------------
@@ -1123,10 +1165,11 @@ extern "C" int hal_attention_mfma(const void* q, int q_row_stride, void* out, in
                                   max_big, merges, max_merges, counts, seg_q_start, seg_q_len,
                                   seg_kv_len, block_table, bt_stride, k_pages, v_pages, part_o, part_ml,
                                   counters, n_counters, H, K, head_dim, page_size, tiled, scale, window,
-                                  0, nullptr, 0, 0, 0.f, nullptr, merge_parts, stream);
+                                  0, nullptr, 0, 0, 0.f, nullptr, 0, merge_parts, stream);
 }
 
-// The same with a rule for the scores.  `chunk`: the work lists must have been cut for it (a
+// The same with a rule for the scores.  `keep` (with a window): the first keys that stay visible;
+// the work lists name them.  `chunk`: the work lists must have been cut for it (a
 // tile's first key is no earlier than the start of its first row's chunk).  `bias_log2`:
 // float32 [H][bias_len], the bias by distance times log2 e.
 extern "C" int hal_attention_mfma_ruled(const void* q, int q_row_stride, void* out, int out_row_stride,
@@ -1139,15 +1182,18 @@ extern "C" int hal_attention_mfma_ruled(const void* q, int q_row_stride, void* o
                                         int* counters, int n_counters, int H, int K, int head_dim,
                                         int page_size, int tiled, float scale, int window, int chunk,
                                         const float* bias_log2, int bias_len, int sink,
-                                        float softcap, const float* sink_log2,
+                                        float softcap, const float* sink_log2, int keep,
                                         int merge_parts, hipStream_t stream) {
+  HAL_REQUIRE(keep >= 0 && (keep == 0 || (window > 0 && chunk == 0)),
+              "hal_attention_mfma: %d kept keys belong to a window alone (window %d, chunk %d)", keep, window, chunk);
   HAL_REQUIRE(chunk >= 0 && (bias_log2 == nullptr || bias_len > 0),
               "hal_attention_mfma: chunk %d, bias table of %d distances", chunk, bias_len);
   HAL_REQUIRE(sink >= HAL_WEIGHTS_SOFTMAX && sink <= HAL_WEIGHTS_SIGMOID, "hal_attention_mfma: weights of kind %d", sink);
   HAL_REQUIRE(softcap >= 0.f && (sink_log2 == nullptr || sink == HAL_WEIGHTS_SINK),
               "hal_attention_mfma: a cap of %g, or sink values without a sink", (double)softcap);
-  const hal_score_rule rule = {window, chunk, bias_len, sink, bias_log2, softcap, sink_log2};
+  const hal_score_rule rule = {window, chunk, bias_len, sink, bias_log2, softcap, sink_log2, keep};
   const bool ruled = bias_log2 != nullptr || sink || softcap > 0.f;
+  HAL_REQUIRE(!ruled || keep == 0, "hal_attention_mfma: kept keys with a bias, a sink, sigmoid weights or a cap have no build");
   HAL_REQUIRE(head_dim == D, "hal_attention_mfma: built for head size %d, called with %d", D,
               head_dim);
   HAL_REQUIRE(H > 0 && K > 0 && H % K == 0, "hal_attention_mfma: %d heads, %d kv heads", H, K);
@@ -1168,18 +1214,20 @@ extern "C" int hal_attention_mfma_ruled(const void* q, int q_row_stride, void* o
   if ((page_size & (page_size - 1)) == 0)
     for (page_shift = 0; (1 << page_shift) < page_size; ++page_shift) {}
   const int waves = WAVES;
+#define PICK_ATTENTION(RT_, SHARED_, KB_, HV_, RU_, KE_)                                           \
+  {                                                                                               \
+    kernel = attention_mfma_kernel<RT_, false, false, SHARED_, false, KB_, HV_, RU_, KE_>;         \
+    if (tiled) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, D % 32 == 0, KB_, HV_, RU_, KE_>; \
+    else if (page_shift >= 5) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, false, KB_, HV_, RU_, KE_>; \
+    else if (page_shift >= 0) kernel = attention_mfma_kernel<RT_, true, false, SHARED_, false, KB_, HV_, RU_, KE_>; \
+  }
 #define LAUNCH_ATTENTION(RT_, SHARED_, KB_, HV_, LIST, MAX, COUNT)                                 \
   {                                                                                               \
     dim3 grid(((MAX) + waves - 1) / waves, K);                                                    \
-    auto kernel = attention_mfma_kernel<RT_, false, false, SHARED_, false, KB_, HV_, false>;      \
-    if (ruled) {                                                                                  \
-      kernel = attention_mfma_kernel<RT_, false, false, SHARED_, false, KB_, HV_, true>;          \
-      if (tiled) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, D % 32 == 0, KB_, HV_, true>; \
-      else if (page_shift >= 5) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, false, KB_, HV_, true>; \
-      else if (page_shift >= 0) kernel = attention_mfma_kernel<RT_, true, false, SHARED_, false, KB_, HV_, true>; \
-    } else if (tiled) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, D % 32 == 0, KB_, HV_, false>; \
-    else if (page_shift >= 5) kernel = attention_mfma_kernel<RT_, true, true, SHARED_, false, KB_, HV_, false>; \
-    else if (page_shift >= 0) kernel = attention_mfma_kernel<RT_, true, false, SHARED_, false, KB_, HV_, false>; \
+    auto kernel = attention_mfma_kernel<RT_, false, false, SHARED_, false, KB_, HV_, false, false>; \
+    if (ruled) PICK_ATTENTION(RT_, SHARED_, KB_, HV_, true, false)                                \
+    else if (keep > 0) PICK_ATTENTION(RT_, SHARED_, KB_, HV_, false, true)                        \
+    else PICK_ATTENTION(RT_, SHARED_, KB_, HV_, false, false)                                     \
     hipLaunchKernelGGL(kernel, grid, dim3(waves * HAL_WAVE * HV_), 0, stream, (const bf16_t*)q,   \
                        q_row_stride, (bf16_t*)out, out_row_stride, LIST, COUNT, seg_q_start,      \
                        seg_q_len, seg_kv_len, block_table, bt_stride, (const bf16_t*)k_pages,     \
@@ -1195,6 +1243,7 @@ extern "C" int hal_attention_mfma_ruled(const void* q, int q_row_stride, void* o
   if (max_items > 0) LAUNCH_ATTENTION(1, false, 32, 1, items, max_items, counts)
   if (max_big > 0) LAUNCH_ATTENTION(RT_BIG, true, KB_BIG, HALVES_BIG, big_items, max_big, counts + 1)
 #undef LAUNCH_ATTENTION
+#undef PICK_ATTENTION
   if (max_merges > 0) {
     if (merge_parts > 0 && merge_parts <= MERGE_FEW_PARTS)
       hipLaunchKernelGGL(attention_merge_few_kernel, dim3(max_merges, K, 4), dim3(256), 0, stream,

@@ -113,7 +113,7 @@ static inline size_t plain_lds_floats(int D, int keys, int rows) {
 // A block's keys and values on their way to LDS, for both kernels below.  Where a key lies
 // (its page's part for this key/value head, its slot) is looked up once per key, by the
 // block's first threads, two blocks ahead, and left in LDS.  Keys outside [lo_min, p_max] are
-// not read (their pages may not be held) and count as zero; a hole in the block table inside
+// not read, unless they are below `keep` (their pages may not be held) and count as zero; a hole in the block table inside
 // that range gives NaN keys, so that it shows.  Of the keys, thread `tid` brings vector kc of
 // the rows kr0, kr0 + rows_per_pass, ...; of the values, four keys of a dimension each time.
 // (the entry of the block table is asked for in one step of the walk and put down in the
@@ -127,15 +127,16 @@ struct plain_tiles {
   float* k_tile;      // [KEYS][KS]
   float* v_tile;      // [D][VS]
   int2* key_place;    // [2][KEYS]: (page * K + key/value head, slot); -1: a hole, -2: not read
-  int KS, VS, D, dv, page_size, page_shift, n_pages, K, g, lo_min, p_max, tid, kc, kr0, rows_per_pass;
+  int KS, VS, D, dv, page_size, page_shift, n_pages, K, g, lo_min, p_max, keep, tid, kc, kr0, rows_per_pass;
   int asked_page, asked_slot;
   float kreg[NV][4], vreg[NV][4];
 
+  // j0: the block's first key (its keys follow each other)
   __device__ __forceinline__ void ask_place(int j0) {
     asked_slot = -1;
     if (tid < KEYS) {
       const int j = j0 + tid;
-      if (j >= lo_min && j <= p_max) {
+      if ((j >= lo_min || j < keep) && j <= p_max) {
         const int pg = page_shift >= 0 ? j >> page_shift : j / page_size;
         asked_page = bt[pg];
         asked_slot = j - pg * page_size;
@@ -258,11 +259,14 @@ attention_plain_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict_
     const int* bt = block_table + (size_t)seg * bt_stride;
     const int n_rows = (tb - ta) * heads_here;
     // the keys this workgroup walks for the run
-    int j_begin = lo_min / KEYS * KEYS, j_end = p_max + 1;
+    // (j: places in the walk, which are the keys themselves where none are kept in front)
+    const hal_key_walk walk(rule, lo_min);
+    const int v_first = walk.first(lo_min), v_last = walk.last(p_max);
+    int j_begin = v_first / KEYS * KEYS, j_end = v_last + 1;
     // (pieces as workgroups: a token a workgroup, so the run's range is the range of its rows)
-    const int piece_shift = split ? plain_piece_shift(lo_min, p_max, max_pieces) : PLAIN_PIECE_SHIFT;
+    const int piece_shift = split ? plain_piece_shift(v_first, v_last, max_pieces) : PLAIN_PIECE_SHIFT;
     if (split) {
-      const int pc = (lo_min >> piece_shift) + (int)blockIdx.z;
+      const int pc = (v_first >> piece_shift) + (int)blockIdx.z;
       j_begin = max(j_begin, pc << piece_shift);
       j_end = min(j_end, (pc + 1) << piece_shift);
     }
@@ -301,36 +305,38 @@ attention_plain_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict_
     tiles.k_tile = k_tile, tiles.v_tile = v_tile, tiles.key_place = key_place;
     tiles.KS = KS, tiles.VS = VS, tiles.D = D, tiles.dv = dv, tiles.page_size = page_size, tiles.page_shift = page_shift;
     tiles.n_pages = n_pages, tiles.K = K, tiles.g = g, tiles.lo_min = lo_min, tiles.p_max = p_max, tiles.tid = tid;
+    tiles.keep = rule.keep;
     tiles.kc = tid & ((1 << cw_shift) - 1), tiles.kr0 = tid >> cw_shift, tiles.rows_per_pass = PLAIN_THREADS >> cw_shift;
     tiles.asked_page = 0, tiles.asked_slot = -1;
 
-    tiles.ask_place(j_begin);
+    tiles.ask_place(walk.key(j_begin));
     tiles.put_place(0);
-    tiles.ask_place(j_begin + KEYS);
+    tiles.ask_place(walk.key(j_begin + KEYS));
     tiles.put_place(1);
     __syncthreads();
     tiles.fetch(0);
-    tiles.ask_place(j_begin + 2 * KEYS);
+    tiles.ask_place(walk.key(j_begin + 2 * KEYS));
     int buf = 0;
     for (int j0 = j_begin; j0 < j_end; j0 += KEYS, buf ^= 1) {
       __syncthreads();  // every wave has read the block before
       tiles.commit();
       tiles.put_place(buf);  // of the block after the next
       if (j0 + KEYS < j_end) tiles.fetch(buf ^ 1);
-      tiles.ask_place(j0 + 3 * KEYS);
+      tiles.ask_place(walk.key(j0 + 3 * KEYS));
       __syncthreads();
+      const int key0 = walk.key(j0);  // the block's first key
       const bool piece_ends = ((j0 + KEYS) & ((1 << piece_shift) - 1)) == 0 || j0 + KEYS >= j_end;
 #pragma unroll
       for (int rr = 0; rr < RW; ++rr) {
         const int r = wave + PLAIN_WAVES * rr;
         const bool have_row = r < n_rows;  // (the same for the whole wave)
         const int p = row_p[rr], lo = row_lo[rr];
-        if (have_row && j0 <= p && j0 + KEYS > lo) {  // the block holds keys of this row
+        if (have_row && key0 <= p && (key0 + KEYS > lo || key0 < rule.keep)) {  // the block holds keys of this row
           // ---- scores: a lane is a key (blocks of 32: the two halves of the wave take a
           // half of the dimensions each, where that is a whole number of vectors) ----
           const int key_lane = lane % KEYS;
-          const int j = j0 + key_lane;
-          const bool valid = j >= lo && j <= p;
+          const int j = key0 + key_lane;
+          const bool valid = hal_rule_sees(rule, lo, j) && j <= p;
           float s = -INFINITY;
           {
             const bool halves = KEYS == 32 && D % 8 == 0;  // (the same for every lane)
@@ -391,8 +397,9 @@ attention_plain_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict_
           // Only pieces that hold keys of the row count (the others would join as nothing,
           // but where pieces are workgroups of their own nobody computes them).
           const int pc = j0 >> piece_shift;
-          const bool mine = pc >= (lo >> piece_shift) && pc <= (p >> piece_shift);
-          const bool only_piece = (lo >> piece_shift) == (p >> piece_shift);
+          const int pc_first = walk.first(lo) >> piece_shift, pc_last = walk.last(p) >> piece_shift;
+          const bool mine = pc >= pc_first && pc <= pc_last;
+          const bool only_piece = pc_first == pc_last;
           if (mine && split && !only_piece) {
             float* dst = part + (((size_t)(ta + r / heads_here) * H + h_first + r % heads_here) * max_pieces + blockIdx.z) * (D + 2);
 #pragma unroll
@@ -425,7 +432,7 @@ attention_plain_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict_
     for (int rr = 0; rr < RW; ++rr) {
       const int r = wave + PLAIN_WAVES * rr;
       const int p = row_p[rr], lo = row_lo[rr];
-      const bool only_piece = (lo >> piece_shift) == (p >> piece_shift);
+      const bool only_piece = (walk.first(lo) >> piece_shift) == (walk.last(p) >> piece_shift);
       if (r >= n_rows || (split && !(only_piece && blockIdx.z == 0))) continue;
       T* op = out + (size_t)(ta + r / heads_here) * out_row_stride + (size_t)(h_first + r % heads_here) * D;
       const float inv = hal_rule_inverse(rule, M[rr], L[rr], h_first + r % heads_here);
@@ -448,8 +455,10 @@ attention_plain_merge_kernel(T* __restrict__ out, int out_row_stride, const int*
   const int t = blockIdx.x, h = blockIdx.y, lane = threadIdx.x;
   const int p = positions[t];
   const int lo = hal_rule_lo(rule, p);
-  const int piece_shift = plain_piece_shift(lo, p, max_pieces);
-  const int first = lo >> piece_shift, last = p >> piece_shift;
+  const hal_key_walk walk(rule, lo);
+  const int v_first = walk.first(lo), v_last = walk.last(p);
+  const int piece_shift = plain_piece_shift(v_first, v_last, max_pieces);
+  const int first = v_first >> piece_shift, last = v_last >> piece_shift;
   if (first == last) return;  // written by the piece's own workgroup
   float M = -INFINITY, L = 0.f, A[R];
 #pragma unroll
@@ -559,7 +568,8 @@ attention_rows_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict__
     const int lo_min = hal_rule_lo(rule, p_first);
     const int* bt = block_table + (size_t)seg * bt_stride;
     const int n_rows = (tb - ta) * heads_here;
-    const int j_begin = lo_min / KEYS * KEYS, j_end = p_max + 1;
+    const hal_key_walk walk(rule, lo_min);  // (j: places in the walk)
+    const int j_begin = walk.first(lo_min) / KEYS * KEYS, j_end = walk.last(p_max) + 1;
 
     // this lane's row (both halves of the wave have the same 32 rows)
     const int r = wave * 32 + col;
@@ -596,25 +606,26 @@ attention_rows_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict__
     tiles.KS = KS, tiles.VS = VS, tiles.D = D, tiles.dv = D / 4, tiles.page_size = page_size, tiles.page_shift = page_shift;
     tiles.n_pages = n_pages, tiles.K = K, tiles.g = g, tiles.lo_min = lo_min, tiles.p_max = p_max, tiles.tid = tid;
     tiles.kc = tid & ((1 << cw_shift) - 1), tiles.kr0 = tid >> cw_shift, tiles.rows_per_pass = PLAIN_THREADS >> cw_shift;
-    tiles.asked_page = 0, tiles.asked_slot = -1;
+    tiles.asked_page = 0, tiles.asked_slot = -1, tiles.keep = rule.keep;
 
     __syncthreads();  // the walk before is done with the tiles and the places
-    tiles.ask_place(j_begin);
+    tiles.ask_place(walk.key(j_begin));
     tiles.put_place(0);
-    tiles.ask_place(j_begin + KEYS);
+    tiles.ask_place(walk.key(j_begin + KEYS));
     tiles.put_place(1);
     __syncthreads();
     tiles.fetch(0);
-    tiles.ask_place(j_begin + 2 * KEYS);
+    tiles.ask_place(walk.key(j_begin + 2 * KEYS));
     int buf = 0;
     for (int j0 = j_begin; j0 < j_end; j0 += KEYS, buf ^= 1) {
       __syncthreads();  // every wave has read the block before
       tiles.commit();
       tiles.put_place(buf);  // of the block after the next
       if (j0 + KEYS < j_end) tiles.fetch(buf ^ 1);
-      tiles.ask_place(j0 + 3 * KEYS);
+      tiles.ask_place(walk.key(j0 + 3 * KEYS));
       __syncthreads();
-      if (!wave_has_rows || j0 > wave_p || j0 + KEYS <= wave_lo) continue;  // (the same for the whole wave)
+      const int key0 = walk.key(j0);
+      if (!wave_has_rows || key0 > wave_p || (key0 + KEYS <= wave_lo && key0 >= rule.keep)) continue;  // (the same for the whole wave)
       // ---- S^T: lane = (key col, half) for the keys, (row col, half) for q ----
       plain_f32x16 st;
 #pragma unroll
@@ -635,8 +646,8 @@ attention_rows_kernel(const T* __restrict__ q, int q_row_stride, T* __restrict__
       bool valid[16];
 #pragma unroll
       for (int v = 0; v < 16; ++v) {
-        const int j = j0 + 8 * (v / 4) + 4 * half + v % 4;
-        valid[v] = j >= lo && j <= p;
+        const int j = key0 + 8 * (v / 4) + 4 * half + v % 4;
+        valid[v] = hal_rule_sees(rule, lo, j) && j <= p;
         st[v] = valid[v] ? hal_rule_cap(rule, st[v] * scale) + (rule.bias ? hal_rule_bias(rule, head, p - j) : 0.f) : -INFINITY;
         if (valid[v] && rule.sink == HAL_WEIGHTS_SIGMOID) st[v] = hal_log_sigmoid(st[v]);
         mx = fmaxf(mx, st[v]);
@@ -755,7 +766,7 @@ extern "C" int hal_attention_simple(const void* q, int q_row_stride, void* out,
                                     hipStream_t stream) {
   return hal_attention_simple_ruled(q, q_row_stride, out, out_row_stride, dtype, positions, token_seg,
                                     block_table, bt_stride, k_pages, v_pages, part, n_tokens, H, K, D,
-                                    page_size, n_pages, scale, window, 0, nullptr, 0, 0, 0.f, nullptr,
+                                    page_size, n_pages, scale, window, 0, nullptr, 0, 0, 0.f, nullptr, 0,
                                     max_kv_len, min_q_len, stream);
 }
 
@@ -766,14 +777,16 @@ extern "C" int hal_attention_simple_ruled(const void* q, int q_row_stride, void*
                                           int n_tokens, int H, int K, int D, int page_size, int n_pages,
                                           float scale, int window, int chunk, const float* bias,
                                           int bias_len, int sink, float softcap,
-                                          const float* sink_value, int max_kv_len, int min_q_len,
+                                          const float* sink_value, int keep, int max_kv_len, int min_q_len,
                                           hipStream_t stream) {
+  HAL_REQUIRE(keep >= 0 && (keep == 0 || (window > 0 && chunk == 0)),
+              "hal_attention_simple: %d kept keys belong to a window alone (window %d, chunk %d)", keep, window, chunk);
   HAL_REQUIRE(chunk >= 0 && (bias == nullptr || bias_len > 0),
               "hal_attention_simple: chunk %d, bias table of %d distances", chunk, bias_len);
   HAL_REQUIRE(sink >= HAL_WEIGHTS_SOFTMAX && sink <= HAL_WEIGHTS_SIGMOID, "hal_attention_simple: weights of kind %d", sink);
   HAL_REQUIRE(softcap >= 0.f && (sink_value == nullptr || sink == HAL_WEIGHTS_SINK),
               "hal_attention_simple: a cap of %g, or sink values without a sink", (double)softcap);
-  const hal_score_rule rule = {window, chunk, bias_len, sink, bias, softcap, sink_value};
+  const hal_score_rule rule = {window, chunk, bias_len, sink, bias, softcap, sink_value, keep};
   HAL_REQUIRE(n_tokens >= 0 && H > 0 && K > 0 && D > 0 && page_size > 0 && n_pages > 0,
               "hal_attention_simple: bad sizes T=%d H=%d K=%d D=%d page=%d pages=%d", n_tokens, H,
               K, D, page_size, n_pages);

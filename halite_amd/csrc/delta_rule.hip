@@ -450,9 +450,9 @@ extern "C" int hal_delta_rule(const float* r, int ldr, const float* k, int ldk, 
   return 0;
 }
 
-// ---- out = y / rms(y over each head) * w * sigmoid(z): a wave a (token, head) -------------
+// ---- out = y / rms(y over each head) * w * sigmoid(z) (or silu(z)): a wave a (token, head) -------------
 template <typename T>
-__global__ void head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ z, int ldz,
+__global__ void head_norm_gate_kernel(const float* __restrict__ y, const float* __restrict__ z, int ldz, bool silu,
                                       const void* __restrict__ w, int w_dtype, float eps, T* __restrict__ out,
                                       int n_tokens, int H, int D) {
   const int lane = threadIdx.x % HAL_WAVE;
@@ -466,7 +466,8 @@ __global__ void head_norm_gate_kernel(const float* __restrict__ y, const float* 
   const float rstd = 1.0f / sqrtf(wave_sum(ss) / (float)D + eps);
   for (int i = lane; i < D; i += HAL_WAVE) {
     const size_t c = (size_t)h * D + i;
-    const float g = z ? delta_sigmoid(z[t * ldz + c]) : 1.0f;
+    const float zv = z ? z[t * ldz + c] : 0.f;
+    const float g = z ? delta_sigmoid(zv) * (silu ? zv : 1.0f) : 1.0f;
     const float wt = w ? load_as_f32(w, w_dtype, c) : 1.0f;
     out[t * H * D + c] = from_f32<T>(yr[i] * rstd * wt * g);
   }
@@ -475,7 +476,7 @@ __global__ void head_norm_gate_kernel(const float* __restrict__ y, const float* 
 // The same for heads of many channels: a workgroup a (token, head).
 template <typename T>
 __global__ void __launch_bounds__(256)
-head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict__ z, int ldz,
+head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict__ z, int ldz, bool silu,
                            const void* __restrict__ w, int w_dtype, float eps, T* __restrict__ out, int H, int D) {
   __shared__ float scratch[16];
   const size_t t = blockIdx.x;
@@ -486,13 +487,14 @@ head_norm_gate_wide_kernel(const float* __restrict__ y, const float* __restrict_
   const float rstd = 1.0f / sqrtf(block_sum(ss, scratch) / (float)D + eps);
   for (int i = threadIdx.x; i < D; i += blockDim.x) {
     const size_t c = (size_t)h * D + i;
-    const float g = z ? delta_sigmoid(z[t * ldz + c]) : 1.0f;
+    const float zv = z ? z[t * ldz + c] : 0.f;
+    const float g = z ? delta_sigmoid(zv) * (silu ? zv : 1.0f) : 1.0f;
     const float wt = w ? load_as_f32(w, w_dtype, c) : 1.0f;
     out[t * H * D + c] = from_f32<T>(yr[i] * rstd * wt * g);
   }
 }
 
-extern "C" int hal_head_norm_gate(const float* y, const float* z, int ldz, const void* w, int w_dtype, float eps,
+extern "C" int hal_head_norm_gate(const float* y, const float* z, int ldz, int silu, const void* w, int w_dtype, float eps,
                                   void* out, int dtype, int n_tokens, int H, int D, hipStream_t stream) {
   HAL_REQUIRE(n_tokens >= 0 && H > 0 && D > 0 && (z == nullptr || ldz >= H * D),
               "hal_head_norm_gate: bad sizes T=%d heads=%d dim=%d", n_tokens, H, D);
@@ -501,10 +503,10 @@ extern "C" int hal_head_norm_gate(const float* y, const float* z, int ldz, const
   if (D >= 512 && H <= 65535) {
     const dim3 wide(n_tokens, H);
     if (dtype == HAL_F32)
-      hipLaunchKernelGGL(head_norm_gate_wide_kernel<float>, wide, dim3(256), 0, stream, y, z, ldz, w, w_dtype, eps,
+      hipLaunchKernelGGL(head_norm_gate_wide_kernel<float>, wide, dim3(256), 0, stream, y, z, ldz, silu != 0, w, w_dtype, eps,
                          (float*)out, H, D);
     else
-      hipLaunchKernelGGL(head_norm_gate_wide_kernel<bf16_t>, wide, dim3(256), 0, stream, y, z, ldz, w, w_dtype, eps,
+      hipLaunchKernelGGL(head_norm_gate_wide_kernel<bf16_t>, wide, dim3(256), 0, stream, y, z, ldz, silu != 0, w, w_dtype, eps,
                          (bf16_t*)out, H, D);
     HAL_LAUNCH_CHECK();
     return 0;
@@ -512,10 +514,10 @@ extern "C" int hal_head_norm_gate(const float* y, const float* z, int ldz, const
   const long long units = (long long)n_tokens * H;
   const dim3 grid((unsigned)((units + 3) / 4));
   if (dtype == HAL_F32)
-    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, stream, y, z, ldz, w, w_dtype, eps,
+    hipLaunchKernelGGL(head_norm_gate_kernel<float>, grid, dim3(256), 0, stream, y, z, ldz, silu != 0, w, w_dtype, eps,
                        (float*)out, n_tokens, H, D);
   else
-    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, stream, y, z, ldz, w, w_dtype, eps,
+    hipLaunchKernelGGL(head_norm_gate_kernel<bf16_t>, grid, dim3(256), 0, stream, y, z, ldz, silu != 0, w, w_dtype, eps,
                        (bf16_t*)out, n_tokens, H, D);
   HAL_LAUNCH_CHECK();
   return 0;

@@ -44,6 +44,78 @@ __global__ void embedding_vec_kernel(const int* __restrict__ ids, const TT* __re
   }
 }
 
+// The same with a row of a second table added, chosen by a hash of the token before and the token
+// (the first token of a request has the table's last row).
+template <typename TT>
+__global__ void pair_embedding_kernel(const int* __restrict__ ids, const TT* __restrict__ table,
+                                      const TT* __restrict__ pairs, float scale, int buckets, long long mul_prev,
+                                      long long mul_cur, const int* __restrict__ positions,
+                                      const int* __restrict__ token_seg, const int* __restrict__ seg_q_start,
+                                      const int* __restrict__ token_slot, int* __restrict__ last_id, bool single,
+                                      float* __restrict__ out, int d, int vocab) {
+  const int t = blockIdx.x;
+  const int id = ids[t];
+  float* o = out + (size_t)t * d;
+  const bool first = single || t == seg_q_start[token_seg[t]];
+  const int before = first ? last_id[token_slot[t]] : ids[t - 1];
+  if (single) {
+    __syncthreads();  // every thread has read the id before
+    if (threadIdx.x == 0) last_id[token_slot[t]] = id;
+  }
+  if (id < 0 || id >= vocab) {  // as above
+    for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = __uint_as_float(0x7fc00000u);
+    return;
+  }
+  long long at = buckets;
+  if (positions[t] != 0) {
+    at = ((long long)before * mul_prev + (long long)id * mul_cur) % buckets;
+    if (at < 0) at += buckets;
+  }
+  const TT* row = table + (size_t)id * d;
+  const TT* pair = pairs + (size_t)at * d;
+  for (int i = threadIdx.x; i < d; i += blockDim.x) o[i] = fmaf(to_f32(row[i]), scale, to_f32(pair[i]));
+}
+
+__global__ void carry_ids_kernel(const int* __restrict__ ids, int* __restrict__ last_id,
+                                 const int* __restrict__ seg_q_start, const int* __restrict__ seg_q_len,
+                                 const int* __restrict__ token_slot, int n_segs) {
+  const int s = blockIdx.x * blockDim.x + threadIdx.x;
+  if (s >= n_segs || seg_q_len[s] <= 0) return;
+  const int t = seg_q_start[s] + seg_q_len[s] - 1;
+  last_id[token_slot[t]] = ids[t];
+}
+
+extern "C" int hal_pair_embedding(const int* ids, const void* table, const void* pairs, int dtype, float scale,
+                                  int buckets, long long mul_prev, long long mul_cur, const int* positions,
+                                  const int* token_seg, const int* seg_q_start, const int* token_slot, int* last_id,
+                                  int single, float* out, int n_tokens, int d, int vocab, hipStream_t stream) {
+  HAL_REQUIRE(n_tokens >= 0 && d > 0 && vocab > 0 && buckets > 0, "hal_pair_embedding: bad sizes T=%d d=%d V=%d buckets=%d",
+              n_tokens, d, vocab, buckets);
+  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_pair_embedding: unknown table dtype %d", dtype);
+  if (n_tokens == 0) return 0;
+  const int threads = d >= 1024 ? 256 : (d >= 256 ? 128 : 64);
+  if (dtype == HAL_F32)
+    hipLaunchKernelGGL(pair_embedding_kernel<float>, dim3(n_tokens), dim3(threads), 0, stream, ids, (const float*)table,
+                       (const float*)pairs, scale, buckets, mul_prev, mul_cur, positions, token_seg, seg_q_start,
+                       token_slot, last_id, single != 0, out, d, vocab);
+  else
+    hipLaunchKernelGGL(pair_embedding_kernel<bf16_t>, dim3(n_tokens), dim3(threads), 0, stream, ids,
+                       (const bf16_t*)table, (const bf16_t*)pairs, scale, buckets, mul_prev, mul_cur, positions,
+                       token_seg, seg_q_start, token_slot, last_id, single != 0, out, d, vocab);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+extern "C" int hal_carry_ids(const int* ids, int* last_id, const int* seg_q_start, const int* seg_q_len,
+                             const int* token_slot, int n_segs, hipStream_t stream) {
+  HAL_REQUIRE(n_segs >= 0, "hal_carry_ids: %d segments", n_segs);
+  if (n_segs == 0) return 0;
+  hipLaunchKernelGGL(carry_ids_kernel, dim3((n_segs + 255) / 256), dim3(256), 0, stream, ids, last_id, seg_q_start,
+                     seg_q_len, token_slot, n_segs);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
 // Token ids that an earlier step left on the device: tokens[i] holds a row of `src` on
 // entry and that row's value on return.
 __global__ void take_tokens_kernel(const int* __restrict__ src, int n_src, int* __restrict__ tokens,
@@ -266,13 +338,13 @@ extern "C" int hal_residual_add(float* h, const void* delta, int dtype, long lon
 }
 
 // ---------------------------------------------------------------------------------
-// out[t, f] = up[t, f] * silu(gate[t, f]); gate and up are the two halves of one
-// row of `gu` ([T, 2F], gate first).  silu(x) = x * sigmoid(x) in float32.
+// out[t, f] = up[t, f] * act(gate[t, f]); gate and up are the two halves of one
+// row of `gu` ([T, 2F], gate first).  act in float32: silu(x) = x * sigmoid(x), or gelu's tanh form.
 // src/halite/transformers/feedforward.py:204-212
 // ---------------------------------------------------------------------------------
 template <typename T>
-__global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
-                                int F) {
+__global__ void gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
+                                int F, int act) {
   const size_t n = (size_t)n_tokens * F;
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   const size_t stride = (size_t)gridDim.x * blockDim.x;
@@ -280,8 +352,7 @@ __global__ void silu_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, i
     const size_t t = i / F, f = i % F;
     const float g = to_f32(gu[t * 2 * F + f]);
     const float u = to_f32(gu[t * 2 * F + F + f]);
-    const float s = g / (1.0f + expf(-g));
-    out[i] = from_f32<T>(u * s);
+    out[i] = from_f32<T>(u * hal_gate_act(act, g));
   }
 }
 
@@ -319,8 +390,8 @@ extern "C" int hal_scale_normed_rows(const void* x, int ldx, const float* ss, in
 
 // four elements per access; F is a multiple of 4
 template <typename T>
-__global__ void silu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
-                                    int F) {
+__global__ void gate_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
+                                    int F, int act) {
   const int f4 = F / 4;
   const size_t n = (size_t)n_tokens * f4;
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -331,26 +402,27 @@ __global__ void silu_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ ou
     load4(gu + t * 2 * F + f, g);
     load4(gu + t * 2 * F + F + f, u);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) y[e] = u[e] * (g[e] / (1.0f + expf(-g[e])));
+    for (int e = 0; e < 4; ++e) y[e] = u[e] * hal_gate_act(act, g[e]);
     store4(out + t * F + f, y);
   }
 }
 
-extern "C" int hal_silu_mul(const void* gu, void* out, int dtype, int n_tokens, int F,
+extern "C" int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act,
                             hipStream_t stream) {
-  HAL_REQUIRE(n_tokens >= 0 && F > 0, "hal_silu_mul: bad sizes T=%d F=%d", n_tokens, F);
+  HAL_REQUIRE(act == HAL_ACT_SILU || act == HAL_ACT_GELU_TANH, "hal_gate_mul: activation %d", act);
+  HAL_REQUIRE(n_tokens >= 0 && F > 0, "hal_gate_mul: bad sizes T=%d F=%d", n_tokens, F);
   if (n_tokens == 0) return 0;
-  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_silu_mul: unknown dtype %d", dtype);
+  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_gate_mul: unknown dtype %d", dtype);
   if (F % 4 == 0) {
     const size_t n4 = (size_t)n_tokens * (F / 4);
     const size_t want4 = (n4 + 255) / 256;
     const int blocks4 = (int)(want4 < 16384 ? want4 : 16384);
     if (dtype == HAL_F32)
-      hipLaunchKernelGGL(silu_mul_vec_kernel<float>, dim3(blocks4), dim3(256), 0, stream,
-                         (const float*)gu, (float*)out, n_tokens, F);
+      hipLaunchKernelGGL(gate_mul_vec_kernel<float>, dim3(blocks4), dim3(256), 0, stream,
+                         (const float*)gu, (float*)out, n_tokens, F, act);
     else
-      hipLaunchKernelGGL(silu_mul_vec_kernel<bf16_t>, dim3(blocks4), dim3(256), 0, stream,
-                         (const bf16_t*)gu, (bf16_t*)out, n_tokens, F);
+      hipLaunchKernelGGL(gate_mul_vec_kernel<bf16_t>, dim3(blocks4), dim3(256), 0, stream,
+                         (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, act);
     HAL_LAUNCH_CHECK();
     return 0;
   }
@@ -359,13 +431,13 @@ extern "C" int hal_silu_mul(const void* gu, void* out, int dtype, int n_tokens, 
   const size_t want = (n + threads - 1) / threads;
   const int blocks = (int)(want < 8192 ? want : 8192);
   if (dtype == HAL_F32)
-    hipLaunchKernelGGL(silu_mul_kernel<float>, dim3(blocks), dim3(threads), 0, stream,
-                       (const float*)gu, (float*)out, n_tokens, F);
+    hipLaunchKernelGGL(gate_mul_kernel<float>, dim3(blocks), dim3(threads), 0, stream,
+                       (const float*)gu, (float*)out, n_tokens, F, act);
   else if (dtype == HAL_BF16)
-    hipLaunchKernelGGL(silu_mul_kernel<bf16_t>, dim3(blocks), dim3(threads), 0, stream,
-                       (const bf16_t*)gu, (bf16_t*)out, n_tokens, F);
+    hipLaunchKernelGGL(gate_mul_kernel<bf16_t>, dim3(blocks), dim3(threads), 0, stream,
+                       (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, act);
   else
-    return hal_fail("hal_silu_mul: unknown dtype %d", dtype);
+    return hal_fail("hal_gate_mul: unknown dtype %d", dtype);
   HAL_LAUNCH_CHECK();
   return 0;
 }

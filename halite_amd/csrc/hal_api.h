@@ -26,7 +26,8 @@ int hal_rmsnorm(float* h, const void* delta, const int* rows, const void* w, int
 
 int hal_residual_add(float* h, const void* delta, int dtype, long long n, hipStream_t stream);
 
-int hal_silu_mul(const void* gu, void* out, int dtype, int n_tokens, int F, hipStream_t stream);
+// out = up * act(gate) of rows [gate | up]; act: 0 silu, 1 gelu's tanh form
+int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act, hipStream_t stream);
 
 // out [m, d] = bf16(x * rsqrt(sum_p ss[p][row] / d + eps)): the rows of an RMSNorm whose
 // scaling was left to the reader (x = bf16(w * bf16(h)), ss [n_parts, row_width] partial
@@ -58,23 +59,25 @@ int hal_attention_simple(const void* q, int q_row_stride, void* out, int out_row
 // [H][bias_len], added to the scaled score of the key n tokens back at
 // [head][min(n, bias_len - 1)]; `sink`: one more term of score 0 and no value in the softmax
 // (`sink_value`, or null: float32 [H], that term's score per head instead of 0); `softcap` > 0:
-// the scaled score s becomes softcap * tanh(s / softcap) before the bias.
+// the scaled score s becomes softcap * tanh(s / softcap) before the bias; `keep` > 0 (with a
+// window): a request's first `keep` keys stay visible to every later query.
 int hal_attention_simple_ruled(const void* q, int q_row_stride, void* out, int out_row_stride,
                                int dtype, const int* positions, const int* token_seg,
                                const int* block_table, int bt_stride, const void* k_pages,
                                const void* v_pages, float* part, int n_tokens, int H, int K, int D,
                                int page_size, int n_pages, float scale, int window, int chunk,
                                const float* bias, int bias_len, int sink, float softcap,
-                               const float* sink_value, int max_kv_len, int min_q_len,
+                               const float* sink_value, int keep, int max_kv_len, int min_q_len,
                                hipStream_t stream);
 
 int hal_gemm_f32(const float* A, int lda, const float* W, int ldw, float* C, int ldc, int M,
                  int N, int K, hipStream_t stream);
 
-// X [M <= 64, K] bf16, W [N, K] bf16, optional W2 [N, K] (gated: up * silu(gate), W the gate).
+// X [M <= 64, K] bf16, W [N, K] bf16, optional W2 [N, K] (gated: up * act(gate), W the gate's;
+// act as for hal_gate_mul).
 // out_mode: 0 bf16, 1 float32, 2 add into float32, 3 bf16 of the square of relu of the result.
 int hal_gemm_bf16_skinny(const void* X, int ldx, const void* W, const void* W2, int ldw, void* C,
-                         int ldc, int out_mode, int M, int N, int K, hipStream_t stream);
+                         int ldc, int out_mode, int act, int M, int N, int K, hipStream_t stream);
 
 // The packed q, k, v projection of M <= 32 tokens with the rotation of q and k (pairs
 // (j, j + D/2), whole head) and the append of k and v to the pages in its epilogue.  W:
@@ -277,8 +280,8 @@ int hal_delta_rule(const float* r, int ldr, const float* k, int ldk, const float
                    float unit_eps, float* pre, float* state, const int* seg_q_start,
                    const int* seg_q_len, const int* token_slot, float* o, int n_tokens, int n_segs,
                    int H, int D, hipStream_t stream);
-// out = y / rms(y over each head of D) * w * sigmoid(z)  (w, z: null for none)
-int hal_head_norm_gate(const float* y, const float* z, int ldz, const void* w, int w_dtype, float eps,
+// out = y / rms(y over each head of D) * w * sigmoid(z), or silu(z)  (w, z: null for none)
+int hal_head_norm_gate(const float* y, const float* z, int ldz, int silu, const void* w, int w_dtype, float eps,
                        void* out, int dtype, int n_tokens, int H, int D, hipStream_t stream);
 
 // ---- several copies of the residual stream, per-head norms, per-head gates (stream_ops.hip) --
@@ -286,11 +289,12 @@ int hal_head_norm_gate(const float* y, const float* z, int ldz, const void* w, i
 // x_t <- sum_s mix[s][t] x_s + m * out[t] * y for every copy t, from the old copies.  With
 // read: u = sum_s in[s] x_s (in null: ones) of the new copies, written to result as it is
 // (norm_w null, float32) or as u / sqrt(mean(u^2) + eps) * (offset + norm_w).  rows (or null;
-// only without y): the rows to take, results in that order.
+// only without y): the rows to take, results in that order, ld_result elements from one to the next.
 int hal_streams_step(float* x, long long copy_stride, int S, const float* y, const void* mix,
                      const void* outw, float m, const void* inw, int c_dtype, int read,
                      const void* norm_w, int norm_dtype, float offset, float eps, void* result,
-                     int result_dtype, const int* rows, int n_rows, int W, hipStream_t stream);
+                     int ld_result, int result_dtype, const int* rows, int n_rows, int W,
+                     hipStream_t stream);
 // Every head of float32 q [T, H * dq], k [T, K * dq], v [T, K * dv] divided by its own root
 // mean square, packed as hal_qk_norm_pack packs (and appended to the pages, if given).
 // w_q, w_k (or null): a weight [dq] for every normed head of q / k; norm_v 0: the values are not
@@ -308,9 +312,75 @@ int hal_silu_rows(const float* a, int lda, void* out, int dtype, int n_rows, int
 // out[t, j] = gelu_tanh(g[t, j]) * table[tokens[t]][col0 + j], j < dim (a token out of range: NaN)
 int hal_token_gate(const float* g, int ldg, const void* table, int t_dtype, int ld_table, int col0,
                    const int* tokens, int vocab, void* out, int dtype, int n_rows, int dim, hipStream_t stream);
-// y[t, h * n + j] = x[t, h * x_head + j] * sigmoid(g[t, h]), j < n
+// y[t, h * n + j] = x[t, h * x_head + j] * sigmoid(g[t, h]), j < n; with cos_t, sin_t [table_len, n / 2]
+// (or null) every head is first turned back by its token's position: (u, v) -> (u c + v s, v c - u s)
 int hal_head_gate_cols(const void* x, int ldx, int x_head, const float* g, int ldg, void* y, int n, int H,
-                       int dtype, int n_tokens, hipStream_t stream);
+                       const int* positions, const float* cos_t, const float* sin_t, int table_len,
+                       int interleaved, int dtype, int n_tokens, hipStream_t stream);
+// float32 q [T, H * dq], k [T, K * dq], v [T, K * dv] turned by the tokens' positions and packed
+// (and appended) as hal_head_norm_pack packs: the first rot entries of every head of q and k by the
+// table cos_t, sin_t [table_len, rot / 2], all dv entries of the heads of v by cos_v, sin_v
+// [table_len, dv / 2] (null: not).
+int hal_turn_pack(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                  const int* positions, const float* cos_t, const float* sin_t, int rot, const float* cos_v,
+                  const float* sin_v, int table_len, int interleaved, void* out, int row_stride, int dtype,
+                  int n_tokens, int H, int K, int dq, int dv, int D, const int* token_seg,
+                  const int* block_table, int bt_stride, void* k_pages, void* v_pages, int page_size,
+                  int n_pages, int tiled, hipStream_t stream);
+// y[r] (add: +)= s1 * a[r] / sqrt(mean(a[r]^2) + eps) * w1 (+ the same of b, w2, s2; null: not)
+int hal_normed_sum(float* y, const float* a, const void* w1, float s1, const float* b, const void* w2, float s2,
+                   int w_dtype, float eps, int n_rows, int d, int add, hipStream_t stream);
+// out[r, c] = T(h[r, c]), c < d, rows of out ld_out elements apart
+int hal_cast_cols(const float* h, void* out, int ld_out, int dtype, int n_rows, int d, hipStream_t stream);
+// x = cap * tanh(x / cap), in place
+int hal_soft_cap_f32(float* x, float cap, long long n, hipStream_t stream);
+
+// ---- embedding with a table of pairs; gated scan; time mixing (time_mix.hip) ----------------------
+// out[t] = table[ids[t]] * scale + pairs[row(t)], row(t) = (previous id * mul_prev + ids[t] * mul_cur)
+// mod buckets, or `buckets` (the table's last row) at position 0; the id before a segment's first
+// token is last_id[token_slot].  single: every segment is one token, and last_id moves on here.
+int hal_pair_embedding(const int* ids, const void* table, const void* pairs, int dtype, float scale, int buckets,
+                       long long mul_prev, long long mul_cur, const int* positions, const int* token_seg,
+                       const int* seg_q_start, const int* token_slot, int* last_id, int single, float* out,
+                       int n_tokens, int d, int vocab, hipStream_t stream);
+// last_id[slot] = the segment's last id
+int hal_carry_ids(const int* ids, int* last_id, const int* seg_q_start, const int* seg_q_len, const int* token_slot,
+                  int n_segs, hipStream_t stream);
+// The gated scan over rows a [T, lda] = [z | x | g] of float32 projections, C channels each:
+// z = sigmoid(. + z_bias), u = . + x_bias, c = u + 1/2 (u >= 0) or sigmoid(u),
+// S <- (1 - z) S + z c, out = S * silu(g).  state float32 [slots][C].  chunks, seg_chunks as for
+// hal_ssd_scan (or null) with room for n_chunks * C floats each in sums and decays.
+int hal_gated_scan(const float* a, int lda, const void* z_bias, const void* x_bias, int b_dtype, float* state,
+                   const int* seg_q_start, const int* seg_q_len, const int* token_slot, void* out, int dtype,
+                   int n_segs, int C, const int* chunks, const int* seg_chunks, int n_chunks, float* sums,
+                   float* decays, hipStream_t stream);
+// Token shift: for s of n_mixes, out_s[t] = x[t] + (x[t - 1] - x[t]) * mu[s]; the row before a segment's first
+// token is last[token_slot] (float32 [slots][W]).  out_s lies at out + s * mix_stride, rows
+// row_stride apart, for s < n_mixes - 1; the last one at out_last, rows W apart.  single: every
+// segment is one token, and `last` moves on here; else hal_carry_rows does it.
+int hal_token_shift(const void* x, int dtype, const void* mu, int mu_dtype, int n_mixes, float* last,
+                    const int* token_seg, const int* seg_q_start, const int* token_slot, int single, void* out,
+                    long long mix_stride, int row_stride, void* out_last, int n_tokens, int W, hipStream_t stream);
+int hal_carry_rows(const void* x, int dtype, float* last, const int* seg_q_start, const int* seg_q_len,
+                   const int* token_slot, int n_segs, int W, hipStream_t stream);
+// decay[t, c] = exp(-exp(w0[c] + sum_j w2[c, j] tanh(x1[t, j]))), rows of decay ldd apart
+int hal_wkv_decay(const float* x1, int ldx1, const void* w2, const void* w0, int w_dtype, int rank, float* decay,
+                  int ldd, int n_tokens, int n, hipStream_t stream);
+// Per head o_t = (S + diag(u) k v^T)^T r with the old state, then S <- diag(decay) S + k v^T.
+// r, k, v, decay float32, rows ld apart, heads of D; bonus u [H * D]; state float32 [slots][H][D][D]
+// (key channel, value channel); o float32 [T, H * D].  chunks as for hal_ssd_scan with room for
+// n_chunks * H * D * D floats in sums and n_chunks * H * D in decays.
+int hal_wkv_scan(const float* r, const float* k, const float* v, const float* decay, int ld, const void* bonus,
+                 int b_dtype, float* state, const int* seg_q_start, const int* seg_q_len, const int* token_slot,
+                 float* o, int n_segs, int H, int D, const int* chunks, const int* seg_chunks, int n_chunks,
+                 float* sums, float* decays, hipStream_t stream);
+// The same for a step in which every request brings one token, with the decay made from x1 and the
+// result normed, weighted and gated: out = o / rms(o over the head) * norm_w * silu(gate).
+// D is 16, 32, 64 or 128.
+int hal_wkv_step(const float* r, const float* k, const float* v, const float* gate, int ld, const float* x1,
+                 int ldx1, const void* w2, const void* w0, const void* bonus, const void* norm_w, int w_dtype,
+                 int rank, float eps, float* state, const int* token_slot, void* out, int dtype, int n_tokens,
+                 int H, int D, hipStream_t stream);
 
 // ---- the head-size-specific library (attention_mfma.hip) ---------------------------------
 int hal_attention_mfma_head_dim();
@@ -342,6 +412,6 @@ int hal_attention_mfma_ruled(const void* q, int q_row_stride, void* out, int out
                              int n_counters, int H, int K, int head_dim, int page_size, int tiled,
                              float scale, int window, int chunk, const float* bias_log2,
                              int bias_len, int sink, float softcap, const float* sink_log2,
-                             int merge_parts, hipStream_t stream);
+                             int keep, int merge_parts, hipStream_t stream);
 
 }  // extern "C"

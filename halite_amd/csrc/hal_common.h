@@ -103,6 +103,14 @@ __device__ __forceinline__ void load4_any(const void* p, int dtype, size_t i, fl
   else load4((const bf16_t*)p + i, v);
 }
 
+// ---- activations of a gated product: act(gate) * up -------------------------------------
+enum { HAL_ACT_SILU = 0, HAL_ACT_GELU_TANH = 1 };
+__device__ __forceinline__ float hal_gate_act(int act, float g) {
+  if (act == HAL_ACT_GELU_TANH)
+    return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+  return g / (1.0f + expf(-g));
+}
+
 // ---- reductions -----------------------------------------------------------------
 __device__ __forceinline__ float wave_sum(float v) {
 #pragma unroll
@@ -151,6 +159,8 @@ __host__ __device__ __forceinline__ size_t kv_value_offset(bool tiled, int page_
 // exp(m) where a softmax's is divided by its sum.  `softcap` > 0: the scaled score s becomes
 // softcap * tanh(s / softcap) before anything is added to it.  `sink_value` (or null, with
 // HAL_WEIGHTS_SINK): float32 [heads], the score of the sink's term of every head instead of 0.
+// `keep` (with a window): the first `keep` keys of a request stay visible to every later query;
+// a query at p then sees the keys below min(keep, p + 1) and lo(p) .. p.
 enum { HAL_WEIGHTS_SOFTMAX = 0, HAL_WEIGHTS_SINK = 1, HAL_WEIGHTS_SIGMOID = 2 };
 struct hal_score_rule {
   int window;
@@ -160,6 +170,7 @@ struct hal_score_rule {
   const float* bias;
   float softcap;
   const float* sink_value;
+  int keep;
 };
 __host__ __device__ __forceinline__ int hal_rule_lo(const hal_score_rule& r, int p) {
   int lo = 0;
@@ -167,6 +178,30 @@ __host__ __device__ __forceinline__ int hal_rule_lo(const hal_score_rule& r, int
   if (r.chunk > 0 && p - p % r.chunk > lo) lo = p - p % r.chunk;
   return lo;
 }
+// whether a key that is not behind the query is seen (lo: hal_rule_lo of the query)
+__device__ __forceinline__ bool hal_rule_sees(const hal_score_rule& r, int lo, int j) { return j >= lo || j < r.keep; }
+
+// The keys of a walk over a request's keys, one after the other: all from the first visible one
+// on, or, with kept first keys, the kept ones (in whole units of HAL_KEPT_UNIT) and then those
+// from the unit of the walk's first window on.  v: place in the walk; key(v): the key there.
+// Blocks of up to HAL_KEPT_UNIT places cut at multiples of their size are runs of keys.
+#define HAL_KEPT_UNIT 64
+__host__ __device__ __forceinline__ int hal_kept_units(int keep) {
+  return (keep + HAL_KEPT_UNIT - 1) / HAL_KEPT_UNIT * HAL_KEPT_UNIT;
+}
+struct hal_key_walk {
+  int kept, gap;
+  __device__ __forceinline__ hal_key_walk(const hal_score_rule& r, int lo) {
+    kept = r.keep > 0 ? hal_kept_units(r.keep) : 0;
+    const int from = lo / HAL_KEPT_UNIT * HAL_KEPT_UNIT;
+    gap = (r.keep > 0 && from > kept) ? from - kept : 0;
+  }
+  __device__ __forceinline__ int key(int v) const { return v < kept ? v : v + gap; }
+  // the places of a row's first and last visible key
+  __device__ __forceinline__ int first(int lo) const { return kept > 0 ? 0 : lo; }
+  __device__ __forceinline__ int last(int p) const { return p - gap; }
+};
+
 __device__ __forceinline__ float hal_rule_bias(const hal_score_rule& r, int head, int back) {
   return r.bias[(size_t)head * r.bias_len + (back < r.bias_len ? back : r.bias_len - 1)];
 }

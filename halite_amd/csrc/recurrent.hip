@@ -11,6 +11,9 @@
 //   S_t = exp(-exp(A_log) * dt_t) S_(t-1) + dt_t * B_t x_t^T,  y_t = S_t^T C_t + D x_t,
 //   dt_t = softplus(dt_raw_t + dt_bias)
 //
+// and a gated scan per channel whose gates read the token alone:
+//   S_t = (1 - z_t) S_(t-1) + z_t c_t,  z = sigmoid(.), c = u + 1/2 where u >= 0, else sigmoid(u)
+//
 // Decays, step sizes, the state and the sums over it are float32 whatever the activations'
 // type is.
 #include "hal_common.h"
@@ -370,6 +373,100 @@ extern "C" int hal_ssd_scan(const void* xbc, int ldx, int dtype, const float* dt
 #undef SCAN_BY_STATE
 #undef SCAN_STEPS
 #undef SCAN_LAUNCH
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- the gated scan: a thread a (run, channel).  a: rows [z | x | g] of C channels each, without
+// their biases; out = S * silu(g).  MODE 0: a run is a segment; MODE 1, the carry and MODE 2: the
+// segments cut into chunks, as for the recurrence above. -----------------------------------------
+template <typename T, int MODE>
+__global__ void __launch_bounds__(256)
+gated_scan_kernel(const float* __restrict__ a, int lda, const void* __restrict__ z_bias, const void* __restrict__ x_bias,
+                  int b_dtype, float* __restrict__ state, const int* __restrict__ seg_q_start,
+                  const int* __restrict__ seg_q_len, const int* __restrict__ token_slot, T* __restrict__ out, int C,
+                  const int* __restrict__ chunks, float* __restrict__ sums, float* __restrict__ decays) {
+  const int s = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (c >= C) return;
+  const int t0 = MODE == 0 ? seg_q_start[s] : chunks[s * 4], n = MODE == 0 ? seg_q_len[s] : chunks[s * 4 + 1];
+  if (n <= 0) return;
+  float* st = MODE == 0 ? state + (size_t)token_slot[t0] * C + c : sums + (size_t)s * C + c;
+  float S = MODE == 1 ? 0.f : *st, kept = 1.f;
+  const float zb = load_as_f32(z_bias, b_dtype, c), xb = load_as_f32(x_bias, b_dtype, c);
+  const float* row = a + (size_t)t0 * lda + c;
+  T* o = out + (size_t)t0 * C + c;
+  constexpr int AHEAD = 8;
+  for (int i0 = 0; i0 < n; i0 += AHEAD) {
+    float zr[AHEAD], xr[AHEAD], gr[AHEAD];
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i) {
+      const bool have = i0 + i < n;
+      const float* at = row + (size_t)(have ? i0 + i : 0) * lda;
+      zr[i] = at[0];
+      xr[i] = at[C];
+      gr[i] = MODE == 1 ? 0.f : at[2 * C];
+    }
+#pragma unroll
+    for (int i = 0; i < AHEAD; ++i) {
+      if (i0 + i >= n) break;
+      const float zz = zr[i] + zb, u = xr[i] + xb;
+      const float z = 1.0f / (1.0f + expf(-zz)), keep = 1.0f / (1.0f + expf(zz));
+      const float cand = u >= 0.f ? u + 0.5f : 1.0f / (1.0f + expf(-u));
+      S = fmaf(keep, S, z * cand);
+      if (MODE == 1) kept *= keep;
+      else o[(size_t)(i0 + i) * C] = from_f32<T>(S * silu_f32(gr[i]));
+    }
+  }
+  if (MODE != 2) *st = S;
+  if (MODE == 1) decays[(size_t)s * C + c] = kept;
+}
+
+__global__ void __launch_bounds__(256)
+gated_carry_kernel(float* __restrict__ state, float* __restrict__ sums, const float* __restrict__ decays,
+                   const int* __restrict__ seg_chunks, const int* __restrict__ seg_q_start,
+                   const int* __restrict__ seg_q_len, const int* __restrict__ token_slot, int C) {
+  const int s = blockIdx.x, c = blockIdx.y * blockDim.x + threadIdx.x;
+  if (seg_q_len[s] <= 0 || c >= C) return;
+  const int c0 = seg_chunks[s * 2], nc = seg_chunks[s * 2 + 1];
+  float* st = state + (size_t)token_slot[seg_q_start[s]] * C + c;
+  float S = *st;
+  constexpr int AHEAD = 8;
+  for (int k0 = 0; k0 < nc; k0 += AHEAD) {
+    float left[AHEAD], kept[AHEAD];
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const size_t at = (size_t)(c0 + (k0 + u < nc ? k0 + u : nc - 1)) * C + c;
+      left[u] = sums[at];
+      kept[u] = decays[at];
+    }
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      if (k0 + u >= nc) break;
+      sums[(size_t)(c0 + k0 + u) * C + c] = S;
+      S = fmaf(kept[u], S, left[u]);
+    }
+  }
+  *st = S;
+}
+
+extern "C" int hal_gated_scan(const float* a, int lda, const void* z_bias, const void* x_bias, int b_dtype, float* state,
+                              const int* seg_q_start, const int* seg_q_len, const int* token_slot, void* out, int dtype,
+                              int n_segs, int C, const int* chunks, const int* seg_chunks, int n_chunks, float* sums,
+                              float* decays, hipStream_t stream) {
+  HAL_REQUIRE(n_segs >= 0 && C > 0 && lda >= 3 * C, "hal_gated_scan: bad sizes segments=%d C=%d rows of %d", n_segs, C, lda);
+  HAL_REQUIRE((C + 255) / 256 <= 65535, "hal_gated_scan: %d channels exceed the grid limit", C);
+  HAL_REQUIRE((dtype == HAL_F32 || dtype == HAL_BF16) && (b_dtype == HAL_F32 || b_dtype == HAL_BF16),
+              "hal_gated_scan: dtypes %d, %d", dtype, b_dtype);
+  const bool cut = chunks != nullptr;
+  HAL_REQUIRE(!cut || (seg_chunks && sums && decays && n_chunks >= 0), "hal_gated_scan: chunks without their buffers");
+  if (n_segs == 0) return 0;
+  const int by = (C + 255) / 256;
+#define GATED_LAUNCH(T_, MODE_, RUNS_)                                                                                  hipLaunchKernelGGL((gated_scan_kernel<T_, MODE_>), dim3(RUNS_, by), dim3(256), 0, stream, a, lda, z_bias, x_bias,                          b_dtype, state, seg_q_start, seg_q_len, token_slot, (T_*)out, C, chunks, sums, decays)
+#define GATED_STEPS(T_)                                                                                                do {                                                                                                                   if (!cut) {                                                                                                            GATED_LAUNCH(T_, 0, n_segs);                                                                                       } else if (n_chunks > 0) {                                                                                             GATED_LAUNCH(T_, 1, n_chunks);                                                                                       hipLaunchKernelGGL(gated_carry_kernel, dim3(n_segs, by), dim3(256), 0, stream, state, sums, decays, seg_chunks,                          seg_q_start, seg_q_len, token_slot, C);                                                           GATED_LAUNCH(T_, 2, n_chunks);                                                                                     }                                                                                                                  } while (0)
+  if (dtype == HAL_F32) GATED_STEPS(float);
+  else GATED_STEPS(bf16_t);
+#undef GATED_STEPS
+#undef GATED_LAUNCH
   HAL_LAUNCH_CHECK();
   return 0;
 }

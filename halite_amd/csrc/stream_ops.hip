@@ -417,7 +417,7 @@ __global__ void streams_step_kernel(float* __restrict__ x, size_t copy_stride, i
                                     const void* __restrict__ mix, const void* __restrict__ outw, float m,
                                     const void* __restrict__ inw, int c_dtype, int read,
                                     const void* __restrict__ norm_w, int norm_dtype, float offset, float eps,
-                                    TO* __restrict__ result, const int* __restrict__ rows, int W) {
+                                    TO* __restrict__ result, int ld_result, const int* __restrict__ rows, int W) {
   extern __shared__ float u_row[];
   __shared__ float scratch[16];
   const size_t t = rows ? (size_t)rows[blockIdx.x] : (size_t)blockIdx.x;
@@ -458,7 +458,7 @@ __global__ void streams_step_kernel(float* __restrict__ x, size_t copy_stride, i
         u_row[i] = u;
         ss += u * u;
       } else {
-        result[(size_t)blockIdx.x * W + i] = from_f32<TO>(u);
+        result[(size_t)blockIdx.x * ld_result + i] = from_f32<TO>(u);
       }
     }
   }
@@ -466,13 +466,15 @@ __global__ void streams_step_kernel(float* __restrict__ x, size_t copy_stride, i
   const float total = block_sum(ss, scratch);
   const float rstd = 1.0f / sqrtf(total / (float)W + eps);
   for (int i = threadIdx.x; i < W; i += blockDim.x)  // (a thread reads back what it wrote itself)
-    result[(size_t)blockIdx.x * W + i] = from_f32<TO>(u_row[i] * rstd * (offset + load_as_f32(norm_w, norm_dtype, i)));
+    result[(size_t)blockIdx.x * ld_result + i] = from_f32<TO>(u_row[i] * rstd * (offset + load_as_f32(norm_w, norm_dtype, i)));
 }
 
 extern "C" int hal_streams_step(float* x, long long copy_stride, int S, const float* y, const void* mix,
                                 const void* outw, float m, const void* inw, int c_dtype, int read,
                                 const void* norm_w, int norm_dtype, float offset, float eps, void* result,
-                                int result_dtype, const int* rows, int n_rows, int W, hipStream_t stream) {
+                                int ld_result, int result_dtype, const int* rows, int n_rows, int W,
+                                hipStream_t stream) {
+  HAL_REQUIRE(!read || ld_result >= W, "hal_streams_step: rows of %d for a width of %d", ld_result, W);
   HAL_REQUIRE(S >= 1 && S <= 8, "hal_streams_step: %d copies of the stream (1 to 8)", S);
   HAL_REQUIRE(n_rows >= 0 && W > 0 && W <= 16384, "hal_streams_step: bad sizes rows=%d width=%d", n_rows, W);
   HAL_REQUIRE(y == nullptr || (mix && outw && rows == nullptr), "hal_streams_step: an update needs its weights and all rows");
@@ -483,7 +485,7 @@ extern "C" int hal_streams_step(float* x, long long copy_stride, int S, const fl
   const size_t lds = (read && norm_w) ? (size_t)W * sizeof(float) : 0;
 #define STREAMS_LAUNCH(T_, M_)                                                                                      \
   hipLaunchKernelGGL((streams_step_kernel<T_, M_>), dim3(n_rows), dim3(256), lds, stream, x, (size_t)copy_stride, S, y, \
-                     mix, outw, m, inw, c_dtype, read, norm_w, norm_dtype, offset, eps, (T_*)result, rows, W)
+                     mix, outw, m, inw, c_dtype, read, norm_w, norm_dtype, offset, eps, (T_*)result, ld_result, rows, W)
 #define STREAMS_BY_COUNT(T_)                \
   do {                                      \
     if (S <= 2) STREAMS_LAUNCH(T_, 2);      \
@@ -586,30 +588,276 @@ extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int l
 }
 
 // ---- y[t, h * n + j] = x[t, h * x_head + j] * sigmoid(g[t, h]) for j < n: every head's result
-// times one number of its own, the heads' padding dropped on the way -------------------------
+// times one number of its own, the heads' padding dropped on the way.  With a rotation table
+// (cos_t, sin_t [table_len, n / 2]) every head's n entries are turned back by the token's position
+// first: (u, v) of the pair (i, i + n / 2), or (2i, 2i + 1), becomes (u c + v s, v c - u s). ------
+__device__ __forceinline__ int pair_of(int j, int n, bool interleaved, int& partner, bool& second) {
+  if (interleaved) {
+    second = (j & 1) != 0;
+    partner = j ^ 1;
+    return j / 2;
+  }
+  const int half = n / 2;
+  second = j >= half;
+  partner = second ? j - half : j + half;
+  return second ? j - half : j;
+}
+
 template <typename T>
 __global__ void head_gate_cols_kernel(const T* __restrict__ x, int ldx, int x_head, const float* __restrict__ g, int ldg,
-                                      T* __restrict__ y, int n, int H) {
+                                      T* __restrict__ y, int n, int H, const int* __restrict__ positions,
+                                      const float* __restrict__ cos_t, const float* __restrict__ sin_t, int table_len,
+                                      bool interleaved) {
   const size_t t = blockIdx.x;
+  const int pos = cos_t ? positions[t] : 0;
+  const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
   for (int e = threadIdx.x; e < H * n; e += blockDim.x) {
     const int h = e / n, j = e % n;
     const float gate = 1.0f / (1.0f + expf(-g[t * ldg + h]));
-    y[t * H * n + e] = from_f32<T>(to_f32(x[t * ldx + (size_t)h * x_head + j]) * gate);
+    const T* xr = x + t * ldx + (size_t)h * x_head;
+    float f = to_f32(xr[j]);
+    if (cos_t) {
+      int partner;
+      bool second;
+      const int i = pair_of(j, n, interleaved, partner, second);
+      const float c = known ? cos_t[(size_t)pos * (n / 2) + i] : NAN, s = known ? sin_t[(size_t)pos * (n / 2) + i] : NAN;
+      const float o = to_f32(xr[partner]);
+      f = second ? f * c - o * s : f * c + o * s;
+    }
+    y[t * H * n + e] = from_f32<T>(f * gate);
   }
 }
 
+// ---- q, k and v of float32 projections with their heads turned by the tokens' positions, packed
+// as [H heads of D | K heads of D | K heads of D] with zeros beyond a head's entries, keys and
+// values appended to the pages as well (k_pages null: not).  q and k: the pairs of their first `rot`
+// entries, by the table cos_t, sin_t [table_len, rot / 2] (rot 0: as they are); v: all of its
+// dv entries by a table of its own, cos_v, sin_v [table_len, dv / 2] (null: as they are).  A
+// wave a (token, head). -----------------------------------------------------------------------
+template <typename T>
+__global__ void turn_pack_kernel(const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk,
+                                 const float* __restrict__ v, int ldv, const int* __restrict__ positions,
+                                 const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot,
+                                 const float* __restrict__ cos_v, const float* __restrict__ sin_v, int table_len,
+                                 bool interleaved, T* __restrict__ out, int row_stride, int n_tokens, int H, int K,
+                                 int dq, int dv, int D, const int* __restrict__ token_seg,
+                                 const int* __restrict__ block_table, int bt_stride, T* __restrict__ k_pages,
+                                 T* __restrict__ v_pages, int page_size, int n_pages, bool tiled) {
+  const int lane = threadIdx.x % HAL_WAVE, slots = H + 2 * K;
+  const size_t unit = (size_t)blockIdx.x * (blockDim.x / HAL_WAVE) + threadIdx.x / HAL_WAVE;
+  if (unit >= (size_t)n_tokens * slots) return;
+  const size_t t = unit / slots;
+  const int hs = (int)(unit % slots);
+  const int kind = hs < H ? 0 : (hs < H + K ? 1 : 2);
+  const int head = kind == 0 ? hs : (kind == 1 ? hs - H : hs - H - K);
+  const int n = kind == 2 ? dv : dq;
+  const float* src = kind == 0 ? q + t * ldq + (size_t)head * dq
+                               : (kind == 1 ? k + t * ldk + (size_t)head * dq : v + t * ldv + (size_t)head * dv);
+  const float* ct = kind == 2 ? cos_v : cos_t;
+  const float* st = kind == 2 ? sin_v : sin_t;
+  const int turned = ct == nullptr ? 0 : (kind == 2 ? dv : rot);
+  const int pos = positions[t];
+  const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
+  long long page = -1;
+  int off = 0;
+  if (k_pages && kind != 0) {
+    page = block_table[(size_t)token_seg[t] * bt_stride + pos / page_size];
+    off = pos % page_size;
+    if (page < 0 || page >= n_pages) page = -1;  // checked on the host
+  }
+  T* o = out + t * row_stride + (size_t)hs * D;
+  for (int d = lane; d < D; d += HAL_WAVE) {
+    float f = d < n ? src[d] : 0.f;
+    if (d < turned) {
+      int partner;
+      bool second;
+      const int i = pair_of(d, turned, interleaved, partner, second);
+      const float c = known ? ct[(size_t)pos * (turned / 2) + i] : NAN, s = known ? st[(size_t)pos * (turned / 2) + i] : NAN;
+      const float other = src[partner];
+      f = second ? f * c + other * s : f * c - other * s;
+    }
+    const T x = from_f32<T>(f);
+    o[d] = x;
+    if (page >= 0) {
+      if (kind == 1) k_pages[((size_t)page * K + head) * page_size * D + kv_key_offset(tiled, page_size, D, off, d)] = x;
+      else v_pages[((size_t)page * K + head) * D * page_size + kv_value_offset(tiled, page_size, D, off, d)] = x;
+    }
+  }
+}
+
+extern "C" int hal_turn_pack(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv,
+                             const int* positions, const float* cos_t, const float* sin_t, int rot, const float* cos_v,
+                             const float* sin_v, int table_len, int interleaved, void* out, int row_stride, int dtype,
+                             int n_tokens, int H, int K, int dq, int dv, int D, const int* token_seg,
+                             const int* block_table, int bt_stride, void* k_pages, void* v_pages, int page_size,
+                             int n_pages, int tiled, hipStream_t stream) {
+  HAL_REQUIRE(k_pages == nullptr || (v_pages && token_seg && block_table && page_size > 0 && n_pages > 0),
+              "hal_turn_pack: pages without the arrays that say where a token's key goes");
+  HAL_REQUIRE(n_tokens >= 0 && H > 0 && K > 0 && dq > 0 && dv > 0 && D >= dq && D >= dv,
+              "hal_turn_pack: bad sizes T=%d H=%d K=%d dq=%d dv=%d D=%d", n_tokens, H, K, dq, dv, D);
+  HAL_REQUIRE(row_stride >= (H + 2 * K) * D && ldq >= H * dq && ldk >= K * dq && ldv >= K * dv,
+              "hal_turn_pack: rows too short");
+  HAL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dq && (rot == 0 || (cos_t && sin_t)), "hal_turn_pack: %d turned entries of %d",
+              rot, dq);
+  HAL_REQUIRE((cos_v == nullptr) == (sin_v == nullptr) && (cos_v == nullptr || dv % 2 == 0),
+              "hal_turn_pack: values of %d entries are turned in pairs", dv);
+  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_turn_pack: dtype %d", dtype);
+  if (n_tokens == 0) return 0;
+  HAL_REQUIRE(positions && table_len > 0, "hal_turn_pack: no positions or tables");
+  const float* ct = rot > 0 ? cos_t : nullptr;
+  const long long units = (long long)n_tokens * (H + 2 * K);
+  const dim3 grid((unsigned)((units + 3) / 4));
+#define TURN_LAUNCH(T_)                                                                                              \
+  hipLaunchKernelGGL(turn_pack_kernel<T_>, grid, dim3(256), 0, stream, q, ldq, k, ldk, v, ldv, positions, ct, sin_t, rot, \
+                     cos_v, sin_v, table_len, interleaved != 0, (T_*)out, row_stride, n_tokens, H, K, dq, dv, D,      \
+                     token_seg, block_table, bt_stride, (T_*)k_pages, (T_*)v_pages, page_size, n_pages, tiled != 0)
+  if (dtype == HAL_F32) TURN_LAUNCH(float);
+  else TURN_LAUNCH(bf16_t);
+#undef TURN_LAUNCH
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
 extern "C" int hal_head_gate_cols(const void* x, int ldx, int x_head, const float* g, int ldg, void* y, int n, int H,
-                                  int dtype, int n_tokens, hipStream_t stream) {
+                                  const int* positions, const float* cos_t, const float* sin_t, int table_len,
+                                  int interleaved, int dtype, int n_tokens, hipStream_t stream) {
+  HAL_REQUIRE(cos_t == nullptr || (sin_t && positions && table_len > 0 && n % 2 == 0),
+              "hal_head_gate_cols: heads of %d entries are turned back in pairs, by a table and positions", n);
   HAL_REQUIRE(n_tokens >= 0 && H > 0 && n > 0 && x_head >= n && ldx >= H * x_head && ldg >= H,
               "hal_head_gate_cols: bad sizes T=%d heads=%d n=%d of %d", n_tokens, H, n, x_head);
   HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_head_gate_cols: dtype %d", dtype);
   if (n_tokens == 0) return 0;
   if (dtype == HAL_F32)
     hipLaunchKernelGGL(head_gate_cols_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, (const float*)x, ldx, x_head,
-                       g, ldg, (float*)y, n, H);
+                       g, ldg, (float*)y, n, H, positions, cos_t, sin_t, table_len, interleaved != 0);
   else
     hipLaunchKernelGGL(head_gate_cols_kernel<bf16_t>, dim3(n_tokens), dim3(256), 0, stream, (const bf16_t*)x, ldx, x_head,
-                       g, ldg, (bf16_t*)y, n, H);
+                       g, ldg, (bf16_t*)y, n, H, positions, cos_t, sin_t, table_len, interleaved != 0);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- y[r] (+)= s1 * norm(a[r]) * w1 (+ s2 * norm(b[r]) * w2), norm(x) = x / sqrt(mean(x^2) + eps):
+// the sum of results that are normed each on its own; float32 rows, a workgroup a row -------------
+template <int VMAX>
+__global__ void __launch_bounds__(256)
+normed_sum_vec_kernel(float* __restrict__ y, const float* __restrict__ a, const void* __restrict__ w1, float s1,
+                      const float* __restrict__ b, const void* __restrict__ w2, float s2, int w_dtype, float eps, int d,
+                      bool add) {
+  __shared__ float2 parts[4];
+  const size_t r = blockIdx.x;
+  const int nv = d / 4;
+  float x[VMAX][4], z[VMAX][4];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int u = 0; u < VMAX; ++u) {
+    const int v = threadIdx.x + u * blockDim.x;
+    if (v < nv) {
+      load4(a + r * d + v * 4, x[u]);
+      sa += (x[u][0] * x[u][0] + x[u][1] * x[u][1]) + (x[u][2] * x[u][2] + x[u][3] * x[u][3]);
+      if (b) {
+        load4(b + r * d + v * 4, z[u]);
+        sb += (z[u][0] * z[u][0] + z[u][1] * z[u][1]) + (z[u][2] * z[u][2] + z[u][3] * z[u][3]);
+      }
+    }
+  }
+  sa = wave_sum(sa), sb = wave_sum(sb);
+  if (threadIdx.x % HAL_WAVE == 0) parts[threadIdx.x / HAL_WAVE] = float2{sa, sb};
+  __syncthreads();
+  sa = sb = 0.f;
+  for (int w = 0; w < (int)blockDim.x / HAL_WAVE; ++w) sa += parts[w].x, sb += parts[w].y;
+  const float ra = s1 / sqrtf(sa / (float)d + eps), rb = s2 / sqrtf(sb / (float)d + eps);
+#pragma unroll
+  for (int u = 0; u < VMAX; ++u) {
+    const int v = threadIdx.x + u * blockDim.x;
+    if (v < nv) {
+      float wa[4], wb[4], out[4] = {0.f, 0.f, 0.f, 0.f};
+      load4_any(w1, w_dtype, (size_t)v * 4, wa);
+      if (add) load4(y + r * d + v * 4, out);
+      if (b) load4_any(w2, w_dtype, (size_t)v * 4, wb);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        out[i] += x[u][i] * ra * wa[i];
+        if (b) out[i] += z[u][i] * rb * wb[i];
+      }
+      store4(y + r * d + v * 4, out);
+    }
+  }
+}
+
+__global__ void __launch_bounds__(256)
+normed_sum_kernel(float* __restrict__ y, const float* __restrict__ a, const void* __restrict__ w1, float s1,
+                  const float* __restrict__ b, const void* __restrict__ w2, float s2, int w_dtype, float eps, int d,
+                  bool add) {
+  __shared__ float scratch[16];
+  const size_t r = blockIdx.x;
+  float sa = 0.f, sb = 0.f;
+  for (int i = threadIdx.x; i < d; i += blockDim.x) {
+    const float x = a[r * d + i], z = b ? b[r * d + i] : 0.f;
+    sa += x * x, sb += z * z;
+  }
+  const float ra = s1 / sqrtf(block_sum(sa, scratch) / (float)d + eps), rb = s2 / sqrtf(block_sum(sb, scratch) / (float)d + eps);
+  for (int i = threadIdx.x; i < d; i += blockDim.x) {
+    float out = add ? y[r * d + i] : 0.f;
+    out += a[r * d + i] * ra * load_as_f32(w1, w_dtype, i);
+    if (b) out += b[r * d + i] * rb * load_as_f32(w2, w_dtype, i);
+    y[r * d + i] = out;
+  }
+}
+
+extern "C" int hal_normed_sum(float* y, const float* a, const void* w1, float s1, const float* b, const void* w2, float s2,
+                              int w_dtype, float eps, int n_rows, int d, int add, hipStream_t stream) {
+  HAL_REQUIRE(n_rows >= 0 && d > 0, "hal_normed_sum: bad sizes rows=%d d=%d", n_rows, d);
+  HAL_REQUIRE((b == nullptr) == (w2 == nullptr) && (w_dtype == HAL_F32 || w_dtype == HAL_BF16),
+              "hal_normed_sum: every term has a weight, float32 or bf16");
+  if (n_rows == 0) return 0;
+  constexpr int VMAX = 8;
+  const bool aligned = d % 4 == 0 && ((uintptr_t)y % 16) == 0 && ((uintptr_t)a % 16) == 0 && ((uintptr_t)b % 16) == 0 &&
+                       ((uintptr_t)w1 % 16) == 0 && ((uintptr_t)w2 % 16) == 0;
+  if (aligned && d <= 4 * VMAX * 256) {
+    const int nv = d / 4, threads = nv >= 512 ? 256 : (nv >= 128 ? 128 : 64);
+    if (nv <= 2 * threads)
+      hipLaunchKernelGGL(normed_sum_vec_kernel<2>, dim3(n_rows), dim3(threads), 0, stream, y, a, w1, s1, b, w2, s2, w_dtype, eps, d, add != 0);
+    else if (nv <= 4 * threads)
+      hipLaunchKernelGGL(normed_sum_vec_kernel<4>, dim3(n_rows), dim3(threads), 0, stream, y, a, w1, s1, b, w2, s2, w_dtype, eps, d, add != 0);
+    else
+      hipLaunchKernelGGL(normed_sum_vec_kernel<VMAX>, dim3(n_rows), dim3(threads), 0, stream, y, a, w1, s1, b, w2, s2, w_dtype, eps, d, add != 0);
+  } else {
+    hipLaunchKernelGGL(normed_sum_kernel, dim3(n_rows), dim3(256), 0, stream, y, a, w1, s1, b, w2, s2, w_dtype, eps, d, add != 0);
+  }
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- float32 rows [n_rows, d] rounded into a column range of wider rows ---------------------------
+template <typename T>
+__global__ void cast_cols_kernel(const float* __restrict__ h, T* __restrict__ out, int ld_out, int d) {
+  const size_t r = blockIdx.x;
+  for (int i = threadIdx.x; i < d; i += blockDim.x) out[r * ld_out + i] = from_f32<T>(h[r * d + i]);
+}
+
+extern "C" int hal_cast_cols(const float* h, void* out, int ld_out, int dtype, int n_rows, int d, hipStream_t stream) {
+  HAL_REQUIRE(n_rows >= 0 && d > 0 && ld_out >= d, "hal_cast_cols: bad sizes rows=%d d=%d of %d", n_rows, d, ld_out);
+  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_cast_cols: dtype %d", dtype);
+  if (n_rows == 0) return 0;
+  if (dtype == HAL_F32)
+    hipLaunchKernelGGL(cast_cols_kernel<float>, dim3(n_rows), dim3(256), 0, stream, h, (float*)out, ld_out, d);
+  else
+    hipLaunchKernelGGL(cast_cols_kernel<bf16_t>, dim3(n_rows), dim3(256), 0, stream, h, (bf16_t*)out, ld_out, d);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- x = cap * tanh(x / cap), in place ---------------------------------------------------------
+__global__ void soft_cap_kernel(float* __restrict__ x, float cap, long long n) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i < n) x[i] = cap * tanhf(x[i] / cap);
+}
+
+extern "C" int hal_soft_cap_f32(float* x, float cap, long long n, hipStream_t stream) {
+  HAL_REQUIRE(n >= 0 && cap > 0.f, "hal_soft_cap_f32: %lld elements, cap %g", n, (double)cap);
+  if (n == 0) return 0;
+  hipLaunchKernelGGL(soft_cap_kernel, dim3((unsigned)((n + 255) / 256)), dim3(256), 0, stream, x, cap, n);
   HAL_LAUNCH_CHECK();
   return 0;
 }

@@ -185,15 +185,15 @@ class StepContext:
     # The plans of the attention kernel are part of the same upload, so they are
     # declared before the first device access.
     def plan_attention(self, group_id: int, n_heads: int, n_kv_heads: int, window: int,
-                       head_dim: int, late=False, chunk: int = 0) -> None:
-        key = (group_id, n_heads // n_kv_heads, window, chunk)
+                       head_dim: int, late=False, chunk: int = 0, keep: int = 0) -> None:
+        key = (group_id, n_heads // n_kv_heads, window, chunk, keep)
         if key in self._plan_host:
             return
         if self._dev is not None and not late:
             return
         plan = attention_kernels.plan_items(
             self.seg_q_len_host, self.seg_kv_len_host, n_heads // n_kv_heads, n_kv_heads, window,
-            attention_kernels.rows_per_big_item(head_dim), chunk,
+            attention_kernels.rows_per_big_item(head_dim), chunk, keep,
         )
         self._plan_host[key] = plan
         plan.name = f"plan{len(self._plan_host)}"
@@ -276,11 +276,11 @@ class StepContext:
 
     def attention(self, q, q_row_stride, kv, group: GroupStep, n_heads, scale, window, rule=None) -> torch.Tensor:
         """Attention of every token of the step over its request's cached keys; ``rule``
-        (``kernels.ops.ScoreRule``): a chunked mask, a bias by distance, a sink."""
+        (``kernels.ops.ScoreRule``): a chunked mask, kept first keys, a bias by distance, a sink."""
         return attention_kernels.paged_attention(self, q, q_row_stride, kv, group, n_heads, scale, window, rule)
 
-    def device_plan(self, group_id: int, group_size: int, window: int, chunk: int = 0):
-        key = (group_id, group_size, window, chunk)
+    def device_plan(self, group_id: int, group_size: int, window: int, chunk: int = 0, keep: int = 0):
+        key = (group_id, group_size, window, chunk, keep)
         plan = self._plan_host.get(key)
         if plan is None:
             return None

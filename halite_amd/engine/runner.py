@@ -19,7 +19,7 @@ import torch
 from ..cache import CacheManager, NoSpace
 from ..config.engine import ModelConfig, ServerConfig, check_stated_sizes
 from ..config.registry import read_config
-from ..parts.decoder import Decoder
+from ..parts.decoder import EMBEDDING_RUN, Decoder
 from ..weights import fill_random, load_weights
 from ..kernels import attention as attention_kernels
 from ..kernels import ops
@@ -71,6 +71,8 @@ class ModelRunner:
             st = mixer.state_need()
             if st:
                 state_needs[i] = st
+        if model.embedding.state_need():
+            state_needs[EMBEDDING_RUN] = model.embedding.state_need()
         sizes = [model.mixer_of_run(i).attention_sizes() for i in range(len(spec.order))]
         check_stated_sizes(self.model_config, len(spec.order), [s for s in sizes if s is not None])
         page_size = self.server_config.page_size
@@ -83,6 +85,7 @@ class ModelRunner:
         for run in model.runs:
             run.kv = self.cache.layer_pages(run.index)
             run.state = self.cache.state_of_run(run.index)
+        model.embedding_run.state = self.cache.state_of_run(EMBEDDING_RUN)
         self._staging = _Staging(self.device) if self.device.type == "cuda" else None
         self.max_total_tokens = self.cache.token_capacity
         # position tables for the whole context, so that their addresses never change
@@ -187,12 +190,10 @@ class ModelRunner:
         self._ahead = self._token_feed = self._staging = None
         for run in self.model.runs:
             run.kv, run.state = None, {}
+        self.model.embedding_run.state = {}
         self.cache.release_storage()
-        holders = list(self.model.named_parts().values()) + list(self.model.positions.values())
-        for part in holders:
-            for name, value in list(vars(part).items()):
-                if isinstance(value, torch.Tensor):
-                    setattr(part, name, None)
+        for part in list(self.model.named_parts().values()) + list(self.model.positions.values()):
+            part.drop_tensors()
         self.released, self.has_weights = True, False
         gc.collect()
         if self.device.type == "cuda":

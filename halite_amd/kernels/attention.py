@@ -37,6 +37,8 @@ MIN_PIECE_KEYS = 384
 # kernel behind it); more go to the merge kernel, which spreads a tile's partial results over
 # many workgroups (16 and 32 pieces measured 1 to 2 us faster so).
 MERGED_IN_KERNEL = 8
+# Kept first keys are walked in whole units of this many keys (``HAL_KEPT_UNIT`` of the kernels)
+KEPT_UNIT = 64
 N_COUNTERS = 1 << 14  # one per (tile that the kernel merges, key/value head); a tile has pieces only while these are few
 
 
@@ -71,12 +73,15 @@ class AttentionPlan:
     one piece of a tile's key range cut in four (some may be empty), which the workgroup
     joins itself, into the output or, where the range has several pieces, into the run's
     partial slot.  Places 8 and 9: the tile's first partial slot and number of pieces if the
-    kernel is to merge them itself (then the tile has no merge entry), else 0;
+    kernel is to merge them itself (then the tile has no merge entry), else 0.  Places 10 and
+    11: the first and the number of the kept first keys (multiples of 32) that the wave walks
+    before its range;
     ``big_items`` [n, 16] for longer segments: the first five the same, then the first rows
     of the item's further tiles (-1: none), ``rows_big`` rows per item; then the segment's
     first token, number of tokens and number of keys, and the first and end key of the walk
     of the item's run of four (a workgroup's waves), so that a workgroup knows all it needs
-    after one trip to memory;
+    after one trip to memory; place 13: how many kept keys the run walks in front (a multiple
+    of 64), place 14: up to which key they count for the item (0: not for this one);
     ``merges`` [n, 8]: segment, first row of a 16-row tile, first partial slot, number of
     partials, slots between partials, the segment's first token and number of tokens.
     A segment's first token is the sum of the lengths of the segments before it."""
@@ -150,10 +155,17 @@ def rows_per_big_item(head_dim: int) -> int:
     return int(library.attention_library(head_dim).hal_attention_mfma_rows_per_big_item())
 
 
-def _tiles(seg_q_len, seg_kv_len, group_size, window, rows_per_tile, pick, chunk=0):
+def kept_units(keep: int) -> int:
+    """``keep`` kept first keys in whole units."""
+    return -(-keep // KEPT_UNIT) * KEPT_UNIT
+
+
+def _tiles(seg_q_len, seg_kv_len, group_size, window, rows_per_tile, pick, chunk=0, keep=0):
     """The tiles of ``rows_per_tile`` rows of the segments whose row count ``pick``
     accepts: segment, first row, first and end key of each (arrays).  ``chunk``: a row sees
-    no key before the start of its own chunk of that many positions."""
+    no key before the start of its own chunk of that many positions.  ``keep``: the first
+    ``keep`` keys stay visible under a window; a tile whose range begins among them (in
+    whole units) takes all keys from 0 on, a later one walks them in front of its range."""
     ql = np.asarray(seg_q_len, dtype=np.int64)
     kl = np.asarray(seg_kv_len, dtype=np.int64)
     rows = ql * group_size
@@ -171,11 +183,13 @@ def _tiles(seg_q_len, seg_kv_len, group_size, window, rows_per_tile, pick, chunk
     b = np.zeros_like(r0) if window <= 0 else np.maximum(0, pos0 + first_q - window + 1)
     if chunk > 0:
         b = np.maximum(b, (pos0 + first_q) // chunk * chunk)
+    if keep > 0:
+        b = np.where(b <= kept_units(keep), 0, b)
     e = pos0 + last_q + 1
     return seg_ids, r0, b, e
 
 
-def _cut_long(seg_ids, rho0s, kv_b, kv_e, chunk, slots_per_tile, first_slot, seg_scalars, more_tiles):
+def _cut_long(seg_ids, rho0s, kv_b, kv_e, chunk, slots_per_tile, first_slot, seg_scalars, more_tiles, keep=0):
     """Items and merge entries of the long segments' items, whose key ranges are cut into
     pieces of ``chunk`` keys (pieces end on multiples of 32 keys).  ``more_tiles`` [n, k]
     holds the first rows of an item's further 16-row tiles (-1: none); ``seg_scalars``
@@ -204,19 +218,21 @@ def _cut_long(seg_ids, rho0s, kv_b, kv_e, chunk, slots_per_tile, first_slot, seg
     cut = np.nonzero(n_pieces > 1)[0]
     firsts = np.concatenate((rho0s[cut][:, None], more_tiles[cut]), axis=1)
     sub = np.broadcast_to(np.arange(firsts.shape[1]), firsts.shape)
-    keep = firsts >= 0
-    rows_of = np.broadcast_to(cut[:, None], firsts.shape)[keep]
-    merges = np.zeros((int(keep.sum()), 8), dtype=np.int32)
+    real = firsts >= 0
+    rows_of = np.broadcast_to(cut[:, None], firsts.shape)[real]
+    merges = np.zeros((int(real.sum()), 8), dtype=np.int32)
     merges[:, 0] = seg_ids[rows_of]
-    merges[:, 1] = firsts[keep]
-    merges[:, 2] = items[first_item[rows_of], 4] + sub[keep]
+    merges[:, 1] = firsts[real]
+    merges[:, 2] = items[first_item[rows_of], 4] + sub[real]
     merges[:, 3] = n_pieces[rows_of]
     merges[:, 4] = slots_per_tile
     merges[:, 5:7] = seg_scalars[merges[:, 0], :2]
-    return _group_items(items, piece, WAVES_PER_GROUP, seg_scalars), merges, first_slot + n_split * slots_per_tile
+    # the kept first keys go with the first piece of every range that does not begin at 0
+    kept = np.where((piece == 0) & (kv_b[tile_of] > 0), keep, 0)
+    return _group_items(items, piece, WAVES_PER_GROUP, seg_scalars, kept), merges, first_slot + n_split * slots_per_tile
 
 
-def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars):
+def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars, keep=0):
     """Items and merge entries of one-tile items whose key ranges are cut into at most
     ``most_pieces`` pieces, one per workgroup, and every piece into four, one per wave (in
     blocks of 32 keys, as evenly as they go; where a piece is short some of the four are
@@ -228,8 +244,10 @@ def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars
     if n == 0:
         return np.zeros((0, SMALL_ITEM_INTS), np.int32), np.zeros((0, 8), np.int32), first_slot
     base = kv_b - kv_b % KEYS_PER_BLOCK
-    blocks = -(-(kv_e - base) // KEYS_PER_BLOCK)
-    n_pieces = np.clip((kv_e - base) // MIN_PIECE_KEYS, 1, most_pieces)
+    # (kept first keys are walked in front of a range that does not begin at 0)
+    front = np.where(kv_b > 0, kept_units(keep) // KEYS_PER_BLOCK, 0)
+    blocks = front + -(-(kv_e - base) // KEYS_PER_BLOCK)
+    n_pieces = np.clip((front * KEYS_PER_BLOCK + kv_e - base) // MIN_PIECE_KEYS, 1, most_pieces)
     total = int(n_pieces.sum())
     tile_of = np.repeat(np.arange(n), n_pieces)
     first_item = np.concatenate(([0], np.cumsum(n_pieces)[:-1]))
@@ -237,7 +255,9 @@ def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars
     # wave w of all the range's waves takes the blocks from ceil(w * blocks / waves) on
     waves = (n_pieces * WAVES_PER_GROUP)[tile_of][:, None]
     w = piece[:, None] * WAVES_PER_GROUP + np.arange(WAVES_PER_GROUP + 1)[None, :]
-    edge = base[tile_of][:, None] + -(-(w * blocks[tile_of][:, None]) // waves) * KEYS_PER_BLOCK
+    edge = -(-(w * blocks[tile_of][:, None]) // waves)  # in blocks of the walk
+    in_front = np.minimum(edge, front[tile_of][:, None]) * KEYS_PER_BLOCK
+    edge = base[tile_of][:, None] + np.maximum(edge - front[tile_of][:, None], 0) * KEYS_PER_BLOCK
     b = np.maximum(kv_b[tile_of][:, None], edge[:, :-1])
     e = np.minimum(kv_e[tile_of][:, None], edge[:, 1:])
     empty = b >= e
@@ -250,6 +270,9 @@ def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars
     items[:, :, 2] = np.where(empty, b[:, :1], b)
     items[:, :, 3] = np.where(empty, b[:, :1], e)
     items[:, :, 5:8] = seg_scalars[seg_ids[tile_of]][:, None, :]
+    n_front = in_front[:, 1:] - in_front[:, :-1]
+    items[:, :, 10] = np.where(n_front > 0, in_front[:, :-1], 0)
+    items[:, :, 11] = n_front
     split = n_pieces[tile_of] > 1
     n_split = int(split.sum())
     slots = np.full(total, -1, dtype=np.int64)
@@ -267,15 +290,16 @@ def _cut_joined(seg_ids, rho0s, kv_b, kv_e, most_pieces, first_slot, seg_scalars
     merges[:, 3] = n_pieces[cut]
     merges[:, 4] = 1
     merges[:, 5:7] = seg_scalars[seg_ids[cut], :2]
-    keys = np.where(empty, 0, e).max(axis=1) - b[:, 0]  # a piece's first wave always has keys
+    keys = (np.where(empty, 0, e - b) + n_front).sum(axis=1)
     order = np.argsort(-keys, kind="stable")
     return items[order].reshape(total * WAVES_PER_GROUP, SMALL_ITEM_INTS), merges, first_slot + n_split
 
 
-def _group_items(items: np.ndarray, piece: np.ndarray, group: int, seg_scalars: np.ndarray) -> np.ndarray:
+def _group_items(items: np.ndarray, piece: np.ndarray, group: int, seg_scalars: np.ndarray,
+                 kept: np.ndarray) -> np.ndarray:
     """Orders items so that every run of ``group`` items (a workgroup's waves) belongs to
     one segment and to the same piece of neighbouring tiles, i.e. walks nearly the same
-    keys; a run that cannot be filled is padded with items that have no rows and no keys.
+    keys; ``kept``: per item, up to which of the kept first keys it takes (0: none); a run that cannot be filled is padded with items that have no rows and no keys.
     The runs with the longest walk come first."""
     n = len(items)
     if n == 0:
@@ -298,12 +322,21 @@ def _group_items(items: np.ndarray, piece: np.ndarray, group: int, seg_scalars: 
     live = runs[:, :, 3] > runs[:, :, 2]
     first_key = np.where(live, runs[:, :, 2], np.iinfo(np.int32).max).min(axis=1)
     end_key = np.where(live, runs[:, :, 3], 0).max(axis=1)
-    walk = np.where(live.any(axis=1), end_key - first_key, 0)
+    # kept first keys: walked in front of the run's range, or part of it where some item's begins at 0
+    kept_of = np.zeros(total, dtype=np.int64)
+    kept_of[dest] = kept[order]
+    kept_of = kept_of.reshape(total // group, group)
+    most_kept = kept_of.max(axis=1)
+    front = np.where((most_kept > 0) & (first_key > 0), kept_units(int(most_kept.max())), 0)
+    end_key = np.maximum(end_key, most_kept)
+    walk = np.where(live.any(axis=1), front + end_key - first_key, 0)
     wide = np.zeros((total // group, group, BIG_ITEM_INTS), dtype=np.int32)
     wide[:, :, :8] = runs
     wide[:, :, 8:11] = seg_scalars[runs[:, 0, 0]][:, None, :]
     wide[:, :, 11] = np.where(live.any(axis=1), first_key, 0)[:, None]
     wide[:, :, 12] = end_key[:, None]
+    wide[:, :, 13] = front[:, None]
+    wide[:, :, 14] = kept_of
     return wide[np.argsort(-walk, kind="stable")].reshape(total, BIG_ITEM_INTS)
 
 
@@ -331,11 +364,12 @@ def _group_tiles(seg_ids, rho0s, kv_b, kv_e, per_item: int):
 
 
 def plan_items(seg_q_len, seg_kv_len, group_size: int, n_kv_heads: int, window: int,
-               rows_big: int = 64, chunk: int = 0) -> AttentionPlan:
+               rows_big: int = 64, chunk: int = 0, keep: int = 0) -> AttentionPlan:
     """Cuts the step's query rows into tiles of 16 rows.  A segment of at most 16 rows or
     of one token (decode tokens) gives one-tile items, four to a workgroup, which takes a
     piece of the tile's key range; a longer segment gives items of ``rows_big / 16`` tiles
-    that share the keys a wave loads.  Where there are too few items to fill the GPU, a key range is cut
+    that share the keys a wave loads.  ``keep`` (with a window): the first keys of a request
+    that stay visible.  Where there are too few items to fill the GPU, a key range is cut
     into pieces whose partial results are merged."""
     ql = np.asarray(seg_q_len, dtype=np.int64).reshape(-1)
     seg_scalars = np.stack((np.cumsum(ql) - ql, ql, np.asarray(seg_kv_len, dtype=np.int64).reshape(-1)), axis=1)
@@ -343,9 +377,9 @@ def plan_items(seg_q_len, seg_kv_len, group_size: int, n_kv_heads: int, window: 
     # (a single token is never a long segment, however many heads share its keys: a decode
     # step then has one-tile items only, whose room is known before the lengths are)
     short = lambda r, q: (r <= ROWS_PER_ITEM) | (q == 1) | (per_item == 1)
-    small = _tiles(seg_q_len, seg_kv_len, group_size, window, ROWS_PER_ITEM, short, chunk)
-    big = _tiles(seg_q_len, seg_kv_len, group_size, window, ROWS_PER_ITEM, lambda r, q: ~short(r, q), chunk)
-    items, merges_s, slot = _cut_joined(*small, pieces_per_tile(len(small[0]), n_kv_heads), 0, seg_scalars)
+    small = _tiles(seg_q_len, seg_kv_len, group_size, window, ROWS_PER_ITEM, short, chunk, keep)
+    big = _tiles(seg_q_len, seg_kv_len, group_size, window, ROWS_PER_ITEM, lambda r, q: ~short(r, q), chunk, keep)
+    items, merges_s, slot = _cut_joined(*small, pieces_per_tile(len(small[0]), n_kv_heads), 0, seg_scalars, keep)
     more = None
     if len(big[0]):
         *big, more = _group_tiles(*big, per_item)
@@ -359,7 +393,7 @@ def plan_items(seg_q_len, seg_kv_len, group_size: int, n_kv_heads: int, window: 
         total = int((big[3] - big[2]).sum()) * n_kv_heads
         chunk = -(-total // target)
         chunk = max(MIN_SPLIT_KEYS, -(-chunk // KEYS_PER_BLOCK) * KEYS_PER_BLOCK)
-    big_items, merges_b, slot = _cut_long(*big, chunk, per_item, slot, seg_scalars, more)
+    big_items, merges_b, slot = _cut_long(*big, chunk, per_item, slot, seg_scalars, more, keep)
     merges = np.concatenate((merges_s, merges_b)) if len(merges_s) or len(merges_b) else np.zeros((0, 8), np.int32)
     return AttentionPlan(items, big_items, merges, slot, rows_big)
 
@@ -423,7 +457,7 @@ def attention_mfma(q, q_row_stride, plan_dev, ctx, group, kv, n_heads, scale, wi
         P(group.block_table), group.block_table.shape[1], P(kv.k), P(kv.v), P(part_o), P(part_ml),
         P(counters), N_COUNTERS, n_heads, n_kv, head_dim, page_size, 1 if getattr(kv, "tiled", False) else 0,
         ctypes.c_float(scale), window, rule.chunk, P(bias), 0 if bias is None else bias.shape[1],
-        rule.weights_code(), ctypes.c_float(rule.softcap), P(sinks), plan.max_parts, ops._stream(),
+        rule.weights_code(), ctypes.c_float(rule.softcap), P(sinks), rule.keep, plan.max_parts, ops._stream(),
     )
     ops._check(lib, rc)
     return out
@@ -437,12 +471,12 @@ def upload_plan(plan: AttentionPlan, device):
 
 def paged_attention(ctx, q, q_row_stride, kv, group, n_heads, scale, window, rule=None):
     n_pages, n_kv, page_size, head_dim = kv.k.shape
-    chunk = rule.chunk if rule is not None else 0
+    chunk, keep = (rule.chunk, rule.keep) if rule is not None else (0, 0)
     if mfma_supported(q.dtype, head_dim, page_size) and q_row_stride % 8 == 0:
-        plan_dev = ctx.device_plan(group.group_id, n_heads // n_kv, window, chunk)
+        plan_dev = ctx.device_plan(group.group_id, n_heads // n_kv, window, chunk, keep)
         if plan_dev is None:
-            ctx.plan_attention(group.group_id, n_heads, n_kv, window, head_dim, late=True, chunk=chunk)
-            plan_dev = ctx.device_plan(group.group_id, n_heads // n_kv, window, chunk)
+            ctx.plan_attention(group.group_id, n_heads, n_kv, window, head_dim, late=True, chunk=chunk, keep=keep)
+            plan_dev = ctx.device_plan(group.group_id, n_heads // n_kv, window, chunk, keep)
         return attention_mfma(q, q_row_stride, plan_dev, ctx, group, kv, n_heads, scale, window, rule)
     if getattr(kv, "tiled", False):
         raise ops.KernelError(

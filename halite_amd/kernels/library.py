@@ -48,6 +48,7 @@ CORE_SOURCES = [
     "stream_ops.hip",
     "recurrent.hip",
     "delta_rule.hip",
+    "time_mix.hip",
 ]
 ATTENTION_SOURCES = ["runtime.hip", "attention_mfma.hip"]
 

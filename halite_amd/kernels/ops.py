@@ -35,7 +35,8 @@ class ScoreRule:
     are not normalised over the keys.  ``softcap`` > 0: the scaled score ``s`` becomes
     ``softcap * tanh(s / softcap)`` before the bias.  ``sink_values`` (with ``sink``): float32
     ``[heads]`` on the device, the score of the sink's term of every head instead of 0 (it is
-    neither scaled nor capped)."""
+    neither scaled nor capped).  ``keep`` (with a window): the first ``keep`` keys of a request
+    stay visible to every later query."""
 
     chunk: int = 0
     bias: torch.Tensor | None = None
@@ -47,10 +48,11 @@ class ScoreRule:
     sink_values: torch.Tensor | None = None
     # the same values times log2 e
     sink_values_log2: torch.Tensor | None = None
+    keep: int = 0
 
     def plain(self) -> bool:
         return (self.chunk == 0 and self.bias is None and not self.sink and not self.sigmoid
-                and self.softcap == 0.0)
+                and self.softcap == 0.0 and self.keep == 0)
 
     def sink_checked(self, n_heads: int, log2: bool) -> torch.Tensor | None:
         """The sinks' values as a kernel takes them (None: every sink has the score 0)."""
@@ -169,6 +171,33 @@ def embedding(ids: torch.Tensor, table: torch.Tensor, out: torch.Tensor | None =
     return out
 
 
+def pair_embedding(ids: torch.Tensor, table: torch.Tensor, pairs: torch.Tensor, scale: float, mul_prev: int,
+                   mul_cur: int, ctx, last_id: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
+    """``embedding`` with a row of ``pairs`` ``[buckets + 1, d]`` added to every token's: row
+    ``(previous id * mul_prev + id * mul_cur) mod buckets``, the last row at position 0.  The
+    id before a segment's first token is ``last_id`` (int32 ``[slots, 1]``), which is left as
+    the step's last ids."""
+    lib = library.core_library()
+    _dev(ids, table, pairs, out, last_id, ctx.positions, ctx.token_seg, ctx.seg_q_start, ctx.token_slot)
+    _i32(ids, "ids"), _i32(last_id, "last_id")
+    n, (vocab, d) = ids.numel(), table.shape
+    _need(pairs.dim() == 2 and pairs.shape[1] == d and pairs.shape[0] > 1 and pairs.dtype == table.dtype,
+          "pair_embedding: a table [buckets + 1, d] of the embedding's type")
+    _need(ctx.positions.numel() == n and ctx.token_seg.numel() == n and ctx.token_slot.numel() == n, "pair_embedding: step arrays")
+    if out is None:
+        out = torch.empty((n, d), dtype=torch.float32, device=table.device)
+    _need(out.dtype == torch.float32 and out.shape == (n, d), "pair_embedding: bad output")
+    single = n == ctx.n_segs
+    _check(lib, lib.hal_pair_embedding(
+        _ptr(ids), _ptr(table), _ptr(pairs), dtype_code(table.dtype), ctypes.c_float(scale), pairs.shape[0] - 1,
+        ctypes.c_longlong(mul_prev), ctypes.c_longlong(mul_cur), _ptr(ctx.positions), _ptr(ctx.token_seg),
+        _ptr(ctx.seg_q_start), _ptr(ctx.token_slot), _ptr(last_id), 1 if single else 0, _ptr(out), n, d, vocab, _stream()))
+    if not single:
+        _check(lib, lib.hal_carry_ids(_ptr(ids), _ptr(last_id), _ptr(ctx.seg_q_start), _ptr(ctx.seg_q_len),
+                                      _ptr(ctx.token_slot), ctx.n_segs, _stream()))
+    return out
+
+
 def take_tokens(src: torch.Tensor, tokens: torch.Tensor) -> None:
     """``tokens[i] = src[tokens[i]]`` in place: token ids that an earlier step left on the
     device go into a step's array without a round over the host."""
@@ -224,18 +253,27 @@ def residual_add(h: torch.Tensor, delta: torch.Tensor):
     return h
 
 
-def silu_mul(gate_up: torch.Tensor):
-    """``up * silu(gate)`` of rows ``[gate | up]``."""
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}  # the kernels' numbers for what a gate goes through
+
+
+def gate_mul(gate_up: torch.Tensor, activation: str = "silu"):
+    """``up * act(gate)`` of rows ``[gate | up]``."""
     lib = library.core_library()
     _dev(gate_up)
     n, two_f = gate_up.shape
-    _need(two_f % 2 == 0, "silu_mul: odd row length")
+    _need(two_f % 2 == 0, "gate_mul: odd row length")
     out = torch.empty((n, two_f // 2), dtype=gate_up.dtype, device=gate_up.device)
     _check(
         lib,
-        lib.hal_silu_mul(_ptr(gate_up), _ptr(out), dtype_code(gate_up.dtype), n, two_f // 2, _stream()),
+        lib.hal_gate_mul(_ptr(gate_up), _ptr(out), dtype_code(gate_up.dtype), n, two_f // 2,
+                         GATE_ACTIVATIONS[activation], _stream()),
     )
     return out
+
+
+def silu_mul(gate_up: torch.Tensor):
+    """``up * silu(gate)`` of rows ``[gate | up]``."""
+    return gate_mul(gate_up)
 
 
 def rope_append(
@@ -412,7 +450,7 @@ def attention_simple(
             _ptr(positions), _ptr(token_seg), _ptr(block_table), block_table.shape[1],
             _ptr(k_pages), _ptr(v_pages), _ptr(part), n, n_heads, n_kv, head_dim, page_size, n_pages,
             ctypes.c_float(scale), window, rule.chunk, _ptr(bias), 0 if bias is None else bias.shape[1],
-            rule.weights_code(), ctypes.c_float(rule.softcap), _ptr(sinks), max_kv_len, min_q_len, _stream(),
+            rule.weights_code(), ctypes.c_float(rule.softcap), _ptr(sinks), rule.keep, max_kv_len, min_q_len, _stream(),
         ),
     )
     return out
@@ -541,9 +579,10 @@ def gemm_bf16_skinny(
     add_to: torch.Tensor | None = None,
     tiled_shape: tuple[int, int] | None = None,
     relu_squared: bool = False,
+    activation: str = "silu",
 ):
     """``x @ w.T`` for at most 64 rows of bf16 ``x``; with ``w_up`` the gated form
-    ``(x @ w_up.T) * silu(x @ w.T)``; ``add_to`` (float32) receives ``+=``;
+    ``(x @ w_up.T) * act(x @ w.T)`` (``activation``: a name of ``GATE_ACTIVATIONS``); ``add_to`` (float32) receives ``+=``;
     ``relu_squared``: the bf16 result is the square of relu of the product."""
     lib = library.core_library()
     _dev(x, add_to)
@@ -578,7 +617,7 @@ def gemm_bf16_skinny(
     _check(
         lib,
         lib.hal_gemm_bf16_skinny(
-            _ptr(x), k, _ptr(w), _ptr(w_up), ldw, _ptr(out), n, mode, m, n, k, _stream()
+            _ptr(x), k, _ptr(w), _ptr(w_up), ldw, _ptr(out), n, mode, GATE_ACTIVATIONS[activation], m, n, k, _stream()
         ),
     )
     return out
@@ -781,6 +820,15 @@ def scale_(x: torch.Tensor, s: float) -> torch.Tensor:
     return x
 
 
+def soft_cap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """``x = cap * tanh(x / cap)`` in place (float32)."""
+    lib = library.core_library()
+    _dev(x)
+    _need(x.dtype == torch.float32 and cap > 0, "soft_cap_: float32 and a positive cap")
+    _check(lib, lib.hal_soft_cap_f32(_ptr(x), ctypes.c_float(cap), ctypes.c_longlong(x.numel()), _stream()))
+    return x
+
+
 def grouped_gemm(
     x: torch.Tensor, w: torch.Tensor, y: torch.Tensor, *, n_rows: int,
     x_group_cols: int = 0, x_col0: int = 0, y_group_cols: int = 0, y_col0: int = 0,
@@ -934,6 +982,33 @@ def cast_rows(h: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
     out = torch.empty(h.shape, dtype=dtype, device=h.device)
     _check(lib, lib.hal_cast_rows(_ptr(h), _ptr(out), dtype_code(dtype), ctypes.c_longlong(h.numel()), _stream()))
     return out
+
+
+def cast_cols(h: torch.Tensor, out: torch.Tensor) -> None:
+    """``out[r, c] = h[r, c]`` rounded to ``out``'s type; ``out`` may be a column range of wider rows."""
+    lib = library.core_library()
+    _dev(h)
+    _need(h.dtype == torch.float32 and h.dim() == 2 and out.is_cuda and out.shape == h.shape and out.stride(1) == 1,
+          "cast_cols: float32 rows into rows of their shape")
+    _check(lib, lib.hal_cast_cols(_ptr(h), _ptr(out), out.stride(0), dtype_code(out.dtype), h.shape[0], h.shape[1], _stream()))
+
+
+def normed_sum(terms: list[tuple[torch.Tensor, torch.Tensor, float]], eps: float) -> torch.Tensor:
+    """``sum_i s_i * a_i / sqrt(mean(a_i^2) + eps) * w_i`` for ``(a_i, w_i, s_i)`` of ``terms``: float32
+    rows ``[T, d]``, each normed on its own, weighted and added up."""
+    lib = library.core_library()
+    a0, w0, _ = terms[0]
+    y = torch.empty_like(a0)
+    for a, w, _ in terms:
+        _dev(a, w)
+        _need(a.dtype == torch.float32 and a.shape == a0.shape and w.shape == (a0.shape[1],) and w.dtype == w0.dtype,
+              "normed_sum: float32 rows of one shape, weights of their width and of one type")
+    for i in range(0, len(terms), 2):
+        a, w, s = terms[i]
+        b, w2, s2 = terms[i + 1] if i + 1 < len(terms) else (None, None, 0.0)
+        _check(lib, lib.hal_normed_sum(_ptr(y), _ptr(a), _ptr(w), ctypes.c_float(s), _ptr(b), _ptr(w2), ctypes.c_float(s2),
+                                       dtype_code(w0.dtype), ctypes.c_float(eps), y.shape[0], y.shape[1], 1 if i else 0, _stream()))
+    return y
 
 
 def post_norm_add(h: torch.Tensor, a: torch.Tensor, weight: torch.Tensor, eps: float,
@@ -1206,10 +1281,10 @@ def delta_rule(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, a_raw: torch.T
 
 
 def head_norm_gate(y: torch.Tensor, z: torch.Tensor | None, weight: torch.Tensor | None, eps: float, heads: int,
-                   out_dtype: torch.dtype) -> torch.Tensor:
+                   out_dtype: torch.dtype, silu: bool = False) -> torch.Tensor:
     """Every head of the float32 rows ``y`` ``[T, heads * dim]`` divided by its own root mean
-    square, times ``weight`` (of the row's length) and ``sigmoid(z)`` (float32, a row-strided
-    view is allowed)."""
+    square, times ``weight`` (of the row's length) and ``sigmoid(z)`` (``silu``: ``silu(z)``;
+    float32, a row-strided view is allowed)."""
     lib = library.core_library()
     _dev(y, weight)
     n, inner = y.shape
@@ -1218,7 +1293,7 @@ def head_norm_gate(y: torch.Tensor, z: torch.Tensor | None, weight: torch.Tensor
         _rows_f32(z, inner, "head_norm_gate z")
     _need(weight is None or weight.numel() == inner, "head_norm_gate: a weight of the row's length")
     out = torch.empty((n, inner), dtype=out_dtype, device=y.device)
-    _check(lib, lib.hal_head_norm_gate(_ptr(y), _ptr(z), 0 if z is None else z.stride(0), _ptr(weight),
+    _check(lib, lib.hal_head_norm_gate(_ptr(y), _ptr(z), 0 if z is None else z.stride(0), 1 if silu else 0, _ptr(weight),
                                        dtype_code(weight.dtype) if weight is not None else F32, ctypes.c_float(eps),
                                        _ptr(out), dtype_code(out_dtype), n, heads, inner // heads, _stream()))
     return out
@@ -1227,13 +1302,15 @@ def head_norm_gate(y: torch.Tensor, z: torch.Tensor | None, weight: torch.Tensor
 def streams_step(x: torch.Tensor, *, y: torch.Tensor | None = None, mix: torch.Tensor | None = None,
                  out: torch.Tensor | None = None, mult: float = 1.0, read: bool = False,
                  inw: torch.Tensor | None = None, norm_weight: torch.Tensor | None = None, offset: float = 0.0,
-                 eps: float = 0.0, dtype: torch.dtype = torch.float32, rows: torch.Tensor | None = None):
+                 eps: float = 0.0, dtype: torch.dtype = torch.float32, rows: torch.Tensor | None = None,
+                 result: torch.Tensor | None = None):
     """One pass over the copies ``x`` (float32 ``[S, T, W]``) of the residual stream.  With
     ``y`` (float32 ``[T, W]``) every copy is made anew from the old ones, ``x_t <- sum_s
     mix[s, t] x_s + mult * out[t] * y``.  With ``read`` the row ``u = sum_s inw[s] x_s``
     (``inw`` None: the plain sum) of the new copies comes back, as it is (float32) or, with
     ``norm_weight``, as ``u / sqrt(mean(u^2) + eps) * (offset + norm_weight)`` in ``dtype``;
-    ``rows`` (only without ``y``): of those rows alone."""
+    ``rows`` (only without ``y``): of those rows alone; ``result``: rows to write them to (of
+    any type, a column range of wider rows is allowed) instead of new ones."""
     lib = library.core_library()
     _dev(x, y, mix, out, inw, norm_weight, rows)
     _i32(rows, "rows")
@@ -1246,14 +1323,16 @@ def streams_step(x: torch.Tensor, *, y: torch.Tensor | None = None, mix: torch.T
     _need(norm_weight is None or norm_weight.numel() == w, "streams_step: a norm weight of the rows' width")
     c_dtype = mix.dtype if mix is not None else (inw.dtype if inw is not None else torch.float32)
     n = t if rows is None else rows.numel()
-    result = None
-    if read:
+    if read and result is not None:
+        _need(result.is_cuda and result.shape == (n, w) and result.stride(1) == 1, "streams_step: result rows")
+    elif read:
         result = torch.empty((n, w), dtype=dtype if norm_weight is not None else torch.float32, device=x.device)
     _check(lib, lib.hal_streams_step(
         _ptr(x), ctypes.c_longlong(t * w), s, _ptr(y), _ptr(mix), _ptr(out), ctypes.c_float(mult), _ptr(inw),
         dtype_code(c_dtype), 1 if read else 0, _ptr(norm_weight),
         dtype_code(norm_weight.dtype) if norm_weight is not None else F32, ctypes.c_float(offset), ctypes.c_float(eps),
-        _ptr(result), dtype_code(result.dtype) if result is not None else F32, _ptr(rows), n, w, _stream()))
+        _ptr(result), 0 if result is None else result.stride(0), dtype_code(result.dtype) if result is not None else F32,
+        _ptr(rows), n, w, _stream()))
     return result
 
 
@@ -1303,19 +1382,219 @@ def head_norm_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float
     return out
 
 
-def head_gate_cols(x: torch.Tensor, x_head: int, gate: torch.Tensor, n: int, n_heads: int) -> torch.Tensor:
+def _table(cos: torch.Tensor | None, sin: torch.Tensor | None, pairs: int, what: str):
+    if cos is not None:
+        _dev(cos, sin)
+        _need(cos.dtype == torch.float32 and sin.dtype == torch.float32 and cos.dim() == 2 and cos.shape == sin.shape
+              and cos.shape[1] == pairs, f"{what}: rotation tables are float32 [positions, {pairs}]")
+
+
+def head_gate_cols(x: torch.Tensor, x_head: int, gate: torch.Tensor, n: int, n_heads: int,
+                   positions: torch.Tensor | None = None, cos: torch.Tensor | None = None,
+                   sin: torch.Tensor | None = None, interleaved: bool = False) -> torch.Tensor:
     """``y[t, h * n + j] = x[t, h * x_head + j] * sigmoid(gate[t, h])`` for ``j < n``: every
     head's first ``n`` entries times a number of the head's own (``gate`` float32, a
-    row-strided view is allowed)."""
+    row-strided view is allowed).  With a rotation table (``cos``, ``sin`` ``[positions, n / 2]``)
+    the ``n`` entries are first turned back by the token's position."""
     lib = library.core_library()
     _dev(x)
     _need(x.dim() == 2 and x.shape[1] >= n_heads * x_head and x_head >= n, "head_gate_cols: rows of padded heads")
     _rows_f32(gate, n_heads, "head_gate_cols gate")
     _need(gate.shape[0] == x.shape[0], "head_gate_cols: one gate row a token")
     y = torch.empty((x.shape[0], n_heads * n), dtype=x.dtype, device=x.device)
+    _table(cos, sin, n // 2, "head_gate_cols")
+    if cos is not None:
+        _dev(positions)
+        _i32(positions, "positions")
+        _need(positions.numel() == x.shape[0], "head_gate_cols: one position a token")
     _check(lib, lib.hal_head_gate_cols(_ptr(x), x.shape[1], x_head, _ptr(gate), gate.stride(0), _ptr(y), n, n_heads,
+                                       _ptr(positions) if cos is not None else None, _ptr(cos), _ptr(sin),
+                                       0 if cos is None else cos.shape[0], 1 if interleaved else 0,
                                        dtype_code(x.dtype), x.shape[0], _stream()))
     return y
+
+
+def turn_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, positions: torch.Tensor, n_heads: int, n_kv_heads: int,
+              qk_dim: int, v_dim: int, head_dim: int, out_dtype: torch.dtype, cos: torch.Tensor | None = None,
+              sin: torch.Tensor | None = None, cos_v: torch.Tensor | None = None, sin_v: torch.Tensor | None = None,
+              interleaved: bool = False, token_seg: torch.Tensor | None = None, block_table: torch.Tensor | None = None,
+              k_pages: torch.Tensor | None = None, v_pages: torch.Tensor | None = None, page_size: int = 0,
+              tiled: bool = False) -> torch.Tensor:
+    """From float32 projections (row-strided views allowed): the leading entries of every head
+    of ``q`` and ``k`` turned by the tokens' positions (``cos``, ``sin`` ``[positions, pairs]``), all
+    entries of every head of ``v`` by a table of their own (``cos_v``, ``sin_v``); the packed
+    rows ``[q heads | k heads | v heads]`` of ``head_dim`` entries a head (zero beyond ``qk_dim`` /
+    ``v_dim``) come back.  With ``k_pages`` and ``v_pages`` keys and values are appended to the
+    pages as well."""
+    lib = library.core_library()
+    n = q.shape[0]
+    _rows_f32(q, n_heads * qk_dim, "turn_pack q"), _rows_f32(k, n_kv_heads * qk_dim, "turn_pack k")
+    _rows_f32(v, n_kv_heads * v_dim, "turn_pack v")
+    _dev(positions)
+    _i32(positions, "positions")
+    _need(positions.numel() == n and head_dim >= max(qk_dim, v_dim), "turn_pack: positions and head sizes")
+    pairs = 0 if cos is None else cos.shape[1]
+    _table(cos, sin, pairs, "turn_pack")
+    _table(cos_v, sin_v, v_dim // 2, "turn_pack")
+    lens = {t.shape[0] for t in (cos, cos_v) if t is not None}
+    out = torch.empty((n, (n_heads + 2 * n_kv_heads) * head_dim), dtype=out_dtype, device=q.device)
+    n_pages = 0
+    if k_pages is not None:
+        _dev(token_seg, block_table, k_pages, v_pages)
+        _i32(token_seg, "token_seg"), _i32(block_table, "block_table")
+        n_pages = k_pages.shape[0]
+        _need(v_pages is not None and k_pages.dtype == out_dtype and v_pages.dtype == out_dtype
+              and k_pages.shape == (n_pages, n_kv_heads, page_size, head_dim)
+              and v_pages.shape == (n_pages, n_kv_heads, head_dim, page_size), "turn_pack: page shapes")
+        _need(token_seg is not None and token_seg.numel() == n and block_table is not None and block_table.dim() == 2,
+              "turn_pack: the step's arrays")
+    _check(lib, lib.hal_turn_pack(
+        _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), _ptr(positions), _ptr(cos), _ptr(sin), 2 * pairs,
+        _ptr(cos_v), _ptr(sin_v), min(lens) if lens else 1 << 30, 1 if interleaved else 0, _ptr(out), out.shape[1],
+        dtype_code(out_dtype), n, n_heads, n_kv_heads, qk_dim, v_dim, head_dim, _ptr(token_seg), _ptr(block_table),
+        0 if block_table is None else block_table.shape[1], _ptr(k_pages), _ptr(v_pages), page_size, n_pages,
+        1 if tiled else 0, _stream()))
+    return out
+
+
+# -- the gated scan; time mixing ------------------------------------------------------------------
+
+
+def _scan_room(chunks, seg_chunks, seg_q_start, sums: tuple, decays: tuple, device, what: str):
+    """Scratch of a scan whose segments are cut into chunks: ``(chunk count, sums, decays)``."""
+    if chunks is None:
+        return 0, None, None
+    _dev(chunks, seg_chunks)
+    _i32(chunks, "chunks"), _i32(seg_chunks, "seg_chunks")
+    _need(chunks.dim() == 2 and chunks.shape[1] == 4 and seg_chunks is not None
+          and seg_chunks.shape == (seg_q_start.numel(), 2), f"{what}: chunk arrays")
+    n = chunks.shape[0]
+    room = lambda shape: torch.empty((n, *shape), dtype=torch.float32, device=device)  # noqa: E731
+    return n, room(sums), room(decays)
+
+
+def gated_scan(a: torch.Tensor, z_bias: torch.Tensor, x_bias: torch.Tensor, state: torch.Tensor, seg_q_start: torch.Tensor,
+               seg_q_len: torch.Tensor, token_slot: torch.Tensor, out_dtype: torch.dtype,
+               chunks: torch.Tensor | None = None, seg_chunks: torch.Tensor | None = None) -> torch.Tensor:
+    """A gated recurrence per channel over every request's tokens of the step: from float32 rows
+    ``a`` = ``[z | x | g]`` (a row-strided view is allowed) ``z = sigmoid(. + z_bias)``, ``u = . +
+    x_bias``, the candidate ``u + 1/2`` where ``u >= 0`` and ``sigmoid(u)`` elsewhere, ``S <- (1 - z) S
+    + z candidate``; returns ``S * silu(g)``.  ``state`` float32 ``[slots, channels]``, read and left as
+    the step's last state.  ``chunks``, ``seg_chunks`` as for ``ssd_scan``."""
+    lib = library.core_library()
+    c = state.shape[1]
+    _rows_f32(a, 3 * c, "gated_scan")
+    _dev(z_bias, x_bias, state, seg_q_start, seg_q_len, token_slot)
+    _i32(seg_q_start, "seg_q_start"), _i32(seg_q_len, "seg_q_len"), _i32(token_slot, "token_slot")
+    _need(state.dtype == torch.float32 and state.dim() == 2, "gated_scan: a float32 state [slots, channels]")
+    _need(z_bias.shape == (c,) and x_bias.shape == (c,) and z_bias.dtype == x_bias.dtype, "gated_scan: biases of one type")
+    _need(token_slot.numel() == a.shape[0] and seg_q_start.numel() == seg_q_len.numel(), "gated_scan: the step's arrays")
+    out = torch.empty((a.shape[0], c), dtype=out_dtype, device=a.device)
+    n_chunks, sums, decays = _scan_room(chunks, seg_chunks, seg_q_start, (c,), (c,), a.device, "gated_scan")
+    _check(lib, lib.hal_gated_scan(
+        _ptr(a), a.stride(0), _ptr(z_bias), _ptr(x_bias), dtype_code(z_bias.dtype), _ptr(state), _ptr(seg_q_start),
+        _ptr(seg_q_len), _ptr(token_slot), _ptr(out), dtype_code(out_dtype), seg_q_start.numel(), c, _ptr(chunks),
+        _ptr(seg_chunks), n_chunks, _ptr(sums), _ptr(decays), _stream()))
+    return out
+
+
+def token_shift(x: torch.Tensor, mu: torch.Tensor, last: torch.Tensor, ctx, side_by_side: bool):
+    """``x_t + (x_(t-1) - x_t) * mu[s]`` for every row ``s`` of ``mu`` ``[n, W]``, in ``x``'s type.  The
+    row before a segment's first token is ``last`` (float32 ``[slots, W]``), which is left as the
+    step's last rows.  Returns the first ``n - 1`` mixes, as columns of one row a token
+    (``[T, (n - 1) * W]``, ``side_by_side``) or one after the other (``[n - 1, T, W]``), and the last."""
+    lib = library.core_library()
+    _dev(x, mu, last, ctx.token_seg, ctx.seg_q_start, ctx.seg_q_len, ctx.token_slot)
+    t, w = x.shape
+    n = mu.shape[0]
+    _need(mu.shape == (n, w) and n > 1 and last.dtype == torch.float32 and last.dim() == 2 and last.shape[1] == w,
+          "token_shift: mu [n, W] and float32 rows [slots, W]")
+    _need(ctx.token_seg.numel() == t and ctx.token_slot.numel() == t, "token_shift: the step's arrays")
+    out = torch.empty((t, (n - 1) * w) if side_by_side else (n - 1, t, w), dtype=x.dtype, device=x.device)
+    out_last = torch.empty((t, w), dtype=x.dtype, device=x.device)
+    single = t == ctx.n_segs
+    _check(lib, lib.hal_token_shift(
+        _ptr(x), dtype_code(x.dtype), _ptr(mu), dtype_code(mu.dtype), n, _ptr(last), _ptr(ctx.token_seg),
+        _ptr(ctx.seg_q_start), _ptr(ctx.token_slot), 1 if single else 0, _ptr(out),
+        ctypes.c_longlong(w if side_by_side else t * w), (n - 1) * w if side_by_side else w, _ptr(out_last), t, w, _stream()))
+    if not single:
+        _check(lib, lib.hal_carry_rows(_ptr(x), dtype_code(x.dtype), _ptr(last), _ptr(ctx.seg_q_start),
+                                       _ptr(ctx.seg_q_len), _ptr(ctx.token_slot), ctx.n_segs, w, _stream()))
+    return out, out_last
+
+
+WKV_STEP_DIMS = (16, 32, 64, 128)  # heads that a step of single tokens has a kernel for
+
+
+def _wkv_rows(tensors, inner: int, what: str) -> int:
+    for t in tensors:
+        _rows_f32(t, inner, what)
+    _need(len({(t.shape[0], t.stride(0)) for t in tensors}) == 1, f"{what}: rows of one length, one a token")
+    return tensors[0].stride(0)
+
+
+def wkv_decay(x1: torch.Tensor, w2: torch.Tensor, w0: torch.Tensor, out: torch.Tensor) -> torch.Tensor:
+    """``exp(-exp(w0 + W2 tanh(x1)))`` of float32 rows ``x1`` ``[T, rank]`` into ``out`` (float32
+    ``[T, channels]``, a row-strided view is allowed)."""
+    lib = library.core_library()
+    n, rank = w2.shape
+    _rows_f32(x1, rank, "wkv_decay x1"), _rows_f32(out, n, "wkv_decay out")
+    _dev(w2, w0)
+    _need(w0.numel() == n and w0.dtype == w2.dtype and out.shape[0] == x1.shape[0], "wkv_decay: w0 [channels] of w2's type")
+    _check(lib, lib.hal_wkv_decay(_ptr(x1), x1.stride(0), _ptr(w2), _ptr(w0), dtype_code(w2.dtype), rank, _ptr(out),
+                                  out.stride(0), x1.shape[0], n, _stream()))
+    return out
+
+
+def wkv_scan(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, decay: torch.Tensor, bonus: torch.Tensor,
+             state: torch.Tensor, seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, token_slot: torch.Tensor,
+             chunks: torch.Tensor | None = None, seg_chunks: torch.Tensor | None = None) -> torch.Tensor:
+    """The recurrence ``o = (S + diag(bonus) k v^T)^T r``, ``S <- diag(decay) S + k v^T`` per head over
+    every request's tokens of the step.  ``r``, ``k``, ``v``, ``decay``: float32 ``[T, heads * dim]``
+    (row-strided views of one row length); ``state`` float32 ``[slots, heads, dim, dim]`` (key
+    channel, value channel), read and left as the step's last state.  ``chunks``, ``seg_chunks`` as
+    for ``ssd_scan``.  Returns float32 ``[T, heads * dim]``."""
+    lib = library.core_library()
+    _, heads, d, d2 = state.shape
+    inner = heads * d
+    ld = _wkv_rows((r, k, v, decay), inner, "wkv_scan")
+    _dev(bonus, state, seg_q_start, seg_q_len, token_slot)
+    _i32(seg_q_start, "seg_q_start"), _i32(seg_q_len, "seg_q_len"), _i32(token_slot, "token_slot")
+    _need(state.dtype == torch.float32 and d == d2 and bonus.numel() == inner, "wkv_scan: a float32 state [slots, heads, dim, dim]")
+    _need(token_slot.numel() == r.shape[0] and seg_q_start.numel() == seg_q_len.numel(), "wkv_scan: the step's arrays")
+    o = torch.empty((r.shape[0], inner), dtype=torch.float32, device=r.device)
+    n_chunks, sums, decays = _scan_room(chunks, seg_chunks, seg_q_start, (heads, d, d), (heads, d), r.device, "wkv_scan")
+    _check(lib, lib.hal_wkv_scan(
+        _ptr(r), _ptr(k), _ptr(v), _ptr(decay), ld, _ptr(bonus), dtype_code(bonus.dtype), _ptr(state), _ptr(seg_q_start),
+        _ptr(seg_q_len), _ptr(token_slot), _ptr(o), seg_q_start.numel(), heads, d, _ptr(chunks), _ptr(seg_chunks), n_chunks,
+        _ptr(sums), _ptr(decays), _stream()))
+    return o
+
+
+def wkv_step(r: torch.Tensor, k: torch.Tensor, v: torch.Tensor, gate: torch.Tensor, x1: torch.Tensor, w2: torch.Tensor,
+             w0: torch.Tensor, bonus: torch.Tensor, norm_weight: torch.Tensor, eps: float, state: torch.Tensor,
+             token_slot: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """A step in which every request brings one token, in one kernel: the decay (``wkv_decay``), the
+    recurrence (``wkv_scan``) and the head's norm, weight and ``silu(gate)``; ``[T, heads * dim]``
+    of ``out_dtype``.  For heads of ``WKV_STEP_DIMS`` channels."""
+    lib = library.core_library()
+    _, heads, d, d2 = state.shape
+    inner = heads * d
+    ld = _wkv_rows((r, k, v, gate), inner, "wkv_step")
+    n, rank = w2.shape
+    _rows_f32(x1, rank, "wkv_step x1")
+    _dev(w2, w0, bonus, norm_weight, state, token_slot)
+    _i32(token_slot, "token_slot")
+    _need(d == d2 and d in WKV_STEP_DIMS and n == inner and state.dtype == torch.float32, "wkv_step: a float32 state [slots, heads, dim, dim]")
+    _need(w0.numel() == inner and bonus.numel() == inner and norm_weight.numel() == inner
+          and w2.dtype == w0.dtype == bonus.dtype == norm_weight.dtype, "wkv_step: weights of one type")
+    _need(token_slot.numel() == r.shape[0] and x1.shape[0] == r.shape[0], "wkv_step: one row a token")
+    out = torch.empty((r.shape[0], inner), dtype=out_dtype, device=r.device)
+    _check(lib, lib.hal_wkv_step(
+        _ptr(r), _ptr(k), _ptr(v), _ptr(gate), ld, _ptr(x1), x1.stride(0), _ptr(w2), _ptr(w0), _ptr(bonus),
+        _ptr(norm_weight), dtype_code(w2.dtype), rank, ctypes.c_float(eps), _ptr(state), _ptr(token_slot), _ptr(out),
+        dtype_code(out_dtype), r.shape[0], heads, d, _stream()))
+    return out
 
 
 # -- small passes over float32 rows of projections ----------------------------------------------

@@ -4,6 +4,7 @@ from .base import (
     EMBEDDINGS,
     FEED_FORWARDS,
     HEADS,
+    JUNCTIONS,
     MIXERS,
     NORMS,
     POSITIONS,
@@ -12,6 +13,7 @@ from .base import (
     Embedding,
     FeedForward,
     Head,
+    Junction,
     Mixer,
     Norm,
     PagedKVNeed,
@@ -27,8 +29,8 @@ from .base import (
 from .decoder import Decoder
 
 __all__ = [
-    "ARRANGEMENTS", "EMBEDDINGS", "FEED_FORWARDS", "HEADS", "MIXERS", "NORMS", "POSITIONS",
-    "Arrangement", "BuildContext", "Decoder", "Embedding", "FeedForward", "Head", "Mixer", "Norm",
+    "ARRANGEMENTS", "EMBEDDINGS", "FEED_FORWARDS", "HEADS", "JUNCTIONS", "MIXERS", "NORMS", "POSITIONS",
+    "Arrangement", "BuildContext", "Decoder", "Embedding", "FeedForward", "Head", "Junction", "Mixer", "Norm",
     "PagedKVNeed", "PagedNeed", "ParamDecl", "Part", "PositionEncoding", "RotaryPositionEncoding", "RunBinding", "StateNeed",
     "register_arrangement",
 ]

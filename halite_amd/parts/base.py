@@ -42,8 +42,9 @@ class PagedNeed:
 
     * ``window`` (an attribute; ``None``: every token's page is kept while the request lives;
       else the tokens a query looks back, itself included, so that pages are given back once
-      every later query has passed them), and ``chunk`` (likewise; else queries see keys of
-      their own chunk of that many positions only);
+      every later query has passed them), ``chunk`` (likewise; else queries see keys of
+      their own chunk of that many positions only), and ``keep`` (with one of the two: the
+      pages of a request's first so many tokens stay all the same);
     * ``page_tensors(page_size)``: name -> shape of one page, the tensors a run keeps per page
       number, all of the cache's element type;
     * ``bind(group_id, tensors, page_size, dtype)``: what the run's mixer finds in ``run.kv``,
@@ -52,6 +53,7 @@ class PagedNeed:
 
     window: int | None = None
     chunk: int | None = None
+    keep: int = 0
 
     def page_tensors(self, page_size: int) -> dict[str, tuple[int, ...]]:
         raise NotImplementedError
@@ -75,6 +77,9 @@ class PagedKVNeed(PagedNeed):
     # True: the pages are kept row by row whatever the sizes (for a reader other than the
     # matrix-core attention kernel)
     plain_layout: bool = False
+    # under a window: every later query sees the request's first tokens too, and the pages of
+    # so many of them are kept
+    keep: int = 0
 
     def page_tensors(self, page_size: int) -> dict[str, tuple[int, ...]]:
         k, d = self.n_kv_heads, self.head_dim
@@ -151,6 +156,12 @@ class Part:
 
     def finalize(self) -> None:
         """Called once after the tensors are filled."""
+
+    def drop_tensors(self) -> None:
+        """Lets go of the part's tensors (the part is not used again)."""
+        for name, value in list(vars(self).items()):
+            if isinstance(value, torch.Tensor):
+                setattr(self, name, None)
 
     def cache_need(self) -> PagedNeed | None:
         return None
@@ -244,8 +255,31 @@ class RotaryPositionEncoding(PositionEncoding):
 
 
 class Embedding(Part):
+    # True: a token's row depends on more than its id, and ``forward`` takes ``ctx`` (the step) and
+    # ``run`` (a binding whose ``state`` holds the embedding's per-request state rows)
+    reads_step: bool = False
+
     def forward(self, tokens: torch.Tensor, out: torch.Tensor | None = None) -> torch.Tensor:
         """The tokens' rows as float32 ``[T, width]``, written to ``out`` if that is given."""
+        raise NotImplementedError
+
+
+class Junction(Part):
+    """Makes the residual stream anew between two runs of the order, from the stream and from
+    what it kept of the embedding's output."""
+
+    def start(self, h0: torch.Tensor) -> torch.Tensor:
+        """At the start of a step: what is kept of the embedding's output ``h0`` (float32 ``[T,
+        width]``) until the step's end."""
+        raise NotImplementedError
+
+    def stream_rows(self, kept: torch.Tensor) -> torch.Tensor:
+        """Where the stream's rows ``[T, width]`` are to be written before ``forward`` (any type, a
+        column range is allowed)."""
+        raise NotImplementedError
+
+    def forward(self, kept: torch.Tensor) -> torch.Tensor:
+        """The new stream, float32 ``[T, width]``."""
         raise NotImplementedError
 
 
@@ -263,9 +297,9 @@ class Connection(Part):
         rows that the next part reads through this connection, normed by ``norm``."""
         raise NotImplementedError
 
-    def leave(self, x: torch.Tensor, pending, rows: torch.Tensor | None) -> torch.Tensor:
+    def leave(self, x: torch.Tensor, pending, rows: torch.Tensor | None, out: torch.Tensor | None = None) -> torch.Tensor:
         """Writes what is ``pending`` and returns the model's one stream (float32; of
-        ``rows`` alone if given)."""
+        ``rows`` alone if given; written to ``out``, in its type, if that is given)."""
         raise NotImplementedError
 
 
@@ -310,6 +344,9 @@ POSITIONS = Registry("position encoding")
 EMBEDDINGS = Registry("embedding")
 CONNECTIONS = Registry("connection")
 HEADS = Registry("head")
+JUNCTIONS = Registry("junction")
+
+
 class Arrangement:
     """The order in which a layer's parts act on the residual stream.
 

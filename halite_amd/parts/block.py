@@ -205,7 +205,7 @@ class HyperPreNormBlock(Arrangement):
             pending = (self.ff.forward(x, ctx), self.ff_link)
         return pending
 
-    def leave(self, h, pending, rows):
-        """The model's one stream after the last block (of ``rows`` alone if given)."""
+    def leave(self, h, pending, rows, out=None):
+        """The model's one stream after the last block (of ``rows`` alone if given; in ``out`` if given)."""
         link = pending[1] if pending is not None else self.mixer_link
-        return link.leave(h, pending, rows)
+        return link.leave(h, pending, rows, out)

@@ -82,7 +82,9 @@ class HyperConnection(Connection):
         return ops.streams_step(x, read=True, inw=self.w_in, norm_weight=norm.weight, offset=norm.p.weight_offset,
                                 eps=norm.p.eps, dtype=self.build.dtype, **self._write_args(pending))
 
-    def leave(self, x, pending, rows):
+    def leave(self, x, pending, rows, out=None):
+        if rows is None:  # (one pass)
+            return ops.streams_step(x, read=True, result=out, **self._write_args(pending))
         if pending is not None:
             ops.streams_step(x, **self._write_args(pending))
-        return ops.streams_step(x, read=True, rows=rows)
+        return ops.streams_step(x, read=True, rows=rows, result=out)

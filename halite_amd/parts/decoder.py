@@ -13,10 +13,12 @@ from dataclasses import dataclass
 import torch
 
 from ..config.spec import ModelSpec
+from ..kernels import ops
 from .base import (
     ARRANGEMENTS,
     EMBEDDINGS,
     HEADS,
+    JUNCTIONS,
     NORMS,
     POSITIONS,
     BuildContext,
@@ -25,6 +27,9 @@ from .base import (
     Part,
     RunBinding,
 )
+
+
+EMBEDDING_RUN = -1  # the index of the embedding's state rows among the runs'
 
 
 @dataclass
@@ -40,8 +45,8 @@ class Decoder:
                  tiled_weights: bool = False):
         # the kinds of parts register themselves when their modules are imported
         from . import (attention, block, capped_attention, connection, decay_attention, embedding, feedforward,  # noqa: F401
-                       general_delta, latent_attention, mixer_sum, moe, norm, normed_attention, rope,
-                       sigmoid_attention, state_space, token_gated)
+                       general_delta, junction, latent_attention, mingru, mixer_sum, moe, norm, normed_attention, rope,
+                       rotated_attention, sigmoid_attention, state_space, time_mix, token_gated)
 
         self.spec = spec
         self.dtype = dtype
@@ -60,11 +65,14 @@ class Decoder:
                 known = ", ".join(sorted(ARRANGEMENTS))
                 raise ConfigError(f"unknown arrangement {lspec.arrangement!r}; known: {known}")
             self.layers[name] = ARRANGEMENTS[lspec.arrangement].build(lspec.arrangement, lspec.parts, build)
+        self.junctions = {name: JUNCTIONS.build(pspec, build) for name, pspec in spec.junctions.items()}
         self.final_norm = NORMS.build(spec.final_norm, build)
         self.head = HEADS.build(spec.head, build)
         self.runs = [
             RunBinding(index=i, appends=run.cache_from is None) for i, run in enumerate(spec.order)
         ]
+        # what an embedding with per-request state is bound to (before the first run)
+        self.embedding_run = RunBinding(index=EMBEDDING_RUN)
         # an arrangement may keep the residual stream in several copies ([copies, T, width]);
         # then every block of the model does, and the last one says how they become one again
         copies = {getattr(self.layers[run.layer], "stream_copies", None) for run in spec.order}
@@ -78,6 +86,8 @@ class Decoder:
         for lname, block in self.layers.items():
             for pname, part in block.parts().items():
                 out[f"layers.{lname}.{pname}"] = part
+        for jname, part in self.junctions.items():
+            out[f"junctions.{jname}"] = part
         out["final_norm"] = self.final_norm
         out["head"] = self.head
         return out
@@ -112,20 +122,27 @@ class Decoder:
     def forward(self, ctx) -> torch.Tensor:
         """float32 logits ``[len(ctx.logit_rows), vocab]``; keys and values of all
         the step's tokens are in the cache afterwards."""
+        reads = dict(ctx=ctx, run=self.embedding_run) if self.embedding.reads_step else {}
         if self.stream_copies is None:
-            h = self.embedding.forward(ctx.tokens)
+            h = h0 = self.embedding.forward(ctx.tokens, **reads)
         else:  # every copy starts as the embedding's output
             h = torch.empty((self.stream_copies, ctx.tokens.numel(), self.spec.hidden_size), dtype=torch.float32,
                             device=self.device)
-            for copy in h:
-                self.embedding.forward(ctx.tokens, out=copy)
+            h0 = self.embedding.forward(ctx.tokens, out=h[0], **reads)
+            for copy in h[1:]:  # (an embedding that reads the step moves its state on: it runs once)
+                copy.copy_(h0) if reads else self.embedding.forward(ctx.tokens, out=copy)
+        kept = {name: junction.start(h0) for name, junction in self.junctions.items()}
         pending = None
         blocks = [self.layers[self.spec.order[run.index].layer] for run in self.runs]
         for i, run in enumerate(self.runs):
+            name = self.spec.order[run.index].junction
+            if name is not None:
+                h = self._through_junction(self.junctions[name], kept[name], h, pending, blocks[max(i - 1, 0)], ctx)
+                pending = None
             # what the next block's first norm lets this block's last product do for it
             # (both are optional abilities of an arrangement: `takes_next_norm` of the one that
             # runs now, `first_norm_for` of the one that runs next)
-            ahead = blocks[i + 1] if i + 1 < len(blocks) else None
+            ahead = blocks[i + 1] if i + 1 < len(blocks) and self.spec.order[i + 1].junction is None else None
             next_norm = None
             if getattr(blocks[i], "takes_next_norm", False) and hasattr(ahead, "first_norm_for"):
                 next_norm = ahead.first_norm_for(h)
@@ -140,3 +157,16 @@ class Decoder:
         else:
             x = self.final_norm.forward(h, delta=pending, rows=ctx.logit_rows)
         return self.head.forward(x)
+
+    def _through_junction(self, junction, kept, h, pending, block, ctx):
+        """The stream that the next run starts from; ``block`` ran last and left ``pending``."""
+        rows = junction.stream_rows(kept)
+        ctx.rounded_rows = None
+        if self.stream_copies is None:
+            if pending is not None:
+                ops.residual_add(h, pending)
+            ops.cast_cols(h, rows)
+            return junction.forward(kept)
+        block.leave(h, pending, None, out=rows)
+        x = junction.forward(kept)
+        return x.unsqueeze(0) if self.stream_copies == 1 else x.unsqueeze(0).repeat(self.stream_copies, 1, 1)

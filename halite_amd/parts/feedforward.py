@@ -5,7 +5,7 @@ from __future__ import annotations
 import torch
 from typing import Literal
 
-from pydantic import BaseModel, Field, StrictBool, StrictInt, field_validator
+from pydantic import BaseModel, Field, StrictBool, StrictInt, field_validator, model_validator
 
 from ..kernels import ops
 from .base import FEED_FORWARDS, FeedForward, ParamDecl
@@ -22,15 +22,21 @@ class GatedParams(BaseModel):
     @field_validator("activation")
     @classmethod
     def _known(cls, v):
-        if v != "silu":
-            raise ValueError(f"activation {v!r}: only 'silu' has a kernel")
+        if v not in ops.GATE_ACTIVATIONS:
+            raise ValueError(f"activation {v!r}: only {sorted(ops.GATE_ACTIVATIONS)} have kernels")
         return v
+
+    @model_validator(mode="after")
+    def _check(self):
+        if self.activation != "silu" and not self.float32_result:
+            raise ValueError("products with a norm folded in compute SiLU; another activation comes with float32_result")
+        return self
 
 
 @FEED_FORWARDS.register("gated")
 class GatedFeedForward(FeedForward):
-    """``linear_out(linear_proj(x) * silu(linear_gate(x)))`` without biases
-    (feedforward.py:204-212).  Gate and up weights live in one tensor
+    """``linear_out(linear_proj(x) * act(linear_gate(x)))`` without biases, ``act`` SiLU
+    (feedforward.py:204-212) or gelu's tanh form.  Gate and up weights live in one tensor
     ``[2F, d]`` (gate first) so that one product serves both; the activation and
     the multiply are float32 on the accumulators or on the product's output."""
 
@@ -108,9 +114,9 @@ class GatedFeedForward(FeedForward):
         f = self.p.intermediate_size
         m, d = x.shape
         if self.t_gate is not None and x.dtype == torch.bfloat16 and d % 8 == 0 and m <= ops.SKINNY_ROWS:
-            act = ops.gemm_bf16_skinny(x, self.t_gate, w_up=self.t_up, tiled_shape=(f, d))
+            act = ops.gemm_bf16_skinny(x, self.t_gate, w_up=self.t_up, tiled_shape=(f, d), activation=self.p.activation)
         else:
-            act = ops.silu_mul(ops.linear(x, self.w_gate_up))
+            act = ops.gate_mul(ops.linear(x, self.w_gate_up), self.p.activation)
         return ops.linear(act, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
 
 

@@ -1,6 +1,9 @@
 """Mixers side by side: every one reads the same rows, and the result is the sum of their
 results, each times a constant.
 
+With ``norm_eps`` every member's result is first divided by its own root mean square over the
+row and multiplied by a weight of its own (``<name>_norm.weight``), in float32.
+
 The mixers are named; the tensors, the per-request state and the cache of a member are the
 member's own, under its name (``<name>.<tensor>``).  At most one member may keep pages (a run
 has one place in one page group); any number may keep state rows.
@@ -9,11 +12,11 @@ has one place in one page group); any number may keep state rows.
 from __future__ import annotations
 
 import torch
-from pydantic import BaseModel, model_validator
+from pydantic import BaseModel, Field, StrictInt, model_validator
 
 from ..config.spec import PartSpec
 from ..kernels import ops
-from .base import MIXERS, Mixer, RunBinding
+from .base import MIXERS, Mixer, ParamDecl, RunBinding
 
 
 class MixerSumParams(BaseModel):
@@ -21,6 +24,9 @@ class MixerSumParams(BaseModel):
     mixers: list[dict]
     """One description a member: ``kind`` and the kind's own parameters."""
     scales: list[float]
+    norm_eps: float | None = Field(default=None, gt=0)
+    size: StrictInt | None = Field(default=None, gt=0)
+    """Of the rows (with ``norm_eps``)."""
 
     @model_validator(mode="after")
     def _check(self):
@@ -28,6 +34,8 @@ class MixerSumParams(BaseModel):
             raise ValueError("a sum of mixers has as many names and scales as members, and at least one")
         if len(set(self.names)) != len(self.names) or any("." in n or not n for n in self.names):
             raise ValueError(f"the members' names {self.names} must differ and hold no dot")
+        if (self.norm_eps is None) != (self.size is None):
+            raise ValueError("members that are normed need the eps and the rows' size")
         return self
 
 
@@ -45,10 +53,20 @@ class MixerSum(Mixer):
             raise ValueError(f"only one member of a sum of mixers may keep pages; {self._paged} all do")
 
     def param_decls(self):
-        return {f"{name}.{k}": d for name, m, _ in self.members for k, d in m.param_decls().items()}
+        decls = {f"{name}.{k}": d for name, m, _ in self.members for k, d in m.param_decls().items()}
+        if self.p.norm_eps is not None:
+            decls.update({f"{name}_norm.weight": ParamDecl((self.p.size,), init="ones") for name, _, _ in self.members})
+        return decls
 
     def allocate(self, dtypes):
-        out = {}
+        out, self.norms = {}, []
+        if self.p.norm_eps is not None:
+            if len({dtypes[f"{name}_norm.weight"] for name, _, _ in self.members}) != 1:
+                raise ValueError("the norms of a sum's members are stored with different element types")
+            for name, _, _ in self.members:
+                key = f"{name}_norm.weight"
+                out[key] = torch.empty((self.p.size,), dtype=dtypes[key], device=self.build.device)
+                self.norms.append(out[key])
         for name, m, _ in self.members:
             own = {k[len(name) + 1 :]: v for k, v in dtypes.items() if k.startswith(name + ".")}
             out.update({f"{name}.{k}": t for k, t in m.allocate(own).items()})
@@ -57,6 +75,12 @@ class MixerSum(Mixer):
     def finalize(self):
         for _, m, _ in self.members:
             m.finalize()
+
+    def drop_tensors(self):
+        super().drop_tensors()
+        self.norms = []
+        for _, m, _ in self.members:
+            m.drop_tensors()
 
     def cache_need(self):
         for _, m, _ in self.members:
@@ -80,7 +104,12 @@ class MixerSum(Mixer):
 
     def forward_terms(self, x, ctx, run):
         """The members' results and their constants, for a caller that adds them up itself
-        (an arrangement whose next kernel reads the sum anyway)."""
+        (an arrangement whose next kernel reads the sum anyway); None where they are normed."""
+        if self.p.norm_eps is not None:
+            return None
+        return self._results(x, ctx, run)
+
+    def _results(self, x, ctx, run):
         terms = []
         for name, m, scale in self.members:
             a = m.forward(x, ctx, self._member_run(run, name))
@@ -88,6 +117,8 @@ class MixerSum(Mixer):
         return terms
 
     def forward(self, x, ctx, run):
+        if self.p.norm_eps is not None:
+            return ops.normed_sum([(a, w, s) for (a, s), w in zip(self._results(x, ctx, run), self.norms)], self.p.norm_eps)
         total = None
         for name, m, scale in self.members:
             a = m.forward(x, ctx, self._member_run(run, name))

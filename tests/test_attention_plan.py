@@ -233,3 +233,50 @@ def test_recorded_decode_steps_have_room_for_any_lengths():
         assert plan.max_parts <= first.max_parts
         if plan.n_partials:  # some range is cut: by the kernel itself or by the merge kernel, as recorded
             assert plan.merged_in_kernel == first.merged_in_kernel and (plan.n_merges > 0) == (first.cap_merges > 0)
+
+
+def seen_keys(plan, seg, row, q_len, kv_len, group, window, keep):
+    """The keys that a query row meets under the plan, as the kernels walk and mask them: for
+    every work item that holds the row, the keys its walk comes by (in the walk's blocks of 32)
+    that lie in one of the item's ranges and that the row sees."""
+    pos = kv_len[seg] - q_len[seg] + row // group
+    met = []
+    visible = lambda j: j <= pos and (window <= 0 or j > pos - window or j < keep)  # noqa: E731
+    for it in plan.items.tolist():
+        if it[0] != seg or not it[1] <= row < it[1] + 16:
+            continue
+        b, e, pre0, n_pre = it[2], it[3], it[10], it[11]
+        assert pre0 % 32 == 0 and n_pre % 32 == 0 and (n_pre == 0 or b // 32 * 32 >= pre0 + n_pre)
+        walk = list(range(pre0, pre0 + n_pre)) + (list(range(b // 32 * 32, e)) if e > b else [])
+        met += [j for j in walk if (b <= j < e or pre0 <= j < pre0 + n_pre) and visible(j)]
+    per_item = max(1, plan.rows_big // 16)
+    for r in range(0, plan.n_big, 4):
+        for it in plan.big_items[r : r + 4].tolist():
+            tiles = [it[1]] + it[5 : 5 + per_item - 1]
+            if it[0] != seg or not any(t >= 0 and t <= row < t + 16 for t in tiles):
+                continue
+            b, e, walk_b, walk_e, n_pre, kept_end = it[2], it[3], it[11], it[12], it[13], it[14]
+            assert n_pre % 64 == 0 and kept_end in (0, keep) and (n_pre == 0 or walk_b // 32 * 32 >= n_pre)
+            walk = list(range(n_pre)) + list(range(walk_b // 32 * 32, walk_e))
+            met += [j for j in walk if (b <= j < e or j < kept_end) and visible(j)]
+    return sorted(met), [j for j in range(pos + 1) if visible(j)]
+
+
+@pytest.mark.parametrize("rows_big", [64, 16])
+@pytest.mark.parametrize("keep", [0, 1, 20, 64, 65, 200])
+@pytest.mark.parametrize("window", [1, 33, 96, 400])
+@pytest.mark.parametrize("heads", [(1, 1), (8, 1), (20, 2)])
+def test_kept_first_keys_are_met_once(rows_big, keep, window, heads):
+    """Every visible key, the kept first ones included, is met by exactly one item of a row:
+    decoded tokens and portions at the start, around the place where the window leaves the kept
+    keys, and far behind it; short and long ones (cut and not cut)."""
+    group, n_kv = heads
+    q_len = [1, 1, 1, 1, 2, 90, 300, 40, 1, 700]
+    kv_len = [5, window + 3, window + keep + 70, 3000, 2500, 90, 300 + window, 2000, 9000, 5000]
+    plan = plan_items(q_len, kv_len, group, n_kv, window, rows_big, keep=keep)
+    for seg in range(len(q_len)):
+        rows = q_len[seg] * group
+        for row in sorted({0, 1, 15, 16, 17, rows // 2, rows // 3, rows - 1}):
+            if row < rows:
+                met, want = seen_keys(plan, seg, row, q_len, kv_len, group, window, keep)
+                assert met == want, (seg, row)
