@@ -335,3 +335,29 @@ def write_model_folder(folder, cfg, weights, dtype=torch.bfloat16):
         json.dump(cfg, f)
     save_file({k: v.to(dtype).contiguous() for k, v in weights.items()}, os.path.join(folder, "model.safetensors"))
     return folder
+
+
+# a loop over two of three layers, both kinds of mixer, kept first tokens, a table of pairs
+NOD_A = model_cfg(64, 331, [
+    parallel_layer(4, 2, 16, 16, 0.3, rotation(5000.0, 16, 2.5), 2, 16, window(24, 5), dense(96)),
+    mingru_layer(40, dense(72)),
+    parallel_layer(4, 1, 16, 32, 0.35, rotation(900.0, 8, 1.5), 4, 8, window(40, 21), dense(80)),
+], scale=3.0, bigram=(37, 5, 11), loop=(1, 3, 2), residual_mult=0.6, softcap=8.0)
+NOD_A_RANKS = {0: 8, 2: 6}
+# the loop begins at the first layer and runs three times; no table of pairs, no multiplier, no cap; no
+# window; a window shorter than what is kept; value heads larger and smaller than the keys'; a layer
+# without feed-forward; one head of 48 channels
+NOD_B = model_cfg(48, 257, [
+    mingru_layer(56),
+    parallel_layer(6, 3, 8, 24, 0.5, rotation(10.0, 4), 1, 48, None, dense(40)),
+    parallel_layer(2, 2, 24, 8, 0.25, rotation(300.0, 24), 2, 24, window(7, 20), dense(52)),
+], loop=(0, 2, 3))
+NOD_B_RANKS = {1: 5, 2: 3}
+# sizes that are multiples of nothing; a window without kept tokens; a loop of one pass; a hash that
+# passes the token before over
+NOD_C = model_cfg(42, 203, [
+    parallel_layer(5, 1, 12, 20, 0.2, rotation(77.0, 6, 3.0), 2, 20, window(33), dense(50)),
+    mingru_layer(30, dense(38)),
+    parallel_layer(3, 3, 10, 6, 0.4, rotation(20.0, 10), 3, 10, window(17, 1), None),
+], scale=0.5, bigram=(7, 0, 3), loop=(1, 2, 1), residual_mult=1.3, softcap=30.0, eps=1e-6)
+NOD_C_RANKS = {0: 6, 2: 2}
