@@ -101,8 +101,10 @@ class Families:
     ELEMENTWISE = ("rmsnorm", "silu_mul", "rope_append", "embedding", "residual_add", "rmsnorm_exact", "latent_prep",
                    "head_cols", "scale_", "moe_route", "moe_sort", "moe_route_sort", "moe_combine", "clamped_gate_mul", "cast_rows",
                    "post_norm_add", "relu_squared", "scaled_sum_", "qk_norm_pack", "gated_part_norm", "head_norm_gate",
-                   "streams_step", "head_norm_pack", "head_gate_cols", "bias_rows_", "silu_rows", "token_gate")
-    RECURRENT = ("short_conv", "short_conv_carry", "ssd_scan", "delta_rule")
+                   "streams_step", "head_norm_pack", "head_gate_cols", "bias_rows_", "silu_rows", "token_gate", "gate_mul",
+                   "turn_pack", "normed_sum", "soft_cap_", "cast_cols", "token_shift", "pair_embedding", "stream_step")
+    RECURRENT = ("short_conv", "short_conv_carry", "short_conv_through", "ssd_scan", "delta_rule", "wkv_decay", "wkv_scan",
+                 "wkv_step", "gated_scan")
 
     def __init__(self):
         self.spans = []
@@ -379,7 +381,7 @@ def zabunex_layer_kinds(n_layers):
     return ["parallel" if i % 4 == 3 else "attention" for i in range(n_layers)]
 
 
-def zabunex_config(s, n_layers, window):
+def zabunex_config(s, n_layers, window, kinds=None):
     attention = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5,
                      bias_max=s["bias_max"], bias_buckets=32, q_temp=dict(coef=0.1, every=1024))
     left = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5, conv=4,
@@ -388,7 +390,7 @@ def zabunex_config(s, n_layers, window):
     mlp = dict(kind="dense", ff=s["ff"])
     layers = [dict(type="attention", mixer=attention, mlp=mlp) if kind == "attention" else
               dict(type="parallel", mixer=dict(left=left, right=right, left_scale=0.5, right_scale=1.0), mlp=mlp)
-              for kind in zabunex_layer_kinds(n_layers)]
+              for kind in kinds or zabunex_layer_kinds(n_layers)]
     return dict(architecture="Zabunex", vocab=COMPARISON_VOCAB, width=s["width"], norm=dict(eps=1e-5), max_positions=8192,
                 layers=layers)
 
@@ -399,12 +401,12 @@ def llama_beside_zabunex(s, n_layers):
                 intermediate_size=s["llama_ff"], max_position_embeddings=8192, rope_scaling=None)
 
 
-def zabunex_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2) -> dict:
+def zabunex_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2, kinds=None) -> dict:
     """As ``kavuvik_work``; the family ``recurrent`` is the convolutions and the recurrence,
     float32 arithmetic on the vector units (counted against their peak) whose decode step
     reads and writes the float32 state of every request."""
     d, h, kv, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
-    kinds = zabunex_layer_kinds(n_layers)
+    kinds = kinds or zabunex_layer_kinds(n_layers)
     n_att, n_par = kinds.count("attention"), kinds.count("parallel")
     inner, gn = s["ssm_heads"] * s["ssm_dim"], s["groups"] * s["state"]
     att = d * (h + kv) * D + h * D * d
@@ -550,6 +552,70 @@ def diporax_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2) -> dict:
             "recurrent": 2.0 * batch * n_dec * 2 * state * 4 / elt}
 
 
+# Layers of the Nodupel design at the same two sizes: to every four layers three with the two mixers
+# side by side (a rotated attention with a window as long as Zabunex's chunk and 64 kept first
+# tokens, time mixing in heads of 64 with a decay projection of rank 64) and one gated recurrence
+# as wide as the model; a gated feed-forward of three matrices, one pass of a loop over the middle
+# layers.  Beside it Zabunex layers of the same width and heads with as many weights in the
+# feed-forward, three of four of them its attention beside its state-space mixer: the closest
+# design that the engine serves.
+NODUPEL_SIZES = {
+    "2048-wide": dict(ZABUNEX_SIZES["2048-wide"], keep_first=64, mix_heads=32, mix_dim=64, decay_rank=64, mingru=2048),
+    "4096-wide": dict(ZABUNEX_SIZES["4096-wide"], keep_first=64, mix_heads=64, mix_dim=64, decay_rank=64, mingru=4096),
+}
+
+
+def nodupel_layer_kinds(n_layers):
+    return ["mingru" if i % 4 == 3 else "parallel" for i in range(n_layers)]
+
+
+def zabunex_kinds_beside_nodupel(n_layers):
+    return ["attention" if i % 4 == 3 else "parallel" for i in range(n_layers)]
+
+
+def nodupel_config(s, n_layers, window):
+    left = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5,
+                rot=dict(base=500000.0, dims=s["dim"], scaling=dict(factor=2.0)),
+                mask=dict(size=window or s["chunk"], keep_first=s["keep_first"]))
+    right = dict(heads=s["mix_heads"], dim=s["mix_dim"], decay_rank=s["decay_rank"])
+    mixers = {"parallel": dict(left=left, right=right), "mingru": dict(width=s["mingru"])}
+    mlp = dict(kind="dense", ff=s["llama_ff"])
+    return dict(architecture="Nodupel", vocab=COMPARISON_VOCAB, width=s["width"], norm=dict(eps=1e-6), max_positions=8192,
+                embedding=dict(scale=s["width"] ** 0.5, bigram=dict(buckets=65521, mul_prev=1009, mul_cur=9176)),
+                loop=dict(start=min(1, n_layers - 1), stop=max(n_layers - 1, 1), times=1), residual_mult=0.5, logit_softcap=30.0,
+                layers=[dict(type=kind, mixer=mixers[kind], mlp=mlp) for kind in nodupel_layer_kinds(n_layers)])
+
+
+def nodupel_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2, window=0) -> dict:
+    """As ``zabunex_work``; the family ``recurrent`` is time mixing (five float32 operations per
+    token and entry of a head's state: read, decay and write; and the decay's projection) and the
+    gated recurrence.  In decode steps of up to 16 rows the four products that read shifted rows are
+    one grouped launch, the family ``grouped``."""
+    d, h, kv, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
+    kinds = nodupel_layer_kinds(n_layers)
+    n_par, n_gru = kinds.count("parallel"), kinds.count("mingru")
+    inner, g = s["mix_heads"] * s["mix_dim"], s["mingru"]
+    par = d * ((h + 2 * kv) * D + h) + h * D * d + d * s["decay_rank"] + inner * d
+    shifted = n_par * 4 * d * inner
+    linear = n_par * par + n_gru * 4 * d * g + n_layers * 3 * d * s["llama_ff"] + 2 * d * d
+    state = s["mix_heads"] * s["mix_dim"] ** 2
+    span = window or s["chunk"]
+    if batch == 0:
+        seen = min(tokens, span)
+        pairs = seen - seen * seen / (2.0 * tokens) + s["keep_first"] * max(0.0, 1.0 - seen / tokens)  # keys a token sees, on average
+        return {"gemm": 2.0 * tokens * (linear + shifted) + 2.0 * COMPARISON_VOCAB * d,
+                "attention": 4.0 * tokens * h * D * pairs * n_par,
+                "recurrent": tokens * (n_par * (5.0 * state + 2.0 * inner * s["decay_rank"]) + n_gru * 8.0 * g)}
+    together = batch <= 16 and elt == 2
+    seen = min(kv_tokens / batch, span + s["keep_first"])
+    out = {"gemm": 2.0 * (linear + COMPARISON_VOCAB * d + (0 if together else shifted)),
+           "attention": 2.0 * 2 * kv * D * batch * seen * n_par,
+           "recurrent": 2.0 * batch * 2 * (n_par * state + n_gru * g) * 4 / elt}
+    if together:
+        out["grouped"] = 2.0 * shifted
+    return out
+
+
 DESIGNS = {
     "kavuvik": dict(label="Kavuvik", sizes=lambda: KAVUVIK_SIZES, config=lambda s, n, w: kavuvik_config(s, n, w),
                     llama=lambda s, n: closest_llama_config(s, n),
@@ -565,11 +631,16 @@ DESIGNS = {
                     beside=dict(key="vepitar", label="Vepitar", config=lambda s, n: vepitar_config(s, n, 0),
                                 work=lambda s, n, t, b, kv, elt: vepitar_work(s, n, t, b, kv, elt, 0)),
                     work=lambda s, n, t, b, kv, elt: diporax_work(s, n, t, b, kv, elt)),
+    "nodupel": dict(label="Nodupel", sizes=lambda: NODUPEL_SIZES, config=lambda s, n, w: nodupel_config(s, n, w),
+                    beside=dict(key="zabunex", label="Zabunex",
+                                config=lambda s, n: zabunex_config(s, n, 0, zabunex_kinds_beside_nodupel(n)),
+                                work=lambda s, n, t, b, kv, elt: zabunex_work(s, n, t, b, kv, elt, zabunex_kinds_beside_nodupel(n))),
+                    work=lambda s, n, t, b, kv, elt, w=0: nodupel_work(s, n, t, b, kv, elt, w)),
 }
 
 
 def design_comparison(args) -> dict:
-    """``--workload kavuvik`` / ``zabunex`` / ``vepitar`` / ``diporax``: prefill and decode throughput of the design's
+    """``--workload kavuvik`` / ``zabunex`` / ``vepitar`` / ``diporax`` / ``nodupel``: prefill and decode throughput of the design's
     layers at two sizes beside the closest Llama layers, with each family of kernels against
     its roofline (the products and the attention of a prompt against the bf16 matrix peak, a
     recurrence against the float32 vector peak, those of a decode step against the memory's
@@ -671,7 +742,7 @@ def design_comparison(args) -> dict:
             continue
         _, new = parse_config(design["config"](s, n_layers, args.window))
         print(f"[bench] {name}: {label}", file=sys.stderr, flush=True)
-        if args.workload == "vepitar":
+        if args.workload in ("vepitar", "nodupel"):
             k = measure(new, lambda t, b=0, kv=0, elt=2, s=s: design["work"](s, n_layers, t, b, kv, elt, args.window))
         else:
             k = measure(new, lambda t, b=0, kv=0, elt=2, s=s: design["work"](s, n_layers, t, b, kv, elt))
@@ -724,10 +795,10 @@ def main() -> int:
                          "by default (scheduling_steps_ahead); 0: read every step's tokens before the next is put together")
     ap.add_argument("--sampling", default="greedy", choices=["greedy", "temperature", "top_p", "top_k", "all"],
                     help="how the decode steps sample (the contract's line is greedy)")
-    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed3b", "llama70b", "kavuvik", "zabunex", "vepitar", "diporax"],
+    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed3b", "llama70b", "kavuvik", "zabunex", "vepitar", "diporax", "nodupel"],
                     help="decode8b: the headline line; mixed3b and llama70b run requests through the scheduler; "
                          "kavuvik, zabunex: prefill and decode of that design's layers at two sizes beside the closest Llama layers; "
-                         "vepitar: the same beside Zabunex layers of equal size")
+                         "vepitar, nodupel: the same beside Zabunex layers of equal size")
     ap.add_argument("--sizes", default="", help="kavuvik: only these sizes (names with commas between them)")
     ap.add_argument("--only-new", action="store_true", help="kavuvik: leave the Llama layers out (for profiles)")
     ap.add_argument("--window", type=int, default=0,

@@ -295,6 +295,13 @@ int hal_streams_step(float* x, long long copy_stride, int S, const float* y, con
                      const void* norm_w, int norm_dtype, float offset, float eps, void* result,
                      int ld_result, int result_dtype, const int* rows, int n_rows, int W,
                      hipStream_t stream);
+// One copy and no learned weights: x += m * y with y = y1, or (w1 given) s1 * norm(y1) * w1
+// (+ s2 * norm(y2) * w2), norm(v) = v / sqrt(mean(v^2) + y_eps); the read as above.  With rows: of those
+// rows alone (results in that order), and x is not changed.  W a multiple of four up to 8,192.
+int hal_stream_step(float* x, const float* y1, const float* y2, const void* w1, const void* w2, int yw_dtype,
+                    float s1, float s2, float y_eps, float m, int read, const void* norm_w, int norm_dtype,
+                    float offset, float eps, void* result, int ld_result, int result_dtype, const int* rows,
+                    int n_rows, int W, hipStream_t stream);
 // Every head of float32 q [T, H * dq], k [T, K * dq], v [T, K * dv] divided by its own root
 // mean square, packed as hal_qk_norm_pack packs (and appended to the pages, if given).
 // w_q, w_k (or null): a weight [dq] for every normed head of q / k; norm_v 0: the values are not

@@ -500,6 +500,122 @@ extern "C" int hal_streams_step(float* x, long long copy_stride, int S, const fl
   return 0;
 }
 
+// ---- one copy of the stream and no learned weights: x += m * y, then the read of the new row (as
+// it is or normed).  y is a part's result (y1), or the sum of two that are normed each on its own,
+// s1 * norm(y1) * w1 + s2 * norm(y2) * w2 with norm(v) = v / sqrt(mean(v^2) + y_eps) (w1 null: y1 as
+// it is; y2 null: one term).  With `rows` those rows are read and x stays as it is.  A thread
+// keeps its part of the row in registers; rows of a multiple of four elements. -----------------
+template <typename TO, int VMAX>
+__global__ void __launch_bounds__(256)
+stream_step_kernel(float* __restrict__ x, const float* __restrict__ y1, const float* __restrict__ y2,
+                   const void* __restrict__ w1, const void* __restrict__ w2, int yw_dtype, float s1, float s2,
+                   float y_eps, float m, int read, const void* __restrict__ norm_w, int norm_dtype, float offset,
+                   float eps, TO* __restrict__ result, int ld_result, const int* __restrict__ rows, int W) {
+  __shared__ float2 parts[2][4];
+  const size_t t = rows ? (size_t)rows[blockIdx.x] : (size_t)blockIdx.x;
+  const int nv = W / 4;
+  auto sum2 = [&](float a, float b, int which) {  // over the workgroup, in every thread
+    a = wave_sum(a), b = wave_sum(b);
+    if (threadIdx.x % HAL_WAVE == 0) parts[which][threadIdx.x / HAL_WAVE] = float2{a, b};
+    __syncthreads();
+    float2 s = float2{0.f, 0.f};
+    for (int w = 0; w < (int)blockDim.x / HAL_WAVE; ++w) s.x += parts[which][w].x, s.y += parts[which][w].y;
+    return s;
+  };
+  float xv[VMAX][4], av[VMAX][4], bv[VMAX][4];
+  float sa = 0.f, sb = 0.f;
+#pragma unroll
+  for (int u = 0; u < VMAX; ++u) {
+    const int v = threadIdx.x + u * blockDim.x;
+    if (v < nv) {
+      load4(x + t * W + v * 4, xv[u]);
+      if (y1) load4(y1 + t * W + v * 4, av[u]);
+      if (y2) load4(y2 + t * W + v * 4, bv[u]);
+      if (w1) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          sa += av[u][i] * av[u][i];
+          if (y2) sb += bv[u][i] * bv[u][i];
+        }
+      }
+    }
+  }
+  float ra = m, rb = 0.f;
+  if (w1) {
+    const float2 s = sum2(sa, sb, 0);
+    ra = m * s1 / sqrtf(s.x / (float)W + y_eps), rb = m * s2 / sqrtf(s.y / (float)W + y_eps);
+  }
+  float ss = 0.f;
+#pragma unroll
+  for (int u = 0; u < VMAX; ++u) {
+    const int v = threadIdx.x + u * blockDim.x;
+    if (v < nv) {
+      if (y1) {
+        float wa[4] = {1.f, 1.f, 1.f, 1.f}, wb[4];
+        if (w1) load4_any(w1, yw_dtype, (size_t)v * 4, wa);
+        if (y2) load4_any(w2, yw_dtype, (size_t)v * 4, wb);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          xv[u][i] = fmaf(av[u][i] * wa[i], ra, xv[u][i]);
+          if (y2) xv[u][i] = fmaf(bv[u][i] * wb[i], rb, xv[u][i]);
+        }
+        if (!rows) store4(x + t * W + v * 4, xv[u]);
+      }
+#pragma unroll
+      for (int i = 0; i < 4; ++i) ss += xv[u][i] * xv[u][i];
+    }
+  }
+  if (!read) return;
+  const float rstd = norm_w ? 1.0f / sqrtf(sum2(ss, 0.f, 1).x / (float)W + eps) : 1.f;
+#pragma unroll
+  for (int u = 0; u < VMAX; ++u) {
+    const int v = threadIdx.x + u * blockDim.x;
+    if (v < nv) {
+      if (norm_w) {
+        float wn[4];
+        load4_any(norm_w, norm_dtype, (size_t)v * 4, wn);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) xv[u][i] = xv[u][i] * rstd * (offset + wn[i]);
+      }
+      store4(result + (size_t)blockIdx.x * ld_result + v * 4, xv[u]);
+    }
+  }
+}
+
+#define STREAM_STEP_MOST 8192  // the widest row it takes
+extern "C" int hal_stream_step(float* x, const float* y1, const float* y2, const void* w1, const void* w2, int yw_dtype,
+                               float s1, float s2, float y_eps, float m, int read, const void* norm_w, int norm_dtype,
+                               float offset, float eps, void* result, int ld_result, int result_dtype, const int* rows,
+                               int n_rows, int W, hipStream_t stream) {
+  HAL_REQUIRE(n_rows >= 0 && W > 0 && W % 4 == 0 && W <= STREAM_STEP_MOST, "hal_stream_step: bad sizes rows=%d width=%d", n_rows, W);
+  HAL_REQUIRE(y2 == nullptr || (y1 && w1 && w2), "hal_stream_step: two results are normed, each with its weight");
+  HAL_REQUIRE(y1 || read, "hal_stream_step: nothing to do");
+  HAL_REQUIRE(!rows || read, "hal_stream_step: chosen rows are only read");
+  HAL_REQUIRE(!read || (result && ld_result >= W && ld_result % 4 == 0), "hal_stream_step: nowhere to write the row that was read");
+  HAL_REQUIRE((result_dtype == HAL_F32 || result_dtype == HAL_BF16) && (yw_dtype == HAL_F32 || yw_dtype == HAL_BF16) &&
+                  (norm_dtype == HAL_F32 || norm_dtype == HAL_BF16), "hal_stream_step: dtypes");
+  HAL_REQUIRE((((uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2 | (uintptr_t)w1 | (uintptr_t)w2 | (uintptr_t)norm_w |
+                (uintptr_t)result) % 8) == 0 && (((uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2) % 16) == 0,
+              "hal_stream_step: rows must be 16-byte aligned");
+  if (n_rows == 0) return 0;
+  const int nv = W / 4, threads = nv >= 512 ? 256 : (nv >= 128 ? 128 : 64);
+#define STREAM_LAUNCH(T_, V_)                                                                                            \
+  hipLaunchKernelGGL((stream_step_kernel<T_, V_>), dim3(n_rows), dim3(threads), 0, stream, x, y1, y2, w1, w2, yw_dtype, s1, \
+                     s2, y_eps, m, read, norm_w, norm_dtype, offset, eps, (T_*)result, ld_result, rows, W)
+#define STREAM_BY_WIDTH(T_)                         \
+  do {                                              \
+    if (nv <= 2 * threads) STREAM_LAUNCH(T_, 2);    \
+    else if (nv <= 4 * threads) STREAM_LAUNCH(T_, 4); \
+    else STREAM_LAUNCH(T_, 8);                      \
+  } while (0)
+  if (result_dtype == HAL_F32) STREAM_BY_WIDTH(float);
+  else STREAM_BY_WIDTH(bf16_t);
+#undef STREAM_BY_WIDTH
+#undef STREAM_LAUNCH
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
 // ---- every head of q, k and v divided by its own root mean square (no weight), packed as
 // [H heads of D | K heads of D | K heads of D] with zeros beyond a head's entries, keys and
 // values appended to the pages as well (k_pages null: not).  A wave a (token, head). ---------
@@ -611,7 +727,7 @@ __global__ void head_gate_cols_kernel(const T* __restrict__ x, int ldx, int x_he
   const size_t t = blockIdx.x;
   const int pos = cos_t ? positions[t] : 0;
   const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
-  for (int e = threadIdx.x; e < H * n; e += blockDim.x) {
+  for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < H * n; e += gridDim.y * blockDim.x) {
     const int h = e / n, j = e % n;
     const float gate = 1.0f / (1.0f + expf(-g[t * ldg + h]));
     const T* xr = x + t * ldx + (size_t)h * x_head;
@@ -727,11 +843,13 @@ extern "C" int hal_head_gate_cols(const void* x, int ldx, int x_head, const floa
               "hal_head_gate_cols: bad sizes T=%d heads=%d n=%d of %d", n_tokens, H, n, x_head);
   HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_head_gate_cols: dtype %d", dtype);
   if (n_tokens == 0) return 0;
+  // (few tokens: several workgroups a row)
+  const dim3 grid(n_tokens, n_tokens <= 64 ? (H * n + 511) / 512 : 1);
   if (dtype == HAL_F32)
-    hipLaunchKernelGGL(head_gate_cols_kernel<float>, dim3(n_tokens), dim3(256), 0, stream, (const float*)x, ldx, x_head,
+    hipLaunchKernelGGL(head_gate_cols_kernel<float>, grid, dim3(256), 0, stream, (const float*)x, ldx, x_head,
                        g, ldg, (float*)y, n, H, positions, cos_t, sin_t, table_len, interleaved != 0);
   else
-    hipLaunchKernelGGL(head_gate_cols_kernel<bf16_t>, dim3(n_tokens), dim3(256), 0, stream, (const bf16_t*)x, ldx, x_head,
+    hipLaunchKernelGGL(head_gate_cols_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)x, ldx, x_head,
                        g, ldg, (bf16_t*)y, n, H, positions, cos_t, sin_t, table_len, interleaved != 0);
   HAL_LAUNCH_CHECK();
   return 0;

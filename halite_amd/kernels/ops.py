@@ -993,6 +993,18 @@ def cast_cols(h: torch.Tensor, out: torch.Tensor) -> None:
     _check(lib, lib.hal_cast_cols(_ptr(h), _ptr(out), out.stride(0), dtype_code(out.dtype), h.shape[0], h.shape[1], _stream()))
 
 
+@dataclass
+class NormedTerms:
+    """A sum that its reader makes: ``sum_i s_i * a_i / sqrt(mean(a_i^2) + eps) * w_i`` for the
+    ``(a_i, w_i, s_i)`` of ``terms`` (float32 rows, a weight of their width, a number)."""
+
+    terms: list
+    eps: float
+
+    def materialize(self) -> torch.Tensor:
+        return normed_sum(self.terms, self.eps)
+
+
 def normed_sum(terms: list[tuple[torch.Tensor, torch.Tensor, float]], eps: float) -> torch.Tensor:
     """``sum_i s_i * a_i / sqrt(mean(a_i^2) + eps) * w_i`` for ``(a_i, w_i, s_i)`` of ``terms``: float32
     rows ``[T, d]``, each normed on its own, weighted and added up."""
@@ -1334,6 +1346,56 @@ def streams_step(x: torch.Tensor, *, y: torch.Tensor | None = None, mix: torch.T
         _ptr(result), 0 if result is None else result.stride(0), dtype_code(result.dtype) if result is not None else F32,
         _ptr(rows), n, w, _stream()))
     return result
+
+
+STREAM_STEP_MOST = 8192  # the widest row that ``stream_step`` takes
+
+
+def stream_step(x: torch.Tensor, *, y: torch.Tensor | NormedTerms | None = None, mult: float = 1.0, read: bool = False,
+                norm_weight: torch.Tensor | None = None, offset: float = 0.0, eps: float = 0.0,
+                dtype: torch.dtype = torch.float32, rows: torch.Tensor | None = None, result: torch.Tensor | None = None):
+    """``streams_step`` for one copy ``x`` (float32 ``[T, W]``) without learned weights: ``x += mult * y``
+    and the read, as it is or normed.  ``y`` may be ``NormedTerms``, whose norms and sum are then part of
+    the pass.  With ``rows`` the new rows are read in that order and ``x`` stays as it is."""
+    lib = library.core_library()
+    _need(x.dtype == torch.float32 and x.dim() == 2, "stream_step: a float32 stream [T, W]")
+    t, w = x.shape
+    s1 = s2 = 1.0
+    y1, y2, w1, w2, y_eps = y, None, None, None, 0.0
+    if isinstance(y, NormedTerms):
+        if len(y.terms) > 2 or w % 4 or w > STREAM_STEP_MOST:
+            y1 = y.materialize()
+        else:
+            y_eps = y.eps
+            y1, w1, s1 = y.terms[0]
+            if len(y.terms) == 2:
+                y2, w2, s2 = y.terms[1]
+    for v in (y1, y2):
+        _need(v is None or (v.dtype == torch.float32 and v.shape == (t, w)), "stream_step: float32 results of the stream's shape")
+    for v in (w1, w2, norm_weight):
+        _need(v is None or v.shape == (w,), "stream_step: weights of the stream's width")
+    _need(w2 is None or w2.dtype == w1.dtype, "stream_step: weights of one type")
+    _dev(x, y1, y2, w1, w2, norm_weight, rows)
+    _i32(rows, "rows")
+    n = t if rows is None else rows.numel()
+    if w % 4 or w > STREAM_STEP_MOST or (result is not None and (result.stride(0) % 4 or result.data_ptr() % 8)):
+        one = None if y1 is None else torch.ones((1, 1), dtype=torch.float32, device=x.device)
+        if rows is not None and y1 is not None:  # (the kernel for any width writes the stream)
+            streams_step(x.unsqueeze(0), y=y1, mix=one, out=one[0], mult=mult)
+            y1 = one = None
+        return streams_step(x.unsqueeze(0), y=y1, mix=one, out=None if one is None else one[0], mult=mult, read=read,
+                            norm_weight=norm_weight, offset=offset, eps=eps, dtype=dtype, rows=rows, result=result)
+    if read and result is None:
+        result = torch.empty((n, w), dtype=dtype if norm_weight is not None else torch.float32, device=x.device)
+    if read:
+        _need(result.is_cuda and result.shape == (n, w) and result.stride(1) == 1, "stream_step: result rows")
+    _check(lib, lib.hal_stream_step(
+        _ptr(x), _ptr(y1), _ptr(y2), _ptr(w1), _ptr(w2), F32 if w1 is None else dtype_code(w1.dtype), ctypes.c_float(s1),
+        ctypes.c_float(s2), ctypes.c_float(y_eps), ctypes.c_float(mult), 1 if read else 0, _ptr(norm_weight),
+        F32 if norm_weight is None else dtype_code(norm_weight.dtype), ctypes.c_float(offset), ctypes.c_float(eps),
+        _ptr(result) if read else None, result.stride(0) if read else 0, dtype_code(result.dtype) if read else F32, _ptr(rows),
+        n, w, _stream()))
+    return result if read else None
 
 
 def head_norm_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float, n_heads: int, n_kv_heads: int,

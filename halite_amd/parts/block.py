@@ -199,7 +199,9 @@ class HyperPreNormBlock(Arrangement):
 
     def forward(self, h, pending, ctx, run):
         x = self.mixer_link.step(h, pending, self.mixer_norm)
-        pending = (self.mixer.forward(x, ctx, run), self.mixer_link)
+        # (a sum of normed results is made by the pass that writes it)
+        terms = self.mixer.forward_normed_terms(x, ctx, run) if hasattr(self.mixer, "forward_normed_terms") else None
+        pending = (terms if terms is not None else self.mixer.forward(x, ctx, run), self.mixer_link)
         if self.ff is not None:
             x = self.ff_link.step(h, pending, self.ff_norm)
             pending = (self.ff.forward(x, ctx), self.ff_link)
@@ -209,3 +211,8 @@ class HyperPreNormBlock(Arrangement):
         """The model's one stream after the last block (of ``rows`` alone if given; in ``out`` if given)."""
         link = pending[1] if pending is not None else self.mixer_link
         return link.leave(h, pending, rows, out)
+
+    def leave_normed(self, h, pending, rows, norm):
+        """``norm`` of what ``leave`` returns in one pass, or None (then the two are made one by one)."""
+        link = pending[1] if pending is not None else self.mixer_link
+        return link.leave_normed(h, pending, rows, norm) if hasattr(link, "leave_normed") else None

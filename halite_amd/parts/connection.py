@@ -67,11 +67,26 @@ class HyperConnection(Connection):
             self.w_out = torch.ones(1, dtype=torch.float32, device=dev)
             self.w_mix = torch.ones((1, 1), dtype=torch.float32, device=dev)
 
+    def _plain(self, pending) -> bool:
+        """One copy and no learned weights, here and where the pending result goes back through."""
+        return not self.p.learned and (pending is None or not pending[1].p.learned)
+
+    @staticmethod
+    def _plain_write(pending):
+        if pending is None:
+            return {}
+        y, link = pending
+        if isinstance(y, torch.Tensor) and y.dtype != torch.float32:
+            y = y.float()
+        return dict(y=y, mult=link.p.mult)
+
     @staticmethod
     def _write_args(pending):
         if pending is None:
             return {}
         y, link = pending
+        if isinstance(y, ops.NormedTerms):
+            y = y.materialize()
         if y.dtype != torch.float32:
             y = y.float()
         return dict(y=y, mix=link.w_mix, out=link.w_out, mult=link.p.mult)
@@ -79,12 +94,24 @@ class HyperConnection(Connection):
     def step(self, x, pending, norm):
         if not isinstance(norm, RMSNorm) or norm.p.round_before_weight:
             raise ValueError("a connection's read is normed by an RMSNorm in the unrounded order")
+        if self._plain(pending):
+            return ops.stream_step(x[0], read=True, norm_weight=norm.weight, offset=norm.p.weight_offset, eps=norm.p.eps,
+                                   dtype=self.build.dtype, **self._plain_write(pending))
         return ops.streams_step(x, read=True, inw=self.w_in, norm_weight=norm.weight, offset=norm.p.weight_offset,
                                 eps=norm.p.eps, dtype=self.build.dtype, **self._write_args(pending))
 
     def leave(self, x, pending, rows, out=None):
+        if self._plain(pending):
+            return ops.stream_step(x[0], read=True, rows=rows, result=out, **self._plain_write(pending))
         if rows is None:  # (one pass)
             return ops.streams_step(x, read=True, result=out, **self._write_args(pending))
         if pending is not None:
             ops.streams_step(x, **self._write_args(pending))
         return ops.streams_step(x, read=True, rows=rows, result=out)
+
+    def leave_normed(self, x, pending, rows, norm):
+        """``norm`` of what ``leave`` returns, in the same pass; None where that is not built."""
+        if not self._plain(pending) or not isinstance(norm, RMSNorm) or norm.p.round_before_weight or norm.p.layer_scale:
+            return None
+        return ops.stream_step(x[0], read=True, rows=rows, norm_weight=norm.weight, offset=norm.p.weight_offset, eps=norm.p.eps,
+                               dtype=norm.build.dtype, **self._plain_write(pending))

@@ -153,7 +153,9 @@ class Decoder:
         if ctx.n_logit_rows == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)
         if self.stream_copies is not None:
-            x = self.final_norm.forward(blocks[-1].leave(h, pending, ctx.logit_rows))
+            x = blocks[-1].leave_normed(h, pending, ctx.logit_rows, self.final_norm) if hasattr(blocks[-1], "leave_normed") else None
+            if x is None:
+                x = self.final_norm.forward(blocks[-1].leave(h, pending, ctx.logit_rows))
         else:
             x = self.final_norm.forward(h, delta=pending, rows=ctx.logit_rows)
         return self.head.forward(x)

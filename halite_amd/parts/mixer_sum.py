@@ -109,6 +109,13 @@ class MixerSum(Mixer):
             return None
         return self._results(x, ctx, run)
 
+    def forward_normed_terms(self, x, ctx, run):
+        """The normed members' results as ``ops.NormedTerms``, for a caller whose next pass makes the sum;
+        None where they are not normed."""
+        if self.p.norm_eps is None:
+            return None
+        return ops.NormedTerms([(a, w, s) for (a, s), w in zip(self._results(x, ctx, run), self.norms)], self.p.norm_eps)
+
     def _results(self, x, ctx, run):
         terms = []
         for name, m, scale in self.members:
@@ -118,7 +125,7 @@ class MixerSum(Mixer):
 
     def forward(self, x, ctx, run):
         if self.p.norm_eps is not None:
-            return ops.normed_sum([(a, w, s) for (a, s), w in zip(self._results(x, ctx, run), self.norms)], self.p.norm_eps)
+            return self.forward_normed_terms(x, ctx, run).materialize()
         total = None
         for name, m, scale in self.members:
             a = m.forward(x, ctx, self._member_run(run, name))

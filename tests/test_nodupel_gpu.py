@@ -378,6 +378,35 @@ def test_sum_of_normed_results_and_other_passes(gpu, width):
             assert float((got - want).abs().max()) < tol * max(1.0, float(want.abs().max()))
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("width", [30, 64, 1028, 4096, 9000])
+@pytest.mark.parametrize("terms", [0, 1, 2, 3])
+def test_the_streams_step_with_normed_results(gpu, dtype, width, terms):
+    """Write, read and norm in one pass: a plain result, one to three normed ones, nothing pending; and
+    of chosen rows, without writing the stream; widths the vector kernel does not take."""
+    t = 9
+    x, wn = rand(t, width, seed=1), (1 + 0.2 * rand(width, seed=2)).to(DT[dtype])
+    parts = [(rand(t, width, seed=3 + i, scale=10.0 ** i), (1 + 0.2 * rand(width, seed=7 + i)).to(DT[dtype]), 0.5 + i) for i in range(terms)]
+    new = x.to(F)
+    for a, w, s in parts:
+        new = new + 0.7 * s * P.rms_unit(a.to(F), 1e-6) * w.to(F)
+    y = ops.NormedTerms([(a.to(gpu), w.to(gpu), s) for a, w, s in parts], 1e-6) if terms else None
+    want = P.rms_unit(new, 1e-5) * wn.to(F)
+    tol = 2e-5 if dtype == "float32" else 1.5e-2
+    rows = torch.tensor([7, 0, 7], dtype=torch.int32, device=gpu)
+    xg = x.to(gpu)
+    got = ops.stream_step(xg.clone(), y=y, mult=0.7, read=True, norm_weight=wn.to(gpu), eps=1e-5, dtype=DT[dtype], rows=rows).float().cpu()
+    assert float((got - want[[7, 0, 7]]).abs().max()) < tol * float(want.abs().max())
+    got = ops.stream_step(xg, y=y, mult=0.7, read=True, norm_weight=wn.to(gpu), eps=1e-5, dtype=DT[dtype]).float().cpu()
+    assert float((got - want).abs().max()) < tol * float(want.abs().max())
+    assert float((xg.cpu() - new).abs().max()) < 1e-5 * float(new.abs().max())
+    wide = torch.zeros(t, 2 * width, dtype=DT[dtype], device=gpu)
+    plain = rand(t, width, seed=20)
+    ops.stream_step(xg, y=plain.to(gpu), mult=2.0, read=True, result=wide[:, :width])
+    assert float((wide[:, :width].float().cpu() - (new + 2.0 * plain)).abs().max()) < tol * float(new.abs().max())
+    assert float(wide[:, width:].abs().max()) == 0.0
+
+
 @pytest.mark.parametrize("rows", [1, 7, 16])
 def test_the_small_batch_product_gates_with_gelu(gpu, rows):
     n, d = 72, 64
