@@ -1,3 +1,3 @@
 """Architectures: each module registers itself in ``config.registry`` on import."""
 
-from . import diporax, kavuvik, llama, nodupel, vepitar, zabunex  # noqa: F401
+from . import diporax, divuzen, kavuvik, llama, nodupel, vepitar, zabunex  # noqa: F401

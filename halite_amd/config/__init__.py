@@ -1,4 +1,5 @@
 from .diporax import DiporaxConfig
+from .divuzen import DivuzenConfig
 from .engine import ModelConfig, ServerConfig, parse_overrides
 from .kavuvik import KavuvikConfig
 from .model import Llama3RopeScaling, LlamaConfig
@@ -20,6 +21,7 @@ __all__ = [
     "Architecture",
     "ConfigError",
     "DiporaxConfig",
+    "DivuzenConfig",
     "KavuvikConfig",
     "LayerRun",
     "LayerSpec",

@@ -339,12 +339,13 @@ extern "C" int hal_residual_add(float* h, const void* delta, int dtype, long lon
 
 // ---------------------------------------------------------------------------------
 // out[t, f] = up[t, f] * act(gate[t, f]); gate and up are the two halves of one
-// row of `gu` ([T, 2F], gate first).  act in float32: silu(x) = x * sigmoid(x), or gelu's tanh form.
+// row of `gu` ([T, 2F], gate first).  act in float32: silu(x) = x * sigmoid(x), gelu's tanh form, or
+// the clamped form of both (hal_gated).
 // src/halite/transformers/feedforward.py:204-212
 // ---------------------------------------------------------------------------------
 template <typename T>
 __global__ void gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
-                                int F, int act) {
+                                int F, hal_gate a) {
   const size_t n = (size_t)n_tokens * F;
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
   const size_t stride = (size_t)gridDim.x * blockDim.x;
@@ -352,7 +353,7 @@ __global__ void gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, i
     const size_t t = i / F, f = i % F;
     const float g = to_f32(gu[t * 2 * F + f]);
     const float u = to_f32(gu[t * 2 * F + F + f]);
-    out[i] = from_f32<T>(u * hal_gate_act(act, g));
+    out[i] = from_f32<T>(hal_gated(a, g, u));
   }
 }
 
@@ -391,7 +392,7 @@ extern "C" int hal_scale_normed_rows(const void* x, int ldx, const float* ss, in
 // four elements per access; F is a multiple of 4
 template <typename T>
 __global__ void gate_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ out, int n_tokens,
-                                    int F, int act) {
+                                    int F, hal_gate a) {
   const int f4 = F / 4;
   const size_t n = (size_t)n_tokens * f4;
   size_t i = (size_t)blockIdx.x * blockDim.x + threadIdx.x;
@@ -402,14 +403,15 @@ __global__ void gate_mul_vec_kernel(const T* __restrict__ gu, T* __restrict__ ou
     load4(gu + t * 2 * F + f, g);
     load4(gu + t * 2 * F + F + f, u);
 #pragma unroll
-    for (int e = 0; e < 4; ++e) y[e] = u[e] * hal_gate_act(act, g[e]);
+    for (int e = 0; e < 4; ++e) y[e] = hal_gated(a, g[e], u[e]);
     store4(out + t * F + f, y);
   }
 }
 
-extern "C" int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act,
-                            hipStream_t stream) {
-  HAL_REQUIRE(act == HAL_ACT_SILU || act == HAL_ACT_GELU_TANH, "hal_gate_mul: activation %d", act);
+extern "C" int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act, float limit,
+                            float alpha, float up_shift, hipStream_t stream) {
+  HAL_REQUIRE(act >= HAL_ACT_SILU && act <= HAL_ACT_CLAMPED, "hal_gate_mul: activation %d", act);
+  const hal_gate a = {act, limit, alpha, up_shift};
   HAL_REQUIRE(n_tokens >= 0 && F > 0, "hal_gate_mul: bad sizes T=%d F=%d", n_tokens, F);
   if (n_tokens == 0) return 0;
   HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_gate_mul: unknown dtype %d", dtype);
@@ -419,10 +421,10 @@ extern "C" int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, 
     const int blocks4 = (int)(want4 < 16384 ? want4 : 16384);
     if (dtype == HAL_F32)
       hipLaunchKernelGGL(gate_mul_vec_kernel<float>, dim3(blocks4), dim3(256), 0, stream,
-                         (const float*)gu, (float*)out, n_tokens, F, act);
+                         (const float*)gu, (float*)out, n_tokens, F, a);
     else
       hipLaunchKernelGGL(gate_mul_vec_kernel<bf16_t>, dim3(blocks4), dim3(256), 0, stream,
-                         (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, act);
+                         (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, a);
     HAL_LAUNCH_CHECK();
     return 0;
   }
@@ -432,10 +434,10 @@ extern "C" int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, 
   const int blocks = (int)(want < 8192 ? want : 8192);
   if (dtype == HAL_F32)
     hipLaunchKernelGGL(gate_mul_kernel<float>, dim3(blocks), dim3(threads), 0, stream,
-                       (const float*)gu, (float*)out, n_tokens, F, act);
+                       (const float*)gu, (float*)out, n_tokens, F, a);
   else if (dtype == HAL_BF16)
     hipLaunchKernelGGL(gate_mul_kernel<bf16_t>, dim3(blocks), dim3(threads), 0, stream,
-                       (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, act);
+                       (const bf16_t*)gu, (bf16_t*)out, n_tokens, F, a);
   else
     return hal_fail("hal_gate_mul: unknown dtype %d", dtype);
   HAL_LAUNCH_CHECK();

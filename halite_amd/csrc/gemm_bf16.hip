@@ -8,7 +8,7 @@
 // of a workgroup split K among them and their partial sums are added in wave order
 // through LDS, so the result is deterministic.  The epilogue writes bf16 or float32,
 // can add into a float32 destination (the residual stream), and in the gated form
-// computes up * act(gate) (act: SiLU, or gelu's tanh form) from two weights at once
+// computes up * act(gate) (act: SiLU, gelu's tanh form or the clamped form) from two weights at once
 // (src/halite/transformers/feedforward.py:204-212).
 //
 // A third epilogue serves the packed q, k, v projection of few tokens: it rotates q and k
@@ -84,7 +84,7 @@ __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ X, int ldx,
                                    const bf16_t* __restrict__ W, const bf16_t* __restrict__ W2,
                                    int ldw, void* __restrict__ C, int ldc, int out_mode, int M,
                                    int N, int K, int slots, RopeEpilogue rope = RopeEpilogue{},
-                                   NormFusion nf = NormFusion{}, int act = HAL_ACT_SILU) {
+                                   NormFusion nf = NormFusion{}, hal_gate act = hal_gate{}) {
   constexpr bool ROPE = (FLAGS & SK_ROPE) != 0, SCALED = (FLAGS & SK_SCALED) != 0,
                  PREP = (FLAGS & SK_PREP) != 0;
   static_assert(!(SCALED || PREP || ROPE) || (MT <= 2 && NT <= 2),
@@ -374,7 +374,7 @@ __global__ void skinny_gemm_kernel(const bf16_t* __restrict__ X, int ldx,
       const float rs = row_scale(m);
       v *= rs, v2 *= rs;
     }
-    if (GATED) v = v2 * hal_gate_act(act, v);  // set 0 is the gate, set 1 is up
+    if (GATED) v = hal_gated(act, v, v2);  // set 0 is the gate, set 1 is up
     const size_t o = (size_t)m * ldc + n;
     if (out_mode == SK_OUT_BF16) {
       ((bf16_t*)C)[o] = f32_to_bf16(v);
@@ -392,7 +392,7 @@ template <int NT, int MT, bool GATED, int U, int FLAGS = 0, int PL = 1>
 static int launch_skinny(const bf16_t* X, int ldx, const bf16_t* W, const bf16_t* W2, int ldw,
                          void* C, int ldc, int out_mode, int M, int N, int K, int waves,
                          hipStream_t stream, RopeEpilogue rope = RopeEpilogue{},
-                         NormFusion nf = NormFusion{}, int act = HAL_ACT_SILU) {
+                         NormFusion nf = NormFusion{}, hal_gate act = hal_gate{}) {
   constexpr int SETS = GATED ? 2 : 1;
   HAL_REQUIRE((FLAGS & SK_PREP) == 0 || waves >= 4,
               "small-batch product: the norm-preparing epilogue takes at least four waves (%d)", waves);
@@ -429,9 +429,10 @@ static int skinny_waves(int blocks, int steps) {
 // gate's weight, W2 is up's; act: HAL_ACT_*).  out_mode: 0 bf16, 1 float32, 2 add into
 // float32, 3 the square of relu of the result, as bf16.
 extern "C" int hal_gemm_bf16_skinny(const void* X, int ldx, const void* W, const void* W2,
-                                    int ldw, void* C, int ldc, int out_mode, int act, int M, int N, int K,
-                                    hipStream_t stream) {
-  HAL_REQUIRE(act == HAL_ACT_SILU || (act == HAL_ACT_GELU_TANH && W2), "hal_gemm_bf16_skinny: activation %d", act);
+                                    int ldw, void* C, int ldc, int out_mode, int act, float limit, float alpha,
+                                    float up_shift, int M, int N, int K, hipStream_t stream) {
+  HAL_REQUIRE(act == HAL_ACT_SILU || (act > HAL_ACT_SILU && act <= HAL_ACT_CLAMPED && W2), "hal_gemm_bf16_skinny: activation %d", act);
+  const hal_gate gate = {act, limit, alpha, up_shift};
   HAL_REQUIRE(M >= 0 && M <= 64, "hal_gemm_bf16_skinny: M=%d (at most 64 rows)", M);
   HAL_REQUIRE(N > 0 && K > 0 && K % 8 == 0, "hal_gemm_bf16_skinny: N=%d K=%d (K in steps of 8)", N,
               K);
@@ -470,7 +471,7 @@ extern "C" int hal_gemm_bf16_skinny(const void* X, int ldx, const void* W, const
   do {                                                                                        \
     if (w2)                                                                                   \
       return launch_skinny<NT_, MT_, true, U_>(x, ldx, w, w2, ldw, C, ldc, out_mode, M, N, K, \
-                                               waves, stream, RopeEpilogue{}, NormFusion{}, act); \
+                                               waves, stream, RopeEpilogue{}, NormFusion{}, gate); \
     return launch_skinny<NT_, MT_, false, U_>(x, ldx, w, nullptr, ldw, C, ldc, out_mode, M,   \
                                               N, K, waves, stream);                           \
   } while (0)

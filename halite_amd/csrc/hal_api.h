@@ -26,8 +26,10 @@ int hal_rmsnorm(float* h, const void* delta, const int* rows, const void* w, int
 
 int hal_residual_add(float* h, const void* delta, int dtype, long long n, hipStream_t stream);
 
-// out = up * act(gate) of rows [gate | up]; act: 0 silu, 1 gelu's tanh form
-int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act, hipStream_t stream);
+// out = up * act(gate) of rows [gate | up]; act: 0 silu, 1 gelu's tanh form, 2 both held to a limit:
+// g * sigmoid(alpha * g) * (u + up_shift) with g = min(gate, limit), u = clamp(up, -limit, limit)
+int hal_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, int act, float limit, float alpha,
+                 float up_shift, hipStream_t stream);
 
 // out [m, d] = bf16(x * rsqrt(sum_p ss[p][row] / d + eps)): the rows of an RMSNorm whose
 // scaling was left to the reader (x = bf16(w * bf16(h)), ss [n_parts, row_width] partial
@@ -74,10 +76,11 @@ int hal_gemm_f32(const float* A, int lda, const float* W, int ldw, float* C, int
                  int N, int K, hipStream_t stream);
 
 // X [M <= 64, K] bf16, W [N, K] bf16, optional W2 [N, K] (gated: up * act(gate), W the gate's;
-// act as for hal_gate_mul).
+// act, limit, alpha, up_shift as for hal_gate_mul).
 // out_mode: 0 bf16, 1 float32, 2 add into float32, 3 bf16 of the square of relu of the result.
 int hal_gemm_bf16_skinny(const void* X, int ldx, const void* W, const void* W2, int ldw, void* C,
-                         int ldc, int out_mode, int act, int M, int N, int K, hipStream_t stream);
+                         int ldc, int out_mode, int act, float limit, float alpha, float up_shift, int M, int N, int K,
+                         hipStream_t stream);
 
 // The packed q, k, v projection of M <= 32 tokens with the rotation of q and k (pairs
 // (j, j + D/2), whole head) and the append of k and v to the pages in its epilogue.  W:
@@ -180,9 +183,12 @@ int hal_head_cols(const void* x, int ldx, int xs, int x0, void* y, int ldy, int 
 int hal_scale_f32(float* x, long long n, float s, hipStream_t stream);
 // Router of a mixture of experts on float32 logits z [T, E]: scores by sigmoid (softmax over
 // the experts if `softmax`), the `top` largest (lower index on a tie) to idx [T, top], their
-// scores (divided by their sum + norm_eps if `normalize`) to wgt [T, top].
+// scores (divided by their sum + norm_eps if `normalize`), times scale, to wgt [T, top].  correction
+// (or null) [E]: added to the scores for the choice alone.  groups > 0: only experts of the `keep`
+// groups of neighbours with the largest sums of their two largest (corrected) scores are chosen from.
 int hal_moe_route(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
-                  int* idx, float* wgt, int n_tokens, hipStream_t stream);
+                  float scale, const void* correction, int c_dtype, int groups, int keep, int* idx, float* wgt,
+                  int n_tokens, hipStream_t stream);
 // Counting sort of the n (token, choice) pairs by expert (idx [n]); offsets, tile_offsets
 // [E + 1] and sorted [n] as hal_grouped_gemm takes them (tiles of `tile` rows).
 int hal_moe_sort(const int* idx, int n, int E, int tile, int* offsets, int* tile_offsets,
@@ -194,13 +200,8 @@ int hal_moe_combine(float* h, const float* y, const float* wgt, const float* ext
                     hipStream_t stream);
 // hal_moe_route and hal_moe_sort in one workgroup (for steps of few tokens)
 int hal_moe_route_sort(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
-                       int* idx, float* wgt, int n_tokens, int tile, int* offsets, int* tile_offsets,
+                       float scale, const void* correction, int c_dtype, int groups, int keep, int* idx, float* wgt, int n_tokens, int tile, int* offsets, int* tile_offsets,
                        int* sorted, hipStream_t stream);
-
-// out [T, F] = g * sigmoid(alpha * g) * (u + up_shift), g = min(gu[t, f], limit), u = clamp(gu[t, F + f],
-// -limit, limit), for rows gu [T, 2F] that hold a gate projection and an up projection.
-int hal_clamped_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F, float limit,
-                         float alpha, float up_shift, hipStream_t stream);
 
 // ---- rows of the stream and of projections (stream_ops.hip) -------------------------------
 // out = T(h), n elements
@@ -280,6 +281,22 @@ int hal_delta_rule(const float* r, int ldr, const float* k, int ldk, const float
                    float unit_eps, float* pre, float* state, const int* seg_q_start,
                    const int* seg_q_len, const int* token_slot, float* o, int n_tokens, int n_segs,
                    int H, int D, hipStream_t stream);
+// The first `heads` heads of `dim` entries of float32 rows x turned in place by the tokens' positions:
+// the pairs of their first `rot` entries, by the table cos_t, sin_t [table_len, rot / 2]; the first
+// n_scaled heads are then multiplied by `scale`.  rot 0: scaled alone.
+int hal_rotate_heads(float* x, int ldx, const int* positions, const float* cos_t, const float* sin_t, int rot,
+                     int table_len, int interleaved, int heads, int dim, int n_scaled, float scale, int n_tokens,
+                     hipStream_t stream);
+// One token a request: S <- decay_h S + k v^T, y = S^T q per head (state [slots, H, N, P]) on rows v
+// [T, H * P], k and q [T, H * N], gate [T, H * P] (float32, row length ld); k and q turned as by
+// hal_rotate_heads, k times k_scale; in_silu: v, k and q through SiLU first; then every head divided
+// by its root mean square, times w (or null, [H * P]) and sigmoid(gate), or silu(gate).
+// N <= 256, P a multiple of 4 up to 1024.
+int hal_decay_step(const float* v, const float* k, const float* q, const float* gate, int ld, int in_silu,
+                   const int* positions, const float* cos_t, const float* sin_t, int rot, int table_len,
+                   int interleaved, float k_scale, const float* decay, float* state, const int* token_slot,
+                   const void* w, int w_dtype, int silu, float eps, void* out, int dtype, int n_tokens, int H, int N,
+                   int P, hipStream_t stream);
 // out = y / rms(y over each head of D) * w * sigmoid(z), or silu(z)  (w, z: null for none)
 int hal_head_norm_gate(const float* y, const float* z, int ldz, int silu, const void* w, int w_dtype, float eps,
                        void* out, int dtype, int n_tokens, int H, int D, hipStream_t stream);
@@ -305,10 +322,13 @@ int hal_stream_step(float* x, const float* y1, const float* y2, const void* w1, 
 // Every head of float32 q [T, H * dq], k [T, K * dq], v [T, K * dv] divided by its own root
 // mean square, packed as hal_qk_norm_pack packs (and appended to the pages, if given).
 // w_q, w_k (or null): a weight [dq] for every normed head of q / k; norm_v 0: the values are not
-// divided; v_other (or null): the values become (1 - v_mix) v + v_mix v_other.
+// divided; v_other (or null): the values become (1 - v_mix) v + v_mix v_other.  rot > 0: then the first
+// rot entries of every head of q and k are turned by the token's position, by the table cos_t, sin_t
+// [table_len, rot / 2] (pairs (i, i + rot / 2), or neighbours).  K 0: queries alone, rows of H heads.
 int hal_head_norm_pack(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, float eps,
                        const void* w_q, const void* w_k, int w_dtype, int norm_v, const float* v_other,
-                       int ldvo, float v_mix, const int* positions, void* out, int row_stride, int dtype, int n_tokens, int H,
+                       int ldvo, float v_mix, const int* positions, const float* cos_t, const float* sin_t,
+                       int rot, int table_len, int interleaved, void* out, int row_stride, int dtype, int n_tokens, int H,
                        int K, int dq, int dv, int D, const int* token_seg, const int* block_table,
                        int bt_stride, void* k_pages, void* v_pages, int page_size, int n_pages, int tiled,
                        hipStream_t stream);

@@ -104,11 +104,23 @@ __device__ __forceinline__ void load4_any(const void* p, int dtype, size_t i, fl
 }
 
 // ---- activations of a gated product: act(gate) * up -------------------------------------
-enum { HAL_ACT_SILU = 0, HAL_ACT_GELU_TANH = 1 };
+// HAL_ACT_CLAMPED holds both to a limit: g = min(gate, limit), u = clamp(up, -limit, limit),
+// g * sigmoid(alpha * g) * (u + up_shift)
+enum { HAL_ACT_SILU = 0, HAL_ACT_GELU_TANH = 1, HAL_ACT_CLAMPED = 2 };
+struct hal_gate {
+  int act;
+  float limit, alpha, up_shift;  // of HAL_ACT_CLAMPED
+};
 __device__ __forceinline__ float hal_gate_act(int act, float g) {
   if (act == HAL_ACT_GELU_TANH)
     return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
   return g / (1.0f + expf(-g));
+}
+__device__ __forceinline__ float hal_gated(const hal_gate& a, float g, float u) {
+  if (a.act != HAL_ACT_CLAMPED) return u * hal_gate_act(a.act, g);
+  g = fminf(g, a.limit);
+  u = fminf(fmaxf(u, -a.limit), a.limit);
+  return g / (1.0f + expf(-a.alpha * g)) * (u + a.up_shift);
 }
 
 // ---- reductions -----------------------------------------------------------------

@@ -8,7 +8,8 @@
 //     the query latent and of the key/value latent, and the key and value rows that the
 //     paged attention kernels take;
 //   * column ranges copied head by head;
-//   * the router of a mixture of experts: sigmoid scores, the largest `top`, their weights;
+//   * the router of a mixture of experts: scores, the chosen `top` (also by corrected scores and
+//     among the best groups of neighbours), their weights;
 //   * a counting sort of the (token, choice) pairs by expert, on the device;
 //   * the weighted sum of the chosen experts' results, added into the stream.
 #include "hal_common.h"
@@ -179,16 +180,94 @@ extern "C" int hal_scale_f32(float* x, long long n, float s, hipStream_t stream)
 #define MOE_MAX_EXPERTS 1024
 // Router: z [T, E] float32 logits.  score = sigmoid(z) (or, softmax == 1, the softmax over
 // the experts); the `top` largest scores (the lower index wins a tie); weights = the chosen
-// scores, divided by their sum + norm_eps if `normalize`.
+// scores, divided by their sum + norm_eps if `normalize`, times `scale`.  `correction` (or null)
+// [E]: added to the scores for the choice alone.  `groups` > 0: the experts form so many equal
+// groups of neighbours, and only experts of the `keep` groups with the largest sums of their two
+// largest (corrected) scores are chosen from (the lower group wins a tie).
 // ---------------------------------------------------------------------------------
+// The groups' part: a group's two largest scores are found across the wave, four groups at a time;
+// lane g % 64 keeps the sum of group g in word g / 64, counts the groups before it, and says
+// whether its group stays open; the scores of closed groups become -infinity.
+#define MOE_ROUTE_PER_LANE (MOE_MAX_EXPERTS / HAL_WAVE)
+__device__ __forceinline__ void moe_close_groups(float (&s)[MOE_ROUTE_PER_LANE], int E, int groups, int keep, int lane) {
+  const int per = E / groups, words = (E + HAL_WAVE - 1) / HAL_WAVE, gwords = (groups + HAL_WAVE - 1) / HAL_WAVE;
+  float mine[MOE_ROUTE_PER_LANE];
+#pragma unroll
+  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) mine[u] = -INFINITY;
+  constexpr int SIDE = 4;
+  for (int g0 = 0; g0 < groups; g0 += SIDE) {
+    float a[SIDE], b[SIDE];  // the largest and the second largest
+#pragma unroll
+    for (int v = 0; v < SIDE; ++v) a[v] = b[v] = -INFINITY;
+#pragma unroll
+    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
+      if (u >= words) continue;
+      const int e = lane + u * HAL_WAVE;
+      const int g = e < E ? e / per - g0 : -1;
+#pragma unroll
+      for (int v = 0; v < SIDE; ++v)
+        if (g == v) b[v] = fmaxf(b[v], fminf(a[v], s[u])), a[v] = fmaxf(a[v], s[u]);
+    }
+#pragma unroll
+    for (int off = HAL_WAVE / 2; off > 0; off >>= 1) {
+#pragma unroll
+      for (int v = 0; v < SIDE; ++v) {
+        const float oa = __shfl_xor(a[v], off, HAL_WAVE), ob = __shfl_xor(b[v], off, HAL_WAVE);
+        b[v] = fmaxf(fminf(a[v], oa), fmaxf(b[v], ob));
+        a[v] = fmaxf(a[v], oa);
+      }
+    }
+#pragma unroll
+    for (int v = 0; v < SIDE; ++v) {
+      const int g = g0 + v;
+      const float sum = per > 1 ? a[v] + b[v] : a[v];
+#pragma unroll
+      for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
+        if (g < groups && u == g / HAL_WAVE && lane == g % HAL_WAVE) mine[u] = sum;
+    }
+  }
+  int ahead[MOE_ROUTE_PER_LANE];  // groups that come before mine
+#pragma unroll
+  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) ahead[u] = 0;
+#pragma unroll
+  for (int w = 0; w < MOE_ROUTE_PER_LANE; ++w) {
+    if (w >= gwords) continue;
+    const int n = groups - w * HAL_WAVE < HAL_WAVE ? groups - w * HAL_WAVE : HAL_WAVE;
+    for (int l = 0; l < n; ++l) {
+      const float other = __shfl(mine[w], l, HAL_WAVE);
+#pragma unroll
+      for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
+        if (u < gwords && (other > mine[u] || (other == mine[u] && w * HAL_WAVE + l < u * HAL_WAVE + lane))) ++ahead[u];
+    }
+  }
+#pragma unroll
+  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
+    if (u >= words) continue;
+    const int e = lane + u * HAL_WAVE, g = e < E ? e / per : 0;
+    int before = 0;
+#pragma unroll
+    for (int w = 0; w < MOE_ROUTE_PER_LANE; ++w) {
+      if (w >= gwords) continue;
+      const int got = __shfl(ahead[w], g % HAL_WAVE, HAL_WAVE);
+      if (w == g / HAL_WAVE) before = got;
+    }
+    if (before >= keep) s[u] = -INFINITY;
+  }
+}
 // One wave a token: lane l holds the scores of the experts l, l + 64, ...; each of the `top`
 // rounds finds the largest score that is left (the lower index on a tie) across the wave.
-#define MOE_ROUTE_PER_LANE (MOE_MAX_EXPERTS / HAL_WAVE)
-__device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int ldz, int E, int top, int softmax,
-                                                int normalize, float norm_eps, int* __restrict__ idx,
-                                                float* __restrict__ wgt, int t, int lane) {
+struct MoeChoice {
+  int softmax, normalize;
+  float norm_eps, scale;
+  const void* correction;
+  int c_dtype, groups, keep;
+};
+__device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int ldz, int E, int top, const MoeChoice& how,
+                                                int* __restrict__ idx, float* __restrict__ wgt, int t, int lane) {
   const float* zr = z + (size_t)t * ldz;
   float s[MOE_ROUTE_PER_LANE];
+  float w[MOE_ROUTE_PER_LANE];  // the scores as weights, where the choice is made by other numbers
+  const bool apart = how.correction != nullptr || how.groups > 0;
   float zmax = -INFINITY;
 #pragma unroll
   for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
@@ -196,7 +275,7 @@ __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int
     s[u] = e < E ? zr[e] : -INFINITY;
     zmax = fmaxf(zmax, s[u]);
   }
-  if (softmax) {
+  if (how.softmax) {
     zmax = wave_max(zmax);
     float part = 0.f;
 #pragma unroll
@@ -212,6 +291,15 @@ __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int
     for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
       if (lane + u * HAL_WAVE < E) s[u] = 1.0f / (1.0f + expf(-s[u]));
   }
+  if (apart) {
+#pragma unroll
+    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
+      const int e = lane + u * HAL_WAVE;
+      w[u] = s[u];
+      if (how.correction && e < E) s[u] += load_as_f32(how.correction, how.c_dtype, e);
+    }
+  }
+  if (how.groups > 0) moe_close_groups(s, E, how.groups, how.keep, lane);
   float sum = 0.f;
   float kept[MOE_ROUTE_PER_LANE];  // lane j % 64 keeps the j-th choice's score in kept[j / 64]
   for (int j = 0; j < top; ++j) {
@@ -226,9 +314,14 @@ __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int
       const int oe = __shfl_xor(best_e, off, HAL_WAVE);
       if (ob > best || (ob == best && oe < best_e)) best = ob, best_e = oe;
     }
+    float own = 0.f;
 #pragma unroll
     for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-      if (lane + u * HAL_WAVE == best_e) s[u] = -INFINITY;  // taken
+      if (lane + u * HAL_WAVE == best_e) {
+        s[u] = -INFINITY;  // taken
+        if (apart) own = w[u];
+      }
+    if (apart) best = __shfl(own, best_e % HAL_WAVE, HAL_WAVE);
     sum += best;
     if (lane == 0) idx[(size_t)t * top + j] = best_e;
 #pragma unroll
@@ -238,24 +331,32 @@ __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int
 #pragma unroll
   for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
     const int j = lane + u * HAL_WAVE;
-    if (j < top) wgt[(size_t)t * top + j] = normalize ? kept[u] / (sum + norm_eps) : kept[u];
+    if (j < top) wgt[(size_t)t * top + j] = (how.normalize ? kept[u] / (sum + how.norm_eps) : kept[u]) * how.scale;
   }
 }
 
-__global__ void __launch_bounds__(HAL_WAVE) moe_route_kernel(const float* __restrict__ z, int ldz, int E, int top, int softmax,
-                                                             int normalize, float norm_eps, int* __restrict__ idx,
-                                                             float* __restrict__ wgt, int n_tokens) {
-  moe_route_token(z, ldz, E, top, softmax, normalize, norm_eps, idx, wgt, blockIdx.x, threadIdx.x);
+__global__ void __launch_bounds__(HAL_WAVE) moe_route_kernel(const float* __restrict__ z, int ldz, int E, int top, MoeChoice how,
+                                                             int* __restrict__ idx, float* __restrict__ wgt, int n_tokens) {
+  moe_route_token(z, ldz, E, top, how, idx, wgt, blockIdx.x, threadIdx.x);
 }
 
-extern "C" int hal_moe_route(const float* z, int ldz, int E, int top, int softmax, int normalize,
-                             float norm_eps, int* idx, float* wgt, int n_tokens,
-                             hipStream_t stream) {
+static int moe_check_choice(const MoeChoice& how, int E, int top) {
+  HAL_REQUIRE(how.c_dtype == HAL_F32 || how.c_dtype == HAL_BF16, "router: a correction of type %d", how.c_dtype);
+  HAL_REQUIRE(how.groups >= 0 && (how.groups == 0 || (E % how.groups == 0 && how.keep > 0 && how.keep <= how.groups &&
+                                                      top <= E / how.groups * how.keep)),
+              "router: %d of %d experts in %d groups of which %d are kept", top, E, how.groups, how.keep);
+  return 0;
+}
+
+extern "C" int hal_moe_route(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
+                             float scale, const void* correction, int c_dtype, int groups, int keep, int* idx,
+                             float* wgt, int n_tokens, hipStream_t stream) {
+  const MoeChoice how = {softmax, normalize, norm_eps, scale, correction, c_dtype, groups, keep};
+  if (int rc = moe_check_choice(how, E, top)) return rc;
   HAL_REQUIRE(n_tokens >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E,
               "hal_moe_route: bad sizes T=%d E=%d top=%d", n_tokens, E, top);
   if (n_tokens == 0) return 0;
-  hipLaunchKernelGGL(moe_route_kernel, dim3(n_tokens), dim3(HAL_WAVE), 0, stream, z, ldz, E, top, softmax,
-                     normalize, norm_eps, idx, wgt, n_tokens);
+  hipLaunchKernelGGL(moe_route_kernel, dim3(n_tokens), dim3(HAL_WAVE), 0, stream, z, ldz, E, top, how, idx, wgt, n_tokens);
   HAL_LAUNCH_CHECK();
   return 0;
 }
@@ -309,7 +410,7 @@ __global__ void __launch_bounds__(1024) moe_sort_kernel(const int* __restrict__ 
 // Both in one workgroup, for steps of few tokens: its sixteen waves take the tokens in turn,
 // then all of it sorts the pairs.
 __global__ void __launch_bounds__(1024) moe_route_sort_kernel(const float* __restrict__ z, int ldz, int E, int top,
-                                                              int softmax, int normalize, float norm_eps,
+                                                              MoeChoice how,
                                                               int* __restrict__ idx, float* __restrict__ wgt,
                                                               int n_tokens, int tile, int* __restrict__ offsets,
                                                               int* __restrict__ tile_offsets, int* __restrict__ sorted) {
@@ -317,19 +418,21 @@ __global__ void __launch_bounds__(1024) moe_route_sort_kernel(const float* __res
   __shared__ int cursor[MOE_MAX_EXPERTS];
   const int wave = threadIdx.x / HAL_WAVE, lane = threadIdx.x % HAL_WAVE;
   for (int t = wave; t < n_tokens; t += 1024 / HAL_WAVE)
-    moe_route_token(z, ldz, E, top, softmax, normalize, norm_eps, idx, wgt, t, lane);
+    moe_route_token(z, ldz, E, top, how, idx, wgt, t, lane);
   __threadfence_block();
   __syncthreads();
   moe_sort_pairs(idx, n_tokens * top, E, tile, offsets, tile_offsets, sorted, count, cursor);
 }
 
 extern "C" int hal_moe_route_sort(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
+                                  float scale, const void* correction, int c_dtype, int groups, int keep,
                                   int* idx, float* wgt, int n_tokens, int tile, int* offsets, int* tile_offsets,
                                   int* sorted, hipStream_t stream) {
+  const MoeChoice how = {softmax, normalize, norm_eps, scale, correction, c_dtype, groups, keep};
+  if (int rc = moe_check_choice(how, E, top)) return rc;
   HAL_REQUIRE(n_tokens >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E && tile > 0,
               "hal_moe_route_sort: bad sizes T=%d E=%d top=%d", n_tokens, E, top);
-  hipLaunchKernelGGL(moe_route_sort_kernel, dim3(1), dim3(1024), 0, stream, z, ldz, E, top, softmax, normalize, norm_eps,
-                     idx, wgt, n_tokens, tile, offsets, tile_offsets, sorted);
+  hipLaunchKernelGGL(moe_route_sort_kernel, dim3(1), dim3(1024), 0, stream, z, ldz, E, top, how, idx, wgt, n_tokens, tile, offsets, tile_offsets, sorted);
   HAL_LAUNCH_CHECK();
   return 0;
 }
@@ -369,39 +472,6 @@ extern "C" int hal_moe_combine(float* h, const float* y, const float* wgt, const
   int parts = 1;  // workgroups a row, so that a decode step has a few hundred of them
   while (parts < 16 && n_tokens * parts < 256 && d / (threads * parts * 2) >= 1) parts *= 2;
   hipLaunchKernelGGL(moe_combine_kernel, dim3(n_tokens, parts), dim3(threads), 0, stream, h, y, wgt, extra, extra_gate, ld_gate, top, d, overwrite != 0);
-  HAL_LAUNCH_CHECK();
-  return 0;
-}
-
-// ---------------------------------------------------------------------------------
-// out[t, f] = g * sigmoid(alpha * g) * (u + 1) with g = min(gu[t, f], limit) and
-// u = clamp(gu[t, F + f], -limit, limit): the activation of a clamped gated feed-forward
-// whose gate and up projections are the two halves of one product's rows.
-// ---------------------------------------------------------------------------------
-template <typename T>
-__global__ void clamped_gate_mul_kernel(const T* __restrict__ gu, T* __restrict__ out, int F, float limit,
-                                        float alpha, float up_shift) {
-  const int t = blockIdx.x;
-  const int f = blockIdx.y * blockDim.x + threadIdx.x;
-  if (f >= F) return;
-  const float g = fminf(to_f32(gu[(size_t)t * 2 * F + f]), limit);
-  const float u = fminf(fmaxf(to_f32(gu[(size_t)t * 2 * F + F + f]), -limit), limit);
-  out[(size_t)t * F + f] = from_f32<T>(g / (1.0f + __expf(-alpha * g)) * (u + up_shift));
-}
-
-extern "C" int hal_clamped_gate_mul(const void* gu, void* out, int dtype, int n_tokens, int F,
-                                    float limit, float alpha, float up_shift, hipStream_t stream) {
-  HAL_REQUIRE(n_tokens >= 0 && F > 0, "hal_clamped_gate_mul: bad sizes T=%d F=%d", n_tokens, F);
-  HAL_REQUIRE(dtype == HAL_F32 || dtype == HAL_BF16, "hal_clamped_gate_mul: dtype %d", dtype);
-  HAL_REQUIRE((F + 255) / 256 <= 65535, "hal_clamped_gate_mul: %d columns", F);
-  if (n_tokens == 0) return 0;
-  dim3 grid(n_tokens, (F + 255) / 256);
-  if (dtype == HAL_F32)
-    hipLaunchKernelGGL(clamped_gate_mul_kernel<float>, grid, dim3(256), 0, stream, (const float*)gu,
-                       (float*)out, F, limit, alpha, up_shift);
-  else
-    hipLaunchKernelGGL(clamped_gate_mul_kernel<bf16_t>, grid, dim3(256), 0, stream, (const bf16_t*)gu,
-                       (bf16_t*)out, F, limit, alpha, up_shift);
   HAL_LAUNCH_CHECK();
   return 0;
 }

@@ -11,6 +11,8 @@
 //   S_t = exp(-exp(A_log) * dt_t) S_(t-1) + dt_t * B_t x_t^T,  y_t = S_t^T C_t + D x_t,
 //   dt_t = softplus(dt_raw_t + dt_bias)
 //
+// (with one constant decay a head, unit steps and no D: a linear attention or retention, whose keys and
+// queries may be turned by the tokens' positions first)
 // and a gated scan per channel whose gates read the token alone:
 //   S_t = (1 - z_t) S_(t-1) + z_t c_t,  z = sigmoid(.), c = u + 1/2 where u >= 0, else sigmoid(u)
 //
@@ -373,6 +375,175 @@ extern "C" int hal_ssd_scan(const void* xbc, int ldx, int dtype, const float* dt
 #undef SCAN_BY_STATE
 #undef SCAN_STEPS
 #undef SCAN_LAUNCH
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- queries and keys turned in place by the tokens' positions, before a recurrence reads them: a
+// thread a pair of the first `rot` entries of a head (or an entry behind them, which is only scaled);
+// the first n_scaled heads are multiplied by `scale` behind the turn -----------------------------------
+__device__ __forceinline__ void rot_pair(int i, int rot, bool interleaved, int& a, int& b) {
+  a = interleaved ? 2 * i : i;
+  b = interleaved ? 2 * i + 1 : i + rot / 2;
+}
+
+__global__ void __launch_bounds__(256)
+rotate_heads_kernel(float* __restrict__ x, int ldx, const int* __restrict__ positions, const float* __restrict__ cos_t,
+                    const float* __restrict__ sin_t, int rot, int table_len, bool interleaved, int heads, int dim,
+                    int n_scaled, float scale) {
+  const size_t t = blockIdx.x;
+  const int pairs = rot / 2, per = dim - pairs;
+  const int pos = rot > 0 ? positions[t] : 0;
+  const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
+  for (int e = blockIdx.y * blockDim.x + threadIdx.x; e < heads * per; e += gridDim.y * blockDim.x) {
+    const int h = e / per, i = e % per;
+    const float m = h < n_scaled ? scale : 1.0f;
+    float* xr = x + t * ldx + (size_t)h * dim;
+    if (i < pairs) {
+      int a, b;
+      rot_pair(i, rot, interleaved, a, b);
+      const float c = known ? cos_t[(size_t)pos * pairs + i] : NAN, s = known ? sin_t[(size_t)pos * pairs + i] : NAN;
+      const float u = xr[a], v = xr[b];
+      xr[a] = (u * c - v * s) * m;
+      xr[b] = (v * c + u * s) * m;
+    } else if (m != 1.0f) {
+      xr[i + pairs] *= m;
+    }
+  }
+}
+
+extern "C" int hal_rotate_heads(float* x, int ldx, const int* positions, const float* cos_t, const float* sin_t, int rot,
+                                int table_len, int interleaved, int heads, int dim, int n_scaled, float scale,
+                                int n_tokens, hipStream_t stream) {
+  HAL_REQUIRE(n_tokens >= 0 && heads > 0 && dim > 0 && ldx >= heads * dim && n_scaled >= 0 && n_scaled <= heads,
+              "hal_rotate_heads: bad sizes T=%d heads=%d dim=%d rows of %d", n_tokens, heads, dim, ldx);
+  HAL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dim && (rot == 0 || (cos_t && sin_t && positions && table_len > 0)),
+              "hal_rotate_heads: %d turned entries of %d", rot, dim);
+  if (n_tokens == 0) return 0;
+  const int units = heads * (dim - rot / 2), want = (units + 255) / 256;
+  hipLaunchKernelGGL(rotate_heads_kernel, dim3(n_tokens, want < 64 ? want : 64), dim3(256), 0, stream, x, ldx, positions, cos_t,
+                     sin_t, rot, table_len, interleaved != 0, heads, dim, n_scaled, scale);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
+// ---- a step in which every request brings one token, for a recurrence with constant decays whose
+// heads are normed each on its own: a workgroup takes one head of one request.  It starts the loads
+// of the state (16 bytes a thread, whole rows), turns the token's query and key meanwhile, writes the
+// state back, crosses the threads through LDS for the sum over the key channels, and finishes
+// the head: its root mean square, weight and gate. ---------------------------------------------------
+#define DECAY_STEP_ROWS 8  // of the state a thread holds at a time
+template <typename T>
+__global__ void __launch_bounds__(1024)
+decay_step_kernel(const float* __restrict__ v, const float* __restrict__ k, const float* __restrict__ q,
+                  const float* __restrict__ gate, int ld, bool in_silu, const int* __restrict__ positions,
+                  const float* __restrict__ cos_t, const float* __restrict__ sin_t, int rot, int table_len,
+                  bool interleaved, float k_scale, const float* __restrict__ decay, float* __restrict__ state,
+                  const int* __restrict__ token_slot, const void* __restrict__ w, int w_dtype, bool silu, float eps,
+                  T* __restrict__ out, int H, int N, int P) {
+  __shared__ float k_s[256], q_s[256], scratch[16];
+  __shared__ float4 red[1024];
+  const size_t t = blockIdx.x;
+  const int h = blockIdx.y, tid = threadIdx.x, threads = blockDim.x;
+  const int CG = P / 4, RG = threads / CG;  // threads across a row of the state, rows side by side
+  const int cg = tid % CG, rg = tid / CG;
+  const bool works = rg < RG;
+  float* st = state + ((size_t)token_slot[t] * H + h) * N * P + cg * 4;
+  float4 S[DECAY_STEP_ROWS];
+  auto load = [&](int row0) {
+#pragma unroll
+    for (int j = 0; j < DECAY_STEP_ROWS; ++j)
+      if (works && row0 + j * RG < N) S[j] = *(const float4*)(st + (size_t)(row0 + j * RG) * P);
+  };
+  load(rg);
+  auto in = [&](const float* p) { return in_silu ? silu_f32(*p) : *p; };
+  float vv[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) vv[i] = works ? in(v + t * ld + (size_t)h * P + cg * 4 + i) : 0.f;
+  const int pos = rot > 0 ? positions[t] : 0;
+  const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
+  const float* kr = k + t * ld + (size_t)h * N;
+  const float* qr = q + t * ld + (size_t)h * N;
+  for (int i = tid; i < N - rot / 2; i += threads) {
+    if (i < rot / 2) {
+      int a, b;
+      rot_pair(i, rot, interleaved, a, b);
+      const float c = known ? cos_t[(size_t)pos * (rot / 2) + i] : NAN, s = known ? sin_t[(size_t)pos * (rot / 2) + i] : NAN;
+      const float ka = in(kr + a), kb = in(kr + b), qa = in(qr + a), qb = in(qr + b);
+      k_s[a] = (ka * c - kb * s) * k_scale, k_s[b] = (kb * c + ka * s) * k_scale;
+      q_s[a] = qa * c - qb * s, q_s[b] = qb * c + qa * s;
+    } else {
+      k_s[i + rot / 2] = in(kr + i + rot / 2) * k_scale;
+      q_s[i + rot / 2] = in(qr + i + rot / 2);
+    }
+  }
+  __syncthreads();
+  const float d = decay[h];
+  float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
+  for (int row0 = rg; row0 < N && works; row0 += RG * DECAY_STEP_ROWS) {
+    if (row0 != rg) load(row0);
+#pragma unroll
+    for (int j = 0; j < DECAY_STEP_ROWS; ++j) {
+      const int row = row0 + j * RG;
+      if (row >= N) break;
+      const float kk = k_s[row], qq = q_s[row];
+      S[j].x = fmaf(d, S[j].x, kk * vv[0]), acc.x = fmaf(S[j].x, qq, acc.x);
+      S[j].y = fmaf(d, S[j].y, kk * vv[1]), acc.y = fmaf(S[j].y, qq, acc.y);
+      S[j].z = fmaf(d, S[j].z, kk * vv[2]), acc.z = fmaf(S[j].z, qq, acc.z);
+      S[j].w = fmaf(d, S[j].w, kk * vv[3]), acc.w = fmaf(S[j].w, qq, acc.w);
+      *(float4*)(st + (size_t)row * P) = S[j];
+    }
+  }
+  if (works) red[rg * CG + cg] = acc;
+  __syncthreads();
+  const float* sums = (const float*)red;  // [RG][P]
+  float y[4], ss = 0.f;  // (P is at most four times the threads)
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int p = tid + u * threads;
+    y[u] = 0.f;
+    if (p < P)
+      for (int r = 0; r < RG; ++r) y[u] += sums[r * P + p];
+    ss += y[u] * y[u];
+  }
+  const float rstd = 1.0f / sqrtf(block_sum(ss, scratch) / (float)P + eps);
+#pragma unroll
+  for (int u = 0; u < 4; ++u) {
+    const int p = tid + u * threads;
+    if (p >= P) break;
+    const size_t c = (size_t)h * P + p;
+    const float z = gate[t * ld + c], s = 1.0f / (1.0f + expf(-z));
+    const float wt = w ? load_as_f32(w, w_dtype, c) : 1.0f;
+    out[t * H * P + c] = from_f32<T>(y[u] * rstd * wt * (silu ? z * s : s));
+  }
+}
+
+extern "C" int hal_decay_step(const float* v, const float* k, const float* q, const float* gate, int ld, int in_silu,
+                              const int* positions, const float* cos_t, const float* sin_t, int rot, int table_len,
+                              int interleaved, float k_scale, const float* decay, float* state, const int* token_slot,
+                              const void* w, int w_dtype, int silu, float eps, void* out, int dtype, int n_tokens, int H,
+                              int N, int P, hipStream_t stream) {
+  HAL_REQUIRE(n_tokens >= 0 && H > 0 && H <= 65535 && N > 0 && N <= 256 && P > 0 && P % 4 == 0 && P <= 1024,
+              "hal_decay_step: bad sizes T=%d heads=%d state %d x %d", n_tokens, H, N, P);
+  HAL_REQUIRE(ld >= H * P && ld >= H * N && v && k && q && gate && decay && state && token_slot, "hal_decay_step: rows");
+  HAL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= N && (rot == 0 || (cos_t && sin_t && positions && table_len > 0)),
+              "hal_decay_step: %d turned entries of %d", rot, N);
+  HAL_REQUIRE((dtype == HAL_F32 || dtype == HAL_BF16) && (w == nullptr || w_dtype == HAL_F32 || w_dtype == HAL_BF16),
+              "hal_decay_step: dtypes %d, %d", dtype, w_dtype);
+  HAL_REQUIRE(((uintptr_t)state % 16) == 0, "hal_decay_step: the state must be 16-byte aligned");
+  if (n_tokens == 0) return 0;
+  // as many threads as take the state in one go, DECAY_STEP_ROWS rows each
+  int threads = (N * (P / 4) / DECAY_STEP_ROWS + 63) / 64 * 64;
+  if (threads < (P / 4 + 63) / 64 * 64) threads = (P / 4 + 63) / 64 * 64;
+  if (threads < 64) threads = 64;
+  if (threads > 1024) threads = 1024;
+#define DECAY_STEP(T_)                                                                                                   \
+  hipLaunchKernelGGL(decay_step_kernel<T_>, dim3(n_tokens, H), dim3(threads), 0, stream, v, k, q, gate, ld, in_silu != 0, \
+                     positions, cos_t, sin_t, rot, table_len, interleaved != 0, k_scale, decay, state, token_slot, w,      \
+                     w_dtype, silu != 0, eps, (T_*)out, H, N, P)
+  if (dtype == HAL_F32) DECAY_STEP(float);
+  else DECAY_STEP(bf16_t);
+#undef DECAY_STEP
   HAL_LAUNCH_CHECK();
   return 0;
 }

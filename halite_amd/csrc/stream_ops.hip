@@ -616,15 +616,31 @@ extern "C" int hal_stream_step(float* x, const float* y1, const float* y2, const
   return 0;
 }
 
+// The pair of entry j of n turned entries: its number, its partner, whether j is the second of the two.
+__device__ __forceinline__ int pair_of(int j, int n, bool interleaved, int& partner, bool& second) {
+  if (interleaved) {
+    second = (j & 1) != 0;
+    partner = j ^ 1;
+    return j / 2;
+  }
+  const int half = n / 2;
+  second = j >= half;
+  partner = second ? j - half : j + half;
+  return second ? j - half : j;
+}
+
 // ---- every head of q, k and v divided by its own root mean square (no weight), packed as
 // [H heads of D | K heads of D | K heads of D] with zeros beyond a head's entries, keys and
-// values appended to the pages as well (k_pages null: not).  A wave a (token, head). ---------
+// values appended to the pages as well (k_pages null: not).  cos_t: the first `rot` entries of every
+// normed head of q and k are turned by the token's position.  K 0: queries alone.  A wave a (token, head). --
 template <typename T>
 __global__ void head_norm_pack_kernel(const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk,
                                       const float* __restrict__ v, int ldv, float eps,
                                       const void* __restrict__ w_q, const void* __restrict__ w_k, int w_dtype,
                                       bool norm_v, const float* __restrict__ v_other, int ldvo, float v_mix,
-                                      const int* __restrict__ positions, T* __restrict__ out, int row_stride,
+                                      const int* __restrict__ positions, const float* __restrict__ cos_t,
+                                      const float* __restrict__ sin_t, int rot, int table_len, bool interleaved,
+                                      T* __restrict__ out, int row_stride,
                                       int n_tokens, int H, int K, int dq, int dv, int D,
                                       const int* __restrict__ token_seg, const int* __restrict__ block_table,
                                       int bt_stride, T* __restrict__ k_pages, T* __restrict__ v_pages, int page_size,
@@ -648,6 +664,9 @@ __global__ void head_norm_pack_kernel(const float* __restrict__ q, int ldq, cons
   // (a weight of the head's size, shared by the heads; values: a blend with another layer's)
   const void* w = kind == 0 ? w_q : (kind == 1 ? w_k : nullptr);
   const float* other = (kind == 2 && v_other) ? v_other + t * ldvo + (size_t)head * dv : nullptr;
+  const int turned = (cos_t && kind != 2) ? rot : 0;
+  const int at = turned > 0 ? positions[t] : 0;
+  const bool known = at >= 0 && at < table_len;  // checked on the host; else the row shows it
   long long page = -1;
   int off = 0;
   if (k_pages && kind != 0) {
@@ -660,6 +679,15 @@ __global__ void head_norm_pack_kernel(const float* __restrict__ q, int ldq, cons
   for (int d = lane; d < D; d += HAL_WAVE) {
     float f = d < n ? src[d] * rstd : 0.f;
     if (w && d < n) f *= load_as_f32(w, w_dtype, d);
+    if (d < turned) {
+      int partner;
+      bool second;
+      const int i = pair_of(d, turned, interleaved, partner, second);
+      const float c = known ? cos_t[(size_t)at * (turned / 2) + i] : NAN, s = known ? sin_t[(size_t)at * (turned / 2) + i] : NAN;
+      float o = src[partner] * rstd;
+      if (w) o *= load_as_f32(w, w_dtype, partner);
+      f = second ? f * c + o * s : f * c - o * s;
+    }
     if (other && d < n) f = (1.0f - v_mix) * f + v_mix * other[d];
     const T x = from_f32<T>(f);
     o[d] = x;
@@ -672,13 +700,14 @@ __global__ void head_norm_pack_kernel(const float* __restrict__ q, int ldq, cons
 
 extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, float eps,
                                   const void* w_q, const void* w_k, int w_dtype, int norm_v, const float* v_other,
-                                  int ldvo, float v_mix, const int* positions, void* out, int row_stride, int dtype, int n_tokens, int H,
+                                  int ldvo, float v_mix, const int* positions, const float* cos_t, const float* sin_t,
+                                  int rot, int table_len, int interleaved, void* out, int row_stride, int dtype, int n_tokens, int H,
                                   int K, int dq, int dv, int D, const int* token_seg, const int* block_table,
                                   int bt_stride, void* k_pages, void* v_pages, int page_size, int n_pages, int tiled,
                                   hipStream_t stream) {
   HAL_REQUIRE(k_pages == nullptr || (v_pages && token_seg && block_table && positions && page_size > 0 && n_pages > 0),
               "hal_head_norm_pack: pages without the arrays that say where a token's key goes");
-  HAL_REQUIRE(n_tokens >= 0 && H > 0 && K > 0 && dq > 0 && dv > 0 && D >= dq && D >= dv,
+  HAL_REQUIRE(n_tokens >= 0 && H > 0 && K >= 0 && dq > 0 && dv > 0 && D >= dq && D >= dv && (K > 0 || !k_pages),
               "hal_head_norm_pack: bad sizes T=%d H=%d K=%d dq=%d dv=%d D=%d", n_tokens, H, K, dq, dv, D);
   HAL_REQUIRE(row_stride >= (H + 2 * K) * D && ldq >= H * dq && ldk >= K * dq && ldv >= K * dv,
               "hal_head_norm_pack: rows too short");
@@ -686,17 +715,20 @@ extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int l
   HAL_REQUIRE((w_q == nullptr) == (w_k == nullptr) && (w_q == nullptr || w_dtype == HAL_F32 || w_dtype == HAL_BF16),
               "hal_head_norm_pack: weights for both q and k or for neither, float32 or bf16");
   HAL_REQUIRE(v_other == nullptr || ldvo >= K * dv, "hal_head_norm_pack: rows of the other values too short");
+  HAL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= dq && (rot == 0 || (cos_t && sin_t && positions && table_len > 0)),
+              "hal_head_norm_pack: %d turned entries of %d", rot, dq);
+  if (rot == 0) cos_t = nullptr;
   if (n_tokens == 0) return 0;
   const long long units = (long long)n_tokens * (H + 2 * K);
   const dim3 grid((unsigned)((units + 3) / 4));
   if (dtype == HAL_F32)
     hipLaunchKernelGGL(head_norm_pack_kernel<float>, grid, dim3(256), 0, stream, q, ldq, k, ldk, v, ldv, eps, w_q, w_k,
-                       w_dtype, norm_v != 0, v_other, ldvo, v_mix, positions,
+                       w_dtype, norm_v != 0, v_other, ldvo, v_mix, positions, cos_t, sin_t, rot, table_len, interleaved != 0,
                        (float*)out, row_stride, n_tokens, H, K, dq, dv, D, token_seg, block_table, bt_stride,
                        (float*)k_pages, (float*)v_pages, page_size, n_pages, tiled != 0);
   else
     hipLaunchKernelGGL(head_norm_pack_kernel<bf16_t>, grid, dim3(256), 0, stream, q, ldq, k, ldk, v, ldv, eps, w_q, w_k,
-                       w_dtype, norm_v != 0, v_other, ldvo, v_mix, positions,
+                       w_dtype, norm_v != 0, v_other, ldvo, v_mix, positions, cos_t, sin_t, rot, table_len, interleaved != 0,
                        (bf16_t*)out, row_stride, n_tokens, H, K, dq, dv, D, token_seg, block_table, bt_stride,
                        (bf16_t*)k_pages, (bf16_t*)v_pages, page_size, n_pages, tiled != 0);
   HAL_LAUNCH_CHECK();
@@ -707,18 +739,6 @@ extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int l
 // times one number of its own, the heads' padding dropped on the way.  With a rotation table
 // (cos_t, sin_t [table_len, n / 2]) every head's n entries are turned back by the token's position
 // first: (u, v) of the pair (i, i + n / 2), or (2i, 2i + 1), becomes (u c + v s, v c - u s). ------
-__device__ __forceinline__ int pair_of(int j, int n, bool interleaved, int& partner, bool& second) {
-  if (interleaved) {
-    second = (j & 1) != 0;
-    partner = j ^ 1;
-    return j / 2;
-  }
-  const int half = n / 2;
-  second = j >= half;
-  partner = second ? j - half : j + half;
-  return second ? j - half : j;
-}
-
 template <typename T>
 __global__ void head_gate_cols_kernel(const T* __restrict__ x, int ldx, int x_head, const float* __restrict__ g, int ldg,
                                       T* __restrict__ y, int n, int H, const int* __restrict__ positions,

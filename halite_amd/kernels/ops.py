@@ -9,6 +9,7 @@ functions: without a GPU and the built library they raise.
 from __future__ import annotations
 
 import ctypes
+import math
 from dataclasses import dataclass
 
 import torch
@@ -253,11 +254,24 @@ def residual_add(h: torch.Tensor, delta: torch.Tensor):
     return h
 
 
-GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1}  # the kernels' numbers for what a gate goes through
+GATE_ACTIVATIONS = {"silu": 0, "gelu_tanh": 1, "clamped": 2}  # the kernels' numbers for what a gate goes through
 
 
-def gate_mul(gate_up: torch.Tensor, activation: str = "silu"):
-    """``up * act(gate)`` of rows ``[gate | up]``."""
+@dataclass(frozen=True)
+class Clamp:
+    """The constants of the activation ``clamped``: ``g * sigmoid(alpha * g) * (u + up_shift)`` with ``g =
+    min(gate, limit)`` and ``u = clamp(up, -limit, limit)`` (``limit`` ``inf``: neither is held)."""
+
+    limit: float = math.inf
+    alpha: float = 1.0
+    up_shift: float = 0.0
+
+    def args(self):
+        return ctypes.c_float(self.limit), ctypes.c_float(self.alpha), ctypes.c_float(self.up_shift)
+
+
+def gate_mul(gate_up: torch.Tensor, activation: str = "silu", clamp: Clamp = Clamp()):
+    """``up * act(gate)`` of rows ``[gate | up]`` (``clamped``: see ``Clamp``)."""
     lib = library.core_library()
     _dev(gate_up)
     n, two_f = gate_up.shape
@@ -266,7 +280,7 @@ def gate_mul(gate_up: torch.Tensor, activation: str = "silu"):
     _check(
         lib,
         lib.hal_gate_mul(_ptr(gate_up), _ptr(out), dtype_code(gate_up.dtype), n, two_f // 2,
-                         GATE_ACTIVATIONS[activation], _stream()),
+                         GATE_ACTIVATIONS[activation], *clamp.args(), _stream()),
     )
     return out
 
@@ -580,9 +594,11 @@ def gemm_bf16_skinny(
     tiled_shape: tuple[int, int] | None = None,
     relu_squared: bool = False,
     activation: str = "silu",
+    clamp: Clamp = Clamp(),
 ):
     """``x @ w.T`` for at most 64 rows of bf16 ``x``; with ``w_up`` the gated form
-    ``(x @ w_up.T) * act(x @ w.T)`` (``activation``: a name of ``GATE_ACTIVATIONS``); ``add_to`` (float32) receives ``+=``;
+    ``(x @ w_up.T) * act(x @ w.T)`` (``activation``: a name of ``GATE_ACTIVATIONS``,
+    ``clamp`` its constants if it is ``clamped``); ``add_to`` (float32) receives ``+=``;
     ``relu_squared``: the bf16 result is the square of relu of the product."""
     lib = library.core_library()
     _dev(x, add_to)
@@ -617,7 +633,7 @@ def gemm_bf16_skinny(
     _check(
         lib,
         lib.hal_gemm_bf16_skinny(
-            _ptr(x), k, _ptr(w), _ptr(w_up), ldw, _ptr(out), n, mode, GATE_ACTIVATIONS[activation], m, n, k, _stream()
+            _ptr(x), k, _ptr(w), _ptr(w_up), ldw, _ptr(out), n, mode, GATE_ACTIVATIONS[activation], *clamp.args(), m, n, k, _stream()
         ),
     )
     return out
@@ -886,28 +902,51 @@ def grouped_gemm(
     return y
 
 
-def moe_route(z: torch.Tensor, top: int, softmax: bool = False, normalize: bool = True, norm_eps: float = 0.0):
+@dataclass(frozen=True)
+class RouterChoice:
+    """How a router's scores become the chosen experts and their weights.  ``softmax``: the scores are
+    the softmax over the experts, else sigmoids.  ``correction`` ``[E]`` (on the device): added to
+    the scores for the choice alone.  ``groups`` > 0: the experts form so many equal groups of
+    neighbours and the choice is among the ``keep`` groups with the largest sums of their two
+    largest (corrected) scores.  The weights are the chosen experts' scores without the correction,
+    divided by their sum + ``norm_eps`` if ``normalize``, times ``scale``."""
+
+    softmax: bool = False
+    normalize: bool = True
+    norm_eps: float = 0.0
+    scale: float = 1.0
+    correction: torch.Tensor | None = None
+    groups: int = 0
+    keep: int = 0
+
+    def args(self, n_experts: int):
+        c = self.correction
+        _need(c is None or (c.is_cuda and c.is_contiguous() and c.shape == (n_experts,)), "router: a correction [E] on the GPU")
+        return (1 if self.softmax else 0, 1 if self.normalize else 0, ctypes.c_float(self.norm_eps), ctypes.c_float(self.scale),
+                _ptr(c), F32 if c is None else dtype_code(c.dtype), self.groups, self.keep)
+
+
+def moe_route(z: torch.Tensor, top: int, **how):
     """The ``top`` experts of every token from float32 router logits ``z`` ``[T, E]``: indices
-    ``[T, top]`` int32 and weights ``[T, top]`` float32 (sigmoid scores, or the softmax over
-    the experts; divided by their sum + ``norm_eps`` if ``normalize``)."""
+    ``[T, top]`` int32 and weights ``[T, top]`` float32 (``how``: the fields of ``RouterChoice``)."""
     lib = library.core_library()
+    choice = RouterChoice(**how)
     _need(z.is_cuda and z.dtype == torch.float32 and z.dim() == 2 and z.stride(1) == 1,
           "moe_route: float32 logits [T, E] (a row-strided view is allowed)")
     t, e = z.shape
     idx = torch.empty((t, top), dtype=torch.int32, device=z.device)
     wgt = torch.empty((t, top), dtype=torch.float32, device=z.device)
-    _check(lib, lib.hal_moe_route(_ptr(z), z.stride(0), e, top, 1 if softmax else 0, 1 if normalize else 0,
-                                  ctypes.c_float(norm_eps), _ptr(idx), _ptr(wgt), t, _stream()))
+    _check(lib, lib.hal_moe_route(_ptr(z), z.stride(0), e, top, *choice.args(e), _ptr(idx), _ptr(wgt), t, _stream()))
     return idx, wgt
 
 
 ROUTE_SORT_MAX_TOKENS = 16  # up to so many tokens (one a wave) one workgroup routes and sorts
 
 
-def moe_route_sort(z: torch.Tensor, top: int, n_experts: int, softmax: bool = False, normalize: bool = True,
-                   norm_eps: float = 0.0):
+def moe_route_sort(z: torch.Tensor, top: int, n_experts: int, **how):
     """``moe_route`` and ``moe_sort`` in one launch: ``(idx, wgt, offsets, tile_offsets, sorted)``."""
     lib = library.core_library()
+    choice = RouterChoice(**how)
     _need(z.is_cuda and z.dtype == torch.float32 and z.dim() == 2 and z.stride(1) == 1 and z.shape[1] == n_experts,
           "moe_route_sort: float32 logits [T, E] (a row-strided view is allowed)")
     t = z.shape[0]
@@ -916,8 +955,7 @@ def moe_route_sort(z: torch.Tensor, top: int, n_experts: int, softmax: bool = Fa
     offsets = torch.empty(n_experts + 1, dtype=torch.int32, device=z.device)
     tile_offsets = torch.empty(n_experts + 1, dtype=torch.int32, device=z.device)
     order = torch.empty(max(t * top, 1), dtype=torch.int32, device=z.device)
-    _check(lib, lib.hal_moe_route_sort(_ptr(z), z.stride(0), n_experts, top, 1 if softmax else 0, 1 if normalize else 0,
-                                       ctypes.c_float(norm_eps), _ptr(idx), _ptr(wgt), t, GROUP_TILE_ROWS, _ptr(offsets),
+    _check(lib, lib.hal_moe_route_sort(_ptr(z), z.stride(0), n_experts, top, *choice.args(n_experts), _ptr(idx), _ptr(wgt), t, GROUP_TILE_ROWS, _ptr(offsets),
                                        _ptr(tile_offsets), _ptr(order), _stream()))
     return idx, wgt, offsets, tile_offsets, order
 
@@ -959,14 +997,7 @@ def moe_combine(h: torch.Tensor, y: torch.Tensor, wgt: torch.Tensor, extra: torc
 def clamped_gate_mul(gate_up: torch.Tensor, limit: float, alpha: float, up_shift: float = 1.0) -> torch.Tensor:
     """``g * sigmoid(alpha * g) * (u + up_shift)`` with ``g = min(gate, limit)`` and
     ``u = clamp(up, -limit, limit)`` of rows ``[gate | up]``."""
-    lib = library.core_library()
-    _dev(gate_up)
-    n, two_f = gate_up.shape
-    _need(two_f % 2 == 0, "clamped_gate_mul: odd row length")
-    out = torch.empty((n, two_f // 2), dtype=gate_up.dtype, device=gate_up.device)
-    _check(lib, lib.hal_clamped_gate_mul(_ptr(gate_up), _ptr(out), dtype_code(gate_up.dtype), n, two_f // 2,
-                                         ctypes.c_float(limit), ctypes.c_float(alpha), ctypes.c_float(up_shift), _stream()))
-    return out
+    return gate_mul(gate_up, "clamped", Clamp(limit, alpha, up_shift))
 
 
 # -- rows of the stream and of projections; mixers with a carried state -----------------------
@@ -1398,19 +1429,85 @@ def stream_step(x: torch.Tensor, *, y: torch.Tensor | NormedTerms | None = None,
     return result if read else None
 
 
-def head_norm_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float, n_heads: int, n_kv_heads: int,
+def _rotation(cos, sin, positions, n: int, dim: int, what: str) -> int:
+    """How many entries of a head of ``dim`` a rotation table turns (0 without one)."""
+    if cos is None:
+        return 0
+    _dev(cos, sin, positions)
+    _i32(positions, "positions")
+    _need(cos.dtype == torch.float32 and sin.dtype == torch.float32 and cos.dim() == 2 and cos.shape == sin.shape
+          and cos.is_contiguous() and sin.is_contiguous() and 2 * cos.shape[1] <= dim, f"{what}: float32 tables [positions, pairs]")
+    _need(positions is not None and positions.numel() == n, f"{what}: one position a row")
+    return 2 * cos.shape[1]
+
+
+def rotate_heads_(x: torch.Tensor, heads: int, dim: int, positions: torch.Tensor | None = None, cos: torch.Tensor | None = None,
+                  sin: torch.Tensor | None = None, interleaved: bool = False, n_scaled: int = 0, scale: float = 1.0):
+    """The heads of ``dim`` entries of float32 rows ``x`` (a row-strided view is allowed) turned in place:
+    the pairs of a head's first entries by the token's position (``cos``, ``sin`` ``[positions,
+    pairs]``; None: not); the first ``n_scaled`` heads are then multiplied by ``scale``."""
+    lib = library.core_library()
+    _rows_f32(x, heads * dim, "rotate_heads_")
+    rot = _rotation(cos, sin, positions, x.shape[0], dim, "rotate_heads_")
+    _check(lib, lib.hal_rotate_heads(_ptr(x), x.stride(0), _ptr(positions), _ptr(cos), _ptr(sin), rot,
+                                     0 if cos is None else cos.shape[0], 1 if interleaved else 0, heads, dim, n_scaled,
+                                     ctypes.c_float(scale), x.shape[0], _stream()))
+    return x
+
+
+def decay_step_fits(n_state: int, v_dim: int) -> bool:
+    """Whether ``decay_step`` has a kernel for states of ``n_state x v_dim`` numbers."""
+    return n_state <= 256 and v_dim % 4 == 0 and v_dim <= 1024
+
+
+def decay_step(v: torch.Tensor, k: torch.Tensor, q: torch.Tensor, gate: torch.Tensor, decay: torch.Tensor,
+               state: torch.Tensor, token_slot: torch.Tensor, eps: float, out_dtype: torch.dtype, *,
+               positions: torch.Tensor | None = None, cos: torch.Tensor | None = None, sin: torch.Tensor | None = None,
+               interleaved: bool = False, k_scale: float = 1.0, in_silu: bool = False,
+               weight: torch.Tensor | None = None, silu: bool = False) -> torch.Tensor:
+    """A step in which every request brings one token, for a recurrence with constant decays, in one
+    kernel: ``rotate_heads_`` of ``k`` and ``q`` (``k`` times ``k_scale``), the recurrence ``S <- decay S + k
+    v^T``, ``y = S^T q`` (``ssd_scan`` with ``fixed_decay``) and ``head_norm_gate`` head by head.  ``v`` and
+    ``gate`` float32 ``[T, heads * P]``, ``k`` and ``q`` ``[T, heads * N]`` (views of one row length); ``state``
+    float32 ``[slots, heads, N, P]``.  Returns ``[T, heads * P]`` of ``out_dtype``."""
+    lib = library.core_library()
+    _, heads, n_state, p = state.shape
+    n = v.shape[0]
+    for t, cols in ((v, heads * p), (gate, heads * p), (k, heads * n_state), (q, heads * n_state)):
+        _rows_f32(t, cols, "decay_step")
+    _need(len({(t.shape[0], t.stride(0)) for t in (v, k, q, gate)}) == 1, "decay_step: rows of one length, one a token")
+    _dev(decay, state, token_slot, weight)
+    _i32(token_slot, "token_slot")
+    _need(decay_step_fits(n_state, p), f"decay_step: no kernel for states of {n_state} x {p}")
+    _need(decay.dtype == torch.float32 and decay.shape == (heads,) and state.dtype == torch.float32 and state.is_contiguous(),
+          "decay_step: float32 decays [heads] and states")
+    _need(token_slot.numel() == n and (weight is None or weight.numel() == heads * p), "decay_step: one slot a token")
+    rot = _rotation(cos, sin, positions, n, n_state, "decay_step")
+    out = torch.empty((n, heads * p), dtype=out_dtype, device=v.device)
+    _check(lib, lib.hal_decay_step(
+        _ptr(v), _ptr(k), _ptr(q), _ptr(gate), v.stride(0), 1 if in_silu else 0, _ptr(positions), _ptr(cos), _ptr(sin), rot,
+        0 if cos is None else cos.shape[0], 1 if interleaved else 0, ctypes.c_float(k_scale), _ptr(decay), _ptr(state),
+        _ptr(token_slot), _ptr(weight), F32 if weight is None else dtype_code(weight.dtype), 1 if silu else 0,
+        ctypes.c_float(eps), _ptr(out), dtype_code(out_dtype), n, heads, n_state, p, _stream()))
+    return out
+
+
+def head_norm_pack(q: torch.Tensor, k: torch.Tensor | None, v: torch.Tensor | None, eps: float, n_heads: int, n_kv_heads: int,
                    qk_dim: int, v_dim: int, head_dim: int, out_dtype: torch.dtype,
                    positions: torch.Tensor | None = None, token_seg: torch.Tensor | None = None,
                    block_table: torch.Tensor | None = None, k_pages: torch.Tensor | None = None,
                    v_pages: torch.Tensor | None = None, page_size: int = 0, tiled: bool = False,
                    w_q: torch.Tensor | None = None, w_k: torch.Tensor | None = None, norm_v: bool = True,
-                   v_other: torch.Tensor | None = None, v_mix: float = 0.0) -> torch.Tensor:
+                   v_other: torch.Tensor | None = None, v_mix: float = 0.0, cos: torch.Tensor | None = None,
+                   sin: torch.Tensor | None = None, interleaved: bool = False) -> torch.Tensor:
     """From float32 projections (row-strided views allowed): every head of ``q``, ``k`` and
     (with ``norm_v``) ``v`` divided by its own root mean square; the packed rows ``[q heads | k
     heads | v heads]`` of ``head_dim`` entries a head (zero beyond ``qk_dim`` / ``v_dim``) come
     back.  ``w_q`` / ``w_k`` ``[qk_dim]``: a weight that multiplies every normed head of q / k.
     ``v_other`` (float32 rows like ``v``): the values become ``(1 - v_mix) v + v_mix v_other``.
-    With ``k_pages`` and ``v_pages`` keys and values are appended to the pages as well."""
+    ``cos``, ``sin`` (float32 ``[positions, pairs]``): the pairs of the first entries of every normed
+    head of q and k are turned by the token's position.  ``k`` and ``v`` None (``n_kv_heads`` 0):
+    queries alone.  With ``k_pages`` and ``v_pages`` keys and values are appended to the pages as well."""
     lib = library.core_library()
     _dev(w_q, w_k)
     _need((w_q is None) == (w_k is None) and (w_q is None or (w_q.shape == (qk_dim,) and w_k.shape == (qk_dim,)
@@ -1420,8 +1517,11 @@ def head_norm_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float
         _rows_f32(v_other, n_kv_heads * v_dim, "head_norm_pack v_other")
         _need(v_other.shape[0] == q.shape[0], "head_norm_pack: one row of other values a token")
     n = q.shape[0]
-    _rows_f32(q, n_heads * qk_dim, "head_norm_pack q"), _rows_f32(k, n_kv_heads * qk_dim, "head_norm_pack k")
-    _rows_f32(v, n_kv_heads * v_dim, "head_norm_pack v")
+    _rows_f32(q, n_heads * qk_dim, "head_norm_pack q")
+    _need((k is None) == (v is None) == (n_kv_heads == 0), "head_norm_pack: keys and values, or neither")
+    if k is not None:
+        _rows_f32(k, n_kv_heads * qk_dim, "head_norm_pack k"), _rows_f32(v, n_kv_heads * v_dim, "head_norm_pack v")
+    rot = _rotation(cos, sin, positions, n, qk_dim, "head_norm_pack")
     _need(head_dim >= max(qk_dim, v_dim), "head_norm_pack: head sizes")
     out = torch.empty((n, (n_heads + 2 * n_kv_heads) * head_dim), dtype=out_dtype, device=q.device)
     n_pages = 0
@@ -1435,9 +1535,10 @@ def head_norm_pack(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, eps: float
         _need(positions is not None and positions.numel() == n and token_seg is not None and token_seg.numel() == n
               and block_table is not None and block_table.dim() == 2, "head_norm_pack: the step's arrays")
     _check(lib, lib.hal_head_norm_pack(
-        _ptr(q), q.stride(0), _ptr(k), k.stride(0), _ptr(v), v.stride(0), ctypes.c_float(eps),
-        _ptr(w_q), _ptr(w_k), dtype_code(w_q.dtype) if w_q is not None else F32, 1 if norm_v else 0,
+        _ptr(q), q.stride(0), _ptr(k), 0 if k is None else k.stride(0), _ptr(v), 0 if v is None else v.stride(0),
+        ctypes.c_float(eps), _ptr(w_q), _ptr(w_k), dtype_code(w_q.dtype) if w_q is not None else F32, 1 if norm_v else 0,
         _ptr(v_other), 0 if v_other is None else v_other.stride(0), ctypes.c_float(v_mix), _ptr(positions),
+        _ptr(cos), _ptr(sin), rot, 0 if cos is None else cos.shape[0], 1 if interleaved else 0,
         _ptr(out), out.shape[1], dtype_code(out_dtype), n, n_heads, n_kv_heads, qk_dim, v_dim, head_dim,
         _ptr(token_seg), _ptr(block_table), 0 if block_table is None else block_table.shape[1],
         _ptr(k_pages), _ptr(v_pages), page_size, n_pages, 1 if tiled else 0, _stream()))

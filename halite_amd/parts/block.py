@@ -173,16 +173,19 @@ class HyperPreNormBlock(Arrangement):
     """A pre-norm block on a residual stream that is kept in copies: each of the two parts
     reads its input through a connection of its own (``mixer_link``, ``ff_link``), which also
     says how the part's result gets back into the copies.  A layer may leave the
-    feed-forward (with its norm and connection) out.
+    feed-forward (with its norm and connection) out, and may norm what a part returns on its
+    way there (``mixer_out_norm``, ``ff_out_norm``).
 
     The stream handed from block to block is ``[copies, T, width]`` float32.  A part's
-    result is left pending, with its connection, for whoever reads next: the write of one
-    part and the read and norm of the next are one pass over the copies."""
+    result is left pending, with its connection (and its norm, as a sum of one normed term), for
+    whoever reads next: the write of one part and the read and norm of the next are one pass
+    over the copies."""
 
     graph_safe = True
     roles = {"mixer_norm": NORMS, "mixer": MIXERS, "mixer_link": CONNECTIONS,
-             "ff_norm": NORMS, "ff": FEED_FORWARDS, "ff_link": CONNECTIONS}
-    optional = ("ff_norm", "ff", "ff_link")
+             "ff_norm": NORMS, "ff": FEED_FORWARDS, "ff_link": CONNECTIONS,
+             "mixer_out_norm": NORMS, "ff_out_norm": NORMS}
+    optional = ("ff_norm", "ff", "ff_link", "mixer_out_norm", "ff_out_norm")
 
     def __init__(self, parts):
         super().__init__(parts)
@@ -192,6 +195,20 @@ class HyperPreNormBlock(Arrangement):
             raise ValueError("a block has a feed-forward with its norm and connection, or none of them")
         if self.ff_link is not None and self.ff_link.copies != self.mixer_link.copies:
             raise ValueError("a block's connections keep different numbers of copies")
+        self.mixer_out_norm, self.ff_out_norm = parts.get("mixer_out_norm"), parts.get("ff_out_norm")
+        if self.ff is None and self.ff_out_norm is not None:
+            raise ValueError("a norm on the result of a feed-forward that the block does not have")
+        for norm in (self.mixer_out_norm, self.ff_out_norm):
+            if norm is not None and not (isinstance(norm, RMSNorm) and not norm.p.round_before_weight):
+                raise ValueError("a part's result is normed by an RMSNorm in the unrounded order")
+        if self.mixer_out_norm is not None and hasattr(self.mixer, "forward_normed_terms"):
+            raise ValueError("a sum of normed results is not normed once more")
+
+    @staticmethod
+    def _normed(y, norm):
+        if norm is None:
+            return y
+        return ops.NormedTerms([(y if y.dtype == torch.float32 else y.float(), norm.multiplier, 1.0)], norm.p.eps)
 
     @property
     def stream_copies(self) -> int:
@@ -201,10 +218,11 @@ class HyperPreNormBlock(Arrangement):
         x = self.mixer_link.step(h, pending, self.mixer_norm)
         # (a sum of normed results is made by the pass that writes it)
         terms = self.mixer.forward_normed_terms(x, ctx, run) if hasattr(self.mixer, "forward_normed_terms") else None
-        pending = (terms if terms is not None else self.mixer.forward(x, ctx, run), self.mixer_link)
+        y = terms if terms is not None else self._normed(self.mixer.forward(x, ctx, run), self.mixer_out_norm)
+        pending = (y, self.mixer_link)
         if self.ff is not None:
             x = self.ff_link.step(h, pending, self.ff_norm)
-            pending = (self.ff.forward(x, ctx), self.ff_link)
+            pending = (self._normed(self.ff.forward(x, ctx), self.ff_out_norm), self.ff_link)
         return pending
 
     def leave(self, h, pending, rows, out=None):

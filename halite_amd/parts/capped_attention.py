@@ -14,7 +14,12 @@ parameter:
   ``(1 - lambda) v + lambda v_first`` with the learned number ``value_mix.weight`` and the
   values that a ``"first"`` layer left for the same tokens; the blended values are cached.
 * ``window``: a query sees itself and the ``window - 1`` tokens before it.
-* every head's result is multiplied by ``sigmoid(W_gate x)`` of that head, one number a head.
+* ``head_gate``: every head's result is multiplied by ``sigmoid(W_gate x)`` of that head, one number
+  a head.
+* ``learned_sink``: the softmax's denominator has one more term per head, the exponential of a
+  learned number (tensor ``sink``; it has no key and no value and is neither scaled nor capped).
+* ``own_kv`` false: the mixer has no keys and values (projections, norm, convolutions) of its own and
+  attends to those that an earlier run has left in the cache (the run order says which).
 
 The key and value heads may differ in size; pages hold heads of the larger size (in steps
 of 16), the rest zero.  The result is float32 (the accumulators of the output projection).
@@ -22,6 +27,7 @@ of 16), the rest zero.  The result is float32 (the accumulators of the output pr
 
 from __future__ import annotations
 
+import math
 from typing import Literal
 
 import torch
@@ -47,11 +53,16 @@ class CappedAttentionParams(BaseModel):
     value_mix: Literal["first", "blend"] | None = None
     value_mix_name: str = "values"
     window: StrictInt | None = Field(default=None, gt=0)
+    head_gate: StrictBool = True
+    learned_sink: StrictBool = False
+    own_kv: StrictBool = True
 
     @model_validator(mode="after")
     def _check(self):
         if self.n_heads % self.n_kv_heads:
             raise ValueError(f"{self.n_heads} heads are not a multiple of {self.n_kv_heads} kv heads")
+        if not self.own_kv and (self.bias or self.conv_taps is not None or self.value_mix is not None):
+            raise ValueError("biases, convolutions and a blend of values come with keys and values of the layer's own")
         return self
 
 
@@ -64,7 +75,11 @@ class CappedAttention(Mixer):
         super().__init__(params, build)
         p = params
         self.head_dim = -(-max(p.qk_dim, p.v_dim) // 16) * 16
-        self.n_q, self.n_k, self.n_v = p.n_heads * p.qk_dim, p.n_kv_heads * p.qk_dim, p.n_kv_heads * p.v_dim
+        self.n_q = p.n_heads * p.qk_dim
+        self.n_k, self.n_v = (p.n_kv_heads * p.qk_dim, p.n_kv_heads * p.v_dim) if p.own_kv else (0, 0)
+        # the projections of one product, by the rows each takes of it
+        self.rows = {"q": self.n_q, **({"k": self.n_k, "v": self.n_v} if p.own_kv else {}),
+                     **({"gate": p.n_heads} if p.head_gate else {})}
         self.n_conv = self.n_q + self.n_k + self.n_v
         self.position = None
         if p.position is not None:
@@ -82,8 +97,7 @@ class CappedAttention(Mixer):
     def param_decls(self):
         p = self.p
         d = p.hidden_size
-        decls = {"q.weight": ParamDecl((self.n_q, d)), "k.weight": ParamDecl((self.n_k, d)),
-                 "v.weight": ParamDecl((self.n_v, d)), "gate.weight": ParamDecl((p.n_heads, d))}
+        decls = {f"{name}.weight": ParamDecl((n, d)) for name, n in self.rows.items()}
         if p.bias:
             decls.update({"q.bias": ParamDecl((self.n_q,)), "k.bias": ParamDecl((self.n_k,)),
                           "v.bias": ParamDecl((self.n_v,))})
@@ -92,7 +106,10 @@ class CappedAttention(Mixer):
             decls["k_conv.weight"] = ParamDecl((self.n_k, p.conv_taps))
             decls["v_conv.weight"] = ParamDecl((self.n_v, p.conv_taps))
         decls["q_norm.weight"] = ParamDecl((p.qk_dim,), init="ones")
-        decls["k_norm.weight"] = ParamDecl((p.qk_dim,), init="ones")
+        if p.own_kv:
+            decls["k_norm.weight"] = ParamDecl((p.qk_dim,), init="ones")
+        if p.learned_sink:
+            decls["sink"] = ParamDecl((p.n_heads,))
         if p.value_mix == "blend":
             decls["value_mix.weight"] = ParamDecl(())
         decls["out.weight"] = ParamDecl((d, p.n_heads * p.v_dim))
@@ -101,12 +118,11 @@ class CappedAttention(Mixer):
     def allocate(self, dtypes):
         p = self.p
         dev = self.build.device
-        names = ("q", "k", "v", "gate")
-        if len({dtypes[f"{n}.weight"] for n in names}) != 1:
+        rows = self.rows
+        if len({dtypes[f"{n}.weight"] for n in rows}) != 1:
             raise ValueError("q, k, v and gate weights are stored with different element types")
-        if dtypes["q_norm.weight"] != dtypes["k_norm.weight"]:
+        if p.own_kv and dtypes["q_norm.weight"] != dtypes["k_norm.weight"]:
             raise ValueError("the norms of q and k are stored with different element types")
-        rows = {"q": self.n_q, "k": self.n_k, "v": self.n_v, "gate": p.n_heads}
         # one product for q, k, v and the gate; one bias row and one convolution over the
         # channels of q, k and v
         self.w_in = torch.empty((sum(rows.values()), p.hidden_size), dtype=dtypes["q.weight"], device=dev)
@@ -120,7 +136,7 @@ class CappedAttention(Mixer):
                 raise ValueError("the biases of q, k and v are stored with different element types")
             self.w_bias = torch.empty((self.n_conv,), dtype=dtypes["q.bias"], device=dev)
         out, at = {}, 0
-        for n in names:
+        for n in rows:
             out[f"{n}.weight"] = self.w_in[at : at + rows[n]]
             if n != "gate":
                 if self.w_conv is not None:
@@ -144,7 +160,12 @@ class CappedAttention(Mixer):
                 self.t_in = ops.tile_weight(self.w_in)
             if (p.n_heads * p.v_dim) % 8 == 0 and self.w_out.dtype == torch.bfloat16:
                 self.t_out = ops.tile_weight(self.w_out)
-        self.rule = ops.ScoreRule(softcap=p.softcap) if p.softcap is not None else None
+        sink = {}
+        if p.learned_sink:
+            values = self.w_sink.float().contiguous()
+            sink = dict(sink=True, sink_values=values, sink_values_log2=(values.double() * math.log2(math.e)).float().contiguous())
+        rule = ops.ScoreRule(softcap=p.softcap or 0.0, **sink)
+        self.rule = None if rule.plain() else rule
         # the blend's learned number is a constant once the weights are loaded
         self.blend = float(self.w_value_mix.float().cpu()) if p.value_mix == "blend" else 0.0
 
@@ -176,7 +197,12 @@ class CappedAttention(Mixer):
                                  ctx.token_slot, torch.float32, in_bias=self.w_bias)
         elif self.w_bias is not None:
             ops.bias_rows_(qkv, self.w_bias)
-        q, k, v = qkv[:, : self.n_q], qkv[:, self.n_q : self.n_q + self.n_k], qkv[:, self.n_q + self.n_k :]
+        q = qkv[:, : self.n_q]
+        k = v = None
+        if p.own_kv:
+            k, v = qkv[:, self.n_q : self.n_q + self.n_k], qkv[:, self.n_q + self.n_k :]
+        elif run.appends:
+            raise ValueError("a mixer without keys and values runs on an earlier run's cache")
         other = None
         if p.value_mix is not None:
             left = ctx.__dict__.setdefault("values_left", {})
@@ -186,16 +212,21 @@ class CappedAttention(Mixer):
                 other = left.get(p.value_mix_name)
                 if other is None or other.shape != v.shape:
                     raise ValueError(f"no layer before this one left values {p.value_mix_name!r} of this layer's shape to blend with")
-        pages = dict(token_seg=ctx.token_seg, block_table=group.block_table, k_pages=kv.k, v_pages=kv.v,
-                     page_size=group.page_size, tiled=kv.tiled)
-        appends_here = self.position is None and run.appends
-        packed = ops.head_norm_pack(q, k, v, p.eps, p.n_heads, p.n_kv_heads, p.qk_dim, p.v_dim, D, x.dtype,
-                                    w_q=self.w_q_norm, w_k=self.w_k_norm, norm_v=False, v_other=other, v_mix=self.blend,
-                                    **(dict(positions=ctx.positions, **pages) if appends_here else {}))
+        pages, turn = {}, {}
+        if run.appends:
+            pages = dict(token_seg=ctx.token_seg, block_table=group.block_table, k_pages=kv.k, v_pages=kv.v,
+                         page_size=group.page_size, tiled=kv.tiled)
         if self.position is not None:
             cos, sin = self.position.tables(ctx.max_position + 1)
-            ops.rope_append(packed, ctx.positions, cos, sin, p.n_heads, p.n_kv_heads if run.appends else 0, D,
-                            self.position.rotary_dim, self.position.interleaved, **pages)
+            turn = dict(cos=cos, sin=sin, interleaved=self.position.interleaved)
+        packed = ops.head_norm_pack(q, k, v, p.eps, p.n_heads, p.n_kv_heads if p.own_kv else 0, p.qk_dim, p.v_dim, D, x.dtype,
+                                    w_q=self.w_q_norm, w_k=self.w_k_norm if p.own_kv else self.w_q_norm, norm_v=False,
+                                    v_other=other, v_mix=self.blend, positions=ctx.positions, **turn, **pages)
         out = ctx.attention(packed, packed.shape[1], kv, group, p.n_heads, p.scale, p.window or 0, rule=self.rule)
-        heads = ops.head_gate_cols(out, D, gate, p.v_dim, p.n_heads)
-        return ops.linear(heads, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
+        if p.head_gate:
+            out = ops.head_gate_cols(out, D, gate, p.v_dim, p.n_heads)
+        elif D != p.v_dim:
+            heads = torch.empty((x.shape[0], p.n_heads * p.v_dim), dtype=out.dtype, device=out.device)
+            ops.head_cols(out, D, 0, heads, p.v_dim, 0, p.v_dim, p.n_heads)
+            out = heads
+        return ops.linear(out, self.w_out, out_dtype=torch.float32, tiled=self.t_out)

@@ -1,23 +1,35 @@
-"""A linear attention with one constant decay per head (the "lightning" form): per head a
-state ``S`` of ``qk_dim x v_dim`` numbers, zero when a request starts, that every token decays
-and writes to, ``S_t = decay_h S_(t-1) + k_t v_t^T``, and reads from, ``o_t = S_t^T q_t``, with
-``q = act(W_q x)``, ``k = act(W_k x)``, ``v = act(W_v x)`` (``act`` SiLU) and no other scale.
-The concatenated heads are divided by the root mean square of the whole row, multiplied by a
-weight and by ``sigmoid(W_g x)`` element by element, and projected out.
+"""A linear attention with one constant decay per head ("lightning" attention, retention): per
+head a state ``S`` of ``qk_dim x v_dim`` numbers, zero when a request starts, that every token
+decays and writes to, ``S_t = decay_h S_(t-1) + k_t v_t^T``, and reads from, ``o_t = S_t^T q_t``.
+Its pieces, each a parameter:
+
+* ``activation``: what the projections ``q = act(W_q x)``, ``k = act(W_k x)``, ``v = act(W_v x)`` go
+  through (SiLU, or nothing).
+* ``position``: a rotary encoding of the leading entries of every query and key head.
+* ``key_scale``: a number that the keys are multiplied by (after the rotation).
+* the result is divided by its root mean square, over the whole row of all heads or
+  (``norm_per_head``) each head on its own; with ``norm_weight`` it is multiplied by a weight of the
+  row's size.
+* ``gate``: it is multiplied by ``sigmoid(W_g x)`` or by ``silu(W_g x)`` element by element, and
+  projected out.
 
 Per request the mixer keeps the state (float32); it has no paged cache.  The recurrence is
 the state-space scan's with constant decays and unit step sizes (keys in the place of its
 ``B``, queries of its ``C``, one group a head), so prompts are cut into chunks that are walked
-side by side in the same way.  Decays, state, sums over the state, norm and gate are float32.
+side by side in the same way.  A step of single tokens whose heads are normed each on its own
+is one kernel from the projections to the gated rows.  Rotation, decays, state, sums over the
+state, norm and gate are float32.
 """
 
 from __future__ import annotations
 
+from typing import Literal
+
 import torch
-from pydantic import BaseModel, Field, StrictInt, model_validator
+from pydantic import BaseModel, Field, StrictBool, StrictInt, model_validator
 
 from ..kernels import ops
-from .base import MIXERS, Mixer, ParamDecl, StateNeed
+from .base import MIXERS, Mixer, ParamDecl, RotaryPositionEncoding, StateNeed
 from .state_space import plan_scan_chunks, scan_arrays
 
 
@@ -29,6 +41,12 @@ class DecayAttentionParams(BaseModel):
     decay: list[float]
     """One number in (0, 1] a head."""
     eps: float = Field(gt=0)
+    activation: Literal["silu"] | None = "silu"
+    position: str | None = None
+    key_scale: float = 1.0
+    norm_per_head: StrictBool = False
+    norm_weight: StrictBool = True
+    gate: Literal["sigmoid", "silu"] = "sigmoid"
 
     @model_validator(mode="after")
     def _check(self):
@@ -36,6 +54,8 @@ class DecayAttentionParams(BaseModel):
             raise ValueError(f"{len(self.decay)} decays for {self.n_heads} heads")
         if any(not 0.0 < d <= 1.0 for d in self.decay):
             raise ValueError("a head's decay lies in (0, 1]")
+        if self.activation is not None and (self.position is not None or self.key_scale != 1.0):
+            raise ValueError("queries and keys that are turned or scaled come without an activation")
         return self
 
 
@@ -49,15 +69,27 @@ class DecayAttention(Mixer):
         p = params
         self.inner = p.n_heads * p.v_dim
         self.n_qk = p.n_heads * p.qk_dim
+        self.position = None
+        if p.position is not None:
+            if p.position not in build.positions:
+                raise ValueError(f"linear attention names position encoding {p.position!r}, which the model does not define")
+            self.position = build.positions[p.position]
+            if not isinstance(self.position, RotaryPositionEncoding):
+                raise ValueError(f"position encoding {p.position!r} is not a RotaryPositionEncoding")
+            if self.position.rotary_dim > p.qk_dim:
+                raise ValueError("the position encoding rotates more elements than a head has")
 
     def param_decls(self):
         p = self.p
         d = p.hidden_size
-        return {
+        decls = {
             "v.weight": ParamDecl((self.inner, d)), "k.weight": ParamDecl((self.n_qk, d)),
             "q.weight": ParamDecl((self.n_qk, d)), "gate.weight": ParamDecl((self.inner, d)),
-            "norm.weight": ParamDecl((self.inner,), init="ones"), "out.weight": ParamDecl((d, self.inner)),
         }
+        if p.norm_weight:
+            decls["norm.weight"] = ParamDecl((self.inner,), init="ones")
+        decls["out.weight"] = ParamDecl((d, self.inner))
+        return decls
 
     def allocate(self, dtypes):
         p = self.p
@@ -72,9 +104,12 @@ class DecayAttention(Mixer):
         for n in names:
             out[f"{n}.weight"] = self.w_in[at : at + rows[n]]
             at += rows[n]
-        self.w_norm = torch.empty((self.inner,), dtype=dtypes["norm.weight"], device=dev)
+        self.w_norm = None
+        if p.norm_weight:
+            self.w_norm = torch.empty((self.inner,), dtype=dtypes["norm.weight"], device=dev)
+            out["norm.weight"] = self.w_norm
         self.w_out = torch.empty((p.hidden_size, self.inner), dtype=dtypes["out.weight"], device=dev)
-        out["norm.weight"], out["out.weight"] = self.w_norm, self.w_out
+        out["out.weight"] = self.w_out
         return out
 
     def finalize(self):
@@ -98,8 +133,21 @@ class DecayAttention(Mixer):
         p = self.p
         n_act = self.inner + 2 * self.n_qk
         a = ops.linear(x, self.w_in, out_dtype=torch.float32, tiled=self.t_in)
+        gate, silu = a[:, n_act:], p.gate == "silu"
+        turn = {}
+        if self.position is not None:
+            cos, sin = self.position.tables(ctx.max_position + 1)
+            turn = dict(positions=ctx.positions, cos=cos, sin=sin, interleaved=self.position.interleaved)
+        state = run.state["state"]
+        if p.norm_per_head and x.shape[0] == ctx.n_segs and ops.decay_step_fits(p.qk_dim, p.v_dim):
+            keys, queries = a[:, self.inner : self.inner + self.n_qk], a[:, self.inner + self.n_qk : n_act]
+            gated = ops.decay_step(a[:, : self.inner], keys, queries, gate, self.decay, state, ctx.token_slot, p.eps, x.dtype,
+                                   k_scale=p.key_scale, in_silu=p.activation == "silu", weight=self.w_norm, silu=silu, **turn)
+            return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
+        if turn or p.key_scale != 1.0:
+            ops.rotate_heads_(a[:, self.inner : n_act], 2 * p.n_heads, p.qk_dim, n_scaled=p.n_heads, scale=p.key_scale, **turn)
         # (SiLU of values, keys and queries where the scan reads them: float32 in either mode)
-        y = ops.ssd_scan(a[:, :n_act], None, None, None, None, run.state["state"], ctx.seg_q_start, ctx.seg_q_len,
-                         ctx.token_slot, p.n_heads, fixed_decay=self.decay, in_silu=True, **scan_arrays(ctx))
-        gated = ops.head_norm_gate(y, a[:, n_act:], self.w_norm, p.eps, 1, x.dtype)
+        y = ops.ssd_scan(a[:, :n_act], None, None, None, None, state, ctx.seg_q_start, ctx.seg_q_len, ctx.token_slot,
+                         p.n_heads, fixed_decay=self.decay, in_silu=p.activation == "silu", **scan_arrays(ctx))
+        gated = ops.head_norm_gate(y, gate, self.w_norm, p.eps, p.n_heads if p.norm_per_head else 1, x.dtype, silu=silu)
         return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)

@@ -2,6 +2,8 @@
 
 from __future__ import annotations
 
+import math
+
 import torch
 from typing import Literal
 
@@ -15,6 +17,11 @@ class GatedParams(BaseModel):
     hidden_size: StrictInt = Field(gt=0)
     intermediate_size: StrictInt = Field(gt=0)
     activation: str = "silu"
+    limit: float | None = Field(default=None, gt=0)
+    alpha: float = 1.0
+    up_shift: float = 0.0
+    """Of the activation ``clamped``: ``g * sigmoid(alpha * g) * (u + up_shift)`` with ``g = min(gate,
+    limit)`` and ``u = clamp(up, -limit, limit)`` (no limit: neither is held)."""
     float32_result: StrictBool = False
     """True: the last product's float32 sums come back unrounded (for an arrangement that
     adds them into the float32 stream itself)."""
@@ -30,13 +37,19 @@ class GatedParams(BaseModel):
     def _check(self):
         if self.activation != "silu" and not self.float32_result:
             raise ValueError("products with a norm folded in compute SiLU; another activation comes with float32_result")
+        if self.activation != "clamped" and (self.limit is not None or self.alpha != 1.0 or self.up_shift != 0.0):
+            raise ValueError("limit, alpha and up_shift are the activation 'clamped''s")
         return self
+
+    @property
+    def clamp(self) -> ops.Clamp:
+        return ops.Clamp(math.inf if self.limit is None else self.limit, self.alpha, self.up_shift)
 
 
 @FEED_FORWARDS.register("gated")
 class GatedFeedForward(FeedForward):
     """``linear_out(linear_proj(x) * act(linear_gate(x)))`` without biases, ``act`` SiLU
-    (feedforward.py:204-212) or gelu's tanh form.  Gate and up weights live in one tensor
+    (feedforward.py:204-212), gelu's tanh form, or the clamped form of both products.  Gate and up weights live in one tensor
     ``[2F, d]`` (gate first) so that one product serves both; the activation and
     the multiply are float32 on the accumulators or on the product's output."""
 
@@ -114,9 +127,9 @@ class GatedFeedForward(FeedForward):
         f = self.p.intermediate_size
         m, d = x.shape
         if self.t_gate is not None and x.dtype == torch.bfloat16 and d % 8 == 0 and m <= ops.SKINNY_ROWS:
-            act = ops.gemm_bf16_skinny(x, self.t_gate, w_up=self.t_up, tiled_shape=(f, d), activation=self.p.activation)
+            act = ops.gemm_bf16_skinny(x, self.t_gate, w_up=self.t_up, tiled_shape=(f, d), activation=self.p.activation, clamp=self.p.clamp)
         else:
-            act = ops.gate_mul(ops.linear(x, self.w_gate_up), self.p.activation)
+            act = ops.gate_mul(ops.linear(x, self.w_gate_up), self.p.activation, self.p.clamp)
         return ops.linear(act, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
 
 

@@ -2,7 +2,8 @@
 that every token uses.
 
 The router's logits are a float32 product; a kernel turns them into the chosen experts
-and their weights, a second one sorts the (token, choice) pairs by expert on the device,
+and their weights (by scores with a correction, and among the best groups of experts, where a
+design says so), a second one sorts the (token, choice) pairs by expert on the device,
 and two grouped products run all experts at once on the sorted rows: gate and up with the
 activation in the epilogue, then down.  A last kernel adds the weighted results into the
 float32 stream.  Nothing is read back to the host, so a step's launches depend on its
@@ -44,6 +45,14 @@ class SquaredRelu(BaseModel):
     intermediate_size: StrictInt = Field(gt=0)
 
 
+class ExpertGroups(BaseModel):
+    """The experts form ``count`` equal groups of neighbours; a group counts with the sum of its two
+    largest choice scores, and only experts of the best ``keep`` groups are chosen."""
+
+    count: StrictInt = Field(gt=0)
+    keep: StrictInt = Field(gt=0)
+
+
 class MoEParams(BaseModel):
     hidden_size: StrictInt = Field(gt=0)
     n_experts: StrictInt = Field(gt=0)
@@ -54,6 +63,12 @@ class MoEParams(BaseModel):
     normalize: StrictBool = True
     """The chosen scores are divided by their sum (+ ``norm_eps``)."""
     norm_eps: float = 1e-20
+    weight_scale: float = 1.0
+    """What the (divided) scores are multiplied by to be the experts' weights."""
+    correction: StrictBool = False
+    """True: a tensor ``correction`` ``[n_experts]`` is added to the scores for the choice; the weights are
+    made of the scores without it."""
+    groups: ExpertGroups | None = None
     float32_result: StrictBool = False
     """True: without a stream to add into, the float32 sum comes back unrounded."""
     shared_gate: StrictBool = False
@@ -64,6 +79,10 @@ class MoEParams(BaseModel):
     def _check(self):
         if self.top_k > self.n_experts:
             raise ValueError(f"top_k {self.top_k} of {self.n_experts} experts")
+        g = self.groups
+        if g is not None and (self.n_experts % g.count or g.keep > g.count
+                              or self.top_k > self.n_experts // g.count * g.keep):
+            raise ValueError(f"top_k {self.top_k} of {self.n_experts} experts in {g.count} equal groups of which {g.keep} are kept")
         if self.shared is not None and isinstance(self.expert, SquaredRelu):
             raise ValueError("a shared expert comes with gated experts")
         if self.shared_gate and self.shared is None:
@@ -97,12 +116,14 @@ class MixtureOfExperts(FeedForward):
             decls["shared.down.weight"] = ParamDecl((d, fs))
         if p.shared_gate:
             decls["shared_gate.weight"] = ParamDecl((1, d))
+        if p.correction:
+            decls["correction"] = ParamDecl((p.n_experts,))
         return decls
 
     def allocate(self, dtypes):
         p = self.p
         d, f, n, dev = p.hidden_size, p.expert.intermediate_size, p.n_experts, self.build.device
-        kinds = {dt for name, dt in dtypes.items() if name not in ("router.weight", "shared_gate.weight")}
+        kinds = {dt for name, dt in dtypes.items() if name not in ("router.weight", "shared_gate.weight", "correction")}
         if p.shared_gate and dtypes["shared_gate.weight"] != dtypes["router.weight"]:
             raise ValueError("the router and the shared expert's gate are stored with different element types")
         if len(kinds) != 1:
@@ -117,6 +138,10 @@ class MixtureOfExperts(FeedForward):
         out = {"router.weight": self.w_router[:n]}
         if p.shared_gate:
             out["shared_gate.weight"] = self.w_router[n:]
+        self.w_correction = None
+        if p.correction:
+            self.w_correction = torch.empty((n,), dtype=dtypes["correction"], device=dev)
+            out["correction"] = self.w_correction
         for e in range(n):
             if self.gated:
                 out[f"experts.{e}.gate.weight"] = self.w_gate[e]
@@ -144,7 +169,9 @@ class MixtureOfExperts(FeedForward):
         z = ops.linear(x, self.w_router, out_dtype=torch.float32)
         shared_gate = z[:, p.n_experts:] if p.shared_gate else None
         z = z[:, : p.n_experts]
-        routing = dict(softmax=p.score == "softmax", normalize=p.normalize, norm_eps=p.norm_eps)
+        routing = dict(softmax=p.score == "softmax", normalize=p.normalize, norm_eps=p.norm_eps, scale=p.weight_scale,
+                       correction=self.w_correction, groups=p.groups.count if p.groups else 0,
+                       keep=p.groups.keep if p.groups else 0)
         if n <= ops.ROUTE_SORT_MAX_TOKENS:  # few tokens: one workgroup routes and sorts
             idx, wgt, offsets, tiles, order = ops.moe_route_sort(z, p.top_k, p.n_experts, **routing)
         else:

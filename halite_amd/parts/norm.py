@@ -51,9 +51,13 @@ class RMSNorm(Norm):
         return decls
 
     def finalize(self):
-        # what multiplies the normalised rows: the weight, or weight * scale in float32 (exact
-        # for two 16-bit factors)
-        self.multiplier = self.weight.float() * self.scale.float() if self.p.layer_scale else self.weight
+        # what multiplies the normalised rows: the weight, weight * scale in float32 (exact for
+        # two 16-bit factors), or the weight's distance added up in float32
+        self.multiplier = self.weight
+        if self.p.layer_scale:
+            self.multiplier = self.weight.float() * self.scale.float()
+        elif self.p.weight_offset != 0.0:
+            self.multiplier = self.weight.float() + self.p.weight_offset
 
     def forward(self, h, delta=None, rows=None):
         if self.p.layer_scale:
