@@ -208,3 +208,165 @@ def load_folder(folder: str):
     with open(os.path.join(folder, "config.json")) as f:
         cfg = json.load(f)
     return cfg, load_file(os.path.join(folder, "model.safetensors"))
+
+
+def tokens_with_clear_routing(cfg, w, tokens, margin=0.03, seed=0, tries=600):
+    """``tokens`` with as few replaced as it takes for no router of the model to make a choice (of a
+    group or of an expert) closer than ``margin``: arithmetic in 16 bits moves a score by about a
+    hundredth, and a choice that turns over makes another model of it.  The first token with such a
+    call is drawn anew until there is none (earlier tokens stay as they are: the model is causal)."""
+    gen = torch.Generator().manual_seed(seed)
+    ids = list(tokens)
+    for _ in range(tries):
+        margins = []
+        forward(cfg, w, ids, margins_out=margins)
+        if not margins:
+            return ids
+        close = (torch.stack(margins).min(0).values < margin).nonzero()
+        if close.numel() == 0:
+            return ids
+        ids[int(close[0])] = int(torch.randint(0, cfg["vocab"], (1,), generator=gen))
+    raise RuntimeError("no sequence without a close call of a router")
+
+
+# ---- configurations, tensors and folders for the tests ------------------------------------------
+def rot(base, dims):
+    return {"base": base, "dims": dims}
+
+
+def attention_layer(heads, kv_heads, dim, vdim, scale, rot=None, kv_from=None, mlp=None):
+    mixer = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale}
+    for key, value in (("rot", rot), ("kv_from", kv_from)):
+        if value is not None:
+            mixer[key] = value
+    return {"type": "attention", "mixer": mixer, "mlp": mlp}
+
+
+def retention_layer(heads, dim, vdim, decay, rot=None, mlp=None):
+    mixer = {"heads": heads, "dim": dim, "vdim": vdim, "decay": list(decay)}
+    if rot is not None:
+        mixer["rot"] = rot
+    return {"type": "retention", "mixer": mixer, "mlp": mlp}
+
+
+def dense(ff, limit):
+    return {"kind": "dense", "ff": ff, "limit": limit}
+
+
+def moe(experts, top, ff, scale=1.0, groups=None, shared=None):
+    out = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top, "scale": scale}}
+    if groups is not None:
+        out["router"]["groups"] = {"count": groups[0], "keep": groups[1]}
+    if shared is not None:
+        out["shared"] = {"ff": shared}
+    return out
+
+
+def model_cfg(width, vocab, layers, eps=1e-5, logit_scale=1.0):
+    return {"architecture": "Divuzen", "vocab": vocab, "width": width, "norm": {"eps": eps}, "logit_scale": logit_scale,
+            "layers": layers}
+
+
+def tensor_shapes(cfg) -> dict:
+    """Name -> shape of every tensor of a folder."""
+    W = cfg["width"]
+    out = {"embed": (cfg["vocab"], W), "final.norm": (W,)}
+    for i, layer in enumerate(cfg["layers"]):
+        pre, m = f"l{i}.", layer["mixer"]
+        mix = pre + "mix."
+        out[pre + "norm1"], out[pre + "norm1b"] = (W,), (W,)
+        if layer["type"] == "attention":
+            out[mix + "q"], out[mix + "q.norm"] = (m["heads"] * m["dim"], W), (m["dim"],)
+            out[mix + "sink"], out[mix + "o"] = (m["heads"],), (W, m["heads"] * m["vdim"])
+            if m.get("kv_from") is None:
+                out[mix + "k"], out[mix + "k.norm"] = (m["kv_heads"] * m["dim"], W), (m["dim"],)
+                out[mix + "v"] = (m["kv_heads"] * m["vdim"], W)
+        else:
+            nk, nv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            out[mix + "q"], out[mix + "k"], out[mix + "v"], out[mix + "g"], out[mix + "o"] = (nk, W), (nk, W), (nv, W), (nv, W), (W, nv)
+        f = layer.get("mlp")
+        if f is None:
+            continue
+        out[pre + "norm2"], out[pre + "norm2b"] = (W,), (W,)
+        if f["kind"] == "dense":
+            parts = [("", f["ff"])]
+        else:
+            n = f["router"]["experts"]
+            out[pre + "mlp.router"], out[pre + "mlp.correction"] = (n, W), (n,)
+            parts = [(f"e{e}.", f["expert"]["ff"]) for e in range(n)]
+            if f.get("shared"):
+                parts.append(("shared.", f["shared"]["ff"]))
+                out[pre + "mlp.shared.sg"] = (1, W)
+        for name, ff in parts:
+            out[f"{pre}mlp.{name}gate"], out[f"{pre}mlp.{name}up"], out[f"{pre}mlp.{name}down"] = (ff, W), (ff, W), (W, ff)
+    return out
+
+
+def random_weights(cfg, seed, std=0.12, stored=torch.bfloat16):
+    """Matrices N(0, std); the model's norms around zero, those of q and k around one; sinks of a
+    size that counts and corrections that make choice scores of either sign; rounded to ``stored`` so
+    that engine and plain model hold the same numbers."""
+    gen = torch.Generator().manual_seed(seed)
+    out = {}
+    for name, shape in tensor_shapes(cfg).items():
+        parts = name.split(".")
+        last = parts[-1]
+        r = lambda scale=1.0: scale * torch.randn(shape, generator=gen)  # noqa: E731
+        if name == "embed":
+            t = r(0.7)
+        elif last in ("norm1", "norm1b", "norm2", "norm2b") or name == "final.norm":
+            t = r(0.2)
+        elif last == "norm":
+            t = 1.0 + r(0.2)
+        elif last == "sink":
+            t = 1.0 + r(1.5)
+        elif last == "correction":
+            t = r(0.3) - 0.5
+        elif last == "router":
+            t = r(4 * std)
+        elif last in ("gate", "up", "down"):
+            t = r(1.5 * std)
+        else:
+            t = r(std)
+        out[name] = t.to(stored).float()
+    return out
+
+
+def write_model_folder(folder, cfg, weights, dtype=torch.bfloat16):
+    from safetensors.torch import save_file
+
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(cfg, f)
+    save_file({k: v.to(dtype).contiguous() for k, v in weights.items()}, os.path.join(folder, "model.safetensors"))
+    return folder
+
+
+# both mixers and both feed-forwards; grouped key/value heads; a retention head whose values are
+# longer than its keys; an attention that borrows its keys from the layer before, with a scale of its own;
+# groups of two experts; a limit that holds many products
+DIV_A = model_cfg(64, 331, [
+    retention_layer(2, 16, 24, [0.9, 0.995], rot=rot(1000.0, 8), mlp=dense(48, 0.8)),
+    attention_layer(4, 2, 16, 16, 0.3, rot=rot(500.0, 8), mlp=moe(8, 2, 32, scale=1.7, groups=(4, 2), shared=24)),
+    attention_layer(4, 2, 16, 16, 0.2, rot=rot(500.0, 8), kv_from=1, mlp=dense(48, 1.5)),
+    retention_layer(2, 16, 24, [0.97, 1.0], rot=rot(1000.0, 16), mlp=moe(8, 3, 32, scale=0.8, groups=(2, 1))),
+], logit_scale=0.3)
+# an attention first, without rotation and feed-forward, two layers that borrow from it and one in
+# between with keys of its own that another borrows; values larger and smaller than keys; a whole head rotated;
+# every expert chosen, and one of three, without groups; a retention without rotation
+DIV_B = model_cfg(48, 257, [
+    attention_layer(6, 3, 8, 24, 0.5),
+    retention_layer(3, 8, 16, [0.5, 0.97, 1.0], mlp=moe(5, 5, 24, scale=2.5, shared=16)),
+    attention_layer(6, 3, 8, 24, 0.3, kv_from=0, mlp=moe(3, 1, 36)),
+    attention_layer(2, 2, 24, 8, 0.25, rot=rot(200.0, 24), mlp=dense(40, 3.0)),
+    attention_layer(6, 3, 8, 24, 0.4, kv_from=0),
+    attention_layer(2, 2, 24, 8, 0.3, rot=rot(200.0, 24), kv_from=3, mlp=moe(6, 2, 20, scale=1.2, groups=(3, 2))),
+])
+# sizes that are multiples of nothing; one key/value head; retention states that no fused step takes
+# (value heads of 10) and one head without decay; groups of one expert; a group of six
+DIV_C = model_cfg(42, 203, [
+    attention_layer(5, 1, 12, 20, 0.2, rot=rot(77.0, 6), mlp=moe(6, 3, 20, scale=1.3, groups=(6, 4), shared=28)),
+    retention_layer(3, 14, 10, [0.8, 0.99, 1.0], rot=rot(90.0, 6), mlp=dense(30, 0.5)),
+    attention_layer(5, 1, 12, 20, 0.25, rot=rot(77.0, 6), kv_from=0),
+    retention_layer(1, 20, 12, [1.0], rot=rot(50.0, 20), mlp=moe(12, 2, 20, groups=(2, 1), shared=10)),
+], eps=1e-6, logit_scale=2.0)
