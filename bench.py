@@ -104,7 +104,7 @@ class Families:
                    "streams_step", "head_norm_pack", "head_gate_cols", "bias_rows_", "silu_rows", "token_gate", "gate_mul",
                    "turn_pack", "normed_sum", "soft_cap_", "cast_cols", "token_shift", "pair_embedding", "stream_step")
     RECURRENT = ("short_conv", "short_conv_carry", "short_conv_through", "ssd_scan", "delta_rule", "wkv_decay", "wkv_scan",
-                 "wkv_step", "gated_scan")
+                 "wkv_step", "gated_scan", "rotate_heads_", "decay_step", "decay_chunks")
 
     def __init__(self):
         self.spans = []
@@ -506,7 +506,7 @@ def diporax_layer_kinds(n_layers):
     return [("attention", "attention", "latent_attention", "lightning")[i % 4] for i in range(n_layers)]
 
 
-def diporax_config(s, n_layers, window):
+def diporax_config(s, n_layers, window, kinds=None, side=True):
     rot = dict(base=500000.0, dims=64, scaling=dict(factor=8.0, original=4096, fast=32.0, slow=1.0))
     attention = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5,
                      conv=s["conv"], rot=rot, softcap=30.0, v_mix=True, bias=True)
@@ -518,23 +518,23 @@ def diporax_config(s, n_layers, window):
     moe = dict(kind="moe", router=dict(experts=s["experts"], top=s["top"]), expert=dict(ff=s["gated_ff"]),
                shared=dict(ff=s["shared_ff"]))
     return dict(architecture="Diporax", vocab=COMPARISON_VOCAB, width=s["width"], norm=dict(eps=1e-6),
-                token_side=dict(dim=s["side"]), max_positions=8192,
-                layers=[dict(type=kind, mixer=mixers[kind], mlp=moe) for kind in diporax_layer_kinds(n_layers)])
+                token_side=dict(dim=s["side"]) if side else None, max_positions=8192,
+                layers=[dict(type=kind, mixer=mixers[kind], mlp=moe) for kind in kinds or diporax_layer_kinds(n_layers)])
 
 
-def diporax_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2) -> dict:
+def diporax_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2, kinds=None, side=True) -> dict:
     """As ``vepitar_work``; the family ``recurrent`` is the convolutions and the linear attention
     (four float32 operations per token and entry of a head's state: decay and write, read), whose
     decode step reads and writes every request's state."""
     d, h, kv, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
-    kinds = diporax_layer_kinds(n_layers)
+    kinds = kinds or diporax_layer_kinds(n_layers)
     n_att, n_lat, n_dec = kinds.count("attention"), kinds.count("latent_attention"), kinds.count("lightning")
     DL = -(-(s["rot_dim"] + s["kv_rank"]) // 16) * 16
     inner = s["decay_heads"] * s["decay_dim"]
     att = d * ((h + 2 * kv) * D + h) + h * D * d
     lat = d * (s["q_rank"] + s["kv_rank"] + s["rot_dim"] + h) + s["q_rank"] * h * (D + s["rot_dim"]) + h * D * d
     dec = d * 4 * inner + inner * d
-    every = d * (s["experts"] + 1) + s["shared_ff"] * d + 2 * d * s["side"]  # router, shared down, token input
+    every = d * (s["experts"] + 1) + s["shared_ff"] * d + (2 * d * s["side"] if side else 0)  # router, shared down, token input
     linear = n_att * att + n_lat * lat + n_dec * dec + n_layers * every
     heads = n_lat * (h * D * s["kv_rank"] + h * s["kv_rank"] * D)
     shared_in = 2 * d * s["shared_ff"]
@@ -616,6 +616,75 @@ def nodupel_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2, window=0) -> 
     return out
 
 
+# Layers of the Divuzen design at the same two sizes: retention and rotated attention with sinks in
+# turn, the second attention on the first one's keys and values; a clamped dense feed-forward after
+# every other layer and sixteen experts in four groups of which two are kept after the others.
+# Beside it Diporax layers of the same width, heads, states and experts: linear attention and capped
+# attention in turn, without its token input; the closest design that the engine serves.
+DIVUZEN_SIZES = {
+    "2048-wide": dict(DIPORAX_SIZES["2048-wide"], dense_ff=5120, groups=4, keep=2),
+    "4096-wide": dict(DIPORAX_SIZES["4096-wide"], dense_ff=10240, groups=4, keep=2),
+}
+
+
+def divuzen_layer_kinds(n_layers):
+    """(mixer, feed-forward) of every layer."""
+    mixers = ("retention", "attention", "retention", "borrowing")
+    return [(mixers[i % 4], "dense" if i % 4 in (0, 3) else "moe") for i in range(n_layers)]
+
+
+def diporax_kinds_beside_divuzen(n_layers):
+    return ["lightning" if i % 2 == 0 else "attention" for i in range(n_layers)]
+
+
+def divuzen_config(s, n_layers, window):
+    attention = dict(heads=s["heads"], kv_heads=s["kv_heads"], dim=s["dim"], vdim=s["dim"], scale=s["dim"] ** -0.5,
+                     rot=dict(base=500000.0, dims=64))
+    decay = [1.0 - 2.0 ** -(5 + 8 * h / s["decay_heads"]) for h in range(s["decay_heads"])]
+    retention = dict(heads=s["decay_heads"], dim=s["decay_dim"], vdim=s["decay_dim"], decay=decay,
+                     rot=dict(base=10000.0, dims=s["decay_dim"]))
+    mlps = {"dense": dict(kind="dense", ff=s["dense_ff"], limit=7.0),
+            "moe": dict(kind="moe", router=dict(experts=s["experts"], top=s["top"], scale=2.5,
+                                                groups=dict(count=s["groups"], keep=s["keep"])),
+                        expert=dict(ff=s["gated_ff"]), shared=dict(ff=s["shared_ff"]))}
+    layers = []
+    for mixer, mlp in divuzen_layer_kinds(n_layers):
+        source = [i for i, layer in enumerate(layers) if layer["type"] == "attention" and "kv_from" not in layer["mixer"]]
+        if mixer == "retention":
+            layers.append(dict(type="retention", mixer=retention, mlp=mlps[mlp]))
+        else:
+            layers.append(dict(type="attention", mlp=mlps[mlp],
+                               mixer=dict(attention, kv_from=source[-1]) if mixer == "borrowing" else attention))
+    return dict(architecture="Divuzen", vocab=COMPARISON_VOCAB, width=s["width"], norm=dict(eps=1e-6), max_positions=8192,
+                logit_scale=0.5, layers=layers)
+
+
+def divuzen_work(s, n_layers, tokens, batch=0, kv_tokens=0, elt=2) -> dict:
+    """As ``diporax_work``; the family ``recurrent`` is the rotation of queries and keys and the retention (of
+    a decode step with its norms and gates)."""
+    d, h, kv, D = s["width"], s["heads"], s["kv_heads"], s["dim"]
+    kinds = divuzen_layer_kinds(n_layers)
+    n_own, n_borrow = (sum(mixer == name for mixer, _ in kinds) for name in ("attention", "borrowing"))
+    n_ret = n_layers - n_own - n_borrow
+    n_moe = sum(mlp == "moe" for _, mlp in kinds)
+    inner = s["decay_heads"] * s["decay_dim"]
+    linear = n_own * d * 2 * kv * D + (n_own + n_borrow) * 2 * h * D * d + n_ret * 5 * d * inner
+    linear += (n_layers - n_moe) * 3 * d * s["dense_ff"] + n_moe * (d * (s["experts"] + 1) + s["shared_ff"] * d)
+    shared_in = 2 * d * s["shared_ff"]
+    expert = 3 * d * s["gated_ff"]
+    state = s["decay_heads"] * s["decay_dim"] * s["decay_dim"]
+    if batch == 0:
+        return {"gemm": 2.0 * tokens * linear + 2.0 * COMPARISON_VOCAB * d,
+                "grouped": 2.0 * tokens * n_moe * (shared_in + s["top"] * expert),
+                "attention": 2.0 * tokens * tokens * h * D * (n_own + n_borrow),
+                "recurrent": tokens * n_ret * 4.0 * state}
+    used = min(s["experts"], batch * s["top"])
+    return {"gemm": 2.0 * (linear + COMPARISON_VOCAB * d),
+            "grouped": 2.0 * n_moe * (shared_in + used * expert),
+            "attention": 2.0 * kv_tokens * 2 * kv * D * (n_own + n_borrow),
+            "recurrent": 2.0 * batch * n_ret * 2 * state * 4 / elt}
+
+
 DESIGNS = {
     "kavuvik": dict(label="Kavuvik", sizes=lambda: KAVUVIK_SIZES, config=lambda s, n, w: kavuvik_config(s, n, w),
                     llama=lambda s, n: closest_llama_config(s, n),
@@ -636,11 +705,17 @@ DESIGNS = {
                                 config=lambda s, n: zabunex_config(s, n, 0, zabunex_kinds_beside_nodupel(n)),
                                 work=lambda s, n, t, b, kv, elt: zabunex_work(s, n, t, b, kv, elt, zabunex_kinds_beside_nodupel(n))),
                     work=lambda s, n, t, b, kv, elt, w=0: nodupel_work(s, n, t, b, kv, elt, w)),
+    "divuzen": dict(label="Divuzen", sizes=lambda: DIVUZEN_SIZES, config=lambda s, n, w: divuzen_config(s, n, w),
+                    beside=dict(key="diporax", label="Diporax",
+                                config=lambda s, n: diporax_config(s, n, 0, diporax_kinds_beside_divuzen(n), side=False),
+                                work=lambda s, n, t, b, kv, elt: diporax_work(s, n, t, b, kv, elt, diporax_kinds_beside_divuzen(n),
+                                                                              side=False)),
+                    work=lambda s, n, t, b, kv, elt: divuzen_work(s, n, t, b, kv, elt)),
 }
 
 
 def design_comparison(args) -> dict:
-    """``--workload kavuvik`` / ``zabunex`` / ``vepitar`` / ``diporax`` / ``nodupel``: prefill and decode throughput of the design's
+    """``--workload kavuvik`` / ``zabunex`` / ``vepitar`` / ``diporax`` / ``nodupel`` / ``divuzen``: prefill and decode throughput of the design's
     layers at two sizes beside the closest Llama layers, with each family of kernels against
     its roofline (the products and the attention of a prompt against the bf16 matrix peak, a
     recurrence against the float32 vector peak, those of a decode step against the memory's
@@ -795,10 +870,11 @@ def main() -> int:
                          "by default (scheduling_steps_ahead); 0: read every step's tokens before the next is put together")
     ap.add_argument("--sampling", default="greedy", choices=["greedy", "temperature", "top_p", "top_k", "all"],
                     help="how the decode steps sample (the contract's line is greedy)")
-    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed3b", "llama70b", "kavuvik", "zabunex", "vepitar", "diporax", "nodupel"],
+    ap.add_argument("--workload", default="decode8b", choices=["decode8b", "mixed3b", "llama70b", "kavuvik", "zabunex", "vepitar", "diporax", "nodupel", "divuzen"],
                     help="decode8b: the headline line; mixed3b and llama70b run requests through the scheduler; "
                          "kavuvik, zabunex: prefill and decode of that design's layers at two sizes beside the closest Llama layers; "
-                         "vepitar, nodupel: the same beside Zabunex layers of equal size")
+                         "vepitar, nodupel: the same beside Zabunex layers of equal size; diporax: beside Vepitar layers; "
+                         "divuzen: beside Diporax layers")
     ap.add_argument("--sizes", default="", help="kavuvik: only these sizes (names with commas between them)")
     ap.add_argument("--only-new", action="store_true", help="kavuvik: leave the Llama layers out (for profiles)")
     ap.add_argument("--window", type=int, default=0,
