@@ -198,7 +198,7 @@ int hal_moe_sort(const int* idx, int n, int E, int tile, int* offsets, int* tile
 int hal_moe_combine(float* h, const float* y, const float* wgt, const float* extra,
                     const float* extra_gate, int ld_gate, int top, int d, int n_tokens, int overwrite,
                     hipStream_t stream);
-// hal_moe_route and hal_moe_sort in one workgroup (for steps of few tokens)
+// hal_moe_route and hal_moe_sort in one workgroup (for steps of few tokens; at most 256 experts)
 int hal_moe_route_sort(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
                        float scale, const void* correction, int c_dtype, int groups, int keep, int* idx, float* wgt, int n_tokens, int tile, int* offsets, int* tile_offsets,
                        int* sorted, hipStream_t stream);
@@ -281,6 +281,20 @@ int hal_delta_rule(const float* r, int ldr, const float* k, int ldk, const float
                    float unit_eps, float* pre, float* state, const int* seg_q_start,
                    const int* seg_q_len, const int* token_slot, float* o, int n_tokens, int n_segs,
                    int H, int D, hipStream_t stream);
+// What takes the requests' states through their chunks: S <- decays[c][h] S + sums[c][h] chunk by chunk of
+// a segment, leaving in sums the state that each chunk starts from (NP numbers a head).
+int hal_ssd_carry(float* state, float* sums, const float* decays, const int* seg_chunks, const int* seg_q_start,
+                  const int* seg_q_len, const int* token_slot, int n_segs, int heads, int NP, hipStream_t stream);
+// The recurrence of hal_decay_step over segments cut into chunks of up to 64 tokens (chunks, seg_chunks,
+// sums, decays as for hal_ssd_scan), as float32 products on the matrix cores.  powers [H, 65]: decay_h to
+// the powers 0 .. 64.  gate null: float32 rows y as they are, else normed, weighted and gated as there.
+// N <= 128, P <= 256.
+int hal_decay_chunks(const float* v, const float* k, const float* q, const float* gate, int ld, int in_silu,
+                     const int* positions, const float* cos_t, const float* sin_t, int rot, int table_len,
+                     int interleaved, float k_scale, const float* powers, float* state, const int* seg_q_start,
+                     const int* seg_q_len, const int* token_slot, const int* chunks, const int* seg_chunks,
+                     int n_chunks, float* sums, float* decays, const void* w, int w_dtype, int silu, float eps,
+                     void* out, int dtype, int n_segs, int H, int N, int P, hipStream_t stream);
 // The first `heads` heads of `dim` entries of float32 rows x turned in place by the tokens' positions:
 // the pairs of their first `rot` entries, by the table cos_t, sin_t [table_len, rot / 2]; the first
 // n_scaled heads are then multiplied by `scale`.  rot 0: scaled alone.

@@ -184,93 +184,85 @@ extern "C" int hal_scale_f32(float* x, long long n, float s, hipStream_t stream)
 // [E]: added to the scores for the choice alone.  `groups` > 0: the experts form so many equal
 // groups of neighbours, and only experts of the `keep` groups with the largest sums of their two
 // largest (corrected) scores are chosen from (the lower group wins a tie).
+//
+// One wave a token: lane l holds the scores of the experts l, l + 64, ... in W words (W is the
+// build for so many experts: the code of a step that runs once is mostly fetched, so it is kept
+// short).  A score is shown to all lanes by reading it from its lane at a uniform index.
 // ---------------------------------------------------------------------------------
-// The groups' part: a group's two largest scores are found across the wave, four groups at a time;
-// lane g % 64 keeps the sum of group g in word g / 64, counts the groups before it, and says
-// whether its group stays open; the scores of closed groups become -infinity.
-#define MOE_ROUTE_PER_LANE (MOE_MAX_EXPERTS / HAL_WAVE)
-__device__ __forceinline__ void moe_close_groups(float (&s)[MOE_ROUTE_PER_LANE], int E, int groups, int keep, int lane) {
-  const int per = E / groups, words = (E + HAL_WAVE - 1) / HAL_WAVE, gwords = (groups + HAL_WAVE - 1) / HAL_WAVE;
-  float mine[MOE_ROUTE_PER_LANE];
-#pragma unroll
-  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) mine[u] = -INFINITY;
-  constexpr int SIDE = 4;
-  for (int g0 = 0; g0 < groups; g0 += SIDE) {
-    float a[SIDE], b[SIDE];  // the largest and the second largest
-#pragma unroll
-    for (int v = 0; v < SIDE; ++v) a[v] = b[v] = -INFINITY;
-#pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
-      if (u >= words) continue;
-      const int e = lane + u * HAL_WAVE;
-      const int g = e < E ? e / per - g0 : -1;
-#pragma unroll
-      for (int v = 0; v < SIDE; ++v)
-        if (g == v) b[v] = fmaxf(b[v], fminf(a[v], s[u])), a[v] = fmaxf(a[v], s[u]);
-    }
-#pragma unroll
-    for (int off = HAL_WAVE / 2; off > 0; off >>= 1) {
-#pragma unroll
-      for (int v = 0; v < SIDE; ++v) {
-        const float oa = __shfl_xor(a[v], off, HAL_WAVE), ob = __shfl_xor(b[v], off, HAL_WAVE);
-        b[v] = fmaxf(fminf(a[v], oa), fmaxf(b[v], ob));
-        a[v] = fmaxf(a[v], oa);
-      }
-    }
-#pragma unroll
-    for (int v = 0; v < SIDE; ++v) {
-      const int g = g0 + v;
-      const float sum = per > 1 ? a[v] + b[v] : a[v];
-#pragma unroll
-      for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-        if (g < groups && u == g / HAL_WAVE && lane == g % HAL_WAVE) mine[u] = sum;
-    }
-  }
-  int ahead[MOE_ROUTE_PER_LANE];  // groups that come before mine
-#pragma unroll
-  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) ahead[u] = 0;
-#pragma unroll
-  for (int w = 0; w < MOE_ROUTE_PER_LANE; ++w) {
-    if (w >= gwords) continue;
-    const int n = groups - w * HAL_WAVE < HAL_WAVE ? groups - w * HAL_WAVE : HAL_WAVE;
-    for (int l = 0; l < n; ++l) {
-      const float other = __shfl(mine[w], l, HAL_WAVE);
-#pragma unroll
-      for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-        if (u < gwords && (other > mine[u] || (other == mine[u] && w * HAL_WAVE + l < u * HAL_WAVE + lane))) ++ahead[u];
-    }
-  }
-#pragma unroll
-  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
-    if (u >= words) continue;
-    const int e = lane + u * HAL_WAVE, g = e < E ? e / per : 0;
-    int before = 0;
-#pragma unroll
-    for (int w = 0; w < MOE_ROUTE_PER_LANE; ++w) {
-      if (w >= gwords) continue;
-      const int got = __shfl(ahead[w], g % HAL_WAVE, HAL_WAVE);
-      if (w == g / HAL_WAVE) before = got;
-    }
-    if (before >= keep) s[u] = -INFINITY;
-  }
-}
-// One wave a token: lane l holds the scores of the experts l, l + 64, ...; each of the `top`
-// rounds finds the largest score that is left (the lower index on a tie) across the wave.
 struct MoeChoice {
   int softmax, normalize;
   float norm_eps, scale;
   const void* correction;
   int c_dtype, groups, keep;
 };
+__device__ __forceinline__ float lane_value(float v, int lane) {
+  return __uint_as_float(__builtin_amdgcn_readlane(__float_as_uint(v), lane));
+}
+// how many of the first n numbers (lane l of word w holds number w * 64 + l) come before lane's own
+// ones: larger, or equal and of a lower index
+template <int W>
+__device__ __forceinline__ void places_before(const float (&v)[W], int n, int lane, int (&before)[W]) {
+#pragma unroll
+  for (int u = 0; u < W; ++u) before[u] = 0;
+#pragma unroll
+  for (int w = 0; w < W; ++w) {
+    const int m = n - w * HAL_WAVE < HAL_WAVE ? n - w * HAL_WAVE : HAL_WAVE;
+    for (int l = 0; l < m; ++l) {
+      const float x = lane_value(v[w], l);
+#pragma unroll
+      for (int u = 0; u < W; ++u)
+        before[u] += (x > v[u] || (x == v[u] && w * HAL_WAVE + l < u * HAL_WAVE + lane)) ? 1 : 0;
+    }
+  }
+}
+
+// The scores of experts outside the best groups become -infinity.  Lane g (word g / 64) holds what
+// belongs to group g.
+template <int W>
+__device__ __forceinline__ void moe_close_groups(float (&s)[W], int E, int groups, int keep, int lane) {
+  const int per = E / groups;
+  float first[W], second[W];  // a group's two largest
+#pragma unroll
+  for (int u = 0; u < W; ++u) first[u] = second[u] = -INFINITY;
+  int g = 0, in_group = 0;
+#pragma unroll
+  for (int w = 0; w < W; ++w) {
+    const int m = E - w * HAL_WAVE < HAL_WAVE ? E - w * HAL_WAVE : HAL_WAVE;
+    for (int l = 0; l < m; ++l) {
+      const float x = lane_value(s[w], l);
+#pragma unroll
+      for (int u = 0; u < W; ++u)
+        if (lane + u * HAL_WAVE == g) second[u] = fmaxf(second[u], fminf(first[u], x)), first[u] = fmaxf(first[u], x);
+      if (++in_group == per) in_group = 0, ++g;
+    }
+  }
+  if (per > 1) {
+#pragma unroll
+    for (int u = 0; u < W; ++u) first[u] += second[u];
+  }
+  int before[W];
+  places_before<W>(first, groups, lane, before);
+#pragma unroll
+  for (int u = 0; u < W; ++u) {
+    const int e = lane + u * HAL_WAVE, mine = e < E ? e / per : 0;
+    int place = 0;
+#pragma unroll
+    for (int w = 0; w < W; ++w) {
+      const int got = __shfl(before[w], mine % HAL_WAVE, HAL_WAVE);
+      if (w == mine / HAL_WAVE) place = got;
+    }
+    if (place >= keep) s[u] = -INFINITY;
+  }
+}
+
+template <int W>
 __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int ldz, int E, int top, const MoeChoice& how,
                                                 int* __restrict__ idx, float* __restrict__ wgt, int t, int lane) {
   const float* zr = z + (size_t)t * ldz;
-  float s[MOE_ROUTE_PER_LANE];
-  float w[MOE_ROUTE_PER_LANE];  // the scores as weights, where the choice is made by other numbers
-  const bool apart = how.correction != nullptr || how.groups > 0;
+  float s[W], w[W];  // what the choice is made by, and the scores as weights
   float zmax = -INFINITY;
 #pragma unroll
-  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
+  for (int u = 0; u < W; ++u) {
     const int e = lane + u * HAL_WAVE;
     s[u] = e < E ? zr[e] : -INFINITY;
     zmax = fmaxf(zmax, s[u]);
@@ -279,65 +271,76 @@ __device__ __forceinline__ void moe_route_token(const float* __restrict__ z, int
     zmax = wave_max(zmax);
     float part = 0.f;
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
-      s[u] = lane + u * HAL_WAVE < E ? expf(s[u] - zmax) : -INFINITY;
-      part += lane + u * HAL_WAVE < E ? s[u] : 0.f;
+    for (int u = 0; u < W; ++u) {
+      w[u] = expf(s[u] - zmax);  // (0 beyond the experts)
+      part += w[u];
     }
     const float denom = wave_sum(part);
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) s[u] = s[u] / denom;
+    for (int u = 0; u < W; ++u) w[u] = w[u] / denom;
   } else {
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-      if (lane + u * HAL_WAVE < E) s[u] = 1.0f / (1.0f + expf(-s[u]));
+    for (int u = 0; u < W; ++u) w[u] = 1.0f / (1.0f + expf(-s[u]));
   }
-  if (apart) {
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
-      const int e = lane + u * HAL_WAVE;
-      w[u] = s[u];
-      if (how.correction && e < E) s[u] += load_as_f32(how.correction, how.c_dtype, e);
-    }
+  for (int u = 0; u < W; ++u) {
+    const int e = lane + u * HAL_WAVE;
+    s[u] = w[u];
+    if (how.correction && e < E) s[u] += load_as_f32(how.correction, how.c_dtype, e);
+    if (e >= E || s[u] != s[u]) s[u] = -INFINITY;  // (a choice among numbers that are none is some choice)
   }
-  if (how.groups > 0) moe_close_groups(s, E, how.groups, how.keep, lane);
-  float sum = 0.f;
-  float kept[MOE_ROUTE_PER_LANE];  // lane j % 64 keeps the j-th choice's score in kept[j / 64]
-  for (int j = 0; j < top; ++j) {
-    float best = -INFINITY;
-    int best_e = MOE_MAX_EXPERTS;
+  if (how.groups > 0) moe_close_groups<W>(s, E, how.groups, how.keep, lane);
+  if constexpr (W <= 2) {  // few experts: every expert's place among all
+    int place[W];
+    places_before<W>(s, E, lane, place);
+    float part = 0.f;
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-      if (s[u] > best) best = s[u], best_e = lane + u * HAL_WAVE;  // rising index: the lower one stays on a tie
+    for (int u = 0; u < W; ++u) part += (lane + u * HAL_WAVE < E && place[u] < top) ? w[u] : 0.f;
+    const float sum = wave_sum(part) + how.norm_eps;
 #pragma unroll
-    for (int off = HAL_WAVE / 2; off > 0; off >>= 1) {
-      const float ob = __shfl_xor(best, off, HAL_WAVE);
-      const int oe = __shfl_xor(best_e, off, HAL_WAVE);
-      if (ob > best || (ob == best && oe < best_e)) best = ob, best_e = oe;
+    for (int u = 0; u < W; ++u) {
+      if (lane + u * HAL_WAVE >= E || place[u] >= top) continue;
+      idx[(size_t)t * top + place[u]] = lane + u * HAL_WAVE;
+      wgt[(size_t)t * top + place[u]] = (how.normalize ? w[u] / sum : w[u]) * how.scale;
     }
-    float own = 0.f;
+  } else {  // each of the `top` rounds finds the largest that is left across the wave
+    float sum = 0.f, mine[W];
+    int place[W];
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-      if (lane + u * HAL_WAVE == best_e) {
-        s[u] = -INFINITY;  // taken
-        if (apart) own = w[u];
+    for (int u = 0; u < W; ++u) place[u] = -1;
+    for (int j = 0; j < top; ++j) {
+      float best = -INFINITY;
+      int best_e = MOE_MAX_EXPERTS;
+#pragma unroll
+      for (int u = 0; u < W; ++u)  // rising index: the lower one stays on a tie
+        if (lane + u * HAL_WAVE < E && place[u] < 0 && (s[u] > best || best_e == MOE_MAX_EXPERTS)) best = s[u], best_e = lane + u * HAL_WAVE;
+#pragma unroll
+      for (int off = HAL_WAVE / 2; off > 0; off >>= 1) {
+        const float ob = __shfl_xor(best, off, HAL_WAVE);
+        const int oe = __shfl_xor(best_e, off, HAL_WAVE);
+        if (oe < MOE_MAX_EXPERTS && (best_e == MOE_MAX_EXPERTS || ob > best || (ob == best && oe < best_e))) best = ob, best_e = oe;
       }
-    if (apart) best = __shfl(own, best_e % HAL_WAVE, HAL_WAVE);
-    sum += best;
-    if (lane == 0) idx[(size_t)t * top + j] = best_e;
+      float own = 0.f;
 #pragma unroll
-    for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u)
-      if (u == j / HAL_WAVE && lane == j % HAL_WAVE) kept[u] = best;
-  }
+      for (int u = 0; u < W; ++u)
+        if (lane + u * HAL_WAVE == best_e) place[u] = j, own = w[u];  // taken
+      sum += lane_value(own, __builtin_amdgcn_readfirstlane(best_e % HAL_WAVE));
+    }
+    sum += how.norm_eps;
 #pragma unroll
-  for (int u = 0; u < MOE_ROUTE_PER_LANE; ++u) {
-    const int j = lane + u * HAL_WAVE;
-    if (j < top) wgt[(size_t)t * top + j] = (how.normalize ? kept[u] / (sum + how.norm_eps) : kept[u]) * how.scale;
+    for (int u = 0; u < W; ++u) {
+      mine[u] = (how.normalize ? w[u] / sum : w[u]) * how.scale;
+      if (place[u] < 0) continue;
+      idx[(size_t)t * top + place[u]] = lane + u * HAL_WAVE;
+      wgt[(size_t)t * top + place[u]] = mine[u];
+    }
   }
 }
 
+template <int W>
 __global__ void __launch_bounds__(HAL_WAVE) moe_route_kernel(const float* __restrict__ z, int ldz, int E, int top, MoeChoice how,
                                                              int* __restrict__ idx, float* __restrict__ wgt, int n_tokens) {
-  moe_route_token(z, ldz, E, top, how, idx, wgt, blockIdx.x, threadIdx.x);
+  moe_route_token<W>(z, ldz, E, top, how, idx, wgt, blockIdx.x, threadIdx.x);
 }
 
 static int moe_check_choice(const MoeChoice& how, int E, int top) {
@@ -348,15 +351,26 @@ static int moe_check_choice(const MoeChoice& how, int E, int top) {
   return 0;
 }
 
+#define MOE_BY_WORDS(LAUNCH_, MOST_)               \
+  do {                                             \
+    if (E <= HAL_WAVE) LAUNCH_(1);                 \
+    else if (E <= 2 * HAL_WAVE) LAUNCH_(2);        \
+    else if (E <= 4 * HAL_WAVE) LAUNCH_(4);        \
+    else if (MOST_ > 4) LAUNCH_(MOST_);            \
+  } while (0)
+
 extern "C" int hal_moe_route(const float* z, int ldz, int E, int top, int softmax, int normalize, float norm_eps,
                              float scale, const void* correction, int c_dtype, int groups, int keep, int* idx,
                              float* wgt, int n_tokens, hipStream_t stream) {
   const MoeChoice how = {softmax, normalize, norm_eps, scale, correction, c_dtype, groups, keep};
-  if (int rc = moe_check_choice(how, E, top)) return rc;
   HAL_REQUIRE(n_tokens >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E,
               "hal_moe_route: bad sizes T=%d E=%d top=%d", n_tokens, E, top);
+  if (int rc = moe_check_choice(how, E, top)) return rc;
   if (n_tokens == 0) return 0;
-  hipLaunchKernelGGL(moe_route_kernel, dim3(n_tokens), dim3(HAL_WAVE), 0, stream, z, ldz, E, top, how, idx, wgt, n_tokens);
+#define MOE_ROUTE(W_) \
+  hipLaunchKernelGGL(moe_route_kernel<W_>, dim3(n_tokens), dim3(HAL_WAVE), 0, stream, z, ldz, E, top, how, idx, wgt, n_tokens)
+  MOE_BY_WORDS(MOE_ROUTE, 16);
+#undef MOE_ROUTE
   HAL_LAUNCH_CHECK();
   return 0;
 }
@@ -379,17 +393,28 @@ __device__ __forceinline__ void moe_sort_pairs(const int* idx, int n, int E, int
     if (e >= 0 && e < E) atomicAdd(&count[e], 1);
   }
   __syncthreads();
-  if (threadIdx.x == 0) {
+  if (threadIdx.x < HAL_WAVE) {  // the first wave: running sums, 64 experts at a time
+    const int lane = threadIdx.x;
     int at = 0, tiles = 0;
-    for (int e = 0; e < E; ++e) {
-      offsets[e] = at;
-      tile_offsets[e] = tiles;
-      cursor[e] = at;
-      at += count[e];
-      tiles += (count[e] + tile - 1) / tile;
+    for (int e0 = 0; e0 < E; e0 += HAL_WAVE) {
+      const int e = e0 + lane, c = e < E ? count[e] : 0, ct = (c + tile - 1) / tile;
+      int sum = c, sum_t = ct;
+#pragma unroll
+      for (int off = 1; off < HAL_WAVE; off <<= 1) {
+        const int a = __shfl_up(sum, off, HAL_WAVE), b = __shfl_up(sum_t, off, HAL_WAVE);
+        if (lane >= off) sum += a, sum_t += b;
+      }
+      if (e < E) {
+        offsets[e] = cursor[e] = at + sum - c;
+        tile_offsets[e] = tiles + sum_t - ct;
+      }
+      at += __shfl(sum, HAL_WAVE - 1, HAL_WAVE);
+      tiles += __shfl(sum_t, HAL_WAVE - 1, HAL_WAVE);
     }
-    offsets[E] = at;
-    tile_offsets[E] = tiles;
+    if (lane == 0) {
+      offsets[E] = at;
+      tile_offsets[E] = tiles;
+    }
   }
   __syncthreads();
   for (int i = threadIdx.x; i < n; i += blockDim.x) {
@@ -407,18 +432,19 @@ __global__ void __launch_bounds__(1024) moe_sort_kernel(const int* __restrict__ 
   moe_sort_pairs(idx, n, E, tile, offsets, tile_offsets, sorted, count, cursor);
 }
 
-// Both in one workgroup, for steps of few tokens: its sixteen waves take the tokens in turn,
-// then all of it sorts the pairs.
+// Both in one workgroup, for steps of few tokens and up to 256 experts: its waves take the tokens in
+// turn, then all of it sorts the pairs.
+template <int W>
 __global__ void __launch_bounds__(1024) moe_route_sort_kernel(const float* __restrict__ z, int ldz, int E, int top,
-                                                              MoeChoice how,
-                                                              int* __restrict__ idx, float* __restrict__ wgt,
-                                                              int n_tokens, int tile, int* __restrict__ offsets,
-                                                              int* __restrict__ tile_offsets, int* __restrict__ sorted) {
+                                                              MoeChoice how, int* __restrict__ idx,
+                                                              float* __restrict__ wgt, int n_tokens, int tile,
+                                                              int* __restrict__ offsets, int* __restrict__ tile_offsets,
+                                                              int* __restrict__ sorted) {
   __shared__ int count[MOE_MAX_EXPERTS];
   __shared__ int cursor[MOE_MAX_EXPERTS];
   const int wave = threadIdx.x / HAL_WAVE, lane = threadIdx.x % HAL_WAVE;
-  for (int t = wave; t < n_tokens; t += 1024 / HAL_WAVE)
-    moe_route_token(z, ldz, E, top, how, idx, wgt, t, lane);
+  for (int t = wave; t < n_tokens; t += blockDim.x / HAL_WAVE)
+    moe_route_token<W>(z, ldz, E, top, how, idx, wgt, t, lane);
   __threadfence_block();
   __syncthreads();
   moe_sort_pairs(idx, n_tokens * top, E, tile, offsets, tile_offsets, sorted, count, cursor);
@@ -429,10 +455,15 @@ extern "C" int hal_moe_route_sort(const float* z, int ldz, int E, int top, int s
                                   int* idx, float* wgt, int n_tokens, int tile, int* offsets, int* tile_offsets,
                                   int* sorted, hipStream_t stream) {
   const MoeChoice how = {softmax, normalize, norm_eps, scale, correction, c_dtype, groups, keep};
-  if (int rc = moe_check_choice(how, E, top)) return rc;
-  HAL_REQUIRE(n_tokens >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E && tile > 0,
+  HAL_REQUIRE(n_tokens >= 0 && E > 0 && E <= 4 * HAL_WAVE && top > 0 && top <= E && ldz >= E && tile > 0,
               "hal_moe_route_sort: bad sizes T=%d E=%d top=%d", n_tokens, E, top);
-  hipLaunchKernelGGL(moe_route_sort_kernel, dim3(1), dim3(1024), 0, stream, z, ldz, E, top, how, idx, wgt, n_tokens, tile, offsets, tile_offsets, sorted);
+  if (int rc = moe_check_choice(how, E, top)) return rc;
+  int waves = n_tokens < 4 ? 4 : (n_tokens < 16 ? n_tokens : 16);
+#define MOE_ROUTE_SORT(W_)                                                                                                    \
+  hipLaunchKernelGGL(moe_route_sort_kernel<W_>, dim3(1), dim3(waves * HAL_WAVE), 0, stream, z, ldz, E, top, how, idx, wgt,    \
+                     n_tokens, tile, offsets, tile_offsets, sorted)
+  MOE_BY_WORDS(MOE_ROUTE_SORT, 4);
+#undef MOE_ROUTE_SORT
   HAL_LAUNCH_CHECK();
   return 0;
 }

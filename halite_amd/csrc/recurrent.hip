@@ -323,6 +323,17 @@ ssd_carry_kernel(float* __restrict__ state, float* __restrict__ sums, const floa
   *st = S;
 }
 
+extern "C" int hal_ssd_carry(float* state, float* sums, const float* decays, const int* seg_chunks, const int* seg_q_start,
+                             const int* seg_q_len, const int* token_slot, int n_segs, int heads, int NP, hipStream_t stream) {
+  HAL_REQUIRE(n_segs >= 0 && heads > 0 && heads <= 65535 && NP > 0 && (NP + 255) / 256 <= 65535,
+              "hal_ssd_carry: bad sizes segments=%d heads=%d state of %d", n_segs, heads, NP);
+  if (n_segs == 0) return 0;
+  hipLaunchKernelGGL(ssd_carry_kernel, dim3(n_segs, heads, (NP + 255) / 256), dim3(256), 0, stream, state, sums, decays,
+                     seg_chunks, seg_q_start, seg_q_len, token_slot, heads, NP);
+  HAL_LAUNCH_CHECK();
+  return 0;
+}
+
 // chunks, seg_chunks, sums, decays: all null (a wave walks a whole segment), or the cut of the
 // segments into n_chunks chunks and room for n_chunks * heads * N * P and n_chunks * heads floats.
 extern "C" int hal_ssd_scan(const void* xbc, int ldx, int dtype, const float* dt_raw, int ld_dt,

@@ -47,6 +47,7 @@ CORE_SOURCES = [
     "latent_moe.hip",
     "stream_ops.hip",
     "recurrent.hip",
+    "decay_chunks.hip",
     "delta_rule.hip",
     "time_mix.hip",
 ]

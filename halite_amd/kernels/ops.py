@@ -940,7 +940,8 @@ def moe_route(z: torch.Tensor, top: int, **how):
     return idx, wgt
 
 
-ROUTE_SORT_MAX_TOKENS = 16  # up to so many tokens (one a wave) one workgroup routes and sorts
+ROUTE_SORT_MAX_TOKENS = 16  # up to so many tokens (one a wave) one workgroup routes and sorts,
+ROUTE_SORT_MAX_EXPERTS = 256  # of at most so many experts
 
 
 def moe_route_sort(z: torch.Tensor, top: int, n_experts: int, **how):
@@ -1489,6 +1490,55 @@ def decay_step(v: torch.Tensor, k: torch.Tensor, q: torch.Tensor, gate: torch.Te
         0 if cos is None else cos.shape[0], 1 if interleaved else 0, ctypes.c_float(k_scale), _ptr(decay), _ptr(state),
         _ptr(token_slot), _ptr(weight), F32 if weight is None else dtype_code(weight.dtype), 1 if silu else 0,
         ctypes.c_float(eps), _ptr(out), dtype_code(out_dtype), n, heads, n_state, p, _stream()))
+    return out
+
+
+DECAY_CHUNK = 64  # tokens of a chunk, at most
+
+
+def decay_chunks_fit(n_state: int, v_dim: int) -> bool:
+    """Whether ``decay_chunks`` has a kernel for states of ``n_state x v_dim`` numbers."""
+    return n_state <= 128 and v_dim <= 256
+
+
+def decay_powers(decay: torch.Tensor) -> torch.Tensor:
+    """float32 ``[heads, DECAY_CHUNK + 1]``: the decays (float64 ``[heads]``) to the powers 0, 1, ..."""
+    return (decay[:, None] ** torch.arange(DECAY_CHUNK + 1, dtype=torch.float64)[None, :]).float().contiguous()
+
+
+def decay_chunks(v: torch.Tensor, k: torch.Tensor, q: torch.Tensor, gate: torch.Tensor | None, powers: torch.Tensor,
+                 state: torch.Tensor, seg_q_start: torch.Tensor, seg_q_len: torch.Tensor, token_slot: torch.Tensor,
+                 chunks: torch.Tensor, seg_chunks: torch.Tensor, eps: float = 0.0, out_dtype: torch.dtype = torch.float32, *,
+                 positions: torch.Tensor | None = None, cos: torch.Tensor | None = None, sin: torch.Tensor | None = None,
+                 interleaved: bool = False, k_scale: float = 1.0, in_silu: bool = False,
+                 weight: torch.Tensor | None = None, silu: bool = False) -> torch.Tensor:
+    """``decay_step`` for segments of any number of tokens that are cut into chunks of up to ``DECAY_CHUNK``
+    tokens (``chunks``, ``seg_chunks`` as for ``ssd_scan``): turning, recurrence, norm and gate as float32 products on
+    the matrix cores.  ``powers``: ``decay_powers`` of the decays.  Without a ``gate`` the float32
+    results of the recurrence come back as they are."""
+    lib = library.core_library()
+    _, heads, n_state, p = state.shape
+    n = v.shape[0]
+    rows = [(v, heads * p), (k, heads * n_state), (q, heads * n_state)] + ([(gate, heads * p)] if gate is not None else [])
+    for t, cols in rows:
+        _rows_f32(t, cols, "decay_chunks")
+    _need(len({(t.shape[0], t.stride(0)) for t, _ in rows}) == 1, "decay_chunks: rows of one length, one a token")
+    _dev(powers, state, seg_q_start, seg_q_len, token_slot, weight)
+    _i32(seg_q_start, "seg_q_start"), _i32(seg_q_len, "seg_q_len"), _i32(token_slot, "token_slot")
+    _need(decay_chunks_fit(n_state, p), f"decay_chunks: no kernel for states of {n_state} x {p}")
+    _need(powers.dtype == torch.float32 and powers.shape == (heads, DECAY_CHUNK + 1) and state.dtype == torch.float32,
+          "decay_chunks: float32 powers [heads, 65] and states")
+    _need(token_slot.numel() == n and (weight is None or weight.numel() == heads * p)
+          and (gate is not None or (out_dtype == torch.float32 and weight is None)), "decay_chunks: arguments")
+    rot = _rotation(cos, sin, positions, n, n_state, "decay_chunks")
+    n_chunks, sums, decays = _scan_room(chunks, seg_chunks, seg_q_start, (heads, n_state, p), (heads,), v.device, "decay_chunks")
+    out = torch.empty((n, heads * p), dtype=out_dtype, device=v.device)
+    _check(lib, lib.hal_decay_chunks(
+        _ptr(v), _ptr(k), _ptr(q), _ptr(gate), v.stride(0), 1 if in_silu else 0, _ptr(positions), _ptr(cos), _ptr(sin), rot,
+        0 if cos is None else cos.shape[0], 1 if interleaved else 0, ctypes.c_float(k_scale), _ptr(powers), _ptr(state),
+        _ptr(seg_q_start), _ptr(seg_q_len), _ptr(token_slot), _ptr(chunks), _ptr(seg_chunks), n_chunks, _ptr(sums),
+        _ptr(decays), _ptr(weight), F32 if weight is None else dtype_code(weight.dtype), 1 if silu else 0,
+        ctypes.c_float(eps), _ptr(out), dtype_code(out_dtype), seg_q_start.numel(), heads, n_state, p, _stream()))
     return out
 
 

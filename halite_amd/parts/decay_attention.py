@@ -15,9 +15,10 @@ Its pieces, each a parameter:
 
 Per request the mixer keeps the state (float32); it has no paged cache.  The recurrence is
 the state-space scan's with constant decays and unit step sizes (keys in the place of its
-``B``, queries of its ``C``, one group a head), so prompts are cut into chunks that are walked
-side by side in the same way.  A step of single tokens whose heads are normed each on its own
-is one kernel from the projections to the gated rows.  Rotation, decays, state, sums over the
+``B``, queries of its ``C``, one group a head), so prompts are cut into chunks in the same way; for
+states of up to 128 x 256 a chunk's part is computed as products on the matrix cores (float32),
+larger ones are walked.  A step of single tokens whose heads are normed each on its own is one
+kernel from the projections to the gated rows.  Rotation, decays, state, sums over the
 state, norm and gate are float32.
 """
 
@@ -30,7 +31,7 @@ from pydantic import BaseModel, Field, StrictBool, StrictInt, model_validator
 
 from ..kernels import ops
 from .base import MIXERS, Mixer, ParamDecl, RotaryPositionEncoding, StateNeed
-from .state_space import plan_scan_chunks, scan_arrays
+from .state_space import SCAN_CHUNK, plan_scan_chunks, scan_arrays
 
 
 class DecayAttentionParams(BaseModel):
@@ -114,7 +115,8 @@ class DecayAttention(Mixer):
 
     def finalize(self):
         p = self.p
-        self.decay = torch.tensor(p.decay, dtype=torch.float64).float().to(self.build.device)
+        decay = torch.tensor(p.decay, dtype=torch.float64)
+        self.decay, self.powers = decay.float().to(self.build.device), ops.decay_powers(decay).to(self.build.device)
         self.t_in = self.t_out = None
         if self.build.tiled_weights and self.w_in.is_cuda and self.w_in.dtype == torch.bfloat16:
             if p.hidden_size % 8 == 0:
@@ -139,15 +141,27 @@ class DecayAttention(Mixer):
             cos, sin = self.position.tables(ctx.max_position + 1)
             turn = dict(positions=ctx.positions, cos=cos, sin=sin, interleaved=self.position.interleaved)
         state = run.state["state"]
+        values, keys, queries = a[:, : self.inner], a[:, self.inner : self.inner + self.n_qk], a[:, self.inner + self.n_qk : n_act]
+        recur = dict(k_scale=p.key_scale, in_silu=p.activation == "silu", **turn)
+        finish = dict(eps=p.eps, out_dtype=x.dtype, weight=self.w_norm, silu=silu)
         if p.norm_per_head and x.shape[0] == ctx.n_segs and ops.decay_step_fits(p.qk_dim, p.v_dim):
-            keys, queries = a[:, self.inner : self.inner + self.n_qk], a[:, self.inner + self.n_qk : n_act]
-            gated = ops.decay_step(a[:, : self.inner], keys, queries, gate, self.decay, state, ctx.token_slot, p.eps, x.dtype,
-                                   k_scale=p.key_scale, in_silu=p.activation == "silu", weight=self.w_norm, silu=silu, **turn)
+            # single tokens: one kernel
+            gated = ops.decay_step(values, keys, queries, gate, self.decay, state, ctx.token_slot, **finish, **recur)
+            return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
+        cut = scan_arrays(ctx)
+        if cut["chunks"] is not None and SCAN_CHUNK <= ops.DECAY_CHUNK and ops.decay_chunks_fit(p.qk_dim, p.v_dim):
+            # long segments: chunks as products
+            segs = (ctx.seg_q_start, ctx.seg_q_len, ctx.token_slot)
+            if p.norm_per_head:
+                gated = ops.decay_chunks(values, keys, queries, gate, self.powers, state, *segs, **cut, **finish, **recur)
+            else:
+                y = ops.decay_chunks(values, keys, queries, None, self.powers, state, *segs, **cut, **recur)
+                gated = ops.head_norm_gate(y, gate, self.w_norm, p.eps, 1, x.dtype, silu=silu)
             return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
         if turn or p.key_scale != 1.0:
             ops.rotate_heads_(a[:, self.inner : n_act], 2 * p.n_heads, p.qk_dim, n_scaled=p.n_heads, scale=p.key_scale, **turn)
         # (SiLU of values, keys and queries where the scan reads them: float32 in either mode)
         y = ops.ssd_scan(a[:, :n_act], None, None, None, None, state, ctx.seg_q_start, ctx.seg_q_len, ctx.token_slot,
-                         p.n_heads, fixed_decay=self.decay, in_silu=p.activation == "silu", **scan_arrays(ctx))
+                         p.n_heads, fixed_decay=self.decay, in_silu=p.activation == "silu", **cut)
         gated = ops.head_norm_gate(y, gate, self.w_norm, p.eps, p.n_heads if p.norm_per_head else 1, x.dtype, silu=silu)
         return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)

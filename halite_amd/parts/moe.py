@@ -157,10 +157,14 @@ class MixtureOfExperts(FeedForward):
         return out
 
     def finalize(self):
-        self.t_shared_down = None
-        if (self.p.shared is not None and self.build.tiled_weights and self.ws_down.is_cuda
-                and self.ws_down.dtype == torch.bfloat16 and self.ws_down.shape[1] % 8 == 0):
-            self.t_shared_down = ops.tile_weight(self.ws_down)
+        self.t_shared_gate = self.t_shared_up = self.t_shared_down = None
+        s = self.p.shared
+        if s is not None and self.build.tiled_weights and self.ws_down.is_cuda and self.ws_down.dtype == torch.bfloat16:
+            if s.intermediate_size % 8 == 0:
+                self.t_shared_down = ops.tile_weight(self.ws_down)
+            if self.p.hidden_size % 8 == 0:
+                self.t_shared_gate = ops.tile_weight(self.ws_gate_up[: s.intermediate_size])
+                self.t_shared_up = ops.tile_weight(self.ws_gate_up[s.intermediate_size :])
 
     def forward(self, x, ctx, add_to=None):
         p = self.p
@@ -172,7 +176,7 @@ class MixtureOfExperts(FeedForward):
         routing = dict(softmax=p.score == "softmax", normalize=p.normalize, norm_eps=p.norm_eps, scale=p.weight_scale,
                        correction=self.w_correction, groups=p.groups.count if p.groups else 0,
                        keep=p.groups.keep if p.groups else 0)
-        if n <= ops.ROUTE_SORT_MAX_TOKENS:  # few tokens: one workgroup routes and sorts
+        if n <= ops.ROUTE_SORT_MAX_TOKENS and p.n_experts <= ops.ROUTE_SORT_MAX_EXPERTS:  # few tokens: one workgroup routes and sorts
             idx, wgt, offsets, tiles, order = ops.moe_route_sort(z, p.top_k, p.n_experts, **routing)
         else:
             idx, wgt = ops.moe_route(z, p.top_k, **routing)
@@ -190,8 +194,13 @@ class MixtureOfExperts(FeedForward):
         ops.grouped_gemm(act, self.w_down, y, n_rows=pairs, group_offsets=offsets, tile_offsets=tiles, row_dst=order)
         if p.shared is not None:
             fs = p.shared.intermediate_size
-            if x.dtype == torch.bfloat16 and n <= 16:
-                # few rows: the grouped product of one group, activation in its epilogue
+            if self.t_shared_gate is not None and x.dtype == torch.bfloat16 and n <= ops.SKINNY_ROWS:
+                # few rows: the small-batch product, activation in its epilogue
+                clamp = ops.Clamp(p.shared.limit_or_inf, p.shared.alpha, p.shared.up_shift)
+                acts = ops.gemm_bf16_skinny(x, self.t_shared_gate, w_up=self.t_shared_up, tiled_shape=(fs, d), activation="clamped",
+                                            clamp=clamp)
+            elif x.dtype == torch.bfloat16 and n <= ops.SKINNY_ROWS:
+                # the same without the tiled copies: the grouped product of one group, activation in its epilogue
                 acts = torch.empty((n, fs), dtype=x.dtype, device=x.device)
                 ops.grouped_gemm(x, self.ws_gate_up[:fs].view(1, fs, d), acts, n_rows=n, w_up=self.ws_gate_up[fs:].view(1, fs, d),
                                  limit=p.shared.limit_or_inf, alpha=p.shared.alpha, up_shift=p.shared.up_shift)
