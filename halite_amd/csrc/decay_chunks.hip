@@ -11,6 +11,8 @@
 // outputs may be divided by their root mean square, weighted and gated before they are written.
 // Everything is float32; only the order of the additions differs from the walk token by token.
 //
+// A workgroup takes one head of one chunk, the heads of a chunk are neighbours in the grid (a token's
+// row is read whole at about one time; rows are thousands of entries apart).
 // A wave computes 32 x 32 outputs.  Which k of a product an instruction takes is free as long as
 // both operands agree: half h of a wave takes the four from 8 b + 4 h of every block of eight,
 // so that an operand in LDS is read four entries (16 bytes) at a time.
@@ -34,71 +36,123 @@ struct DecayRows {
   int H, N, P;
 };
 
-__device__ __forceinline__ float dc_in(const DecayRows& a, float x) { return a.in_silu ? x / (1.0f + expf(-x)) : x; }
+// (SILU: the build for rows that may go through SiLU as they are read)
+template <bool SILU>
+__device__ __forceinline__ float dc_in(const DecayRows& a, float x) {
+  if constexpr (SILU) return a.in_silu ? x / (1.0f + expf(-x)) : x;
+  return x;
+}
 
-// The chunk's rows of one head of q or k in LDS [DC_TOKENS][stride], turned, row j times scale(j); zeros
-// beyond the tokens and between N and `width`.
-template <typename F>
-__device__ __forceinline__ void dc_stage(const DecayRows& a, const float* __restrict__ src, int t0, int n, int h, float* dst,
-                                         int stride, int width, F scale) {
-  const int pairs = a.rot / 2, per = width - pairs;
+// A lane's 32 (or 4 NB) numbers of its column of `rows` rows, `stride` apart: those of the rows 8 b + 4 half + i
+// (the last row again beyond the rows: the other operand is zero there).
+template <int BLOCKS>
+__device__ __forceinline__ void dc_column(const float* __restrict__ base, unsigned col, unsigned stride, int rows, int half,
+                                          float (&out)[BLOCKS * 4]) {
+  const unsigned first = 4 * half * stride + col, last = (rows - 1) * stride + col;
+#pragma unroll
+  for (int b = 0; b < BLOCKS; ++b)
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const unsigned at = first + (8 * b + i) * stride;
+      out[b * 4 + i] = base[at < last ? at : last];
+    }
+}
+
+// The chunk's rows of one head of k (and of q, with QUERIES) in LDS [DC_TOKENS][stride], turned, k's row j
+// times scale(j); zeros beyond the tokens and between N and `width`.  A thread brings one pair (or one
+// entry behind the turned ones) of every eighth row, several rows' loads on their way at a time.
+template <bool QUERIES, bool SILU, typename F>
+__device__ __forceinline__ void dc_stage(const DecayRows& a, int t0, int n, int h, float* ks, float* qs, int stride, int width,
+                                         F scale) {
+  constexpr int PASS = 8, AT_ONCE = 4;  // rows side by side (256 threads, 32 to a row), passes whose loads are in flight
+  const int pairs = a.rot / 2, per = width - pairs, j0 = threadIdx.x / 32;
   const int pos0 = a.rot > 0 ? a.positions[t0] : 0;  // (a segment's positions follow one another)
-  for (int e = threadIdx.x; e < DC_TOKENS * per; e += blockDim.x) {
-    const int j = e / per, i = e % per;
-    float* o = dst + j * stride;
-    const float* x = src + (size_t)(t0 + j) * a.ld + (size_t)h * a.N;
-    if (i < pairs) {
-      const int ia = a.interleaved ? 2 * i : i, ib = a.interleaved ? 2 * i + 1 : i + pairs;
-      float u = 0.f, w = 0.f;
-      if (j < n) {
-        const int pos = pos0 + j;
-        const bool known = pos >= 0 && pos < a.table_len;  // checked on the host; else the row shows it
-        const float c = known ? a.cos_t[(size_t)pos * pairs + i] : NAN, s = known ? a.sin_t[(size_t)pos * pairs + i] : NAN;
-        const float xa = dc_in(a, x[ia]), xb = dc_in(a, x[ib]), m = scale(j);
-        u = (xa * c - xb * s) * m;
-        w = (xb * c + xa * s) * m;
+  const size_t head = (size_t)t0 * a.ld + (size_t)h * a.N;
+  for (int i = threadIdx.x % 32; i < per; i += 32) {
+    const bool pair = i < pairs;
+    const int ia = pair ? (a.interleaved ? 2 * i : i) : i + pairs;
+    const int ib = pair ? (a.interleaved ? 2 * i + 1 : i + pairs) : ia;
+    const bool there = ia < a.N;
+#pragma unroll
+    for (int p = 0; p < DC_TOKENS / PASS; p += AT_ONCE) {
+      float ka[AT_ONCE], kb[AT_ONCE], qa[AT_ONCE], qb[AT_ONCE], c[AT_ONCE], s[AT_ONCE];
+#pragma unroll
+      for (int u = 0; u < AT_ONCE; ++u) {
+        const int j = j0 + (p + u) * PASS;
+        const bool have = there && j < n;
+        const float* kr = a.k + head + (size_t)j * a.ld;
+        ka[u] = have ? kr[ia] : 0.f;
+        kb[u] = have && pair ? kr[ib] : 0.f;
+        if (QUERIES) {
+          const float* qr = a.q + head + (size_t)j * a.ld;
+          qa[u] = have ? qr[ia] : 0.f;
+          qb[u] = have && pair ? qr[ib] : 0.f;
+        }
+        c[u] = 1.f, s[u] = 0.f;
+        if (have && pair) {
+          const int pos = pos0 + j;
+          const bool known = pos >= 0 && pos < a.table_len;  // checked on the host; else the row shows it
+          c[u] = known ? a.cos_t[(size_t)pos * pairs + i] : NAN, s[u] = known ? a.sin_t[(size_t)pos * pairs + i] : NAN;
+        }
       }
-      o[ia] = u;
-      o[ib] = w;
-    } else {
-      const int c = i + pairs;
-      o[c] = (j < n && c < a.N) ? dc_in(a, x[c]) * scale(j) : 0.f;
+#pragma unroll
+      for (int u = 0; u < AT_ONCE; ++u) {
+        const int j = j0 + (p + u) * PASS;
+        const float m = j < n ? scale(j) : 0.f, x = dc_in<SILU>(a, ka[u]), y = dc_in<SILU>(a, kb[u]);
+        ks[j * stride + ia] = (x * c[u] - y * s[u]) * m;
+        if (pair) ks[j * stride + ib] = (y * c[u] + x * s[u]) * m;
+        if (QUERIES) {
+          const float z = dc_in<SILU>(a, qa[u]), w = dc_in<SILU>(a, qb[u]);
+          qs[j * stride + ia] = z * c[u] - w * s[u];
+          if (pair) qs[j * stride + ib] = w * c[u] + z * s[u];
+        }
+      }
     }
   }
 }
 
+template <typename T>
+__device__ __forceinline__ T dc_out(float y);
+template <>
+__device__ __forceinline__ float dc_out<float>(float y) { return y; }
+template <>
+__device__ __forceinline__ bf16_t dc_out<bf16_t>(float y) { return bf16_t{(uint16_t)pack_bf16x2(y, 0.f)}; }
+
 __device__ __forceinline__ int dc_row(int v, int half) { return 8 * (v / 4) + 4 * half + v % 4; }  // of register v
 
 // ---- what every chunk leaves from a zero state: sums [chunk][head][N][P], and d^n ------------------
-__global__ void __launch_bounds__(256)
+template <bool SILU>
+__global__ void __launch_bounds__(256, 3)
 decay_sums_kernel(DecayRows a, float* __restrict__ sums, float* __restrict__ decays, int stride) {
   extern __shared__ float dc_lds[];
   __shared__ float pw[DC_TOKENS + 1];
   float* ks = dc_lds;  // [DC_TOKENS][stride]
-  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid % HAL_WAVE, wave = tid / HAL_WAVE;
+  const int h = blockIdx.x, c = blockIdx.y, tid = threadIdx.x, lane = tid % HAL_WAVE, wave = tid / HAL_WAVE;
   const int half = lane / 32, l32 = lane % 32;
   const int t0 = a.chunks[c * 4], n = a.chunks[c * 4 + 1];
   if (n <= 0) return;
   if (tid <= DC_TOKENS) pw[tid] = a.powers[(size_t)h * (DC_TOKENS + 1) + tid];
-  __syncthreads();
   const int row_tiles = (a.N + 31) / 32, col_tiles = (a.P + 31) / 32;
-  dc_stage(a, a.k, t0, n, h, ks, stride, row_tiles * 32, [&](int j) { return a.k_scale * pw[n - 1 - j]; });
-  if (blockIdx.z == 0 && tid == 0) decays[(size_t)c * a.H + h] = pw[n];
-  __syncthreads();
   // a wave takes a tile of 32 columns and the tiles of 32 rows in turn (few columns: the waves share one)
   const int across = col_tiles >= 4 ? 4 : (col_tiles >= 2 ? 2 : 1), down = 4 / across;
-  float* out = sums + ((size_t)c * a.H + h) * a.N * a.P;
-  for (int ct = wave % across + across * blockIdx.z; ct < col_tiles; ct += across * gridDim.z) {
+  const int ct0 = wave % across + across * blockIdx.z;
+  float vr[DC_TOKENS / 2];
+  const float* vbase = a.v + (size_t)t0 * a.ld + (size_t)h * a.P;
+  auto values = [&](int ct) {
     const int col = ct * 32 + l32;
-    const float* vc = a.v + (size_t)h * a.P + (col < a.P ? col : a.P - 1);
-    float vr[DC_TOKENS / 2];
+    dc_column<DC_TOKENS / 8>(vbase, col < a.P ? col : a.P - 1, a.ld, n, half, vr);
+  };
+  values(ct0);
+  __syncthreads();
+  dc_stage<false, SILU>(a, t0, n, h, ks, nullptr, stride, row_tiles * 32, [&](int j) { return a.k_scale * pw[n - 1 - j]; });
+  if (blockIdx.z == 0 && tid == 0) decays[(size_t)c * a.H + h] = pw[n];
+  __syncthreads();
+  float* out = sums + ((size_t)c * a.H + h) * a.N * a.P;
+  for (int ct = ct0; ct < col_tiles; ct += across * gridDim.z) {
+    const int col = ct * 32 + l32;
+    if (ct != ct0) values(ct);
 #pragma unroll
-    for (int b = 0; b < DC_TOKENS / 8; ++b)
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int j = 8 * b + 4 * half + i;  // (keys beyond the tokens are zero)
-        vr[b * 4 + i] = dc_in(a, vc[(size_t)(t0 + (j < n ? j : n - 1)) * a.ld]);
-      }
+    for (int i = 0; i < DC_TOKENS / 2; ++i) vr[i] = dc_in<SILU>(a, vr[i]);
     for (int rt = wave / across; rt < row_tiles; rt += down) {
       dc_f32x16 acc = {};
 #pragma unroll
@@ -117,26 +171,56 @@ decay_sums_kernel(DecayRows a, float* __restrict__ sums, float* __restrict__ dec
 
 // ---- the outputs of every chunk from the state it starts from (`starts`, as the carry left it) -------
 // NB: blocks of eight entries of a key, at most; CT: column tiles a wave.  GATED: normed, weighted and
-// gated rows of T; else float32 rows as they are.
+// gated rows of T; else float32 rows as they are (and the rows read may go through SiLU).
 template <int NB, int CT, bool GATED, typename T>
-__global__ void __launch_bounds__(256)
+__global__ void __launch_bounds__(256, CT == 1 && NB < 16 ? 3 : 2)
 decay_outputs_kernel(DecayRows a, const float* __restrict__ starts, const void* __restrict__ w, int w_dtype, bool silu,
                      float eps, T* __restrict__ out) {
   extern __shared__ float dc_lds[];
   __shared__ float pw[DC_TOKENS + 1];
-  __shared__ float part[2][DC_TOKENS];
+  __shared__ float part[2][DC_TOKENS], rstd[DC_TOKENS];
   constexpr int LD = NB * 8 + 4, LP = DC_TOKENS + 4;
+  constexpr bool SILU = !GATED;
   float* qs = dc_lds;                   // [DC_TOKENS][LD]
   float* ks = dc_lds + DC_TOKENS * LD;  // [DC_TOKENS][LD], then the scores [DC_TOKENS][LP]
-  const int c = blockIdx.x, h = blockIdx.y, tid = threadIdx.x, lane = tid % HAL_WAVE, wave = tid / HAL_WAVE;
+  const int h = blockIdx.x, c = blockIdx.y, tid = threadIdx.x, lane = tid % HAL_WAVE, wave = tid / HAL_WAVE;
   const int half = lane / 32, l32 = lane % 32;
   const int t0 = a.chunks[c * 4], n = a.chunks[c * 4 + 1];
   if (n <= 0) return;
   if (tid <= DC_TOKENS) pw[tid] = a.powers[(size_t)h * (DC_TOKENS + 1) + tid];
-  dc_stage(a, a.q, t0, n, h, qs, LD, NB * 8, [](int) { return 1.0f; });
-  dc_stage(a, a.k, t0, n, h, ks, LD, NB * 8, [&](int) { return a.k_scale; });
-  __syncthreads();
   const int rt = wave % 2, side = wave / 2;  // a wave's tile of 32 rows, and which half of the columns
+  // the state's and the values' entries of a wave's column, asked for long before they are needed
+  const float* S0 = starts + ((size_t)c * a.H + h) * a.N * a.P;
+  float s0[NB * 4], vr[DC_TOKENS / 2];
+  auto column = [&](int u) {
+    const int col = (side + 2 * u) * 32 + l32;
+    return col < a.P ? col : a.P - 1;
+  };
+  auto ask_state = [&](int u) { dc_column<NB>(S0, column(u), a.P, a.N, half, s0); };
+  const float* vbase = a.v + (size_t)t0 * a.ld + (size_t)h * a.P;
+  auto ask_values = [&](int u) { dc_column<DC_TOKENS / 8>(vbase, column(u), a.ld, n, half, vr); };
+  ask_state(0);
+  dc_stage<true, SILU>(a, t0, n, h, ks, qs, LD, NB * 8, [&](int) { return a.k_scale; });
+  __syncthreads();
+  ask_values(0);
+  dc_f32x16 acc[CT];
+#pragma unroll
+  for (int u = 0; u < CT; ++u) {  // what the queries read of the state before the chunk
+    acc[u] = dc_f32x16{};
+    if ((side + 2 * u) * 32 >= a.P) continue;
+    if (u > 0) ask_state(u);
+    const float* qr = qs + (rt * 32 + l32) * LD + 4 * half;
+#pragma unroll
+    for (int b = 0; b < NB; ++b) {
+      const float4 x = *(const float4*)(qr + 8 * b);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, s0[b * 4], acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, s0[b * 4 + 1], acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, s0[b * 4 + 2], acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, s0[b * 4 + 3], acc[u], 0, 0, 0);
+    }
+#pragma unroll
+    for (int v = 0; v < 16; ++v) acc[u][v] *= pw[rt * 32 + dc_row(v, half) + 1];
+  }
   // scores: wave 0 the tile (0, 0), wave 1 (1, 0), wave 3 (1, 1); (0, 1) lies behind every query
   dc_f32x16 sc = {};
   const bool scores = wave != 2;
@@ -162,45 +246,17 @@ decay_outputs_kernel(DecayRows a, const float* __restrict__ starts, const void* 
     }
   }
   __syncthreads();
-  const float* S0 = starts + ((size_t)c * a.H + h) * a.N * a.P;
-  dc_f32x16 acc[CT];
 #pragma unroll
-  for (int u = 0; u < CT; ++u) {
-    acc[u] = dc_f32x16{};
-    const int ct = side + 2 * u;
-    if (ct * 32 >= a.P) continue;
-    const int col = ct * 32 + l32, colc = col < a.P ? col : a.P - 1;
-    const float* qr = qs + (rt * 32 + l32) * LD + 4 * half;
-#pragma unroll
-    for (int b = 0; b < NB; ++b) {
-      const float4 x = *(const float4*)(qr + 8 * b);
-      float s[4];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int k = 8 * b + 4 * half + i;  // (queries beyond N are zero)
-        s[i] = S0[(size_t)(k < a.N ? k : a.N - 1) * a.P + colc];
-      }
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, s[0], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, s[1], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, s[2], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, s[3], acc[u], 0, 0, 0);
-    }
-#pragma unroll
-    for (int v = 0; v < 16; ++v) acc[u][v] *= pw[rt * 32 + dc_row(v, half) + 1];
-    const float* vc = a.v + (size_t)h * a.P + colc;
+  for (int u = 0; u < CT; ++u) {  // the chunk's own values by the scores
+    if ((side + 2 * u) * 32 >= a.P) continue;
+    if (u > 0) ask_values(u);
     const float* pr = ps + (rt * 32 + l32) * LP + 4 * half;
     auto weigh = [&](int b) {
       const float4 x = *(const float4*)(pr + 8 * b);
-      float s[4];
-#pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int j = 8 * b + 4 * half + i;  // (scores beyond the tokens are zero)
-        s[i] = dc_in(a, vc[(size_t)(t0 + (j < n ? j : n - 1)) * a.ld]);
-      }
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, s[0], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, s[1], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, s[2], acc[u], 0, 0, 0);
-      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, s[3], acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.x, dc_in<SILU>(a, vr[b * 4]), acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.y, dc_in<SILU>(a, vr[b * 4 + 1]), acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.z, dc_in<SILU>(a, vr[b * 4 + 2]), acc[u], 0, 0, 0);
+      acc[u] = __builtin_amdgcn_mfma_f32_32x32x2f32(x.w, dc_in<SILU>(a, vr[b * 4 + 3]), acc[u], 0, 0, 0);
     };
 #pragma unroll
     for (int b = 0; b < 4; ++b) weigh(b);
@@ -234,24 +290,36 @@ decay_outputs_kernel(DecayRows a, const float* __restrict__ starts, const void* 
     r[0] += __shfl_xor(r[0], 1, HAL_WAVE);
     if (lane % 2 == 0) part[side][rt * 32 + dc_row(l32 / 2, half)] = r[0];
     __syncthreads();
+    if (tid < DC_TOKENS) rstd[tid] = 1.0f / sqrtf((part[0][tid] + part[1][tid]) / (float)a.P + eps);
+    __syncthreads();
   }
+  const size_t head = (size_t)t0 * a.H * a.P + (size_t)h * a.P;
+  const float* gbase = GATED ? a.gate + (size_t)t0 * a.ld + (size_t)h * a.P : nullptr;
 #pragma unroll
-  for (int v = 0; v < 16; ++v) {
-    const int i = rt * 32 + dc_row(v, half);
-    if (i >= n) continue;
-    float rstd = 1.0f;
-    if constexpr (GATED) rstd = 1.0f / sqrtf((part[0][i] + part[1][i]) / (float)a.P + eps);
+  for (int u = 0; u < CT; ++u) {
+    const int col = (side + 2 * u) * 32 + l32;
+    if (col >= a.P) continue;
+    if constexpr (GATED) {
+      const float wt = w ? load_as_f32(w, w_dtype, (size_t)h * a.P + col) : 1.0f;
+      float z[16];
+      const unsigned first = (rt * 32 + 4 * half) * a.ld + col, last = (n - 1) * a.ld + col;
 #pragma unroll
-    for (int u = 0; u < CT; ++u) {
-      const int col = (side + 2 * u) * 32 + l32;
-      if (col >= a.P) continue;
-      float y = acc[u][v];
-      const size_t cc = (size_t)h * a.P + col;
-      if constexpr (GATED) {
-        const float z = a.gate[(size_t)(t0 + i) * a.ld + cc], s = 1.0f / (1.0f + expf(-z));
-        y *= rstd * (w ? load_as_f32(w, w_dtype, cc) : 1.0f) * (silu ? z * s : s);
+      for (int v = 0; v < 16; ++v) {
+        const unsigned at = first + (8 * (v / 4) + v % 4) * a.ld;
+        z[v] = gbase[at < last ? at : last];
       }
-      out[(size_t)(t0 + i) * a.H * a.P + cc] = from_f32<T>(y);
+#pragma unroll
+      for (int v = 0; v < 16; ++v) {
+        // (one rounding of the reciprocal more or less: it is 1 + something)
+        const float s = __builtin_amdgcn_rcpf(1.0f + expf(-z[v]));
+        acc[u][v] *= rstd[rt * 32 + dc_row(v, half)] * wt * (silu ? z[v] * s : s);
+      }
+    }
+    T* o = out + head + col;
+#pragma unroll
+    for (int v = 0; v < 16; ++v) {
+      const int i = rt * 32 + dc_row(v, half);
+      if (i < n) o[(unsigned)i * (unsigned)(a.H * a.P)] = dc_out<T>(acc[u][v]);
     }
   }
 }
@@ -264,7 +332,7 @@ static int dc_outputs(const DecayRows& a, int n_chunks, const float* starts, con
   if (smem > 48 * 1024)
     HAL_CHECK_HIP(hipFuncSetAttribute((const void*)decay_outputs_kernel<NB, CT, GATED, T>,
                                       hipFuncAttributeMaxDynamicSharedMemorySize, (int)smem));
-  hipLaunchKernelGGL((decay_outputs_kernel<NB, CT, GATED, T>), dim3(n_chunks, a.H), dim3(256), smem, stream, a, starts, w,
+  hipLaunchKernelGGL((decay_outputs_kernel<NB, CT, GATED, T>), dim3(a.H, n_chunks), dim3(256), smem, stream, a, starts, w,
                      w_dtype, silu, eps, (T*)out);
   HAL_LAUNCH_CHECK();
   return 0;
@@ -297,17 +365,22 @@ extern "C" int hal_decay_chunks(const float* v, const float* k, const float* q, 
               "hal_decay_chunks: arguments");
   HAL_REQUIRE(rot >= 0 && rot % 2 == 0 && rot <= N && (rot == 0 || (cos_t && sin_t && positions && table_len > 0)),
               "hal_decay_chunks: %d turned entries of %d", rot, N);
-  HAL_REQUIRE((dtype == HAL_F32 || dtype == HAL_BF16) && (gate || dtype == HAL_F32) &&
+  HAL_REQUIRE((dtype == HAL_F32 || dtype == HAL_BF16) && (gate ? !in_silu : dtype == HAL_F32) &&
                   (w == nullptr || w_dtype == HAL_F32 || w_dtype == HAL_BF16),
               "hal_decay_chunks: dtypes %d, %d", dtype, w_dtype);
+  HAL_REQUIRE(n_chunks <= 65535, "hal_decay_chunks: %d chunks exceed the grid limit", n_chunks);
   if (n_segs == 0 || n_chunks == 0) return 0;
   const DecayRows a = {v, k, q, gate, ld, in_silu != 0, positions, cos_t, sin_t, rot, table_len, interleaved != 0,
                        k_scale, powers, chunks, H, N, P};
   const int stride = (N + 31) / 32 * 32 + 8, col_tiles = (P + 31) / 32;
   int z = 1;  // few chunks and heads: the columns of a state are shared by several workgroups
   while (z < 4 && (long long)n_chunks * H * z < 512 && z * 4 < col_tiles) z *= 2;
-  hipLaunchKernelGGL(decay_sums_kernel, dim3(n_chunks, H, z), dim3(256), sizeof(float) * DC_TOKENS * stride, stream, a, sums,
-                     decays, stride);
+  if (in_silu)
+    hipLaunchKernelGGL(decay_sums_kernel<true>, dim3(H, n_chunks, z), dim3(256), sizeof(float) * DC_TOKENS * stride, stream, a,
+                       sums, decays, stride);
+  else
+    hipLaunchKernelGGL(decay_sums_kernel<false>, dim3(H, n_chunks, z), dim3(256), sizeof(float) * DC_TOKENS * stride, stream, a,
+                       sums, decays, stride);
   HAL_LAUNCH_CHECK();
   if (int rc = hal_ssd_carry(state, sums, decays, seg_chunks, seg_q_start, seg_q_len, token_slot, n_segs, H, N * P, stream))
     return rc;

@@ -287,7 +287,8 @@ int hal_ssd_carry(float* state, float* sums, const float* decays, const int* seg
                   const int* seg_q_len, const int* token_slot, int n_segs, int heads, int NP, hipStream_t stream);
 // The recurrence of hal_decay_step over segments cut into chunks of up to 64 tokens (chunks, seg_chunks,
 // sums, decays as for hal_ssd_scan), as float32 products on the matrix cores.  powers [H, 65]: decay_h to
-// the powers 0 .. 64.  gate null: float32 rows y as they are, else normed, weighted and gated as there.
+// the powers 0 .. 64.  gate null: float32 rows y as they are, else normed, weighted and gated as there
+// (then without in_silu).
 // N <= 128, P <= 256.
 int hal_decay_chunks(const float* v, const float* k, const float* q, const float* gate, int ld, int in_silu,
                      const int* positions, const float* cos_t, const float* sin_t, int rot, int table_len,
@@ -332,7 +333,10 @@ int hal_streams_step(float* x, long long copy_stride, int S, const float* y, con
 int hal_stream_step(float* x, const float* y1, const float* y2, const void* w1, const void* w2, int yw_dtype,
                     float s1, float s2, float y_eps, float m, int read, const void* norm_w, int norm_dtype,
                     float offset, float eps, void* result, int ld_result, int result_dtype, const int* rows,
-                    int n_rows, int W, hipStream_t stream);
+                    int n_rows, int W, const float* wgt, int top, const float* extra, const float* extra_gate, int ld_gate,
+                    hipStream_t stream);
+// (wgt [rows, top], or null: y1 holds rows of experts and stands for what hal_moe_combine makes of them with
+// wgt, extra and extra_gate)
 // Every head of float32 q [T, H * dq], k [T, K * dq], v [T, K * dv] divided by its own root
 // mean square, packed as hal_qk_norm_pack packs (and appended to the pages, if given).
 // w_q, w_k (or null): a weight [dq] for every normed head of q / k; norm_v 0: the values are not

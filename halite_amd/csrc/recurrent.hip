@@ -293,7 +293,7 @@ ssd_scan_kernel(const T* __restrict__ xbc, int ldx, const float* __restrict__ dt
 
 // seg_chunks [segments][2]: a segment's first chunk and number of chunks.  A thread takes one
 // number of the state of one head of one segment through the segment's chunks; the chunks'
-// sums are asked for four at a time (the sums wait for each other, the loads need not).
+// sums are asked for sixteen at a time (the sums wait for each other, the loads need not).
 __global__ void __launch_bounds__(256)
 ssd_carry_kernel(float* __restrict__ state, float* __restrict__ sums, const float* __restrict__ decays,
                  const int* __restrict__ seg_chunks, const int* __restrict__ seg_q_start,
@@ -303,7 +303,7 @@ ssd_carry_kernel(float* __restrict__ state, float* __restrict__ sums, const floa
   const int c0 = seg_chunks[s * 2], nc = seg_chunks[s * 2 + 1];
   float* st = state + ((size_t)token_slot[seg_q_start[s]] * heads + h) * NP + e;
   float S = *st;
-  constexpr int AHEAD = 4;
+  constexpr int AHEAD = 16;
   for (int c = c0; c < c0 + nc; c += AHEAD) {
     float left[AHEAD], decay[AHEAD];
 #pragma unroll

@@ -503,14 +503,22 @@ extern "C" int hal_streams_step(float* x, long long copy_stride, int S, const fl
 // ---- one copy of the stream and no learned weights: x += m * y, then the read of the new row (as
 // it is or normed).  y is a part's result (y1), or the sum of two that are normed each on its own,
 // s1 * norm(y1) * w1 + s2 * norm(y2) * w2 with norm(v) = v / sqrt(mean(v^2) + y_eps) (w1 null: y1 as
-// it is; y2 null: one term).  With `rows` those rows are read and x stays as it is.  A thread
+// it is; y2 null: one term).  With e.wgt y1 is made here from the results y1 [T * top] of the experts that
+// every token uses: sum_j wgt[t, j] y1[t * top + j] (+ sigmoid(gate[t]) extra[t]).  With `rows` those rows are read and x stays as it is.  A thread
 // keeps its part of the row in registers; rows of a multiple of four elements. -----------------
+struct ExpertRows {
+  const float* wgt;    // [T, top], or null
+  int top;
+  const float* extra;  // [T, W], or null
+  const float* gate;   // [T] with rows of ld_gate, or null
+  int ld_gate;
+};
 template <typename TO, int VMAX>
 __global__ void __launch_bounds__(256)
 stream_step_kernel(float* __restrict__ x, const float* __restrict__ y1, const float* __restrict__ y2,
                    const void* __restrict__ w1, const void* __restrict__ w2, int yw_dtype, float s1, float s2,
                    float y_eps, float m, int read, const void* __restrict__ norm_w, int norm_dtype, float offset,
-                   float eps, TO* __restrict__ result, int ld_result, const int* __restrict__ rows, int W) {
+                   float eps, TO* __restrict__ result, int ld_result, const int* __restrict__ rows, int W, ExpertRows e) {
   __shared__ float2 parts[2][4];
   const size_t t = rows ? (size_t)rows[blockIdx.x] : (size_t)blockIdx.x;
   const int nv = W / 4;
@@ -524,12 +532,31 @@ stream_step_kernel(float* __restrict__ x, const float* __restrict__ y1, const fl
   };
   float xv[VMAX][4], av[VMAX][4], bv[VMAX][4];
   float sa = 0.f, sb = 0.f;
+  if (e.wgt) {
+    const float eg = e.gate ? 1.0f / (1.0f + expf(-e.gate[t * e.ld_gate])) : 1.0f;
+#pragma unroll
+    for (int u = 0; u < VMAX; ++u) {
+      const int v = threadIdx.x + u * blockDim.x;
+      if (v >= nv) continue;
+      float r[4] = {0.f, 0.f, 0.f, 0.f};
+      if (e.extra) load4(e.extra + t * W + v * 4, r);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) av[u][i] = r[i] * eg;
+#pragma unroll 4
+      for (int j = 0; j < e.top; ++j) {
+        load4(y1 + (t * e.top + j) * W + v * 4, r);
+        const float m1 = e.wgt[t * e.top + j];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) av[u][i] += m1 * r[i];
+      }
+    }
+  }
 #pragma unroll
   for (int u = 0; u < VMAX; ++u) {
     const int v = threadIdx.x + u * blockDim.x;
     if (v < nv) {
       load4(x + t * W + v * 4, xv[u]);
-      if (y1) load4(y1 + t * W + v * 4, av[u]);
+      if (y1 && !e.wgt) load4(y1 + t * W + v * 4, av[u]);
       if (y2) load4(y2 + t * W + v * 4, bv[u]);
       if (w1) {
 #pragma unroll
@@ -586,7 +613,10 @@ stream_step_kernel(float* __restrict__ x, const float* __restrict__ y1, const fl
 extern "C" int hal_stream_step(float* x, const float* y1, const float* y2, const void* w1, const void* w2, int yw_dtype,
                                float s1, float s2, float y_eps, float m, int read, const void* norm_w, int norm_dtype,
                                float offset, float eps, void* result, int ld_result, int result_dtype, const int* rows,
-                               int n_rows, int W, hipStream_t stream) {
+                               int n_rows, int W, const float* wgt, int top, const float* extra, const float* extra_gate,
+                               int ld_gate, hipStream_t stream) {
+  HAL_REQUIRE(wgt == nullptr || (y1 && !y2 && top > 0), "hal_stream_step: weights of experts without their results");
+  const ExpertRows e = {wgt, top, wgt ? extra : nullptr, wgt ? extra_gate : nullptr, ld_gate};
   HAL_REQUIRE(n_rows >= 0 && W > 0 && W % 4 == 0 && W <= STREAM_STEP_MOST, "hal_stream_step: bad sizes rows=%d width=%d", n_rows, W);
   HAL_REQUIRE(y2 == nullptr || (y1 && w1 && w2), "hal_stream_step: two results are normed, each with its weight");
   HAL_REQUIRE(y1 || read, "hal_stream_step: nothing to do");
@@ -595,13 +625,13 @@ extern "C" int hal_stream_step(float* x, const float* y1, const float* y2, const
   HAL_REQUIRE((result_dtype == HAL_F32 || result_dtype == HAL_BF16) && (yw_dtype == HAL_F32 || yw_dtype == HAL_BF16) &&
                   (norm_dtype == HAL_F32 || norm_dtype == HAL_BF16), "hal_stream_step: dtypes");
   HAL_REQUIRE((((uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2 | (uintptr_t)w1 | (uintptr_t)w2 | (uintptr_t)norm_w |
-                (uintptr_t)result) % 8) == 0 && (((uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2) % 16) == 0,
+                (uintptr_t)result) % 8) == 0 && (((uintptr_t)x | (uintptr_t)y1 | (uintptr_t)y2 | (uintptr_t)extra) % 16) == 0,
               "hal_stream_step: rows must be 16-byte aligned");
   if (n_rows == 0) return 0;
   const int nv = W / 4, threads = nv >= 512 ? 256 : (nv >= 128 ? 128 : 64);
 #define STREAM_LAUNCH(T_, V_)                                                                                            \
   hipLaunchKernelGGL((stream_step_kernel<T_, V_>), dim3(n_rows), dim3(threads), 0, stream, x, y1, y2, w1, w2, yw_dtype, s1, \
-                     s2, y_eps, m, read, norm_w, norm_dtype, offset, eps, (T_*)result, ld_result, rows, W)
+                     s2, y_eps, m, read, norm_w, norm_dtype, offset, eps, (T_*)result, ld_result, rows, W, e)
 #define STREAM_BY_WIDTH(T_)                         \
   do {                                              \
     if (nv <= 2 * threads) STREAM_LAUNCH(T_, 2);    \
@@ -698,6 +728,96 @@ __global__ void head_norm_pack_kernel(const float* __restrict__ q, int ldq, cons
   }
 }
 
+// The same four entries a lane, for sizes and addresses that allow it: LPH lanes (a power of two, at
+// least D / 4) a head, several heads a wave.
+template <typename T>
+__global__ void __launch_bounds__(256)
+head_norm_pack_vec_kernel(const float* __restrict__ q, int ldq, const float* __restrict__ k, int ldk,
+                          const float* __restrict__ v, int ldv, float eps, const void* __restrict__ w_q,
+                          const void* __restrict__ w_k, int w_dtype, bool norm_v, const float* __restrict__ v_other,
+                          int ldvo, float v_mix, const int* __restrict__ positions, const float* __restrict__ cos_t,
+                          const float* __restrict__ sin_t, int rot, int table_len, bool interleaved, T* __restrict__ out,
+                          int row_stride, int n_tokens, int H, int K, int dq, int dv, int D,
+                          const int* __restrict__ token_seg, const int* __restrict__ block_table, int bt_stride,
+                          T* __restrict__ k_pages, T* __restrict__ v_pages, int page_size, int n_pages, bool tiled,
+                          int lph_log2) {
+  const unsigned slots = H + 2 * K, lph = 1u << lph_log2;
+  const unsigned unit = (blockIdx.x * 256u + threadIdx.x) >> lph_log2;
+  if (unit >= n_tokens * slots) return;  // (whole groups of lph lanes leave together)
+  const unsigned t = unit / slots;
+  const int hs = (int)(unit - t * slots);
+  const int kind = hs < H ? 0 : (hs < H + K ? 1 : 2);
+  const int head = kind == 0 ? hs : (kind == 1 ? hs - H : hs - H - K);
+  const int n = kind == 2 ? dv : dq, l = threadIdx.x & (lph - 1), d0 = l * 4;
+  const float* src = kind == 0 ? q + (size_t)t * ldq + head * dq
+                               : (kind == 1 ? k + (size_t)t * ldk + head * dq : v + (size_t)t * ldv + head * dv);
+  const bool turn = cos_t && kind != 2, have = d0 < n;
+  const int turned = turn ? rot : 0;
+  const int pos = (turn || k_pages) ? positions[t] : 0;
+  float f[4] = {0.f, 0.f, 0.f, 0.f};
+  if (have) load4(src + d0, f);
+  const void* w = kind == 0 ? w_q : (kind == 1 ? w_k : nullptr);
+  float wt[4] = {1.f, 1.f, 1.f, 1.f};
+  if (w && have) load4_any(w, w_dtype, d0, wt);
+  // a pair's angle: neighbours hold two pairs of a lane's entries, halves one pair an entry
+  float c[4] = {1.f, 1.f, 1.f, 1.f}, s[4] = {0.f, 0.f, 0.f, 0.f};
+  if (d0 < turned) {
+    const bool known = pos >= 0 && pos < table_len;  // checked on the host; else the row shows it
+    const int half = turned / 2;
+    const size_t row = (size_t)(known ? pos : 0) * half;
+    if (interleaved) {
+      const float2 cc = *(const float2*)(cos_t + row + d0 / 2), ss = *(const float2*)(sin_t + row + d0 / 2);
+      c[0] = c[1] = cc.x, c[2] = c[3] = cc.y, s[0] = s[1] = ss.x, s[2] = s[3] = ss.y;
+    } else {
+      load4(cos_t + row + (d0 < half ? d0 : d0 - half), c);
+      load4(sin_t + row + (d0 < half ? d0 : d0 - half), s);
+    }
+    if (!known) c[0] = c[1] = c[2] = c[3] = NAN;
+  }
+  if (kind != 2 || norm_v) {
+    float ss = (f[0] * f[0] + f[1] * f[1]) + (f[2] * f[2] + f[3] * f[3]);
+    for (unsigned off = lph / 2; off > 0; off >>= 1) ss += __shfl_xor(ss, off, HAL_WAVE);
+    const float rstd = 1.0f / sqrtf(ss / (float)n + eps);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] *= rstd * wt[i];
+  }
+  if (turn) {
+    float o[4];  // the partners, with the sign they enter with
+    if (interleaved) {
+      o[0] = -f[1], o[1] = f[0], o[2] = -f[3], o[3] = f[2];
+    } else {
+      const int half_lanes = turned / 8;
+      const bool second = l >= half_lanes;
+      const int from = (threadIdx.x % HAL_WAVE) + (d0 < turned ? (second ? -half_lanes : half_lanes) : 0);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const float g = __shfl(f[i], from, HAL_WAVE);
+        o[i] = second ? g : -g;
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] = f[i] * c[i] + (d0 < turned ? o[i] * s[i] : 0.f);
+  }
+  if (kind == 2 && v_other && have) {
+    float o[4];
+    load4(v_other + (size_t)t * ldvo + head * dv + d0, o);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) f[i] = (1.0f - v_mix) * f[i] + v_mix * o[i];
+  }
+  if (d0 >= D) return;
+  store4(out + (size_t)t * row_stride + (size_t)hs * D + d0, f);
+  if (!k_pages || kind == 0) return;
+  const int page = block_table[(size_t)token_seg[t] * bt_stride + pos / page_size], off = pos % page_size;
+  if (page < 0 || page >= n_pages) return;  // checked on the host
+  if (kind == 1) {  // (four entries of a key are neighbours in either layout)
+    store4(k_pages + ((size_t)page * K + head) * page_size * D + kv_key_offset(tiled, page_size, D, off, d0), f);
+  } else {
+    T* vp = v_pages + ((size_t)page * K + head) * D * page_size;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) vp[kv_value_offset(tiled, page_size, D, off, d0 + i)] = from_f32<T>(f[i]);
+  }
+}
+
 extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int ldk, const float* v, int ldv, float eps,
                                   const void* w_q, const void* w_k, int w_dtype, int norm_v, const float* v_other,
                                   int ldvo, float v_mix, const int* positions, const float* cos_t, const float* sin_t,
@@ -720,6 +840,27 @@ extern "C" int hal_head_norm_pack(const float* q, int ldq, const float* k, int l
   if (rot == 0) cos_t = nullptr;
   if (n_tokens == 0) return 0;
   const long long units = (long long)n_tokens * (H + 2 * K);
+  const int elt = dtype == HAL_F32 ? 16 : 8;  // bytes of four entries
+  const bool four = D % 4 == 0 && dq % 4 == 0 && dv % 4 == 0 && D <= 256 && ldq % 4 == 0 && ldk % 4 == 0 && ldv % 4 == 0 &&
+                    ldvo % 4 == 0 && row_stride % 4 == 0 && (rot % 8 == 0 || (interleaved && rot % 4 == 0)) &&
+                    (((uintptr_t)q | (uintptr_t)k | (uintptr_t)v | (uintptr_t)v_other | (uintptr_t)cos_t | (uintptr_t)sin_t) % 16) == 0 &&
+                    ((uintptr_t)out % elt) == 0 && ((uintptr_t)k_pages % elt) == 0 &&
+                    (((uintptr_t)w_q | (uintptr_t)w_k) % (w_dtype == HAL_F32 ? 16 : 8)) == 0 && units * 64 < (1ll << 32);
+  if (four) {
+    int lph_log2 = 2;
+    while ((4 << lph_log2) < D) ++lph_log2;
+    const dim3 blocks((unsigned)(((units << lph_log2) + 255) / 256));
+#define PACK_VEC(T_)                                                                                                        \
+  hipLaunchKernelGGL(head_norm_pack_vec_kernel<T_>, blocks, dim3(256), 0, stream, q, ldq, k, ldk, v, ldv, eps, w_q, w_k, w_dtype, \
+                     norm_v != 0, v_other, ldvo, v_mix, positions, cos_t, sin_t, rot, table_len, interleaved != 0, (T_*)out,     \
+                     row_stride, n_tokens, H, K, dq, dv, D, token_seg, block_table, bt_stride, (T_*)k_pages, (T_*)v_pages,      \
+                     page_size, n_pages, tiled != 0, lph_log2)
+    if (dtype == HAL_F32) PACK_VEC(float);
+    else PACK_VEC(bf16_t);
+#undef PACK_VEC
+    HAL_LAUNCH_CHECK();
+    return 0;
+  }
   const dim3 grid((unsigned)((units + 3) / 4));
   if (dtype == HAL_F32)
     hipLaunchKernelGGL(head_norm_pack_kernel<float>, grid, dim3(256), 0, stream, q, ldq, k, ldk, v, ldv, eps, w_q, w_k,

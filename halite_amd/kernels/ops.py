@@ -1034,7 +1034,28 @@ class NormedTerms:
     eps: float
 
     def materialize(self) -> torch.Tensor:
-        return normed_sum(self.terms, self.eps)
+        whole = lambda a: a.materialize() if isinstance(a, ExpertSum) else a  # noqa: E731
+        return normed_sum([(whole(a), w, s) for a, w, s in self.terms], self.eps)
+
+
+@dataclass
+class ExpertSum:
+    """A mixture's result that its reader adds up: ``sum_j wgt[t, j] * y[t * top + j] (+ sigmoid(gate[t]) *
+    extra[t])`` (what ``moe_combine`` makes; all float32).  May be the one term of ``NormedTerms``."""
+
+    y: torch.Tensor
+    wgt: torch.Tensor
+    extra: torch.Tensor | None = None
+    gate: torch.Tensor | None = None
+
+    @property
+    def shape(self):
+        return (self.wgt.shape[0], self.y.shape[1])
+
+    def materialize(self) -> torch.Tensor:
+        out = torch.empty(self.shape, dtype=torch.float32, device=self.y.device)
+        moe_combine(out, self.y, self.wgt, self.extra, extra_gate=self.gate, overwrite=True)
+        return out
 
 
 def normed_sum(terms: list[tuple[torch.Tensor, torch.Tensor, float]], eps: float) -> torch.Tensor:
@@ -1393,23 +1414,38 @@ def stream_step(x: torch.Tensor, *, y: torch.Tensor | NormedTerms | None = None,
     _need(x.dtype == torch.float32 and x.dim() == 2, "stream_step: a float32 stream [T, W]")
     t, w = x.shape
     s1 = s2 = 1.0
-    y1, y2, w1, w2, y_eps = y, None, None, None, 0.0
+    y1, y2, w1, w2, y_eps, experts = y, None, None, None, 0.0, None
     if isinstance(y, NormedTerms):
-        if len(y.terms) > 2 or w % 4 or w > STREAM_STEP_MOST:
+        summed = [isinstance(a, ExpertSum) for a, _, _ in y.terms]
+        if len(y.terms) > 2 or w % 4 or w > STREAM_STEP_MOST or (any(summed) and len(y.terms) > 1):
             y1 = y.materialize()
         else:
             y_eps = y.eps
             y1, w1, s1 = y.terms[0]
+            if summed[0]:
+                experts = y1
+                y1 = experts.y
             if len(y.terms) == 2:
                 y2, w2, s2 = y.terms[1]
-    for v in (y1, y2):
+    for v in (None if experts else y1, y2):
         _need(v is None or (v.dtype == torch.float32 and v.shape == (t, w)), "stream_step: float32 results of the stream's shape")
+    wgt = extra = gate = None
+    if experts:
+        wgt, extra, gate = experts.wgt, experts.extra, experts.gate
+        _dev(wgt, extra)
+        _need(wgt.dtype == torch.float32 and wgt.shape[0] == t and y1.dtype == torch.float32 and y1.shape == (wgt.numel(), w)
+              and (extra is None or (extra.dtype == torch.float32 and extra.shape == (t, w)))
+              and (gate is None or (extra is not None and gate.is_cuda and gate.dtype == torch.float32 and gate.shape == (t, 1))),
+              "stream_step: float32 rows of experts [T * top, W], weights [T, top], an extra row and its gate")
     for v in (w1, w2, norm_weight):
         _need(v is None or v.shape == (w,), "stream_step: weights of the stream's width")
     _need(w2 is None or w2.dtype == w1.dtype, "stream_step: weights of one type")
     _dev(x, y1, y2, w1, w2, norm_weight, rows)
     _i32(rows, "rows")
     n = t if rows is None else rows.numel()
+    if experts and result is not None and (result.stride(0) % 4 or result.data_ptr() % 8):
+        return stream_step(x, y=NormedTerms([(experts.materialize(), w1, s1)], y_eps), mult=mult, read=read, norm_weight=norm_weight,
+                           offset=offset, eps=eps, dtype=dtype, rows=rows, result=result)
     if w % 4 or w > STREAM_STEP_MOST or (result is not None and (result.stride(0) % 4 or result.data_ptr() % 8)):
         one = None if y1 is None else torch.ones((1, 1), dtype=torch.float32, device=x.device)
         if rows is not None and y1 is not None:  # (the kernel for any width writes the stream)
@@ -1426,7 +1462,7 @@ def stream_step(x: torch.Tensor, *, y: torch.Tensor | NormedTerms | None = None,
         ctypes.c_float(s2), ctypes.c_float(y_eps), ctypes.c_float(mult), 1 if read else 0, _ptr(norm_weight),
         F32 if norm_weight is None else dtype_code(norm_weight.dtype), ctypes.c_float(offset), ctypes.c_float(eps),
         _ptr(result) if read else None, result.stride(0) if read else 0, dtype_code(result.dtype) if read else F32, _ptr(rows),
-        n, w, _stream()))
+        n, w, _ptr(wgt), 0 if wgt is None else wgt.shape[1], _ptr(extra), _ptr(gate), 0 if gate is None else gate.stride(0), _stream()))
     return result if read else None
 
 
@@ -1515,7 +1551,7 @@ def decay_chunks(v: torch.Tensor, k: torch.Tensor, q: torch.Tensor, gate: torch.
     """``decay_step`` for segments of any number of tokens that are cut into chunks of up to ``DECAY_CHUNK``
     tokens (``chunks``, ``seg_chunks`` as for ``ssd_scan``): turning, recurrence, norm and gate as float32 products on
     the matrix cores.  ``powers``: ``decay_powers`` of the decays.  Without a ``gate`` the float32
-    results of the recurrence come back as they are."""
+    results of the recurrence come back as they are (``in_silu`` goes with that form alone)."""
     lib = library.core_library()
     _, heads, n_state, p = state.shape
     n = v.shape[0]
@@ -1529,7 +1565,7 @@ def decay_chunks(v: torch.Tensor, k: torch.Tensor, q: torch.Tensor, gate: torch.
     _need(powers.dtype == torch.float32 and powers.shape == (heads, DECAY_CHUNK + 1) and state.dtype == torch.float32,
           "decay_chunks: float32 powers [heads, 65] and states")
     _need(token_slot.numel() == n and (weight is None or weight.numel() == heads * p)
-          and (gate is not None or (out_dtype == torch.float32 and weight is None)), "decay_chunks: arguments")
+          and (not in_silu if gate is not None else (out_dtype == torch.float32 and weight is None)), "decay_chunks: arguments")
     rot = _rotation(cos, sin, positions, n, n_state, "decay_chunks")
     n_chunks, sums, decays = _scan_room(chunks, seg_chunks, seg_q_start, (heads, n_state, p), (heads,), v.device, "decay_chunks")
     out = torch.empty((n, heads * p), dtype=out_dtype, device=v.device)

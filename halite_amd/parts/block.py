@@ -208,7 +208,9 @@ class HyperPreNormBlock(Arrangement):
     def _normed(y, norm):
         if norm is None:
             return y
-        return ops.NormedTerms([(y if y.dtype == torch.float32 else y.float(), norm.multiplier, 1.0)], norm.p.eps)
+        if not isinstance(y, ops.ExpertSum) and y.dtype != torch.float32:
+            y = y.float()
+        return ops.NormedTerms([(y, norm.multiplier, 1.0)], norm.p.eps)
 
     @property
     def stream_copies(self) -> int:
@@ -222,7 +224,10 @@ class HyperPreNormBlock(Arrangement):
         pending = (y, self.mixer_link)
         if self.ff is not None:
             x = self.ff_link.step(h, pending, self.ff_norm)
-            pending = (self._normed(self.ff.forward(x, ctx), self.ff_out_norm), self.ff_link)
+            # (a mixture's weighted sum is made by the pass that norms and writes it)
+            sums = self.ff_out_norm is not None and hasattr(self.ff, "forward_sum")
+            y = self.ff.forward_sum(x, ctx) if sums else self.ff.forward(x, ctx)
+            pending = (self._normed(y, self.ff_out_norm), self.ff_link)
         return pending
 
     def leave(self, h, pending, rows, out=None):

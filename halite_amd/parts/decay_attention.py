@@ -152,11 +152,11 @@ class DecayAttention(Mixer):
         if cut["chunks"] is not None and SCAN_CHUNK <= ops.DECAY_CHUNK and ops.decay_chunks_fit(p.qk_dim, p.v_dim):
             # long segments: chunks as products
             segs = (ctx.seg_q_start, ctx.seg_q_len, ctx.token_slot)
-            if p.norm_per_head:
+            if p.norm_per_head and p.activation is None:
                 gated = ops.decay_chunks(values, keys, queries, gate, self.powers, state, *segs, **cut, **finish, **recur)
             else:
                 y = ops.decay_chunks(values, keys, queries, None, self.powers, state, *segs, **cut, **recur)
-                gated = ops.head_norm_gate(y, gate, self.w_norm, p.eps, 1, x.dtype, silu=silu)
+                gated = ops.head_norm_gate(y, gate, self.w_norm, p.eps, p.n_heads if p.norm_per_head else 1, x.dtype, silu=silu)
             return ops.linear(gated, self.w_out, out_dtype=torch.float32, tiled=self.t_out)
         if turn or p.key_scale != 1.0:
             ops.rotate_heads_(a[:, self.inner : n_act], 2 * p.n_heads, p.qk_dim, n_scaled=p.n_heads, scale=p.key_scale, **turn)

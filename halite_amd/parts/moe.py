@@ -5,8 +5,9 @@ The router's logits are a float32 product; a kernel turns them into the chosen e
 and their weights (by scores with a correction, and among the best groups of experts, where a
 design says so), a second one sorts the (token, choice) pairs by expert on the device,
 and two grouped products run all experts at once on the sorted rows: gate and up with the
-activation in the epilogue, then down.  A last kernel adds the weighted results into the
-float32 stream.  Nothing is read back to the host, so a step's launches depend on its
+activation in the epilogue, then down.  A last kernel adds the weighted results up, into the
+float32 stream or for whoever reads them (an arrangement that norms the result takes the rows and
+adds them up in the kernel that norms, ``forward_sum``).  Nothing is read back to the host, so a step's launches depend on its
 number of tokens alone.
 """
 
@@ -167,9 +168,17 @@ class MixtureOfExperts(FeedForward):
                 self.t_shared_up = ops.tile_weight(self.ws_gate_up[s.intermediate_size :])
 
     def forward(self, x, ctx, add_to=None):
+        s = self.forward_sum(x, ctx)
+        if add_to is not None:
+            ops.moe_combine(add_to, s.y, s.wgt, s.extra, extra_gate=s.gate)
+            return None
+        h = s.materialize()
+        return h if self.p.float32_result else h.to(x.dtype)
+
+    def forward_sum(self, x, ctx) -> ops.ExpertSum:
+        """The result as the rows that its reader adds up."""
         p = self.p
         n, d = x.shape
-        h = add_to if add_to is not None else torch.empty((n, d), dtype=torch.float32, device=x.device)
         z = ops.linear(x, self.w_router, out_dtype=torch.float32)
         shared_gate = z[:, p.n_experts:] if p.shared_gate else None
         z = z[:, : p.n_experts]
@@ -192,6 +201,7 @@ class MixtureOfExperts(FeedForward):
                              group_offsets=offsets, tile_offsets=tiles, row_src=order, src_div=p.top_k)
         y = torch.empty((pairs, d), dtype=torch.float32, device=x.device)
         ops.grouped_gemm(act, self.w_down, y, n_rows=pairs, group_offsets=offsets, tile_offsets=tiles, row_dst=order)
+        extra = None
         if p.shared is not None:
             fs = p.shared.intermediate_size
             if self.t_shared_gate is not None and x.dtype == torch.bfloat16 and n <= ops.SKINNY_ROWS:
@@ -209,8 +219,4 @@ class MixtureOfExperts(FeedForward):
                                             p.shared.up_shift)
             # the shared expert's result rides along with the weighted sum
             extra = ops.linear(acts, self.ws_down, out_dtype=torch.float32, tiled=self.t_shared_down)
-        ops.moe_combine(h, y, wgt, extra if p.shared is not None else None, extra_gate=shared_gate,
-                        overwrite=add_to is None)
-        if add_to is not None:
-            return None
-        return h if p.float32_result else h.to(x.dtype)
+        return ops.ExpertSum(y, wgt, extra, shared_gate)

@@ -338,6 +338,30 @@ def test_a_normed_result_written_and_the_next_row_read(gpu, width):
     close(got, P.model_norm(want, w2.to(F), 1e-5), 2e-6)
 
 
+@pytest.mark.parametrize("width", [64, 42, 1032])
+@pytest.mark.parametrize("shared", [False, True])
+def test_the_experts_sum_in_the_pass_that_norms_it(gpu, width, shared):
+    """The weighted sum of a token's experts (and the gated shared one) made by the stream's step, of all
+    rows and of chosen ones."""
+    t, top = 9, 3
+    x, rows, wgt = rand(t, width, seed=1), rand(t * top, width, seed=2, scale=3.0), rand(t, top, seed=3).abs()
+    extra, gates, w1, w2 = rand(t, width, seed=4), rand(t, 5, seed=5), 0.3 * rand(width, seed=6), 0.3 * rand(width, seed=7)
+    y = (wgt.to(F)[:, :, None] * rows.to(F).view(t, top, width)).sum(1)
+    if shared:
+        y = y + torch.sigmoid(gates[:, 4:].to(F)) * extra.to(F)
+    want = x.to(F) + P.model_norm(y, w1.to(F), 1e-5)
+    term = ops.ExpertSum(rows.to(gpu), wgt.to(gpu), extra.to(gpu) if shared else None, gates.to(gpu)[:, 4:] if shared else None)
+    close(term.materialize(), y, 1e-6)
+    how = dict(read=True, norm_weight=w2.to(gpu), offset=1.0, eps=1e-5, dtype=torch.float32)
+    terms = ops.NormedTerms([(term, (1.0 + w1).to(gpu), 1.0)], 1e-5)
+    some = [4, 0, 7]
+    chosen = ops.stream_step(x.to(gpu), y=terms, rows=i32(some, gpu), **how)
+    close(chosen, P.model_norm(want, w2.to(F), 1e-5)[some], 2e-6)
+    xg = x.to(gpu)
+    close(ops.stream_step(xg, y=terms, **how), P.model_norm(want, w2.to(F), 1e-5), 2e-6)
+    close(xg, want, 1e-6)
+
+
 # -- every mechanism alone ----------------------------------------------------------------------
 
 SMALL_LAYERS = {
