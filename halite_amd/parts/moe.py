@@ -7,8 +7,8 @@ design says so), a second one sorts the (token, choice) pairs by expert on the d
 and two grouped products run all experts at once on the sorted rows: gate and up with the
 activation in the epilogue, then down.  A last kernel adds the weighted results up, into the
 float32 stream or for whoever reads them (an arrangement that norms the result takes the rows and
-adds them up in the kernel that norms, ``forward_sum``).  Nothing is read back to the host, so a step's launches depend on its
-number of tokens alone.
+adds them up in the kernel that norms, ``forward_sum``).  Nothing is read back to the host, so a
+step's launches depend on its number of tokens alone.
 """
 
 from __future__ import annotations
